@@ -13,7 +13,7 @@ cp $ROOT/trackiellm_amd/csrc/common/*.h $OUT/src/common/
 cp $ROOT/trackiellm_amd/csrc/llm/tk_llm_kernels.hip $OUT/src/llm/tk_llm_kernels.hip
 (cd $OUT/src && patch -s -p0 llm/tk_llm_kernels.hip < $ROOT/tools/diag/g32_diagnostics.patch)
 cd $ROOT/trackiellm_amd/csrc
-/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-slp-vectorize -fvisibility=hidden -I$ROOT/include -I$OUT/src/llm -I. -Wall -Wno-unused-function "$@" -c $OUT/src/llm/tk_llm_kernels.hip -o $OUT/k_$NAME.o
+/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-slp-vectorize -Xclang -target-feature -Xclang -packed-fp32-ops -fvisibility=hidden -I$ROOT/include -I$OUT/src/llm -I. -Wall -Wno-unused-function "$@" -c $OUT/src/llm/tk_llm_kernels.hip -o $OUT/k_$NAME.o
 OBJS=$(find $ROOT/build/obj -name '*.o' | grep -v 'llm/tk_llm_kernels.hip.o')
 /opt/rocm/bin/hipcc --offload-arch=gfx950 -shared -fPIC -o $OUT/libtrackie_$NAME.so $OBJS $OUT/k_$NAME.o -lpthread
 echo built $OUT/libtrackie_$NAME.so

@@ -1,10 +1,9 @@
 #!/bin/bash
 # Collects everything under profiles/rNN_* in one GPU call (run through gpurun from the repo root):
 #   1. PMC traffic (FETCH_SIZE, WRITE_SIZE: separate passes) of the W4A8 launch set at 256 and 16 rows and of k_attention at 256 rows x 128 positions
-#   2. kernel traces of the roofline-only run and of the fused default run — of the GRAPH path (the shipped one): rocprofv3's queue
-#      interceptor walks a multi-packet submission linearly and runs off the end of the 16384-packet AQL ring when a hipGraphLaunch
-#      batch straddles it (profiles/r03_rocprofv3_hipgraph_crash_symbolised.txt), so the ring is made large enough never to wrap inside a
-#      profiled run (ROC_AQL_QUEUE_SIZE)
+#   2. kernel traces of the roofline-only run and of the fused default run — of the GRAPH path (the shipped one): under
+#      rocprofv3 a hipGraphLaunch aborts when its batch of packets reaches the end of the AQL ring, so the ring is made large enough never to
+#      wrap inside a profiled run (ROC_AQL_QUEUE_SIZE)
 #   3. the default bench.py line (unprofiled)
 # Everything lands under gpurun_out/; copy what should be judged into profiles/.
 set -o pipefail
@@ -17,9 +16,8 @@ one_csv() { # exactly one counter file per pass, or stop: a stale directory must
   find "$1" -name '*counter_collection.csv'
 }
 # PMC passes run the GRAPH path too (the shipped one): a counter pass yields one dispatch record per kernel node of a replayed graph.
-# ROC_AQL_QUEUE_SIZE: rocprofv3's queue interceptor walks a multi-packet submission linearly and runs off the end of the AQL ring when a
-# hipGraphLaunch batch straddles it (profiles/r03_rocprofv3_hipgraph_crash_symbolised.txt); the ring must therefore never wrap inside a
-# profiled process.  PACKET BUDGET: every profiled command below must submit fewer packets per queue than the ring holds — kernels + a
+# ROC_AQL_QUEUE_SIZE: under rocprofv3 a hipGraphLaunch aborts when its batch of packets reaches the end of the AQL ring; the ring must
+# therefore never wrap inside a profiled process.  PACKET BUDGET: every profiled command below must submit fewer packets per queue than the ring holds — kernels + a
 # barrier packet per graph launch; bench.py --steps 1 --warmup 1 at 3 x 256 is the largest here: 359 k dispatches over its streams' queues
 # (measured, round 4; three LLM groups x (64 prefill passes + 128 decode steps) x ~260 kernels, twice, + perception).  More steps, warm-up or decode length need a larger ring FIRST, or the abort of round 2 comes back.
 export ROC_AQL_QUEUE_SIZE=524288

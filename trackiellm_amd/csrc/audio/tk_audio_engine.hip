@@ -7,13 +7,8 @@
 #include "../nn/tk_gemm_tiled.h"
 #include "../nn/tk_nn_kernels.h"
 
-/* Perception streams run at the highest stream priority: their kernels are small and many, and behind the LLM's large GEMM
- * launches they would otherwise queue for a free CU at every step (the fused cycle's critical path becomes queueing, not work). */
-static inline hipError_t tk_create_perception_stream(hipStream_t* s) {
-    int lo = 0, hi = 0; /* numerically lower = higher priority */
-    if (hipDeviceGetStreamPriorityRange(&lo, &hi) != hipSuccess) return hipStreamCreateWithFlags(s, hipStreamNonBlocking);
-    return hipStreamCreateWithPriority(s, hipStreamNonBlocking, hi);
-}
+/* Every stream of the library keeps the default priority: work on streams of different priorities has been seen to hang. */
+static inline hipError_t tk_create_perception_stream(hipStream_t* s) { return hipStreamCreateWithFlags(s, hipStreamNonBlocking); }
 
 #define HIPQ(expr)                                                                              \
     do {                                                                                        \

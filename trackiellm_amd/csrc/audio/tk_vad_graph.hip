@@ -31,9 +31,7 @@ bool TkVadGraph::check_supported(const TkOnnxGraph& g, std::string* err) {
 bool TkVadGraph::load(const char* path, int device, int window, int sample_rate) {
     device_ = device; window_ = window; sample_rate_ = sample_rate;
     VQ(hipSetDevice(device_));
-    int lo = 0, hi = 0;
-    if (hipDeviceGetStreamPriorityRange(&lo, &hi) == hipSuccess) VQ(hipStreamCreateWithPriority(&stream_, hipStreamNonBlocking, hi));
-    else VQ(hipStreamCreateWithFlags(&stream_, hipStreamNonBlocking));
+    VQ(hipStreamCreateWithFlags(&stream_, hipStreamNonBlocking));
     /* 16 MiB of activations: far more than a 30 ms window needs in any graph of this class */
     if (!exec_.load(path, device_, stream_, (size_t)1 << 22)) { error = exec_.error; return false; }
     const TkOnnxGraph& g = exec_.graph();
