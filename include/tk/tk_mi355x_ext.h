@@ -65,6 +65,19 @@ TK_API void tk_mi355x_llm_model_get_hparams(const tk_mi355x_llm_model_t* m, tk_m
 TK_API uint64_t tk_mi355x_llm_model_weight_bytes(const tk_mi355x_llm_model_t* m);
 TK_API void tk_mi355x_llm_model_destroy(tk_mi355x_llm_model_t** m);
 
+/* ---- decoders described layer by layer (csrc/llm/tk_layered.h): a folder with config.json — "architecture" names the design, registered in
+ * csrc/llm/tk_layer_spec.cpp (Vuvulorn) — and model.safetensors.  tk_model_loader_load_model takes such a folder as its path (with
+ * "?dtype=float32" behind it for 32-bit); sessions, runners, the scheduler, sampling and the decode loop are the ones of every other model.
+ *   load_dir: dtype "bfloat16" (NULL / "": the default; matrix products in bf16 with 32-bit accumulation, norms, scores, routers, the residual
+ *     stream and recurrent state in 32-bit) or "float32" (everything in 32-bit);
+ *   create_layered: random weights of the described shape, made on the device; gate_rank = inner size of the low-rank gates, which only the
+ *     tensors of a checkpoint give;
+ *   config_check: TK_SUCCESS when this build serves the configuration, TK_ERROR_CONFIG_PARSE_FAILED with the reason otherwise (no GPU). ---- */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_model_load_dir(tk_mi355x_llm_model_t** out, const char* dir, const char* dtype, int device);
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_model_create_layered(tk_mi355x_llm_model_t** out, const char* config_json, const char* dtype, int device,
+                                                                       uint64_t seed, int gate_rank);
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_config_check(const char* config_json);
+
 /* continuous batching behind tk_llm_runner_* (csrc/llm/tk_llm_batcher.h): the runners created on one model handle (what
  * tk_model_loader_load_model returns) share decode sessions of `slots` sequences; their prepare_generation / generate_next_token rows
  * are coalesced into passes by one scheduler thread per session.  Set before the first tk_llm_runner_create on the model (default:
@@ -87,12 +100,27 @@ TK_API uint64_t tk_mi355x_llm_model_run_ahead_wasted(void* model_handle);
 /* sessions --------------------------------------------------------------------------------- */
 TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_session_create(tk_mi355x_llm_session_t** out, tk_mi355x_llm_model_t* m, int max_seq,
                                                                  int max_ctx);
+/* the same with a cache for `pool_tokens` positions over all live sequences together (rounded up to pages; 0: max_seq x max_ctx).  Models whose
+ * cache is not paged allocate max_seq x max_ctx all the same. */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_session_create_pool(tk_mi355x_llm_session_t** out, tk_mi355x_llm_model_t* m, int max_seq, int max_ctx, int pool_tokens);
+/* gives back what sequence `seq` holds in the cache; it may start again at position 0 */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_session_release(tk_mi355x_llm_session_t* s, int seq);
+TK_API void tk_mi355x_llm_session_cache_usage(tk_mi355x_llm_session_t* s, int32_t* pages_used, int32_t* pages_total); /* (0, 0): not paged */
+TK_API int tk_mi355x_llm_session_row_capacity(tk_mi355x_llm_session_t* s); /* rows one pass holds; layer-list models split longer forward() calls themselves */
 TK_API void tk_mi355x_llm_session_destroy(tk_mi355x_llm_session_t** s);
 /* rows one pass can hold (16-row MFMA M-tiles x 8): the row capacity of forward(), the column count of decode()'s out_tokens */
 TK_API int tk_mi355x_llm_max_rows(void);
 /* one pass over nrows <= tk_mi355x_llm_max_rows() (sequence, position, token) rows; logits [nrows][vocab] and argmax [nrows] optional */
 TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_forward(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos,
                                                           const int32_t* tok, float* logits, int32_t* argmax);
+/* the same for n_out wanted rows (ascending; 0: none, the rows only extend their sequences): logits [n_out][vocab] and ids [n_out], both optional.
+ * Layer-list models: the rows of a sequence are one run of consecutive positions that continues where the sequence stands, starts at 0, or
+ * replaces the sequence's last pass. */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_forward_rows(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok,
+                                                               int n_out, const int32_t* out_rows, float* logits, int32_t* ids);
+/* a pass that also returns the residual stream after every layer, [layers][nrows][width] (layer-list models) */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_forward_streams(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok,
+                                                                  float* streams);
 /* one pipeline stage of a pass (the LLM layer-sharded over GPUs): layers [layer0, layer1) of this rank's model.  The
  * first stage starts from tok (x_in NULL), later stages from the residual stream x_in [nrows][d_model] fp32; every stage but the last
  * writes the stream to x_out; the last (head != 0, layer1 == n_layer) samples into argmax[nrows].  x_on_host != 0: x_in / x_out are
@@ -116,6 +144,10 @@ typedef struct {
     uint32_t reserved;
 } tk_mi355x_sampling_t;
 struct tk_llm_runner_s;
+/* prompts and continuations as token ids, for models without a vocabulary: prepare_ids = tk_llm_runner_prepare_generation on ids (no BOS is
+ * added); pending_id = the id that the next tk_llm_runner_generate_next_token returns the text of (-1: none) */
+TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_runner_prepare_ids(struct tk_llm_runner_s* runner, const int32_t* ids, int n);
+TK_API int32_t tk_mi355x_llm_runner_pending_id(struct tk_llm_runner_s* runner);
 TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_runner_set_sampling(struct tk_llm_runner_s* runner, float temperature, int32_t top_k, float top_p, float min_p);
 /* tk_mi355x_llm_forward with a sampling state per row (temperature <= 0: that row takes the arg max); ids [nrows] */
 TK_API TK_NODISCARD tk_error_code_t tk_mi355x_llm_forward_sampled(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos,

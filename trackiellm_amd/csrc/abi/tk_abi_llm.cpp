@@ -23,6 +23,7 @@
 #include <vector>
 
 #include "../llm/tk_gguf.h"
+#include "../llm/tk_layered.h"
 #include "../llm/tk_grammar.h"
 #include "../llm/tk_llm_batcher.h"
 #include "../llm/tk_llm_engine.h"
@@ -34,7 +35,10 @@
 #include "tk/tk_model_runner.h"
 
 struct tk_mi355x_llm_model_s {
-    TkLlmModel model;
+    TkLlmModel model; /* GGUF / synthetic Mistral-class checkpoints; unused when `layered` is set */
+    std::unique_ptr<TkLayeredModel> layered;
+    TkDecoderModel* decoder() { return layered ? (TkDecoderModel*)layered.get() : &model; }
+    const TkDecoderModel* decoder() const { return layered ? (const TkDecoderModel*)layered.get() : &model; }
     TkTokenizer tok;
     int context_length = 4096;
     std::string path;
@@ -48,12 +52,18 @@ struct tk_mi355x_llm_model_s {
 };
 
 struct tk_mi355x_llm_session_s {
-    TkLlmSession session;
+    std::unique_ptr<TkDecodeSession> session;
+    TkLlmSession* llm = nullptr;         /* the session as the class the model made, or null */
+    TkLayeredSession* layered = nullptr;
 };
 
 static tk_error_code_t fail(tk_error_code_t code, const std::string& why) {
     tk_error_set_detail("%s", why.c_str());
     return code;
+}
+
+static tk_error_code_t not_this_model(const char* what) {
+    return fail(TK_ERROR_NOT_IMPLEMENTED, std::string(what) + " exists for GGUF-class models only");
 }
 
 static TkLlmHParams to_hp(const tk_mi355x_llm_hparams_t& h) {
@@ -105,18 +115,21 @@ tk_error_code_t tk_mi355x_llm_model_create(tk_mi355x_llm_model_t** out, const tk
 
 tk_error_code_t tk_mi355x_llm_model_fill_synthetic(tk_mi355x_llm_model_t* m, uint64_t seed) {
     if (!m) return TK_ERROR_INVALID_ARGUMENT;
+    if (m->layered) return not_this_model("fill_synthetic");
     if (!m->model.fill_synthetic(seed)) return fail(TK_ERROR_GPU_ROCM_ERROR, m->model.error);
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_model_fill_synthetic_f16(tk_mi355x_llm_model_t* m, uint64_t seed) {
     if (!m) return TK_ERROR_INVALID_ARGUMENT;
+    if (m->layered) return not_this_model("fill_synthetic");
     if (!m->model.fill_synthetic(seed, true)) return fail(TK_ERROR_GPU_ROCM_ERROR, m->model.error);
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_model_set_lora(tk_mi355x_llm_model_t* m, const char* adapter_path) {
     if (!m) return TK_ERROR_INVALID_ARGUMENT;
+    if (m->layered && adapter_path && *adapter_path) return not_this_model("a LoRA adapter");
     if (!adapter_path || !*adapter_path) { m->model.lora = nullptr; m->lora.reset(); return TK_SUCCESS; }
     std::unique_ptr<TkLoraAdapter> ad(new TkLoraAdapter());
     if (!ad->load(adapter_path)) return fail(TK_ERROR_MODEL_LOAD_FAILED, "LoRA adapter: " + ad->error);
@@ -146,22 +159,26 @@ tk_error_code_t tk_mi355x_lora_probe(const char* path, int32_t* rank, float* alp
 
 tk_error_code_t tk_mi355x_llm_model_set_tensor(tk_mi355x_llm_model_t* m, int layer, int which, int type, const void* data, size_t nbytes) {
     if (!m || !data) return TK_ERROR_INVALID_ARGUMENT;
+    if (m->layered) return not_this_model("set_tensor");
     if (!m->model.set_tensor(layer, which, type, data, nbytes)) return fail(TK_ERROR_INVALID_INPUT_TENSOR, m->model.error);
     return TK_SUCCESS;
 }
 
 void tk_mi355x_llm_model_get_hparams(const tk_mi355x_llm_model_t* m, tk_mi355x_llm_hparams_t* out) {
     if (!m || !out) return;
+    if (m->layered) { /* the fields every decoder has; the rest differ layer by layer */
+        const TkLayeredConfig& c = m->layered->cfg;
+        *out = tk_mi355x_llm_hparams_t{};
+        out->n_layer = (int32_t)c.layers.size(); out->d_model = c.width; out->vocab = c.vocab; out->rms_eps = c.eps;
+        return;
+    }
     const TkLlmHParams& h = m->model.hp;
     *out = tk_mi355x_llm_hparams_t{h.n_layer, h.d_model, h.n_head, h.n_kv_head, h.head_dim, h.d_ff, h.vocab, h.rms_eps, h.rope_theta,
                                    h.ks_qkv, h.ks_o, h.ks_gateup, h.ks_down, h.ks_out};
 }
 
 uint64_t tk_mi355x_llm_model_weight_bytes(const tk_mi355x_llm_model_t* m) {
-    if (!m) return 0;
-    uint64_t b = m->model.output.bytes;
-    for (const auto& L : m->model.layers) b += L.q.bytes + L.k.bytes + L.v.bytes + L.o.bytes + L.gate.bytes + L.up.bytes + L.down.bytes;
-    return b;
+    return m ? m->decoder()->step_weight_bytes() : 0;
 }
 
 /* Weights are immutable and 4.3 GB: a model file resident on a device is shared by every loader of the process (the reference caches
@@ -274,13 +291,94 @@ tk_error_code_t tk_mi355x_llm_model_load_gguf_lora(tk_mi355x_llm_model_t** out, 
     return TK_SUCCESS;
 }
 
+/* ---- decoders described layer by layer (csrc/llm/tk_layered.h) ---- */
+
+static bool have_device(int device, tk_error_code_t* rc) {
+    int ndev = 0;
+    if (hipGetDeviceCount(&ndev) != hipSuccess || ndev <= 0) { *rc = fail(TK_ERROR_GPU_DEVICE_NOT_FOUND, "no HIP device visible (the MI355X path has no CPU fallback)"); return false; }
+    if (device < 0 || device >= ndev) { *rc = fail(TK_ERROR_INVALID_ARGUMENT, "device ordinal out of range"); return false; }
+    return true;
+}
+
+tk_error_code_t tk_mi355x_llm_config_check(const char* config_json) {
+    if (!config_json) return TK_ERROR_INVALID_ARGUMENT;
+    TkLayeredConfig c;
+    std::string err;
+    if (!tk_layered_parse(config_json, &c, &err)) return fail(TK_ERROR_CONFIG_PARSE_FAILED, err);
+    return TK_SUCCESS;
+}
+
+tk_error_code_t tk_mi355x_llm_model_load_dir(tk_mi355x_llm_model_t** out, const char* dir, const char* dtype, int device) {
+    if (!out || !dir) return TK_ERROR_INVALID_ARGUMENT;
+    tk_error_code_t rc;
+    if (access((std::string(dir) + "/config.json").c_str(), R_OK) != 0) return fail(TK_ERROR_FILE_NOT_FOUND, std::string("no config.json in ") + dir);
+    if (!have_device(device, &rc)) return rc;
+    std::unique_ptr<tk_mi355x_llm_model_s> m(new tk_mi355x_llm_model_s());
+    m->layered.reset(new TkLayeredModel());
+    if (!m->layered->load(dir, dtype && *dtype ? dtype : "bfloat16", device)) return fail(TK_ERROR_MODEL_LOAD_FAILED, m->layered->error);
+    m->tok.init_bytes(m->layered->cfg.vocab);
+    m->path = dir;
+    *out = m.release();
+    return TK_SUCCESS;
+}
+
+tk_error_code_t tk_mi355x_llm_model_create_layered(tk_mi355x_llm_model_t** out, const char* config_json, const char* dtype, int device, uint64_t seed, int gate_rank) {
+    if (!out || !config_json) return TK_ERROR_INVALID_ARGUMENT;
+    tk_error_code_t rc;
+    if (!have_device(device, &rc)) return rc;
+    std::unique_ptr<tk_mi355x_llm_model_s> m(new tk_mi355x_llm_model_s());
+    m->layered.reset(new TkLayeredModel());
+    if (!m->layered->fill_synthetic(config_json, dtype && *dtype ? dtype : "bfloat16", device, seed, gate_rank)) return fail(TK_ERROR_MODEL_LOAD_FAILED, m->layered->error);
+    m->tok.init_bytes(m->layered->cfg.vocab);
+    *out = m.release();
+    return TK_SUCCESS;
+}
+
 tk_error_code_t tk_mi355x_llm_session_create(tk_mi355x_llm_session_t** out, tk_mi355x_llm_model_t* m, int max_seq, int max_ctx) {
-    if (!out || !m) return TK_ERROR_INVALID_ARGUMENT;
+    return tk_mi355x_llm_session_create_pool(out, m, max_seq, max_ctx, 0);
+}
+
+tk_error_code_t tk_mi355x_llm_session_create_pool(tk_mi355x_llm_session_t** out, tk_mi355x_llm_model_t* m, int max_seq, int max_ctx, int pool_tokens) {
+    if (!out || !m || pool_tokens < 0) return TK_ERROR_INVALID_ARGUMENT;
     std::unique_ptr<tk_mi355x_llm_session_s> s(new tk_mi355x_llm_session_s());
-    if (!s->session.init(&m->model, max_seq, max_ctx)) return fail(TK_ERROR_GPU_MEMORY, s->session.error);
+    std::string err;
+    s->session = m->decoder()->open_session(max_seq, max_ctx, pool_tokens, &err);
+    if (!s->session) return fail(TK_ERROR_GPU_MEMORY, err);
+    if (m->layered) s->layered = (TkLayeredSession*)s->session.get();
+    else s->llm = (TkLlmSession*)s->session.get();
     *out = s.release();
     return TK_SUCCESS;
 }
+
+tk_error_code_t tk_mi355x_llm_forward_rows(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, int n_out,
+                                           const int32_t* out_rows, float* logits, int32_t* ids) {
+    if (!s || !seq || !pos || !tok || n_out < 0 || (n_out > 0 && !out_rows)) return TK_ERROR_INVALID_ARGUMENT;
+    static const int32_t none = 0;
+    if (!s->session->forward(nrows, seq, pos, tok, logits, ids, n_out > 0, nullptr, nullptr, n_out, n_out > 0 ? out_rows : &none)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
+    return TK_SUCCESS;
+}
+
+tk_error_code_t tk_mi355x_llm_forward_streams(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, float* streams) {
+    if (!s || !seq || !pos || !tok || !streams) return TK_ERROR_INVALID_ARGUMENT;
+    if (!s->layered) return fail(TK_ERROR_NOT_IMPLEMENTED, "the streams of a pass are available for layer-list models only");
+    if (!s->layered->forward_streams(nrows, seq, pos, tok, streams)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
+    return TK_SUCCESS;
+}
+
+tk_error_code_t tk_mi355x_llm_session_release(tk_mi355x_llm_session_t* s, int seq) {
+    if (!s) return TK_ERROR_INVALID_ARGUMENT;
+    s->session->release_sequence(seq);
+    return TK_SUCCESS;
+}
+
+void tk_mi355x_llm_session_cache_usage(tk_mi355x_llm_session_t* s, int32_t* pages_used, int32_t* pages_total) {
+    int u = 0, t = 0;
+    if (s) s->session->cache_usage(&u, &t);
+    if (pages_used) *pages_used = u;
+    if (pages_total) *pages_total = t;
+}
+
+int tk_mi355x_llm_session_row_capacity(tk_mi355x_llm_session_t* s) { return s ? s->session->row_capacity() : 0; }
 
 void tk_mi355x_llm_session_destroy(tk_mi355x_llm_session_t** s) {
     if (!s || !*s) return;
@@ -291,7 +389,7 @@ void tk_mi355x_llm_session_destroy(tk_mi355x_llm_session_t** s) {
 tk_error_code_t tk_mi355x_llm_forward(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok,
                                       float* logits, int32_t* argmax) {
     if (!s || !seq || !pos || !tok) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.forward(nrows, seq, pos, tok, logits, argmax, true)) return fail(TK_ERROR_INFERENCE_FAILED, s->session.error);
+    if (!s->session->forward(nrows, seq, pos, tok, logits, argmax, true)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
     return TK_SUCCESS;
 }
 
@@ -306,25 +404,27 @@ tk_error_code_t tk_mi355x_llm_forward_sampled(tk_mi355x_llm_session_t* s, int nr
             return fail(TK_ERROR_INVALID_ARGUMENT, "sampling parameters of row " + std::to_string(r) + " are out of range (temperature >= 0, 0 <= top_k <= 64, 0 < top_p <= 1, 0 <= min_p <= 1)");
         rows[r].temp = p.temperature; rows[r].top_p = p.top_p; rows[r].min_p = p.min_p; rows[r].top_k = p.top_k; rows[r].seed = p.seed; rows[r].counter = p.counter;
     }
-    if (!s->session.forward(nrows, seq, pos, tok, logits, ids, true, nullptr, rows)) return fail(TK_ERROR_INFERENCE_FAILED, s->session.error);
+    if (!s->session->forward(nrows, seq, pos, tok, logits, ids, true, nullptr, rows)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_session_kv_write(tk_mi355x_llm_session_t* s, int layer, int seq, int pos0, int n_pos, const uint16_t* k, const uint16_t* v) {
     if (!s || !k || !v) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.kv_write(layer, seq, pos0, n_pos, k, v)) return fail(TK_ERROR_INVALID_ARGUMENT, s->session.error);
+    if (!s->llm) return not_this_model("kv_write");
+    if (!s->llm->kv_write(layer, seq, pos0, n_pos, k, v)) return fail(TK_ERROR_INVALID_ARGUMENT, s->session->error);
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_session_kv_read(tk_mi355x_llm_session_t* s, int layer, int seq, int pos0, int n_pos, uint16_t* k, uint16_t* v) {
     if (!s || !k || !v) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.kv_read(layer, seq, pos0, n_pos, k, v)) return fail(TK_ERROR_INVALID_ARGUMENT, s->session.error);
+    if (!s->llm) return not_this_model("kv_read");
+    if (!s->llm->kv_read(layer, seq, pos0, n_pos, k, v)) return fail(TK_ERROR_INVALID_ARGUMENT, s->session->error);
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_prefill(tk_mi355x_llm_session_t* s, int nseq, int n_prompt, const int32_t* tokens, int32_t* first_tokens) {
     if (!s || !tokens) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.prefill(nseq, n_prompt, tokens, first_tokens)) return fail(TK_ERROR_INFERENCE_FAILED, s->session.error);
+    if (!s->session->prefill(nseq, n_prompt, tokens, first_tokens)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
     return TK_SUCCESS;
 }
 
@@ -333,8 +433,9 @@ int tk_mi355x_llm_max_rows(void) { return TK_MAX_ROWS; }
 tk_error_code_t tk_mi355x_llm_forward_stage(tk_mi355x_llm_session_t* s, int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok,
                                             const float* x_in, float* x_out, int x_on_host, int layer0, int layer1, int head, int32_t* argmax) {
     if (!s || !seq || !pos) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.forward_stage(nrows, seq, pos, tok, x_in, x_out, x_on_host != 0, layer0, layer1, head != 0, argmax))
-        return fail(TK_ERROR_INFERENCE_FAILED, s->session.error);
+    if (!s->llm) return not_this_model("a pipeline stage");
+    if (!s->llm->forward_stage(nrows, seq, pos, tok, x_in, x_out, x_on_host != 0, layer0, layer1, head != 0, argmax))
+        return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
     return TK_SUCCESS;
 }
 
@@ -345,8 +446,9 @@ static_assert(sizeof(tk_mi355x_pipe_handle_t) == sizeof(TkPipeHandle), "public a
 tk_error_code_t tk_mi355x_pipe_create(tk_mi355x_pipe_t** out, tk_mi355x_llm_session_t* s, int stage, int n_stages, int layer0, int layer1, int payload_f16,
                                       tk_mi355x_pipe_handle_t* my_handle) {
     if (!out || !s) return TK_ERROR_INVALID_ARGUMENT;
+    if (!s->llm) return not_this_model("a pipeline");
     std::unique_ptr<tk_mi355x_pipe_s> p(new tk_mi355x_pipe_s());
-    if (!p->pipe.init(&s->session, stage, n_stages, layer0, layer1, payload_f16 != 0, (TkPipeHandle*)my_handle)) return fail(TK_ERROR_INVALID_ARGUMENT, p->pipe.error);
+    if (!p->pipe.init(s->llm, stage, n_stages, layer0, layer1, payload_f16 != 0, (TkPipeHandle*)my_handle)) return fail(TK_ERROR_INVALID_ARGUMENT, p->pipe.error);
     *out = p.release();
     return TK_SUCCESS;
 }
@@ -402,15 +504,16 @@ tk_error_code_t tk_mi355x_pipe_sync(tk_mi355x_pipe_t* p, int32_t* out_tokens, in
 
 tk_error_code_t tk_mi355x_llm_decode(tk_mi355x_llm_session_t* s, int nrows, int n_steps, int32_t* out_tokens, float* ms_per_step) {
     if (!s) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.decode(nrows, n_steps, out_tokens)) return fail(TK_ERROR_INFERENCE_FAILED, s->session.error);
-    if (ms_per_step) *ms_per_step = s->session.last_step_ms;
+    if (!s->session->decode(nrows, n_steps, out_tokens)) return fail(TK_ERROR_INFERENCE_FAILED, s->session->error);
+    if (ms_per_step) *ms_per_step = s->session->last_step_ms;
     return TK_SUCCESS;
 }
 
 tk_error_code_t tk_mi355x_llm_time_gemv(tk_mi355x_llm_session_t* s, int layer, int which, int nrows, int iters, float* avg_ms,
                                         double* algorithmic_bytes) {
     if (!s || !avg_ms || !algorithmic_bytes || iters <= 0) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.time_gemv(layer, which, nrows, iters, avg_ms, algorithmic_bytes)) return fail(TK_ERROR_GPU_ROCM_ERROR, s->session.error);
+    if (!s->llm) return not_this_model("time_gemv");
+    if (!s->llm->time_gemv(layer, which, nrows, iters, avg_ms, algorithmic_bytes)) return fail(TK_ERROR_GPU_ROCM_ERROR, s->session->error);
     return TK_SUCCESS;
 }
 
@@ -444,7 +547,8 @@ tk_error_code_t tk_mi355x_attention_plan_at(int device, int nrows, int n_head, i
 
 tk_error_code_t tk_mi355x_llm_time_attention(tk_mi355x_llm_session_t* s, int nrows, int ctx, int iters, float* avg_ms, double* kv_bytes) {
     if (!s || !avg_ms || !kv_bytes) return TK_ERROR_INVALID_ARGUMENT;
-    if (!s->session.time_attention(nrows, ctx, iters, avg_ms, kv_bytes)) return fail(TK_ERROR_GPU_ROCM_ERROR, s->session.error);
+    if (!s->llm) return not_this_model("time_attention");
+    if (!s->llm->time_attention(nrows, ctx, iters, avg_ms, kv_bytes)) return fail(TK_ERROR_GPU_ROCM_ERROR, s->session->error);
     return TK_SUCCESS;
 }
 
@@ -570,6 +674,14 @@ static bool parse_synthetic(const std::string& p, std::string* name, uint64_t* s
     return true;
 }
 
+/* a folder with config.json, optionally followed by ?dtype=bfloat16 | float32 */
+static bool is_model_dir(const std::string& p, std::string* dir, std::string* dtype) {
+    const size_t q = p.rfind("?dtype=");
+    *dir = q == std::string::npos ? p : p.substr(0, q);
+    *dtype = q == std::string::npos ? "bfloat16" : p.substr(q + 7);
+    return access((*dir + "/config.json").c_str(), R_OK) == 0;
+}
+
 tk_error_code_t tk_model_loader_load_model(tk_model_loader_t* loader, const tk_model_load_params_t* params, void** out_model_handle) {
     if (!loader || !params || !out_model_handle || !params->model_path || !params->model_path->path_str) return TK_ERROR_INVALID_ARGUMENT;
     if (params->model_type == TK_MODEL_FORMAT_ONNX) return fail(TK_ERROR_NOT_IMPLEMENTED, "ONNX graphs are not interpreted: the detector/ASR/VAD streams have dedicated entry points");
@@ -582,7 +694,7 @@ tk_error_code_t tk_model_loader_load_model(tk_model_loader_t* loader, const tk_m
     const int device = tk_mi355x_get_default_device();
     if (!params->force_reload)
         for (auto* m : g_models)
-            if (m->path == path && m->model.device == device) {
+            if (m->path == path && m->decoder()->device == device) {
                 bool mine = false;
                 for (auto* h : loader->held) mine = mine || h == m;
                 if (!mine && distinct_held(loader) >= loader->max_models) return fail(TK_ERROR_OUT_OF_MEMORY, "model cache full (max_models)");
@@ -593,7 +705,7 @@ tk_error_code_t tk_model_loader_load_model(tk_model_loader_t* loader, const tk_m
             }
     if (distinct_held(loader) >= loader->max_models) return fail(TK_ERROR_OUT_OF_MEMORY, "model cache full (max_models)");
     tk_mi355x_llm_model_t* m = nullptr;
-    std::string name;
+    std::string name, dtype;
     uint64_t seed;
     tk_error_code_t rc;
     if (parse_synthetic(file, &name, &seed)) {
@@ -608,6 +720,11 @@ tk_error_code_t tk_model_loader_load_model(tk_model_loader_t* loader, const tk_m
         if (rc == TK_SUCCESS) rc = f16 ? tk_mi355x_llm_model_fill_synthetic_f16(m, seed) : tk_mi355x_llm_model_fill_synthetic(m, seed);
         if (rc != TK_SUCCESS) { if (m) release_model(m); return rc; } /* g_models_mu is held here */
         if (m->lora) { m->model.lora = nullptr; m->lora->drop_factors(); }
+        m->path = path;
+    } else if (is_model_dir(file, &name, &dtype)) {
+        if (!lora.empty()) return not_this_model("a LoRA adapter");
+        rc = tk_mi355x_llm_model_load_dir(&m, name.c_str(), dtype.c_str(), device);
+        if (rc != TK_SUCCESS) return rc;
         m->path = path;
     } else {
         rc = tk_mi355x_llm_model_load_gguf_lora(&m, file.c_str(), lora.c_str(), device);
@@ -661,7 +778,7 @@ struct tk_llm_runner_s {
     const uint32_t* next_mask() {
         if (!grammar_on) return nullptr;
         if (!trie_built) {
-            std::vector<std::string> pieces((size_t)model->model.hp.vocab);
+            std::vector<std::string> pieces((size_t)model->decoder()->vocab_size());
             for (int i = 0; i < (int)pieces.size(); ++i) pieces[i] = (i == model->tok.eos) ? std::string() : model->tok.piece(i);
             trie.build(pieces);
             trie_built = true;
@@ -696,7 +813,7 @@ tk_error_code_t tk_mi355x_llm_runner_set_sampling(tk_llm_runner_t* runner, float
     /* the device sampler draws from at most TK_SAMPLE_MAX_K = 64 candidates: llama.cpp's default top_k (40) fits; a larger top_k is refused rather than
      * clamped silently, and top_k = 0 ("the whole vocabulary" in llama.cpp) means the 64 largest here (include/tk/tk_mi355x_ext.h) */
     if (top_k > TK_SAMPLE_MAX_K) return fail(TK_ERROR_INVALID_ARGUMENT, "top_k above 64: the sampler keeps at most 64 candidates");
-    if (temperature > 0.0f && runner->model->model.hp.vocab > 65536) return fail(TK_ERROR_NOT_IMPLEMENTED, "stochastic sampling supports vocabularies of at most 65536 tokens");
+    if (temperature > 0.0f && runner->model->decoder()->vocab_size() > 65536) return fail(TK_ERROR_NOT_IMPLEMENTED, "stochastic sampling supports vocabularies of at most 65536 tokens");
     runner->samp.temp = temperature; runner->samp.top_k = top_k; runner->samp.top_p = top_p; runner->samp.min_p = min_p;
     return TK_SUCCESS;
 }
@@ -718,7 +835,7 @@ tk_error_code_t tk_llm_runner_create(tk_llm_runner_t** out_runner, void* model_h
             if (slots <= 0) slots = 16;
             std::unique_ptr<TkLlmBatcher> b(new TkLlmBatcher());
             std::string err;
-            if (!b->init(&r->model->model, slots, r->n_ctx, r->model->tok.eos, &err)) return fail(TK_ERROR_GPU_MEMORY, err);
+            if (!b->init(r->model->decoder(), slots, r->n_ctx, r->model->tok.eos, &err)) return fail(TK_ERROR_GPU_MEMORY, err);
             r->slot = b->acquire_slot();
             r->batcher = b.get();
             r->model->batchers.push_back(std::move(b));
@@ -759,14 +876,12 @@ static tk_error_code_t feed(tk_llm_runner_s* r, const std::vector<int32_t>& toks
     return TK_SUCCESS;
 }
 
-tk_error_code_t tk_llm_runner_prepare_generation(tk_llm_runner_t* runner, const char* prompt, bool use_tool_grammar) {
-    if (!runner || !prompt) return TK_ERROR_INVALID_ARGUMENT;
+static tk_error_code_t prepare_ids(tk_llm_runner_s* runner, const std::vector<int32_t>& toks, bool use_tool_grammar) {
     /* greedy sampling constrained by the tool-call grammar: the arg max runs over the tokens the grammar allows (mask applied on
      * the device), the reference's llama_sampling_set_grammar(sctx, grammar or NULL) (tk_runner_streaming.c:44-48) */
     runner->grammar_on = use_tool_grammar && runner->has_grammar;
     if (runner->grammar_on) runner->gstate.init(&runner->grammar);
     runner->tool_call_text.clear();
-    std::vector<int32_t> toks = runner->model->tok.encode(prompt, true);
     runner->n_past = 0; /* llama_kv_cache_clear: positions restart, stale cache rows are never attended */
     runner->pending = -1;
     tk_error_code_t rc = feed(runner, toks);
@@ -774,6 +889,20 @@ tk_error_code_t tk_llm_runner_prepare_generation(tk_llm_runner_t* runner, const 
     runner->is_processing = true;
     return TK_SUCCESS;
 }
+
+tk_error_code_t tk_llm_runner_prepare_generation(tk_llm_runner_t* runner, const char* prompt, bool use_tool_grammar) {
+    if (!runner || !prompt) return TK_ERROR_INVALID_ARGUMENT;
+    return prepare_ids(runner, runner->model->tok.encode(prompt, true), use_tool_grammar);
+}
+
+tk_error_code_t tk_mi355x_llm_runner_prepare_ids(tk_llm_runner_t* runner, const int32_t* ids, int n) {
+    if (!runner || !ids || n < 1) return TK_ERROR_INVALID_ARGUMENT;
+    for (int i = 0; i < n; ++i)
+        if (ids[i] < 0 || ids[i] >= runner->model->decoder()->vocab_size()) return fail(TK_ERROR_INVALID_ARGUMENT, "token id outside the vocabulary");
+    return prepare_ids(runner, std::vector<int32_t>(ids, ids + n), false);
+}
+
+int32_t tk_mi355x_llm_runner_pending_id(tk_llm_runner_t* runner) { return runner ? runner->pending : -1; }
 
 const char* tk_llm_runner_generate_next_token(tk_llm_runner_t* runner) {
     if (!runner || !runner->is_processing) return NULL;

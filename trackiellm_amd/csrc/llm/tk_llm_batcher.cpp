@@ -22,10 +22,11 @@ TkLlmBatcher::~TkLlmBatcher() {
     }
 }
 
-bool TkLlmBatcher::init(TkLlmModel* model, int slots, int n_ctx, int32_t eos, std::string* err) {
+bool TkLlmBatcher::init(TkDecoderModel* model, int slots, int n_ctx, int32_t eos, std::string* err) {
     if (slots < 1) slots = 1;
     if (slots > TK_MAX_ROWS) slots = TK_MAX_ROWS; /* one decode row per runner must fit one pass */
-    if (!session_.init(model, slots, n_ctx)) { *err = session_.error; return false; }
+    session_ = model->open_session(slots, n_ctx, 0, err);
+    if (!session_) return false;
     n_ctx_ = n_ctx;
     slot_used_.assign((size_t)slots, 0);
     ahead_.assign((size_t)slots, Ahead());
@@ -45,7 +46,11 @@ int TkLlmBatcher::acquire_slot() {
 
 void TkLlmBatcher::release_slot(int slot) {
     std::lock_guard<std::mutex> lk(mu_);
-    if (slot >= 0 && slot < (int)slot_used_.size()) { slot_used_[(size_t)slot] = 0; drop_ahead(slot); }
+    if (slot >= 0 && slot < (int)slot_used_.size()) {
+        slot_used_[(size_t)slot] = 0;
+        drop_ahead(slot);
+        session_->release_sequence(slot);
+    }
 }
 
 void TkLlmBatcher::stats(uint64_t* passes, uint64_t* rows, int* max_rows, uint64_t* wasted) {
@@ -115,7 +120,8 @@ bool TkLlmBatcher::submit(int slot, int pos0, const int32_t* toks, int n, const 
 }
 
 void TkLlmBatcher::loop() {
-    std::vector<int32_t> sq, ps, tk, am;
+    std::vector<int32_t> sq, ps, tk, am, outs, ids;
+    const int max_rows = session_->row_capacity();
     std::vector<const uint32_t*> masks;
     std::vector<TkSampleRow> samps;
     struct Taken { Request* r; int take, last_row; };   /* `take` rows of a request end at row `last_row` of the pass */
@@ -181,11 +187,11 @@ void TkLlmBatcher::loop() {
             const bool decode_first = decode_first_;
             if (decode_first)
                 for (Request* r : queue_) {
-                    if ((int)sq.size() >= TK_MAX_ROWS) break;
+                    if ((int)sq.size() >= max_rows) break;
                     if (r->n - r->done_rows == 1) add_rows(r, 1);
                 }
             auto add_ahead = [&] {
-                for (size_t s = 0; s < ahead_.size() && (int)sq.size() < TK_MAX_ROWS; ++s) {
+                for (size_t s = 0; s < ahead_.size() && (int)sq.size() < max_rows; ++s) {
                     Ahead& a = ahead_[s];
                     if (a.st != Ahead::PLANNED) continue;
                     a.st = Ahead::INFLIGHT;
@@ -199,9 +205,9 @@ void TkLlmBatcher::loop() {
             };
             if (decode_first) add_ahead(); /* one per sequence whose owner holds the id they feed */
             for (Request* r : queue_) {
-                if ((int)sq.size() >= TK_MAX_ROWS) break;
+                if ((int)sq.size() >= max_rows) break;
                 if (decode_first && r->n - r->done_rows == 1) continue; /* taken above */
-                add_rows(r, std::min(r->n - r->done_rows, TK_MAX_ROWS - (int)sq.size()));
+                add_rows(r, std::min(r->n - r->done_rows, max_rows - (int)sq.size()));
             }
             if (!decode_first) add_ahead();
         }
@@ -210,20 +216,28 @@ void TkLlmBatcher::loop() {
         am.assign((size_t)nrows, -1);
         const double t_formed = trace_path_.empty() ? 0.0 : now_ms();
         const bool head = !completing.empty() || !ahead_rows.empty();
-        const bool ok = session_.forward(nrows, sq.data(), ps.data(), tk.data(), nullptr, head ? am.data() : nullptr, head, head && any_mask ? masks.data() : nullptr,
-                                        head && any_samp ? samps.data() : nullptr);
+        /* only the rows that are sampled need the head */
+        outs.clear();
+        for (const Taken& t : in_pass)
+            if (t.r->done_rows + t.take == t.r->n) outs.push_back(t.last_row);
+        for (const AheadRow& a : ahead_rows) outs.push_back(a.row);
+        std::sort(outs.begin(), outs.end());
+        ids.assign(outs.size() + 1, -1);
+        const bool ok = session_->forward(nrows, sq.data(), ps.data(), tk.data(), nullptr, head ? ids.data() : nullptr, head, head && any_mask ? masks.data() : nullptr,
+                                          head && any_samp ? samps.data() : nullptr, (int)outs.size(), head ? outs.data() : nullptr);
+        for (size_t i = 0; i < outs.size() && ok; ++i) am[(size_t)outs[i]] = ids[i];
         {
             std::lock_guard<std::mutex> lk(mu_);
             passes_++;
             if (nrows > max_rows_) max_rows_ = nrows;
-            if (!ok) last_error_ = session_.error;
+            if (!ok) last_error_ = session_->error;
             size_t held = 0; /* completing requests that got no run-ahead row: their owners are waited for */
             for (const Taken& t : in_pass) {
                 Request* r = t.r;
                 const int take = t.take, row = t.last_row + 1;
                 rows_ += (uint64_t)take;
                 r->done_rows += take;
-                if (!ok) { r->ok = false; r->error = session_.error; r->done_rows = r->n; }
+                if (!ok) { r->ok = false; r->error = session_->error; r->done_rows = r->n; }
                 if (r->done_rows == r->n) {
                     r->sampled = ok ? am[(size_t)row - 1] : -1;
                     for (auto it = queue_.begin(); it != queue_.end(); ++it)
@@ -244,7 +258,7 @@ void TkLlmBatcher::loop() {
                     const int pos = a.pos;
                     a = Ahead();
                     w->ok = ok;
-                    if (!ok) w->error = session_.error;
+                    if (!ok) w->error = session_->error;
                     w->sampled = got;
                     rows_++;
                     if (ok) plan_ahead(s, pos, got, false);
@@ -258,7 +272,7 @@ void TkLlmBatcher::loop() {
             }
             expect_ = held;
             if (!trace_path_.empty())
-                trace_.push_back(PassTrace{t_woke, t_formed, now_ms(), nrows, (int)ahead_rows.size(), (int)completing.size(), (int)queue_.size(), session_.n_captures, session_.capture_ms});
+                trace_.push_back(PassTrace{t_woke, t_formed, now_ms(), nrows, (int)ahead_rows.size(), (int)completing.size(), (int)queue_.size(), session_->n_captures, session_->capture_ms});
         }
     }
 }

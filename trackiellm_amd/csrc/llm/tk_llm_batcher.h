@@ -28,13 +28,15 @@
 #include <thread>
 #include <vector>
 
-#include "tk_llm_engine.h"
+#include <memory>
+
+#include "tk_decoder.h"
 
 class TkLlmBatcher {
 public:
     ~TkLlmBatcher();
     /* one session with `slots` sequences of `n_ctx` positions on the model's device; starts the scheduler thread */
-    bool init(TkLlmModel* model, int slots, int n_ctx, int32_t eos, std::string* err);
+    bool init(TkDecoderModel* model, int slots, int n_ctx, int32_t eos, std::string* err);
     int acquire_slot();            /* -1 when every slot is taken */
     void release_slot(int slot);
     int n_ctx() const { return n_ctx_; }
@@ -74,7 +76,7 @@ private:
     int32_t eos_ = -1;
     uint64_t wasted_ = 0;
     std::string last_error_;
-    TkLlmSession session_;
+    std::unique_ptr<TkDecodeSession> session_;
     int n_ctx_ = 0;
     std::vector<char> slot_used_;
     std::mutex mu_;

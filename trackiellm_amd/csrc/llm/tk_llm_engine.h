@@ -18,6 +18,7 @@
 #include <string>
 #include <vector>
 
+#include "tk_decoder.h"
 #include "tk_llm_kernels.h"
 
 struct TkLlmHParams {
@@ -41,16 +42,16 @@ struct TkLlmLayer {
 enum TkLlmTensorId { TK_T_TOKEN_EMBD = 0, TK_T_OUT_NORM = 1, TK_T_OUTPUT = 2 };
 enum TkLlmLayerTensorId { TK_L_ATTN_NORM = 0, TK_L_Q, TK_L_K, TK_L_V, TK_L_O, TK_L_FFN_NORM, TK_L_GATE, TK_L_UP, TK_L_DOWN, TK_L_COUNT };
 
-class TkLlmModel {
+class TkLlmModel : public TkDecoderModel {
 public:
     TkLlmHParams hp{};
-    int device = 0;
     TkDevTensor token_embd, out_norm, output;
     std::vector<TkLlmLayer> layers;
-    std::string error;
-    size_t weight_bytes = 0; /* bytes a decode step streams (matrices only) */
 
-    ~TkLlmModel();
+    ~TkLlmModel() override;
+    int vocab_size() const override { return hp.vocab; }
+    uint64_t step_weight_bytes() const override;
+    std::unique_ptr<TkDecodeSession> open_session(int max_seq, int max_ctx, int pool_tokens, std::string* err) override;
     /* returns false and sets `error` on failure */
     bool init(const TkLlmHParams& hp, int device);
     /* f16: the fp16 checkpoint recipe (every matrix and the embedding IEEE f16, norms f32) instead of Q4_K_M */
@@ -73,41 +74,27 @@ private:
 
 class TkLlmPipe;
 
-class TkLlmSession {
+class TkLlmSession : public TkDecodeSession {
 public:
     TkLlmModel* model = nullptr;
-    int max_seq = 0, max_ctx = 0;
-    std::string error;
-    hipStream_t stream = nullptr;
 
-    ~TkLlmSession();
+    ~TkLlmSession() override;
     bool init(TkLlmModel* m, int max_seq, int max_ctx);
-    /* one pass over nrows <= TK_MAX_ROWS rows (16-row M-tiles); host arrays.  row_masks (optional): row_masks[r] = nullptr or the
-     * (vocab + 31) / 32 words whose bit t says token t may be sampled for row r: grammar-constrained greedy sampling, per row, so
-     * constrained and unconstrained rows share passes (and the captured graphs).  row_samp (optional): [nrows] sampling state, temp > 0
-     * = the reference's default stochastic chain for that row (tk_llm_kernels.h), else greedy */
-    bool forward(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, float* logits_host, int32_t* argmax_host,
-                 bool lm_head = true, const uint32_t* const* row_masks = nullptr, const TkSampleRow* row_samp = nullptr);
+    /* one pass over nrows <= TK_MAX_ROWS rows (16-row M-tiles); see TkDecodeSession.  The head runs over every row of the pass. */
+    bool forward(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, float* logits_host, int32_t* argmax_host, bool lm_head = true,
+                 const uint32_t* const* row_masks = nullptr, const TkSampleRow* row_samp = nullptr, int n_out = 0, const int32_t* out_rows = nullptr) override;
     /* one pipeline stage of a pass: layers [l0, l1) on this GPU.  The first stage starts from `tok` (x_in == nullptr), later stages
      * from the residual stream x_in [nrows][d_model] fp32; every stage but the last writes the stream to x_out; the last one
      * (head == true, l1 == n_layer) samples.  x_on_host: x_in / x_out are host pointers (gloo transport), otherwise device
      * pointers (RCCL transport).  Bit-identical to forward() whatever the split. */
     bool forward_stage(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, const float* x_in, float* x_out, bool x_on_host,
                        int l0, int l1, bool head, int32_t* argmax_host);
-    /* prompts of equal length for sequences 0..nseq-1 (tokens[nseq][n_prompt]); leaves row r = sequence r
-     * holding the first sampled token so decode() can follow; first_tokens_host[nseq] optional */
-    bool prefill(int nseq, int n_prompt, const int32_t* tokens, int32_t* first_tokens_host);
-    /* greedy decode loop, on-device feedback, hipGraph replay.  Starts from the rows' current
-     * (tok, pos) state left by the previous forward()/decode(); out_tokens[n_steps][nrows]. */
-    bool decode(int nrows, int n_steps, int32_t* out_tokens_host);
-    bool reset();
+    bool prefill(int nseq, int n_prompt, const int32_t* tokens, int32_t* first_tokens_host) override;
     /* KV cache import / export: rows [pos0, pos0 + n_pos) of one (layer, sequence) as f16 bits, host arrays in [position][kv head][dim]
      * order (the cache itself is [layer][sequence][kv head][position][dim]).  Restores a saved prompt prefix without re-running it; the
      * parity tests use it to put an attention launch at any context length in one decode step. */
     bool kv_write(int layer, int seq, int pos0, int n_pos, const uint16_t* k, const uint16_t* v);
     bool kv_read(int layer, int seq, int pos0, int n_pos, uint16_t* k, uint16_t* v);
-    /* per-launch timing of the last decode(): average ms of one step measured with HIP events */
-    float last_step_ms = 0.0f;
     /* stand-alone timing of the dominant GEMV (gate/up of layer 0) for bench.py's roofline leg */
     bool time_gemv(int layer, int which, int nrows, int iters, float* avg_ms, double* algo_bytes);
     /* stand-alone timing of the decode attention launch at nrows rows x ctx cached positions, for bench.py's second roofline object */
@@ -120,16 +107,8 @@ private:
     void enqueue_range(int nrows, int l0, int l1, bool embed, bool fold_out, bool lm_head, bool fused_attn);
     int enqueue_matmul(const TkDevTensor* const* t, int nseg, int K, int ks, int n_total, const TkActQ8& act, float* out, int nrows);
     uint16_t *kcache = nullptr, *vcache = nullptr;
-    float *x = nullptr, *x2 = nullptr, *qbuf = nullptr, *partial = nullptr, *partial2 = nullptr, *logits = nullptr, *rope_cos = nullptr, *rope_sin = nullptr;
+    float *x = nullptr, *x2 = nullptr, *qbuf = nullptr, *partial = nullptr, *partial2 = nullptr, *rope_cos = nullptr, *rope_sin = nullptr;
     TkActQ8 act_d{}, act_qd{}, act_ff{};
-    int32_t *d_seq = nullptr, *d_pos = nullptr, *d_tok = nullptr, *d_nsteps = nullptr, *d_hist = nullptr;
-    uint32_t* d_mask = nullptr;     /* [TK_MAX_ROWS][(vocab + 31) / 32] allowed-token bits of the masked rows of the current pass */
-    int32_t* d_mask_row = nullptr;  /* [TK_MAX_ROWS] index into d_mask, -1 = the row samples unconstrained */
-    bool mask_rows_dirty = true;    /* d_mask_row holds something other than all -1 */
-    TkSampleRow* d_samp = nullptr;  /* [TK_MAX_ROWS] sampling state of the rows of the current pass (temp 0 = greedy); decode() continues from it */
-    bool samp_dirty = false;        /* d_samp holds a stochastic row */
-    std::string launch_error; /* set by enqueue_* when a launcher refuses its arguments (no HIP error is raised for that) */
-    int hist_cap = 0;
     hipGraphExec_t graph_exec[2][TK_MAX_ROWS + 1] = {}; /* [long_pass][row count]: decode pass (head + sampling, every sequence once) */
     /* [tiled_pass][row count]: prompt pass (no head, rope/append as its own kernel); sampling pass that holds several positions of one sequence
      * (a prompt's last chunk) */
@@ -150,10 +129,8 @@ private:
     int32_t* d_tiles = nullptr;                         /* [1 + TK_MAX_ROWS] 16-row tiles of a multi-position pass (k_att_tiles) */
     size_t tab_cap = 0;
     bool capture_pass(hipGraphExec_t* slot, int nrows, bool lm_head, bool fused_attn);
-public:
-    uint64_t n_captures = 0; /* passes recorded into a graph so far, and the host time that took (diagnostics: TK_MI355X_BATCHER_TRACE) */
-    double capture_ms = 0.0;
-private:
+    hipGraphExec_t* decode_slot(int nrows, int top) override;
+    void enqueue_decode(int nrows) override;
 };
 
 #endif

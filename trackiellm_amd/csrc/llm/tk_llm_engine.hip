@@ -197,6 +197,18 @@ bool TkLlmModel::fill_synthetic(uint64_t seed, bool f16) {
     return ok;
 }
 
+uint64_t TkLlmModel::step_weight_bytes() const {
+    uint64_t b = output.bytes;
+    for (const auto& L : layers) b += L.q.bytes + L.k.bytes + L.v.bytes + L.o.bytes + L.gate.bytes + L.up.bytes + L.down.bytes;
+    return b;
+}
+
+std::unique_ptr<TkDecodeSession> TkLlmModel::open_session(int max_seq, int max_ctx, int, std::string* err) {
+    std::unique_ptr<TkLlmSession> s(new TkLlmSession());
+    if (!s->init(this, max_seq, max_ctx)) { *err = s->error; return nullptr; }
+    return s;
+}
+
 bool TkLlmModel::ready() const {
     if (!token_embd.data || !out_norm.data || !output.data) return false;
     for (const auto& L : layers) {
@@ -247,8 +259,7 @@ bool TkLlmSession::init(TkLlmModel* m, int mseq, int mctx) {
         error = "max_ctx too large: the attention kernel keeps one score row per query head of a KV group in LDS (about 9000 positions for 4 x 128)";
         return false;
     }
-    HIPQ(hipSetDevice(m->device));
-    HIPQ(hipStreamCreateWithFlags(&stream, hipStreamNonBlocking));
+    if (!init_tables(m->device, h.vocab, TK_MAX_ROWS, 0, nullptr)) return false;
     tk_attention_note_session(m->device, +1);
     counted_ = true;
     const int QD = h.n_head * h.head_dim, KVD = h.n_kv_head * h.head_dim, half = h.head_dim / 2;
@@ -268,26 +279,11 @@ bool TkLlmSession::init(TkLlmModel* m, int mseq, int mctx) {
      * its workgroups write the other */
     HIPQ(hipMalloc((void**)&x2, (size_t)TK_MAX_ROWS * h.d_model * 4));
     HIPQ(hipMalloc((void**)&partial2, pmax * TK_MAX_ROWS * 4));
-    HIPQ(hipMalloc((void**)&logits, (size_t)TK_MAX_ROWS * h.vocab * 4));
     if (!alloc_act(&act_d, h.d_model, m->has_f16, error) || !alloc_act(&act_qd, QD, m->has_f16, error) || !alloc_act(&act_ff, h.d_ff, m->has_f16, error)) return false;
-    HIPQ(hipMalloc((void**)&d_seq, TK_MAX_ROWS * 4));
-    HIPQ(hipMalloc((void**)&d_pos, TK_MAX_ROWS * 4));
-    HIPQ(hipMalloc((void**)&d_tok, TK_MAX_ROWS * 4));
-    HIPQ(hipMalloc((void**)&d_nsteps, TK_MAX_ROWS * 4));
-    HIPQ(hipMemset(d_nsteps, 0, TK_MAX_ROWS * 4));
-    hist_cap = mctx;
-    HIPQ(hipMalloc((void**)&d_hist, (size_t)hist_cap * TK_MAX_ROWS * 4));
     HIPQ(hipMalloc((void**)&d_tiles, (size_t)(1 + TK_MAX_ROWS) * 4));
     HIPQ(hipMemset(d_tiles, 0, (size_t)(1 + TK_MAX_ROWS) * 4));
     if (mctx > TK_LONG_ATT_MIN_POS && tk_attention_long_applies(1, h.n_head, h.n_kv_head, h.head_dim))
         HIPQ(hipMalloc((void**)&d_scores, tk_attention_long_scratch_floats(h.n_head, h.head_dim, mctx) * sizeof(float)));
-    HIPQ(hipMalloc((void**)&d_mask, (size_t)TK_MAX_ROWS * (((size_t)h.vocab + 31) / 32) * 4));
-    HIPQ(hipMalloc((void**)&d_mask_row, TK_MAX_ROWS * 4));
-    HIPQ(hipMemset(d_mask_row, 0xFF, TK_MAX_ROWS * 4));
-    mask_rows_dirty = false;
-    HIPQ(hipMalloc((void**)&d_samp, TK_MAX_ROWS * sizeof(TkSampleRow)));
-    HIPQ(hipMemset(d_samp, 0, TK_MAX_ROWS * sizeof(TkSampleRow))); /* temp 0: every row samples greedily */
-    samp_dirty = false;
     /* RoPE table, double precision on the host (same formula as the oracle) */
     std::vector<float> cs((size_t)mctx * half), sn((size_t)mctx * half);
     for (int p = 0; p < mctx; ++p)
@@ -315,17 +311,9 @@ TkLlmSession::~TkLlmSession() {
     for (auto& v : graph_exec) for (auto& g : v) if (g) (void)hipGraphExecDestroy(g);
     for (auto& v : graph_prefill) for (auto& g : v) if (g) (void)hipGraphExecDestroy(g);
     for (auto& v : graph_head_nf) for (auto& g : v) if (g) (void)hipGraphExecDestroy(g);
-    void* ptrs[] = {kcache, vcache, x, x2, qbuf, partial, partial2, logits, rope_cos, rope_sin, d_seq, d_pos, d_tok, d_nsteps, d_hist, d_mask, d_mask_row, d_samp, d_tab, d_tiles, d_scores};
+    void* ptrs[] = {kcache, vcache, x, x2, qbuf, partial, partial2, rope_cos, rope_sin, d_tab, d_tiles, d_scores};
     for (void* p : ptrs) if (p) (void)hipFree(p);
     free_act(&act_d); free_act(&act_qd); free_act(&act_ff);
-    if (stream) (void)hipStreamDestroy(stream);
-}
-
-bool TkLlmSession::reset() {
-    HIPQ(hipSetDevice(model->device));
-    HIPQ(hipMemsetAsync(d_nsteps, 0, TK_MAX_ROWS * 4, stream));
-    HIPQ(hipStreamSynchronize(stream));
-    return true;
 }
 
 bool TkLlmSession::kv_write(int layer, int seq, int pos0, int n_pos, const uint16_t* k, const uint16_t* v) {
@@ -491,16 +479,6 @@ void TkLlmSession::enqueue_range(int nrows, int l0, int l1, bool embed, bool fol
     tk_launch_argmax(logits, h.vocab, nrows, d_mask, d_mask_row, d_samp, d_tok, d_pos, d_nsteps, d_hist, TK_MAX_ROWS, s);
 }
 
-static bool graphs_enabled() {
-    /* TK_MI355X_NO_GRAPH=1: eager launches, for profilers that cannot follow hipGraphLaunch (see DESIGN.md "Profiling") */
-    const char* ng = getenv("TK_MI355X_NO_GRAPH");
-    return !(ng && ng[0] == '1');
-}
-
-/* one capture at a time per process; relaxed mode: other host threads (detector / ASR / VAD streams) keep calling allocation and copy
- * APIs while this stream records */
-static std::mutex g_capture_mu;
-
 #ifndef TK_TILED_ATT_MIN_POS
 #define TK_TILED_ATT_MIN_POS 128
 #endif
@@ -515,39 +493,21 @@ void TkLlmSession::choose_attention_top(int top, int nrows) {
 }
 
 bool TkLlmSession::capture_pass(hipGraphExec_t* slot, int nrows, bool lm_head, bool fused_attn) {
-    if (*slot) return true;
-    const auto t_cap = std::chrono::steady_clock::now();
-    struct Tally { TkLlmSession* s; std::chrono::steady_clock::time_point t0; ~Tally() { s->n_captures++; s->capture_ms += std::chrono::duration<double, std::milli>(std::chrono::steady_clock::now() - t0).count(); } } tally{this, t_cap};
-    std::lock_guard<std::mutex> lk(g_capture_mu);
-    hipGraph_t g = nullptr;
-    HIPQ(hipStreamBeginCapture(stream, hipStreamCaptureModeRelaxed));
-    launch_error.clear();
-    enqueue_pass(nrows, lm_head, fused_attn);
-    /* from here on the stream must leave capture mode and the graph must be freed whatever fails */
-    const hipError_t e_end = hipStreamEndCapture(stream, &g);
-    hipError_t e_inst = hipSuccess;
-    if (e_end == hipSuccess && launch_error.empty()) e_inst = hipGraphInstantiate(slot, g, nullptr, nullptr, 0);
-    if (g) (void)hipGraphDestroy(g);
-    if (e_end != hipSuccess || e_inst != hipSuccess || !launch_error.empty()) {
-        if (*slot && e_inst != hipSuccess) { (void)hipGraphExecDestroy(*slot); }
-        *slot = nullptr;
-        (void)hipGetLastError();
-        error = !launch_error.empty() ? launch_error
-                : std::string("graph capture of a pass failed: ") + hipGetErrorString(e_end != hipSuccess ? e_end : e_inst);
-        return false;
-    }
-    return true;
+    return capture(slot, [=] { enqueue_pass(nrows, lm_head, fused_attn); });
 }
 
+hipGraphExec_t* TkLlmSession::decode_slot(int nrows, int top) {
+    choose_attention_top(top, nrows);
+    return &graph_exec[long_pass][nrows];
+}
+void TkLlmSession::enqueue_decode(int nrows) { enqueue_pass(nrows, true, true); }
+
 bool TkLlmSession::forward(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, float* logits_host, int32_t* argmax_host,
-                           bool lm_head, const uint32_t* const* row_masks, const TkSampleRow* row_samp) {
+                           bool lm_head, const uint32_t* const* row_masks, const TkSampleRow* row_samp, int n_out, const int32_t* out_rows) {
     if (nrows <= 0 || nrows > TK_MAX_ROWS) { error = "nrows must be in [1,256]"; return false; }
-    for (int r = 0; r < nrows; ++r) {
-        if (seq[r] < 0 || seq[r] >= max_seq || pos[r] < 0 || pos[r] >= max_ctx || tok[r] < 0 || tok[r] >= model->hp.vocab) {
-            error = "row out of range (sequence id, position or token id)";
-            return false;
-        }
-    }
+    if (!rows_in_range(nrows, seq, pos, tok)) return false;
+    for (int i = 0; i < n_out && out_rows; ++i)
+        if (out_rows[i] < 0 || out_rows[i] >= nrows) { error = "wanted row out of range"; return false; }
     HIPQ(hipSetDevice(model->device));
     HIPQ(hipMemcpyAsync(d_seq, seq, nrows * 4, hipMemcpyHostToDevice, stream));
     HIPQ(hipMemcpyAsync(d_pos, pos, nrows * 4, hipMemcpyHostToDevice, stream));
@@ -558,35 +518,7 @@ bool TkLlmSession::forward(int nrows, const int32_t* seq, const int32_t* pos, co
     for (int a = 0; a < nrows && distinct; ++a)
         for (int b = a + 1; b < nrows; ++b)
             if (seq[a] == seq[b]) { distinct = false; break; }
-    if (lm_head) { /* per-row sampling masks: the masks of the constrained rows, compacted, + the row -> mask table the arg max kernel reads */
-        int32_t rowtab[TK_MAX_ROWS];
-        int nmask = 0;
-        const size_t words = ((size_t)model->hp.vocab + 31) / 32;
-        for (int r = 0; r < TK_MAX_ROWS; ++r) rowtab[r] = -1;
-        for (int r = 0; r < nrows; ++r) {
-            if (row_masks && row_masks[r]) {
-                HIPQ(hipMemcpyAsync(d_mask + (size_t)nmask * words, row_masks[r], words * 4, hipMemcpyHostToDevice, stream));
-                rowtab[r] = nmask++;
-            }
-        }
-        if (nmask > 0 || mask_rows_dirty) {
-            HIPQ(hipMemcpyAsync(d_mask_row, rowtab, TK_MAX_ROWS * 4, hipMemcpyHostToDevice, stream)); /* whole table (a wider pass may have left entries); pageable source: staged before the call returns */
-            mask_rows_dirty = nmask > 0;
-        }
-        /* per-row sampling state (temp <= 0: greedy): data of the pass like the masks, so sampled and greedy rows share passes and graphs */
-        bool any_samp = false;
-        for (int r = 0; r < nrows && row_samp; ++r) any_samp = any_samp || row_samp[r].temp > 0.0f;
-        if (any_samp) {
-            if (model->hp.vocab > 65536) { error = "stochastic sampling supports vocabularies of at most 65536 tokens"; return false; }
-            TkSampleRow tab[TK_MAX_ROWS] = {};
-            for (int r = 0; r < nrows; ++r) tab[r] = row_samp[r];
-            HIPQ(hipMemcpyAsync(d_samp, tab, sizeof tab, hipMemcpyHostToDevice, stream));
-            samp_dirty = true;
-        } else if (samp_dirty) {
-            HIPQ(hipMemsetAsync(d_samp, 0, TK_MAX_ROWS * sizeof(TkSampleRow), stream));
-            samp_dirty = false;
-        }
-    }
+    if (lm_head && !stage_sampling(nrows, nullptr, row_masks, row_samp)) return false;
     /* a pass replays a captured graph (one per (row count, form)): a host that asks for one token at a time — the reference's runner
      * API — pays one graph launch, not ~260 kernel launches, per token; masked rows ride the same graphs (the table above is data) */
     hipGraphExec_t* slot = !graphs_enabled() ? nullptr
@@ -601,6 +533,15 @@ bool TkLlmSession::forward(int nrows, const int32_t* seq, const int32_t* pos, co
     if (!launch_error.empty()) { error = launch_error; (void)hipStreamSynchronize(stream); return false; }
     HIPQ(hipGetLastError());
     if (!lm_head) { HIPQ(hipStreamSynchronize(stream)); return true; }
+    if (out_rows) { /* the wanted rows of the pass, in the caller's order */
+        int32_t ids[TK_MAX_ROWS];
+        for (int i = 0; i < n_out && logits_host; ++i)
+            HIPQ(hipMemcpyAsync(logits_host + (size_t)i * vocab_, logits + (size_t)out_rows[i] * vocab_, (size_t)vocab_ * 4, hipMemcpyDeviceToHost, stream));
+        if (argmax_host) HIPQ(hipMemcpyAsync(ids, d_tok, nrows * 4, hipMemcpyDeviceToHost, stream));
+        HIPQ(hipStreamSynchronize(stream));
+        for (int i = 0; i < n_out && argmax_host; ++i) argmax_host[i] = ids[out_rows[i]];
+        return true;
+    }
     if (logits_host) HIPQ(hipMemcpyAsync(logits_host, logits, (size_t)nrows * model->hp.vocab * 4, hipMemcpyDeviceToHost, stream));
     if (argmax_host) HIPQ(hipMemcpyAsync(argmax_host, d_tok, nrows * 4, hipMemcpyDeviceToHost, stream));
     HIPQ(hipStreamSynchronize(stream));
@@ -692,45 +633,6 @@ bool TkLlmSession::prefill(int nseq, int n_prompt, const int32_t* tokens, int32_
     return forward(nseq, sq.data(), ps.data(), tk.data(), nullptr, first_tokens_host, true);
 }
 
-bool TkLlmSession::decode(int nrows, int n_steps, int32_t* out_tokens_host) {
-    if (nrows <= 0 || nrows > TK_MAX_ROWS) { error = "nrows must be in [1,256]"; return false; }
-    if (n_steps <= 0 || n_steps > hist_cap) { error = "n_steps exceeds the session context"; return false; }
-    HIPQ(hipSetDevice(model->device));
-    /* positions must stay inside the cache for the whole loop */
-    int32_t hpos[TK_MAX_ROWS];
-    HIPQ(hipMemcpyAsync(hpos, d_pos, nrows * 4, hipMemcpyDeviceToHost, stream));
-    HIPQ(hipStreamSynchronize(stream));
-    for (int r = 0; r < nrows; ++r)
-        if (hpos[r] + n_steps > max_ctx) { error = "decode would run past max_ctx"; return false; }
-    const bool use_graph = graphs_enabled();
-    int top0 = 0;
-    for (int r = 0; r < nrows; ++r) top0 = hpos[r] > top0 ? hpos[r] : top0;
-    HIPQ(hipMemsetAsync(d_nsteps, 0, TK_MAX_ROWS * 4, stream));
-    if (mask_rows_dirty) { HIPQ(hipMemsetAsync(d_mask_row, 0xFF, TK_MAX_ROWS * 4, stream)); mask_rows_dirty = false; } /* the loop samples unconstrained */
-    hipEvent_t e0, e1;
-    HIPQ(hipEventCreate(&e0));
-    HIPQ(hipEventCreate(&e1));
-    HIPQ(hipEventRecord(e0, stream));
-    for (int i = 0; i < n_steps; ++i) {
-        choose_attention_top(top0 + i, nrows); /* positions advance on the device; the host knows where the loop stands */
-        if (use_graph) {
-            if (!capture_pass(&graph_exec[long_pass][nrows], nrows, true, true)) { (void)hipStreamSynchronize(stream); (void)hipEventDestroy(e0); (void)hipEventDestroy(e1); return false; }
-            HIPQ(hipGraphLaunch(graph_exec[long_pass][nrows], stream));
-        } else { launch_error.clear(); enqueue_pass(nrows, true, true); if (!launch_error.empty()) { error = launch_error; break; } }
-    }
-    if (!launch_error.empty()) { (void)hipStreamSynchronize(stream); (void)hipEventDestroy(e0); (void)hipEventDestroy(e1); launch_error.clear(); return false; }
-    HIPQ(hipGetLastError());
-    HIPQ(hipEventRecord(e1, stream));
-    if (out_tokens_host) HIPQ(hipMemcpyAsync(out_tokens_host, d_hist, (size_t)n_steps * TK_MAX_ROWS * 4, hipMemcpyDeviceToHost, stream));
-    HIPQ(hipStreamSynchronize(stream));
-    float ms = 0.0f;
-    HIPQ(hipEventElapsedTime(&ms, e0, e1));
-    last_step_ms = ms / n_steps;
-    (void)hipEventDestroy(e0);
-    (void)hipEventDestroy(e1);
-    return true;
-}
-
 bool TkLlmSession::time_gemv(int layer, int which, int nrows, int iters, float* avg_ms, double* algo_bytes) {
     const TkLlmHParams& h = model->hp;
     if (layer < 0 || layer >= h.n_layer || nrows < 1 || nrows > TK_MAX_ROWS) { error = "bad layer / nrows"; return false; }
@@ -788,7 +690,7 @@ bool TkLlmSession::time_gemv(int layer, int which, int nrows, int iters, float* 
     const bool use_graph = graphs_enabled();
     hipGraphExec_t ge = nullptr;
     if (use_graph) {
-        std::lock_guard<std::mutex> lk(g_capture_mu);
+        std::lock_guard<std::mutex> lk(tk_capture_mutex());
         hipGraph_t g = nullptr;
         HIPQ(hipStreamBeginCapture(stream, hipStreamCaptureModeRelaxed));
         for (int i = 0; i < iters; ++i) tk_launch_gemv(set[(size_t)i % set.size()], stream);
@@ -847,7 +749,7 @@ bool TkLlmSession::time_attention(int nrows, int ctx, int iters, float* avg_ms, 
     hipGraphExec_t ge = nullptr;
     launch(0);
     if (use_graph) {
-        std::lock_guard<std::mutex> lk(g_capture_mu);
+        std::lock_guard<std::mutex> lk(tk_capture_mutex());
         hipGraph_t g = nullptr;
         HIPQ(hipStreamBeginCapture(stream, hipStreamCaptureModeRelaxed));
         for (int i = 0; i < iters; ++i) launch(i);

@@ -1,0 +1,108 @@
+/*
+ * tk_mixer_kernels.h — launch wrappers of the layer-list decoders' kernels (tk_layered.h): paged attention with a sliding window and kept first
+ * positions, the gated delta rule with its short convolutions, output norms on the residual stream, the grouped sigmoid router.  Sizes and
+ * constants are arguments throughout.  Wrappers only enqueue on `s`.
+ *
+ * Activations that feed a matrix product are operand images (nn/tk_gemm_image.h) of the session's element type; everything else — projections'
+ * results, the residual stream, gates, decays, recurrent state — is f32.
+ */
+#ifndef TK_MIXER_KERNELS_H
+#define TK_MIXER_KERNELS_H
+
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+#include "../nn/tk_gemm_image.h"
+#include "tk_layer_spec.h"
+
+#define TK_PAGE 64 /* positions of a cache page */
+
+/* device tables of one pass.  A segment is a run of consecutive rows that hold consecutive positions of one sequence. */
+struct TkPassTab {
+    const int32_t *seq, *pos, *tok; /* [rows] */
+    const int32_t* seg;             /* [rows] */
+    const int32_t *seg_row0, *seg_n; /* [segments] */
+    int32_t *seg_in, *seg_out;      /* [segments] state copies read (-1: the sequence starts here) and written; never the same copy */
+    const int32_t* page_of;         /* [sequences][max_pages] page ids */
+    int max_pages;
+};
+
+/* keys [page][kv head][TK_PAGE][dim_pad], values transposed [page][kv head][vdim_pad][TK_PAGE]; dim_pad = image k padding, vdim_pad = 16s */
+struct TkKvPool { void *k, *v; int dim_pad, vdim_pad; };
+
+struct TkAttnArgs {
+    int heads, kv_heads, dim, vdim, rot_dims, window, keep_first;
+    float scale, out_scale, eps;
+    int col;                          /* first column of q | k | v in the projections */
+    const float *bias;                /* q | k | v biases or null */
+    const float *q_norm, *k_norm;     /* null: no norm */
+    const float *rope_cos, *rope_sin; /* [max_ctx][rot_dims / 2] */
+    void* q;                          /* [rows][heads][dim_pad] */
+    TkKvPool kv;
+    void* out_img;                    /* next product's image; head h at k = out_k0 + h * vdim */
+    int out_k0, out_ktiles;
+};
+
+struct TkDeltaArgs {
+    int heads, kv_heads, dim, vdim, taps;
+    float out_scale, eps, unit_eps;
+    int col;                          /* first column of q | k | v | b in the projections */
+    const float *conv;                /* [2 kv_heads dim + heads vdim][taps] */
+    const float *a_log, *dt_bias, *norm;
+    const float* low;                 /* [rows][low_ld]: decay inputs (heads x dim) from column low_a on, gate inputs (heads x vdim) from low_g */
+    int low_ld, low_a, low_g;
+    float *q, *k, *v, *g, *beta, *o;  /* [rows][kv_heads dim], same, [rows][heads vdim], [rows][heads dim], [rows][heads], [rows][heads vdim] */
+    float* conv_state;                /* [copies][channels][taps - 1] */
+    float* state;                     /* [copies][heads][dim][vdim padded to 4] */
+    void* out_img;
+    int out_k0, out_ktiles;
+};
+
+void tk_launch_layer_embed(int type, const uint16_t* table, int width, const int32_t* tok, int nrows, float* x, void* img, int ktiles, hipStream_t s);
+
+/* everything between the projections and the mixers: biases, per-head norms, rotation, cache append; convolutions, unit norms, decays, step sizes */
+void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs* attn, const TkDeltaArgs* delta, const TkPassTab& t, int nrows, hipStream_t s);
+
+/* tiles: [2 * n_tiles] = first row, rows (<= 64) of a run of consecutive positions; every head of every tile is one workgroup */
+void tk_launch_attn_tiles(int type, const TkAttnArgs& a, const TkPassTab& t, const int32_t* tiles, int n_tiles, hipStream_t s);
+/* one row at a time (decoding): `splits` workgroups per (row, group of query heads) share the row's pages; scratch for splits > 1 */
+void tk_launch_attn_rows(int type, const TkAttnArgs& a, const TkPassTab& t, int nrows, int splits, float* scratch, hipStream_t s);
+size_t tk_attn_rows_scratch_floats(const TkAttnArgs& a, int nrows, int splits);
+
+/* the recurrence over every segment, token by token, and the gated per-head norm of its output */
+void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, int n_segments, int nrows, hipStream_t s);
+/* the same for passes whose segments are single rows: one launch */
+void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s);
+
+/* where a sublayer's output comes from: a product's rows, or the chosen experts' rows, weighted */
+struct TkSubOut {
+    const float* y; int ld;
+    const float* bias; float bias_scale; /* bias may be null */
+    const int32_t* slot; const float* weight; int top; /* top > 0: y[slot[row * top + j]] * weight[row * top + j] summed over j */
+};
+/* x += norm(output) * w; the image of the new x */
+void tk_launch_post_norm(int type, const TkSubOut& o, const float* w, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s);
+/* norm of the listed rows (null: rows 0 .. n - 1) as an image */
+void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const float* w, float eps, int width, void* img, int ktiles, hipStream_t s);
+
+struct TkMoeTab {
+    int32_t* count;      /* [experts], zero between passes */
+    int32_t* expert;     /* [rows * top] */
+    int32_t* rank;       /* [rows * top] place among the expert's rows */
+    float* weight;       /* [rows * top] */
+    int32_t* tile0;      /* [experts] first 16-row tile */
+    int32_t* slot;       /* [rows * top] row in the gathered image */
+    TkImgBlock* blocks;
+    int32_t* n_blocks;
+};
+void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, const TkMoeTab& t, hipStream_t s);
+void tk_launch_moe_plan(int experts, int block_tiles, const TkMoeTab& t, hipStream_t s);
+void tk_launch_moe_gather(const void* img, void* gathered, int ktiles, int top, int nrows, const TkMoeTab& t, hipStream_t s);
+
+/* end of a pass in a device-driven loop: every single-row segment reads next what it has just written */
+void tk_launch_swap_state(const TkPassTab& t, int n, hipStream_t s);
+
+/* LDS opt-in on the current device; nullptr or an error string */
+const char* tk_mixer_prepare_device();
+
+#endif

@@ -1,0 +1,806 @@
+/* tk_mixer_kernels.hip — see tk_mixer_kernels.h */
+#include "tk_mixer_kernels.h"
+
+#include <math.h>
+
+#include <atomic>
+#include <mutex>
+
+#include "../nn/tk_image_device.h"
+
+namespace {
+
+constexpr float LOG2E = 1.44269504088896340736f;
+
+/* ------------------------------------------------------------------ embedding, norms ------- */
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_layer_embed(const uint16_t* table, int width, const int32_t* tok, float* x, T* img, int ktiles) {
+    const int row = blockIdx.x;
+    const uint16_t* e = table + (size_t)tok[row] * width;
+    for (int k = threadIdx.x; k < width; k += 256) {
+        const float v = tk_bf16_float(e[k]);
+        x[(size_t)row * width + k] = v;
+        tk_img_put(img, row, k, ktiles, v);
+    }
+}
+
+__device__ __forceinline__ float block_sum(float v, float* red /* [16] */) {
+    v = tk_wave_sum(v);
+    const int w = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    if ((threadIdx.x & 63) == 0) red[w] = v;
+    __syncthreads();
+    float t = 0.0f;
+    for (int i = 0; i < nw; ++i) t += red[i];
+    __syncthreads();
+    return t;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_post_norm(TkSubOut o, const float* w, float eps, int width, float* x, T* img, int ktiles) {
+    extern __shared__ __attribute__((aligned(16))) float ybuf[];
+    __shared__ float red[16];
+    const int row = blockIdx.x;
+    float ss = 0.0f;
+    if (o.top > 0) {
+        for (int k = threadIdx.x; k < width; k += 256) {
+            float y = 0.0f;
+            for (int j = 0; j < o.top; ++j) y += o.weight[row * o.top + j] * o.y[(size_t)o.slot[row * o.top + j] * o.ld + k];
+            ybuf[k] = y;
+            ss += y * y;
+        }
+    } else {
+        for (int k = threadIdx.x; k < width; k += 256) {
+            float y = o.y[(size_t)row * o.ld + k];
+            if (o.bias) y += o.bias[k] * o.bias_scale;
+            ybuf[k] = y;
+            ss += y * y;
+        }
+    }
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps); /* block_sum synchronises: ybuf is whole; a thread re-reads its own elements */
+    for (int k = threadIdx.x; k < width; k += 256) {
+        const float v = x[(size_t)row * width + k] + ybuf[k] * r * w[k];
+        x[(size_t)row * width + k] = v;
+        tk_img_put(img, row, k, ktiles, v);
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_rows_norm(const float* x, const int32_t* rows, const float* w, float eps, int width, T* img, int ktiles) {
+    __shared__ float red[16];
+    const int i = blockIdx.x;
+    const float* xr = x + (size_t)(rows ? rows[i] : i) * width;
+    float ss = 0.0f;
+    for (int k = threadIdx.x; k < width; k += 256) ss += xr[k] * xr[k];
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
+    for (int k = threadIdx.x; k < width; k += 256) tk_img_put(img, i, k, ktiles, xr[k] * r * w[k]);
+}
+
+/* ------------------------------------------------------------------ between projections and mixers ---- */
+
+/* one wave: one head of q, k or v of one row */
+template <typename T>
+__device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* p, int row, int u, int lane) {
+    const bool is_q = u < a.heads, is_v = u >= a.heads + a.kv_heads;
+    const int n = is_v ? a.vdim : a.dim;
+    const int head = is_q ? u : is_v ? u - a.heads - a.kv_heads : u - a.heads;
+    const int off = is_q ? head * a.dim : is_v ? (a.heads + a.kv_heads) * a.dim + head * a.vdim : (a.heads + head) * a.dim;
+    const float* src = p + a.col + off;
+    const float* b = a.bias ? a.bias + off : nullptr;
+    const float* w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
+    float v[4];
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e = lane + 64 * i;
+        v[i] = e < n ? src[e] + (b ? b[e] : 0.0f) : 0.0f;
+        ss += v[i] * v[i];
+    }
+    const float r = w ? 1.0f / sqrtf(tk_wave_sum(ss) / (float)n + a.eps) : 1.0f;
+    const int pos = t.pos[row], half = is_v ? 0 : a.rot_dims / 2;
+    const size_t page = is_q ? 0 : (size_t)t.page_of[(size_t)t.seq[row] * t.max_pages + pos / TK_PAGE];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e = lane + 64 * i;
+        if (e >= n) break;
+        float y = w ? v[i] * r * w[e] : v[i];
+        if (e < 2 * half) { /* the other half of the pair: its value times the head's common factor */
+            const int f = e < half ? e + half : e - half, j = e < half ? e : e - half;
+            float z = src[f] + (b ? b[f] : 0.0f);
+            if (w) z = z * r * w[f];
+            const float c = a.rope_cos[(size_t)pos * half + j], s = a.rope_sin[(size_t)pos * half + j];
+            y = e < half ? y * c - z * s : y * c + z * s;
+        }
+        if (is_q) ((T*)a.q)[((size_t)row * a.heads + head) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+        else if (is_v) ((T*)a.kv.v)[((page * a.kv_heads + head) * a.kv.vdim_pad + e) * TK_PAGE + pos % TK_PAGE] = TkImg<T>::from(y);
+        else ((T*)a.kv.k)[((page * a.kv_heads + head) * TK_PAGE + pos % TK_PAGE) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+    }
+}
+
+/* one wave: one head of q, k or v after its convolution, or one head's decays and step size */
+__device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab& t, const float* proj, int ld, int row, int u, int lane) {
+    const int qk = d.kv_heads * d.dim, channels = 2 * qk + d.heads * d.vdim;
+    if (u >= 2 * d.kv_heads + d.heads) {
+        const int h = u - 2 * d.kv_heads - d.heads;
+        const float rate = -expf(d.a_log[h]);
+        for (int e = lane; e < d.dim; e += 64) {
+            const float z = d.low[(size_t)row * d.low_ld + d.low_a + h * d.dim + e] + d.dt_bias[h * d.dim + e];
+            const float sp = fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); /* softplus */
+            d.g[((size_t)row * d.heads + h) * d.dim + e] = expf(rate * sp);
+        }
+        if (lane == 0) d.beta[(size_t)row * d.heads + h] = tk_sigmoid32(proj[(size_t)row * ld + d.col + channels + h]);
+        return;
+    }
+    const int which = u < d.kv_heads ? 0 : u < 2 * d.kv_heads ? 1 : 2;
+    const int head = which == 2 ? u - 2 * d.kv_heads : which == 1 ? u - d.kv_heads : u;
+    const int n = which == 2 ? d.vdim : d.dim, c0 = which == 2 ? 2 * qk + head * d.vdim : which * qk + head * d.dim;
+    const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0, last = t.seg_n[seg] - 1;
+    const int in = t.seg_in[seg], hist = d.taps - 1;
+    /* input of channel c at time `s` of the segment; negative times are the state's */
+    auto input = [&](int c, int s) -> float {
+        if (s >= 0) return proj[(size_t)(row0 + s) * ld + d.col + c];
+        return in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
+    };
+    float v[4];
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e = lane + 64 * i;
+        v[i] = 0.0f;
+        if (e < n) {
+            const int c = c0 + e;
+            float y = 0.0f;
+            for (int j = 0; j < d.taps; ++j) y += d.conv[(size_t)c * d.taps + j] * input(c, at - hist + j);
+            v[i] = tk_silu32(y);
+            ss += v[i] * v[i];
+            if (at == last) {
+                float* out = d.conv_state + ((size_t)t.seg_out[seg] * channels + c) * hist;
+                for (int j = 0; j < hist; ++j) out[j] = input(c, at + 1 - hist + j);
+            }
+        }
+    }
+    float r = 1.0f;
+    if (which < 2) {
+        r = 1.0f / sqrtf(tk_wave_sum(ss) + d.unit_eps);
+        if (which == 0) r *= 1.0f / sqrtf((float)d.dim);
+    }
+    float* dst = which == 0 ? d.q + (size_t)row * qk + head * d.dim : which == 1 ? d.k + (size_t)row * qk + head * d.dim : d.v + ((size_t)row * d.heads + head) * d.vdim;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e = lane + 64 * i;
+        if (e < n) dst[e] = v[i] * r;
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_mixer_prep(const float* proj, int ld, TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int nd) {
+    const int row = blockIdx.y, lane = threadIdx.x & 63;
+    const int u = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
+    if (u < na) attn_unit<T>(a, t, proj + (size_t)row * ld, row, u, lane);
+    else if (u < na + nd) delta_unit(d, t, proj, ld, row, u - na, lane);
+}
+
+/* ------------------------------------------------------------------ attention -------------- */
+
+/* the pages a range of query positions [p0, p1] reads: the kept first ones, then the window's */
+struct PageWalk {
+    int nkeep, first, count;
+    __device__ __forceinline__ PageWalk(int p0, int p1, int window, int keep) {
+        const int lo = window > 0 && p0 - window + 1 > 0 ? p0 - window + 1 : 0;
+        first = lo / TK_PAGE;
+        const int k = keep < p1 + 1 ? keep : p1 + 1;
+        const int kp = (k + TK_PAGE - 1) / TK_PAGE;
+        nkeep = kp < first ? kp : first;
+        count = nkeep + p1 / TK_PAGE - first + 1;
+    }
+    __device__ __forceinline__ int page(int i) const { return i < nkeep ? i : first + i - nkeep; }
+};
+
+/* running softmax of one wave: 16 queries (lane % 16), VT 16-wide tiles of the output (rows 4 (lane / 16) + r) */
+template <typename T, int VT>
+struct Flash {
+    float m, l;
+    tk_v4f o[VT];
+    __device__ __forceinline__ void init() {
+        m = -INFINITY; l = 0.0f;
+#pragma unroll
+        for (int i = 0; i < VT; ++i) o[i] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+    /* s[j]: scores (log2 units) of keys 16 j + 4 g + r of this page; vfrag(vt, j): four values (keys 16 j + 4 g ..) of output column
+     * 16 vt + lane % 16.  The weights stay 32-bit: with bf16 values each weight enters as the sum of two bf16 numbers. */
+    template <typename VF>
+    __device__ __forceinline__ void update(const tk_v4f (&s)[4], int nv, VF vfrag) {
+        float mx = -INFINITY;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[j][r]);
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float mn = fmaxf(m, mx), ms = mn == -INFINITY ? 0.0f : mn;
+        const float al = __builtin_amdgcn_exp2f(m - ms);
+        m = mn;
+        tk_v4f p[4];
+        float sum = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) { p[j][r] = __builtin_amdgcn_exp2f(s[j][r] - ms); sum += p[j][r]; }
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        l = l * al + sum;
+#pragma unroll
+        for (int i = 0; i < VT; ++i) o[i] *= al;
+        accumulate(p, nv, vfrag);
+    }
+    template <typename VF>
+    __device__ __forceinline__ void accumulate(const tk_v4f (&p)[4], int nv, VF vfrag);
+};
+
+template <int VT, typename VF>
+__device__ __forceinline__ void flash_acc(Flash<TkBf16, VT>& f, const tk_v4f (&p)[4], int nv, VF vfrag) {
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+        tk_v4u hi, lo;
+#pragma unroll
+        for (int q = 0; q < 4; ++q) { /* pair q: elements 2 q, 2 q + 1 of [p[2h], p[2h + 1]] */
+            const float x = p[2 * h + (q >> 1)][2 * (q & 1)], y = p[2 * h + (q >> 1)][2 * (q & 1) + 1];
+            const uint16_t xh = tk_bf16_bits(x), yh = tk_bf16_bits(y);
+            hi[q] = (uint32_t)xh | (uint32_t)yh << 16;
+            lo[q] = (uint32_t)tk_bf16_bits(x - tk_bf16_float(xh)) | (uint32_t)tk_bf16_bits(y - tk_bf16_float(yh)) << 16;
+        }
+#pragma unroll
+        for (int i = 0; i < VT; ++i)
+            if (i < nv) {
+                const tk_v2u a = vfrag(i, 2 * h), b = vfrag(i, 2 * h + 1);
+                const tk_v4u v = {a[0], a[1], b[0], b[1]};
+                f.o[i] = TkImg<TkBf16>::mma(v, hi, f.o[i]);
+                f.o[i] = TkImg<TkBf16>::mma(v, lo, f.o[i]);
+            }
+    }
+}
+template <int VT, typename VF>
+__device__ __forceinline__ void flash_acc(Flash<float, VT>& f, const tk_v4f (&p)[4], int nv, VF vfrag) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < VT; ++i)
+            if (i < nv) f.o[i] = TkImg<float>::mma(vfrag(i, j), __builtin_bit_cast(tk_v4u, p[j]), f.o[i]);
+}
+template <typename T, int VT>
+template <typename VF>
+__device__ __forceinline__ void Flash<T, VT>::accumulate(const tk_v4f (&p)[4], int nv, VF vfrag) { flash_acc(*this, p, nv, vfrag); }
+
+/* four values of a transposed value row: 8 bytes (bf16) or 16 (f32) */
+template <typename T> struct VFrag;
+template <> struct VFrag<TkBf16> { typedef tk_v2u type; };
+template <> struct VFrag<float> { typedef tk_v4u type; };
+
+/* head h of `row`, columns 16 i + 4 g + r, times `f` */
+template <typename T, int VT>
+__device__ __forceinline__ void attn_store(const TkAttnArgs& a, const tk_v4f (&o)[VT], int64_t row, int h, int g, float f) {
+    const int k0 = a.out_k0 + h * a.vdim;
+#pragma unroll
+    for (int i = 0; i < VT; ++i) {
+        const int e = 16 * i + 4 * g;
+        if (e >= a.vdim) break;
+        const tk_v4f y = o[i] * f;
+        if ((k0 & 3) == 0 && e + 3 < a.vdim) tk_img_put4((T*)a.out_img, row, k0 + e, a.out_ktiles, y);
+        else
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                if (e + r < a.vdim) tk_img_put((T*)a.out_img, row, k0 + e + r, a.out_ktiles, y[r]);
+    }
+}
+
+/* prompts: 64 consecutive positions of a sequence x one head per workgroup, 16 per wave; pages go through LDS (next page's loads are in flight
+ * in registers while this one is used) */
+template <typename T, int B>
+__global__ __launch_bounds__(256) void k_attn_tiles(TkAttnArgs a, TkPassTab t, const int32_t* tiles) {
+    constexpr int DT = B / TkImg<T>::KT, VT = B / 16, SZ = sizeof(T);
+    typedef typename VFrag<T>::type VF;
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4;
+    const int row0 = tiles[2 * blockIdx.x], n = tiles[2 * blockIdx.x + 1], h = blockIdx.y, kvh = h / (a.heads / a.kv_heads);
+    const int nd = a.kv.dim_pad / TkImg<T>::KT, nv = a.kv.vdim_pad / 16;
+    const int krow = a.kv.dim_pad * SZ + 16, vrow = TK_PAGE * SZ + 16; /* LDS pitches: rows start in different banks */
+    uint8_t *lk = lds, *lv = lds + TK_PAGE * krow;
+    const int p0 = t.pos[row0], seq = t.seq[row0];
+    const int q = wave * 16 + (lane & 15), live = q < n ? q : 0;
+    const int pq = q < n ? p0 + q : -1; /* rows past the tile see nothing and store nothing */
+    tk_v4u qf[DT];
+#pragma unroll
+    for (int d = 0; d < DT; ++d)
+        if (d < nd) qf[d] = *(const tk_v4u*)((const uint8_t*)a.q + (((size_t)(row0 + live) * a.heads + h) * a.kv.dim_pad) * SZ + d * 64 + g * 16);
+    Flash<T, VT> f;
+    f.init();
+    const PageWalk walk(p0, p0 + n - 1, a.window, a.keep_first);
+    const int wave_lo = p0 + wave * 16, wave_hi = p0 + (wave * 16 + 15 < n ? wave * 16 + 15 : n - 1);
+    const int kc = TK_PAGE * a.kv.dim_pad * SZ / 16, vc = a.kv.vdim_pad * TK_PAGE * SZ / 16; /* 16-byte pieces of a page */
+    constexpr int KP = TK_PAGE * B * SZ / 16 / 256, VP = B * TK_PAGE * SZ / 16 / 256;
+    tk_v4u kr[KP], vr[VP];
+    auto fetch = [&](int i) {
+        const size_t page = (size_t)t.page_of[(size_t)seq * t.max_pages + walk.page(i)] * a.kv_heads + kvh;
+        const uint8_t* kp = (const uint8_t*)a.kv.k + page * TK_PAGE * a.kv.dim_pad * SZ;
+        const uint8_t* vp = (const uint8_t*)a.kv.v + page * a.kv.vdim_pad * TK_PAGE * SZ;
+#pragma unroll
+        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (p < kc) kr[c] = *(const tk_v4u*)(kp + (size_t)p * 16); }
+#pragma unroll
+        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (p < vc) vr[c] = *(const tk_v4u*)(vp + (size_t)p * 16); }
+    };
+    const int kpr = a.kv.dim_pad * SZ / 16, vpr = TK_PAGE * SZ / 16; /* pieces of a row */
+    fetch(0);
+    for (int i = 0; i < walk.count; ++i) {
+        __syncthreads();
+#pragma unroll
+        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (p < kc) *(tk_v4u*)(lk + (p / kpr) * krow + (p % kpr) * 16) = kr[c]; }
+#pragma unroll
+        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (p < vc) *(tk_v4u*)(lv + (p / vpr) * vrow + (p % vpr) * 16) = vr[c]; }
+        __syncthreads();
+        if (i + 1 < walk.count) fetch(i + 1);
+        const int k0 = walk.page(i) * TK_PAGE;
+        /* nothing of this page for this wave's rows */
+        if (wave * 16 >= n || k0 > wave_hi || (a.window > 0 && wave_lo - (k0 + TK_PAGE - 1) >= a.window && k0 >= a.keep_first)) continue;
+        tk_v4f s[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            s[j] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+            const uint8_t* kp = lk + (16 * j + (lane & 15)) * krow + g * 16;
+#pragma unroll
+            for (int d = 0; d < DT; ++d)
+                if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + d * 64), qf[d], s[j]);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int key = k0 + 16 * j + 4 * g + r;
+                const bool see = key <= pq && (a.window <= 0 || pq - key < a.window || key < a.keep_first);
+                s[j][r] = see ? s[j][r] * (a.scale * LOG2E) : -INFINITY;
+            }
+        }
+        f.update(s, nv, [&](int vt, int j) { return *(const VF*)(lv + (16 * vt + (lane & 15)) * vrow + (16 * j + 4 * g) * SZ); });
+    }
+    if (q < n) attn_store<T, VT>(a, f.o, row0 + q, h, g, a.out_scale / f.l);
+}
+
+/* decoding: one row x up to 16 query heads of one kv head per workgroup, pages dealt to the waves (and to `splits` workgroups), merged in LDS */
+template <typename T, int B>
+__global__ __launch_bounds__(256) void k_attn_rows(TkAttnArgs a, TkPassTab t, int splits, float* scratch) {
+    constexpr int DT = B / TkImg<T>::KT, VT = B / 16, SZ = sizeof(T);
+    typedef typename VFrag<T>::type VF;
+    __shared__ tk_v4f so[2][VT][64];
+    __shared__ float sm[2][64], sl[2][64];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4;
+    const int row = blockIdx.y, split = blockIdx.z, gq = a.heads / a.kv_heads, per = (gq + 15) / 16;
+    const int kvh = blockIdx.x / per, q = (blockIdx.x % per) * 16 + (lane & 15);
+    const int h = kvh * gq + (q < gq ? q : 0);
+    const int nd = a.kv.dim_pad / TkImg<T>::KT, nv = a.kv.vdim_pad / 16;
+    const int pos = t.pos[row], seq = t.seq[row];
+    tk_v4u qf[DT];
+#pragma unroll
+    for (int d = 0; d < DT; ++d)
+        if (d < nd) qf[d] = *(const tk_v4u*)((const uint8_t*)a.q + (((size_t)row * a.heads + h) * a.kv.dim_pad) * SZ + d * 64 + g * 16);
+    Flash<T, VT> f;
+    f.init();
+    const PageWalk walk(pos, pos, a.window, a.keep_first);
+    for (int i = split * 4 + wave; i < walk.count; i += 4 * splits) {
+        const size_t page = (size_t)t.page_of[(size_t)seq * t.max_pages + walk.page(i)] * a.kv_heads + kvh;
+        const uint8_t* kp = (const uint8_t*)a.kv.k + (page * TK_PAGE + (lane & 15)) * a.kv.dim_pad * SZ + g * 16;
+        const uint8_t* vp = (const uint8_t*)a.kv.v + (page * a.kv.vdim_pad + (lane & 15)) * TK_PAGE * SZ + 4 * g * SZ;
+        const int k0 = walk.page(i) * TK_PAGE;
+        tk_v4f s[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            s[j] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int d = 0; d < DT; ++d)
+                if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64), qf[d], s[j]);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int key = k0 + 16 * j + 4 * g + r;
+                const bool see = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+                s[j][r] = see ? s[j][r] * (a.scale * LOG2E) : -INFINITY;
+            }
+        }
+        f.update(s, nv, [&](int vt, int j) { return *(const VF*)(vp + ((size_t)16 * vt * TK_PAGE + 16 * j) * SZ); });
+    }
+    /* waves 2, 3 into 0, 1, then 1 into 0 */
+#pragma unroll
+    for (int half = 2; half >= 1; half >>= 1) {
+        if (wave >= half && wave < 2 * half) {
+#pragma unroll
+            for (int i = 0; i < VT; ++i) so[wave - half][i][lane] = f.o[i];
+            sm[wave - half][lane] = f.m; sl[wave - half][lane] = f.l;
+        }
+        __syncthreads();
+        if (wave < half) {
+            const float m2 = sm[wave][lane], mn = fmaxf(f.m, m2), ms = mn == -INFINITY ? 0.0f : mn;
+            const float c1 = __builtin_amdgcn_exp2f(f.m - ms), c2 = __builtin_amdgcn_exp2f(m2 - ms);
+            f.l = f.l * c1 + sl[wave][lane] * c2;
+            f.m = mn;
+#pragma unroll
+            for (int i = 0; i < VT; ++i) f.o[i] = f.o[i] * c1 + so[wave][i][lane] * c2;
+        }
+        __syncthreads();
+    }
+    if (wave != 0 || q >= gq) return;
+    if (splits == 1) { attn_store<T, VT>(a, f.o, row, h, g, a.out_scale / f.l); return; }
+    float* out = scratch + (((size_t)row * a.heads + h) * splits + split) * (a.kv.vdim_pad + 2);
+    if (g == 0) { out[0] = f.m; out[1] = f.l; }
+#pragma unroll
+    for (int i = 0; i < VT; ++i)
+        if (i < nv)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) out[2 + 16 * i + 4 * g + r] = f.o[i][r];
+}
+
+template <typename T>
+__global__ __launch_bounds__(64) void k_attn_merge(TkAttnArgs a, int splits, const float* scratch) {
+    const int h = blockIdx.x, row = blockIdx.y, pitch = a.kv.vdim_pad + 2;
+    const float* p = scratch + ((size_t)row * a.heads + h) * splits * pitch;
+    float m = -INFINITY;
+    for (int s = 0; s < splits; ++s) m = fmaxf(m, p[s * pitch]);
+    float l = 0.0f;
+    for (int s = 0; s < splits; ++s) l += p[s * pitch + 1] * __builtin_amdgcn_exp2f(p[s * pitch] - m);
+    const float f = a.out_scale / l;
+    for (int e = threadIdx.x; e < a.vdim; e += 64) {
+        float y = 0.0f;
+        for (int s = 0; s < splits; ++s) y += p[s * pitch + 2 + e] * __builtin_amdgcn_exp2f(p[s * pitch] - m);
+        tk_img_put((T*)a.out_img, row, a.out_k0 + h * a.vdim + e, a.out_ktiles, y * f);
+    }
+}
+
+/* ------------------------------------------------------------------ gated delta rule ------- */
+
+template <int CTRL> __device__ __forceinline__ float dpp_row(float v) { return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false)); }
+/* sum over the 16 lanes of a DPP row (row_ror 8, 4, 2, 1) */
+__device__ __forceinline__ float row16_sum(float v) {
+    v += dpp_row<0x128>(v);
+    v += dpp_row<0x124>(v);
+    v += dpp_row<0x122>(v);
+    v += dpp_row<0x121>(v);
+    return v;
+}
+
+/* A workgroup walks 16 columns of one head's state through a segment; a column is 16 lanes x RPL key rows, so the column's recurrence never
+ * leaves the wave.  q, k, decays, v and step sizes of TC tokens at a time go through LDS, the next TC in flight in registers. */
+template <int RPL>
+__global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) {
+    constexpr int DP = 16 * RPL, TC = RPL > 8 ? 8 : 16, NL = TC * DP / 256;
+    __shared__ __attribute__((aligned(16))) float lq[2][TC][DP], lk[2][TC][DP], lg[2][TC][DP];
+    __shared__ float lv[2][TC][16], lb[2][TC];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int h = blockIdx.y, seg = blockIdx.z, kvh = h / (d.heads / d.kv_heads), vp = (d.vdim + 3) & ~3;
+    const int row0 = t.seg_row0[seg], n = t.seg_n[seg], in = t.seg_in[seg], out = t.seg_out[seg];
+    const int cl = wave * 4 + (lane >> 4), col = blockIdx.x * 16 + cl, r0 = (lane & 15) * RPL;
+    const bool live = col < d.vdim;
+    float S[RPL];
+#pragma unroll
+    for (int i = 0; i < RPL; ++i)
+        S[i] = in >= 0 && live && r0 + i < d.dim ? d.state[(((size_t)in * d.heads + h) * d.dim + r0 + i) * vp + col] : 0.0f;
+    float rq[NL], rk[NL], rg[NL], rv = 0.0f, rb = 0.0f;
+    auto fetch = [&](int t0) {
+#pragma unroll
+        for (int i = 0; i < NL; ++i) {
+            const int idx = tid + 256 * i, tt = t0 + idx / DP, e = idx % DP;
+            const bool ok = tt < n && e < d.dim;
+            const size_t row = row0 + (ok ? tt : 0);
+            rq[i] = ok ? d.q[(row * d.kv_heads + kvh) * d.dim + e] : 0.0f;
+            rk[i] = ok ? d.k[(row * d.kv_heads + kvh) * d.dim + e] : 0.0f;
+            rg[i] = ok ? d.g[(row * d.heads + h) * d.dim + e] : 1.0f;
+        }
+        if (tid < TC * 16) {
+            const int tt = t0 + tid / 16, c = blockIdx.x * 16 + tid % 16;
+            rv = tt < n && c < d.vdim ? d.v[((size_t)(row0 + tt) * d.heads + h) * d.vdim + c] : 0.0f;
+            if (tid % 16 == 0) rb = tt < n ? d.beta[(size_t)(row0 + tt) * d.heads + h] : 0.0f;
+        }
+    };
+    auto put = [&](int b) {
+#pragma unroll
+        for (int i = 0; i < NL; ++i) {
+            const int idx = tid + 256 * i;
+            (&lq[b][0][0])[idx] = rq[i]; (&lk[b][0][0])[idx] = rk[i]; (&lg[b][0][0])[idx] = rg[i];
+        }
+        if (tid < TC * 16) { lv[b][tid / 16][tid % 16] = rv; if (tid % 16 == 0) lb[b][tid / 16] = rb; }
+    };
+    fetch(0);
+    put(0);
+    __syncthreads();
+    for (int t0 = 0, b = 0; t0 < n; t0 += TC, b ^= 1) {
+        if (t0 + TC < n) fetch(t0 + TC);
+        const int m = n - t0 < TC ? n - t0 : TC;
+        for (int i = 0; i < m; ++i) {
+            float sk = 0.0f;
+#pragma unroll
+            for (int e = 0; e < RPL; ++e) { S[e] *= lg[b][i][r0 + e]; sk += S[e] * lk[b][i][r0 + e]; }
+            sk = row16_sum(sk);
+            const float u = lb[b][i] * (lv[b][i][cl] - sk);
+            float so = 0.0f;
+#pragma unroll
+            for (int e = 0; e < RPL; ++e) { S[e] += lk[b][i][r0 + e] * u; so += S[e] * lq[b][i][r0 + e]; }
+            so = row16_sum(so);
+            if ((lane & 15) == 0 && live) d.o[((size_t)(row0 + t0 + i) * d.heads + h) * d.vdim + col] = so;
+        }
+        if (t0 + TC < n) put(b ^ 1); /* the other buffer was last read one iteration ago, before the barrier below */
+        __syncthreads();
+    }
+    if (live)
+#pragma unroll
+        for (int i = 0; i < RPL; ++i)
+            if (r0 + i < d.dim) d.state[(((size_t)out * d.heads + h) * d.dim + r0 + i) * vp + col] = S[i];
+}
+
+/* o over its root mean square, times the norm's weight, times the gate: one wave per (row, head) */
+template <typename T>
+__global__ __launch_bounds__(256) void k_delta_out(TkDeltaArgs d) {
+    const int lane = threadIdx.x & 63, h = blockIdx.x * 4 + (threadIdx.x >> 6), row = blockIdx.y;
+    if (h >= d.heads) return;
+    const float* o = d.o + ((size_t)row * d.heads + h) * d.vdim;
+    float v[4], ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { const int e = lane + 64 * i; v[i] = e < d.vdim ? o[e] : 0.0f; ss += v[i] * v[i]; }
+    const float r = 1.0f / sqrtf(tk_wave_sum(ss) / (float)d.vdim + d.eps);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e = lane + 64 * i;
+        if (e >= d.vdim) break;
+        const float gate = tk_sigmoid32(d.low[(size_t)row * d.low_ld + d.low_g + h * d.vdim + e]);
+        tk_img_put((T*)d.out_img, row, d.out_k0 + h * d.vdim + e, d.out_ktiles, v[i] * r * d.norm[e] * gate * d.out_scale);
+    }
+}
+
+/* one token of one head: the state is read once and written once, a thread holds RPT rows x 4 columns of it.
+ * o = S_new^T q = (g S)^T q + (k . q) u, so both reductions over the key rows run on the decayed old state at once. */
+template <typename T, int THREADS, int RPT>
+__global__ __launch_bounds__(THREADS) void k_delta_step(TkDeltaArgs d, TkPassTab t, int ct_log2) {
+    extern __shared__ __attribute__((aligned(16))) float step_lds[];
+    __shared__ float red[16];
+    const int tid = threadIdx.x, row = blockIdx.y, h = blockIdx.x, kvh = h / (d.heads / d.kv_heads), vp = (d.vdim + 3) & ~3;
+    const int ct = tid & ((1 << ct_log2) - 1), rg = tid >> ct_log2, RG = THREADS >> ct_log2;
+    const bool live = 4 * ct < vp;
+    const int seg = t.seg[row], in = t.seg_in[seg], out = t.seg_out[seg];
+    float *lq = step_lds, *lk = lq + d.dim, *lg = lk + d.dim, *lu = step_lds + (3 * d.dim + 3) / 4 * 4, *pk = lu + vp, *pq = pk + RG * vp;
+    tk_v4f S[RPT];
+    const float* sin = d.state + ((size_t)(in < 0 ? 0 : in) * d.heads + h) * d.dim * vp + 4 * ct;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int e = rg + RG * i;
+        S[i] = in >= 0 && live && e < d.dim ? *(const tk_v4f*)(sin + (size_t)e * vp) : tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+    float kq = 0.0f;
+    for (int e = tid; e < d.dim; e += THREADS) {
+        const float q = d.q[((size_t)row * d.kv_heads + kvh) * d.dim + e], k = d.k[((size_t)row * d.kv_heads + kvh) * d.dim + e];
+        lq[e] = q; lk[e] = k; lg[e] = d.g[((size_t)row * d.heads + h) * d.dim + e];
+        kq += q * k;
+    }
+    kq = block_sum(kq, red); /* also orders the LDS writes above before the reads below */
+    tk_v4f ak = {0.0f, 0.0f, 0.0f, 0.0f}, aq = ak;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int e = rg + RG * i;
+        if (e < d.dim) { S[i] *= lg[e]; ak += S[i] * lk[e]; aq += S[i] * lq[e]; }
+    }
+    if (live) { *(tk_v4f*)(pk + rg * vp + 4 * ct) = ak; *(tk_v4f*)(pq + rg * vp + 4 * ct) = aq; }
+    __syncthreads();
+    const float beta = d.beta[(size_t)row * d.heads + h];
+    float o = 0.0f, ss = 0.0f;
+    if (tid < vp) { /* vdim <= 256 <= THREADS: one column per thread */
+        float sk = 0.0f, sq = 0.0f;
+        for (int i = 0; i < RG; ++i) { sk += pk[i * vp + tid]; sq += pq[i * vp + tid]; }
+        const float v = tid < d.vdim ? d.v[((size_t)row * d.heads + h) * d.vdim + tid] : 0.0f;
+        const float u = tid < d.vdim ? beta * (v - sk) : 0.0f;
+        lu[tid] = u;
+        o = tid < d.vdim ? sq + kq * u : 0.0f;
+        ss = o * o;
+    }
+    ss = block_sum(ss, red);
+    if (live) {
+        const tk_v4f u = *(const tk_v4f*)(lu + 4 * ct);
+        float* so = d.state + ((size_t)out * d.heads + h) * d.dim * vp + 4 * ct;
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) {
+            const int e = rg + RG * i;
+            if (e < d.dim) *(tk_v4f*)(so + (size_t)e * vp) = S[i] + u * lk[e];
+        }
+    }
+    if (tid < d.vdim) {
+        const float r = 1.0f / sqrtf(ss / (float)d.vdim + d.eps);
+        const float gate = tk_sigmoid32(d.low[(size_t)row * d.low_ld + d.low_g + h * d.vdim + tid]);
+        tk_img_put((T*)d.out_img, row, d.out_k0 + h * d.vdim + tid, d.out_ktiles, o * r * d.norm[tid] * gate * d.out_scale);
+    }
+}
+
+__global__ void k_swap_state(TkPassTab t, int n) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) { const int o = t.seg_out[i]; t.seg_in[i] = o; t.seg_out[i] = o ^ 1; }
+}
+
+/* ------------------------------------------------------------------ mixture of experts ----- */
+
+__global__ __launch_bounds__(64) void k_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, TkMoeTab t) {
+    __shared__ float sc[TK_MAX_EXPERTS], gs[64];
+    __shared__ int on[64];
+    const int row = blockIdx.x, lane = threadIdx.x, per = experts / groups;
+    for (int e = lane; e < experts; e += 64) sc[e] = tk_sigmoid32(logits[(size_t)row * ld + e]);
+    __syncthreads();
+    if (lane < groups) { /* a group's score: the sum of its two best */
+        float a = -INFINITY, b = -INFINITY;
+        for (int e = lane * per; e < (lane + 1) * per; ++e) {
+            const float v = sc[e];
+            if (v > a) { b = a; a = v; } else if (v > b) b = v;
+        }
+        gs[lane] = per > 1 ? a + b : a;
+    }
+    __syncthreads();
+    if (lane < groups) {
+        int better = 0;
+        for (int j = 0; j < groups; ++j) better += gs[j] > gs[lane] || (gs[j] == gs[lane] && j < lane);
+        on[lane] = better < keep;
+    }
+    __syncthreads();
+    float c[TK_MAX_EXPERTS / 64]; /* this lane's candidates */
+#pragma unroll
+    for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i) {
+        const int e = lane + 64 * i;
+        c[i] = e < experts && on[e / per] ? sc[e] : -INFINITY;
+    }
+    for (int j = 0; j < top; ++j) {
+        float best = -INFINITY;
+        int id = 0x7fffffff;
+#pragma unroll
+        for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
+            if (c[i] > best) { best = c[i]; id = lane + 64 * i; }
+        for (int s = 32; s >= 1; s >>= 1) {
+            const float ov = __shfl_xor(best, s, 64);
+            const int oi = __shfl_xor(id, s, 64);
+            if (ov > best || (ov == best && oi < id)) { best = ov; id = oi; }
+        }
+        if (id >= experts) id = 0; /* no finite score is left: a defined expert all the same */
+#pragma unroll
+        for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
+            if (lane + 64 * i == id) c[i] = -INFINITY;
+        if (lane == 0) {
+            t.expert[row * top + j] = id;
+            t.weight[row * top + j] = sc[id];
+            t.rank[row * top + j] = atomicAdd(t.count + id, 1);
+        }
+    }
+}
+
+/* experts' row counts -> first tiles and row blocks; the counts are cleared for the next layer */
+__global__ __launch_bounds__(256) void k_moe_plan(int experts, int block_tiles, TkMoeTab t) {
+    __shared__ int st[256], sb[256];
+    const int e = threadIdx.x;
+    const int tiles = e < experts ? (t.count[e] + 15) / 16 : 0, nb = (tiles + block_tiles - 1) / block_tiles;
+    st[e] = tiles; sb[e] = nb;
+    __syncthreads();
+    for (int s = 1; s < 256; s <<= 1) { /* inclusive sums */
+        const int a = e >= s ? st[e - s] : 0, b = e >= s ? sb[e - s] : 0;
+        __syncthreads();
+        st[e] += a; sb[e] += b;
+        __syncthreads();
+    }
+    const int tile0 = st[e] - tiles, b0 = sb[e] - nb;
+    if (e < experts) {
+        t.tile0[e] = tile0;
+        t.count[e] = 0;
+        for (int i = 0; i < nb; ++i) {
+            const int left = tiles - i * block_tiles;
+            t.blocks[b0 + i] = TkImgBlock{e, tile0 + i * block_tiles, left < block_tiles ? left : block_tiles, 0};
+        }
+    }
+    if (e == 255) *t.n_blocks = sb[255];
+}
+
+/* 16-byte pieces of a row of the image to its places among the experts' rows */
+__global__ __launch_bounds__(256) void k_moe_gather(const tk_v4u* img, tk_v4u* out, int ktiles, int top, TkMoeTab t) {
+    const int i = blockIdx.x, row = i / top;
+    const int slot = t.tile0[t.expert[i]] * 16 + t.rank[i];
+    if (blockIdx.y == 0 && threadIdx.x == 0) t.slot[i] = slot;
+    const int p = blockIdx.y * 256 + threadIdx.x; /* piece: k tile p / 4, lane group p % 4 */
+    if (p >= ktiles * 4) return;
+    out[((size_t)(slot >> 4) * ktiles + p / 4) * 64 + (slot & 15) + 16 * (p % 4)] = img[((size_t)(row >> 4) * ktiles + p / 4) * 64 + (row & 15) + 16 * (p % 4)];
+}
+
+} // namespace
+
+/* ------------------------------------------------------------------ launchers -------------- */
+
+#define TK_TYPED(type, ...) do { if ((type) == TK_IMG_F32) { typedef float T; __VA_ARGS__; } else { typedef TkBf16 T; __VA_ARGS__; } } while (0)
+
+void tk_launch_layer_embed(int type, const uint16_t* table, int width, const int32_t* tok, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, hipLaunchKernelGGL((k_layer_embed<T>), dim3(nrows), dim3(256), 0, s, table, width, tok, x, (T*)img, ktiles));
+}
+
+void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs* attn, const TkDeltaArgs* delta, const TkPassTab& t, int nrows, hipStream_t s) {
+    const TkAttnArgs a = attn ? *attn : TkAttnArgs{};
+    const TkDeltaArgs d = delta ? *delta : TkDeltaArgs{};
+    const int na = attn ? a.heads + 2 * a.kv_heads : 0, nd = delta ? 2 * d.kv_heads + 2 * d.heads : 0;
+    TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T>), dim3((na + nd + 3) / 4, nrows), dim3(256), 0, s, proj, ld, a, d, t, na, nd));
+}
+
+static int attn_bucket(const TkAttnArgs& a) {
+    const int m = a.kv.dim_pad > a.kv.vdim_pad ? a.kv.dim_pad : a.kv.vdim_pad;
+    return m <= 64 ? 64 : m <= 128 ? 128 : 256;
+}
+
+void tk_launch_attn_tiles(int type, const TkAttnArgs& a, const TkPassTab& t, const int32_t* tiles, int n_tiles, hipStream_t s) {
+    const int b = attn_bucket(a);
+    TK_TYPED(type, {
+        const size_t lds = (size_t)TK_PAGE * (a.kv.dim_pad * sizeof(T) + 16) + (size_t)a.kv.vdim_pad * (TK_PAGE * sizeof(T) + 16);
+        const dim3 grid(n_tiles, a.heads);
+        if (b == 64) hipLaunchKernelGGL((k_attn_tiles<T, 64>), grid, dim3(256), lds, s, a, t, tiles);
+        else if (b == 128) hipLaunchKernelGGL((k_attn_tiles<T, 128>), grid, dim3(256), lds, s, a, t, tiles);
+        else hipLaunchKernelGGL((k_attn_tiles<T, 256>), grid, dim3(256), lds, s, a, t, tiles);
+    });
+}
+
+size_t tk_attn_rows_scratch_floats(const TkAttnArgs& a, int nrows, int splits) { return splits > 1 ? (size_t)nrows * a.heads * splits * (a.kv.vdim_pad + 2) : 0; }
+
+void tk_launch_attn_rows(int type, const TkAttnArgs& a, const TkPassTab& t, int nrows, int splits, float* scratch, hipStream_t s) {
+    const int b = attn_bucket(a), gq = a.heads / a.kv_heads;
+    TK_TYPED(type, {
+        const dim3 grid(a.kv_heads * ((gq + 15) / 16), nrows, splits);
+        if (b == 64) hipLaunchKernelGGL((k_attn_rows<T, 64>), grid, dim3(256), 0, s, a, t, splits, scratch);
+        else if (b == 128) hipLaunchKernelGGL((k_attn_rows<T, 128>), grid, dim3(256), 0, s, a, t, splits, scratch);
+        else hipLaunchKernelGGL((k_attn_rows<T, 256>), grid, dim3(256), 0, s, a, t, splits, scratch);
+        if (splits > 1) hipLaunchKernelGGL((k_attn_merge<T>), dim3(a.heads, nrows), dim3(64), 0, s, a, splits, scratch);
+    });
+}
+
+void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, int n_segments, int nrows, hipStream_t s) {
+    const dim3 grid((d.vdim + 15) / 16, d.heads, n_segments);
+    const int rpl = (d.dim + 15) / 16;
+    if (rpl <= 2) hipLaunchKernelGGL((k_delta_scan<2>), grid, dim3(256), 0, s, d, t);
+    else if (rpl <= 4) hipLaunchKernelGGL((k_delta_scan<4>), grid, dim3(256), 0, s, d, t);
+    else if (rpl <= 8) hipLaunchKernelGGL((k_delta_scan<8>), grid, dim3(256), 0, s, d, t);
+    else hipLaunchKernelGGL((k_delta_scan<16>), grid, dim3(256), 0, s, d, t);
+    TK_TYPED(type, hipLaunchKernelGGL((k_delta_out<T>), dim3((d.heads + 3) / 4, nrows), dim3(256), 0, s, d));
+}
+
+void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s) {
+    const int vp = (d.vdim + 3) & ~3;
+    int ctl = 0;
+    while ((4 << ctl) < vp) ++ctl;
+    const dim3 grid(d.heads, nrows);
+    auto rpt = [&](int threads) { const int rg = threads >> ctl; return (d.dim + rg - 1) / rg; };
+    auto lds = [&](int threads) { return ((size_t)(3 * d.dim + 3) / 4 * 4 + vp + 2 * (size_t)(threads >> ctl) * vp) * sizeof(float); };
+    TK_TYPED(type, {
+        if (rpt(256) <= 4) hipLaunchKernelGGL((k_delta_step<T, 256, 4>), grid, dim3(256), lds(256), s, d, t, ctl);
+        else if (rpt(256) <= 8) hipLaunchKernelGGL((k_delta_step<T, 256, 8>), grid, dim3(256), lds(256), s, d, t, ctl);
+        else if (rpt(256) <= 16) hipLaunchKernelGGL((k_delta_step<T, 256, 16>), grid, dim3(256), lds(256), s, d, t, ctl);
+        else if (rpt(256) <= 32) hipLaunchKernelGGL((k_delta_step<T, 256, 32>), grid, dim3(256), lds(256), s, d, t, ctl);
+        else hipLaunchKernelGGL((k_delta_step<T, 1024, 16>), grid, dim3(1024), lds(1024), s, d, t, ctl);
+    });
+}
+
+void tk_launch_post_norm(int type, const TkSubOut& o, const float* w, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, hipLaunchKernelGGL((k_post_norm<T>), dim3(nrows), dim3(256), (size_t)width * sizeof(float), s, o, w, eps, width, x, (T*)img, ktiles));
+}
+
+void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const float* w, float eps, int width, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, hipLaunchKernelGGL((k_rows_norm<T>), dim3(n), dim3(256), 0, s, x, rows, w, eps, width, (T*)img, ktiles));
+}
+
+void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, const TkMoeTab& t, hipStream_t s) {
+    hipLaunchKernelGGL(k_moe_select, dim3(nrows), dim3(64), 0, s, logits, ld, experts, top, groups, keep, t);
+}
+void tk_launch_moe_plan(int experts, int block_tiles, const TkMoeTab& t, hipStream_t s) { hipLaunchKernelGGL(k_moe_plan, dim3(1), dim3(256), 0, s, experts, block_tiles, t); }
+void tk_launch_moe_gather(const void* img, void* gathered, int ktiles, int top, int nrows, const TkMoeTab& t, hipStream_t s) {
+    hipLaunchKernelGGL(k_moe_gather, dim3(nrows * top, (ktiles * 4 + 255) / 256), dim3(256), 0, s, (const tk_v4u*)img, (tk_v4u*)gathered, ktiles, top, t);
+}
+void tk_launch_swap_state(const TkPassTab& t, int n, hipStream_t s) { hipLaunchKernelGGL(k_swap_state, dim3((n + 255) / 256), dim3(256), 0, s, t, n); }
+
+const char* tk_mixer_prepare_device() {
+    static std::atomic<bool> done[64];
+    static std::mutex mu;
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return "no current device";
+    if (done[dev].load(std::memory_order_acquire)) return nullptr;
+    std::lock_guard<std::mutex> lk(mu);
+    hipError_t e = hipSuccess;
+    auto opt = [&](const void* f) { if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); };
+    opt((const void*)k_attn_tiles<float, 64>); opt((const void*)k_attn_tiles<float, 128>); opt((const void*)k_attn_tiles<float, 256>);
+    opt((const void*)k_attn_tiles<TkBf16, 64>); opt((const void*)k_attn_tiles<TkBf16, 128>); opt((const void*)k_attn_tiles<TkBf16, 256>);
+    if (e != hipSuccess) return hipGetErrorString(e);
+    done[dev].store(true, std::memory_order_release);
+    return nullptr;
+}

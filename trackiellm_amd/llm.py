@@ -1,5 +1,7 @@
 """LLM stream: tk_model_loader_* / tk_llm_runner_* and the batched tk_mi355x_llm_* extension."""
 import ctypes as C
+import json
+import os
 
 import numpy as np
 
@@ -51,10 +53,24 @@ def _p(a):
     return a.ctypes.data_as(C.c_void_p) if a is not None else None
 
 
+def config_check(config):
+    """raises TkError with the reason when this build does not serve a layer-list configuration (dict or JSON text); no GPU involved"""
+    text = config if isinstance(config, str) else json.dumps(config)
+    check(lib().tk_mi355x_llm_config_check(text.encode()))
+
+
 class LlmModel:
-    def __init__(self, hparams=None, device=0, gguf=None, lora=None):
+    """hparams: a Mistral-class geometry (weights set later); gguf: a checkpoint file; folder: config.json + model.safetensors of a design
+    described layer by layer; config: such a description (dict or JSON text) with random weights"""
+
+    def __init__(self, hparams=None, device=0, gguf=None, lora=None, folder=None, config=None, dtype="bfloat16", seed=1, gate_rank=64):
         self.h = C.c_void_p()
-        if gguf is not None:
+        if folder is not None:
+            check(lib().tk_mi355x_llm_model_load_dir(C.byref(self.h), os.fspath(folder).encode(), dtype.encode(), device))
+        elif config is not None:
+            text = config if isinstance(config, str) else json.dumps(config)
+            check(lib().tk_mi355x_llm_model_create_layered(C.byref(self.h), text.encode(), dtype.encode(), device, C.c_uint64(seed), gate_rank))
+        elif gguf is not None:
             check(lib().tk_mi355x_llm_model_load_gguf_lora(C.byref(self.h), gguf.encode(), lora.encode() if lora else None, device))
         else:
             check(lib().tk_mi355x_llm_model_create(C.byref(self.h), C.byref(hparams), device))
@@ -101,11 +117,42 @@ class LlmModel:
 
 
 class LlmSession:
-    def __init__(self, model, max_seq, max_ctx):
+    """pool_tokens: positions all live sequences hold together, for models with a paged cache (0: max_seq x max_ctx)"""
+
+    def __init__(self, model, max_seq, max_ctx, pool_tokens=0):
         self.model = model
-        self.vocab = model.hparams.vocab
+        hp = model.hparams
+        self.vocab, self.n_layer, self.width = hp.vocab, hp.n_layer, hp.d_model
         self.h = C.c_void_p()
-        check(lib().tk_mi355x_llm_session_create(C.byref(self.h), model.h, max_seq, max_ctx))
+        check(lib().tk_mi355x_llm_session_create_pool(C.byref(self.h), model.h, max_seq, max_ctx, pool_tokens))
+
+    def forward_rows(self, seq, pos, tok, out_rows, want_logits=True, want_ids=False):
+        """one pass; (logits [n_out][vocab] or None, ids [n_out] or None) of the wanted rows (ascending)"""
+        seq, pos, tok, rows = (np.ascontiguousarray(a, dtype=np.int32) for a in (seq, pos, tok, out_rows))
+        logits = np.empty((len(rows), self.vocab), dtype=np.float32) if want_logits else None
+        ids = np.empty(len(rows), dtype=np.int32) if want_ids else None
+        check(lib().tk_mi355x_llm_forward_rows(self.h, len(seq), _p(seq), _p(pos), _p(tok), len(rows), _p(rows), _p(logits), _p(ids)))
+        return logits, ids
+
+    def forward_streams(self, seq, pos, tok):
+        """one pass; the residual stream after every layer [layers][rows][width]"""
+        seq, pos, tok = (np.ascontiguousarray(a, dtype=np.int32) for a in (seq, pos, tok))
+        out = np.empty((self.n_layer, len(seq), self.width), dtype=np.float32)
+        check(lib().tk_mi355x_llm_forward_streams(self.h, len(seq), _p(seq), _p(pos), _p(tok), _p(out)))
+        return out
+
+    def release(self, seq):
+        check(lib().tk_mi355x_llm_session_release(self.h, seq))
+
+    def cache_usage(self):
+        """(pages in use, pages) of a paged cache"""
+        u, t = C.c_int32(0), C.c_int32(0)
+        lib().tk_mi355x_llm_session_cache_usage(self.h, C.byref(u), C.byref(t))
+        return u.value, t.value
+
+    @property
+    def row_capacity(self):
+        return lib().tk_mi355x_llm_session_row_capacity(self.h)
 
     def forward(self, seq, pos, tok, want_logits=True):
         seq = np.ascontiguousarray(seq, dtype=np.int32)
@@ -340,6 +387,16 @@ class LlmRunner:
 
     def prepare(self, prompt, use_tool_grammar=False):
         check(lib().tk_llm_runner_prepare_generation(self.h, prompt.encode(), use_tool_grammar))
+
+    def prepare_ids(self, ids):
+        """prepare() on token ids, for models without a vocabulary"""
+        ids = np.ascontiguousarray(ids, dtype=np.int32)
+        check(lib().tk_mi355x_llm_runner_prepare_ids(self.h, _p(ids), len(ids)))
+
+    @property
+    def pending_id(self):
+        """the id whose text the next next_token() returns, -1 when there is none"""
+        return lib().tk_mi355x_llm_runner_pending_id(self.h)
 
     def set_sampling(self, temperature, top_k=40, top_p=0.95, min_p=0.05):
         """the reference's default stochastic chain (llama_sampling_default_params) instead of greedy; temperature 0 = greedy again"""
