@@ -652,8 +652,77 @@ def hp_weight_bytes(tk, handle):
 COLL_CUDA = True  # collectives on device tensors (RCCL); False in the one-GPU rehearsal (gloo)
 
 
+def layered_config(width, n_layer, attn, delta, mlp, vocab=32000):
+    """a Vuvulorn configuration whose layers are all alike"""
+    layer = {"type": "parallel", "mixer": {"left": attn, "right": delta, "left_scale": 1.0, "right_scale": 1.0}, "mlp": mlp}
+    return {"architecture": "Vuvulorn", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": [layer] * n_layer}
+
+
+def layered_sizes():
+    """name -> (configuration, Mistral-class geometry of the same width, depth and active feed-forward)"""
+    from trackiellm_amd import LlmHParams
+
+    def attn(heads, kv, window):
+        return {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "rot": {"dims": 64, "base": 10000.0}, "scale": 128 ** -0.5, "mask": {"size": window, "keep_first": 4}}
+
+    def delta(heads):
+        return {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}
+    moe = {"kind": "moe", "expert": {"ff": 1024}, "router": {"experts": 64, "top": 8, "groups": {"count": 8, "keep": 4}}}
+    return {"dense-4096": (layered_config(4096, 4, attn(16, 4, 1024), delta(16), {"kind": "dense", "ff": 14336}),
+                           LlmHParams(4, 4096, 32, 8, 128, 14336, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1)),
+            "dense-2048": (layered_config(2048, 8, attn(8, 2, 512), delta(8), {"kind": "dense", "ff": 8192}),
+                           LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1)),
+            "moe-2048": (layered_config(2048, 8, attn(8, 2, 512), delta(8), moe), LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1))}
+
+
+def layered_point(tk, model, prompts, batches, context, steps):
+    """prompt processing (one sequence) and decoding (`batch` sequences at `context` cached positions) of one model"""
+    hp, rng = model.hparams, np.random.default_rng(5)
+    out = {"step_weight_mb": round(model.weight_bytes / 1e6, 1), "prefill": [], "decode": []}
+    for n in prompts:
+        sess = tk.LlmSession(model, 1, n + 8)
+        toks = rng.integers(3, hp.vocab, (1, n)).astype(np.int32)
+        best = 1e9
+        for i in range(4):
+            t0 = time.perf_counter()
+            sess.prefill(toks)
+            best = min(best, time.perf_counter() - t0) if i else best
+        out["prefill"].append({"prompt_tokens": n, "ms": round(1e3 * best, 3), "tok_per_s": round(n / best)})
+        sess.close()
+    for b in batches:
+        sess = tk.LlmSession(model, b, context + 3 * steps + 8)
+        sess.prefill(rng.integers(3, hp.vocab, (b, context)).astype(np.int32))
+        sess.decode(b, steps)
+        ms = min(sess.decode(b, steps)[1] for _ in range(2))
+        out["decode"].append({"batch": b, "context": context, "ms_per_step": round(ms, 3), "tok_per_s": round(1e3 * b / ms)})
+        sess.close()
+    return out
+
+
+def run_layered(args, tk, device):
+    """--layered: the layer-list decoders at sizes that resemble a real model's layers, random weights, beside the Mistral-class model of the same
+    width, depth and active feed-forward (its fp16 and its Q4_K_M checkpoints)"""
+    prompts, batches = (512, 2048), (1, 16, 64, 256)
+    res = {}
+    for name, (cfg, hp) in layered_sizes().items():
+        if args.layered not in ("all", name):
+            continue
+        m = tk.LlmModel(config=cfg, device=device, gate_rank=128)
+        res[name] = {"layered_bf16": layered_point(tk, m, prompts, batches, 512, 24)}
+        m.close()
+        if not args.layered_only:
+            for tag, f16 in (("mistral_f16", True), ("mistral_q4_k_m", False)):
+                m = tk.LlmModel(hp, device=device).fill_synthetic(4, f16=f16)
+                res[name][tag] = layered_point(tk, m, prompts, batches, 512, 24)
+                m.close()
+    print(json.dumps({"metric": "layer-list decoder throughput", "data": "synthetic", "dtype": "bf16", "sizes": res}))
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--layered", default="", choices=["", "all"] + ["dense-4096", "dense-2048", "moe-2048"],
+                    help="instead of the headline: prefill and decode throughput of the layer-list decoders (Vuvulorn) beside the Mistral-class model of equal size; one JSON line of its own")
+    ap.add_argument("--layered-only", action="store_true", help="with --layered: leave the Mistral-class models out (profiling)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
@@ -716,6 +785,8 @@ def main():
         raise SystemExit("bench.py needs one MI355X per rank: no fallback path exists")
     tk.lib().tk_mi355x_set_default_device(local_rank)
 
+    if args.layered:
+        return run_layered(args, tk, local_rank)
     B, P, N = args.batch, args.prompt, args.decode
     G = max(1, args.sessions)
     if args.pipe_rccl:

@@ -118,7 +118,8 @@ private:
     bool alloc(void** p, size_t bytes, bool zero = false);
     bool describe(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, Pass* p);
     void commit(int nrows, const int32_t* seq, const int32_t* pos);
-    bool need_pages(Seq& s, int seq, int last_pos);
+    void need_pages(Seq& s, int seq, int last_pos);
+    void give_back(Seq& s);
     bool upload_pages();
     void gemm(const TkImgGemm& g);
     void enqueue_layers(const Pass& p);

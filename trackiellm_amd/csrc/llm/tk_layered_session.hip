@@ -152,7 +152,7 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
 }
 
 TkLayeredSession::~TkLayeredSession() {
-    if (m_) (void)hipSetDevice(m_->device);
+    (void)hipSetDevice(device_); /* the model may be gone already */
     if (stream) (void)hipStreamSynchronize(stream);
     for (auto& g : graphs_) if (g) (void)hipGraphExecDestroy(g);
     for (void* p : owned_) (void)hipFree(p);
@@ -164,7 +164,10 @@ TkLayeredSession::~TkLayeredSession() {
 void TkLayeredSession::release_sequence(int seq) {
     std::lock_guard<std::mutex> lk(mu_);
     if (seq < 0 || seq >= max_seq) return;
-    Seq& s = seqs_[(size_t)seq];
+    give_back(seqs_[(size_t)seq]);
+}
+
+void TkLayeredSession::give_back(Seq& s) {
     for (auto it = s.pages.rbegin(); it != s.pages.rend(); ++it) free_pages_.push_back(*it);
     s.pages.clear();
     s.len = 0;
@@ -177,16 +180,15 @@ void TkLayeredSession::cache_usage(int* used, int* total) {
     *used = n_pages_ - (int)free_pages_.size();
 }
 
-bool TkLayeredSession::need_pages(Seq& s, int seq, int last_pos) {
+/* the caller has made sure that the pool has them */
+void TkLayeredSession::need_pages(Seq& s, int seq, int last_pos) {
     const size_t want = (size_t)last_pos / TK_PAGE + 1;
     while (s.pages.size() < want) {
-        if (free_pages_.empty()) { error = "cache pool exhausted: " + std::to_string(n_pages_) + " pages of " + std::to_string(TK_PAGE) + " positions are in use"; return false; }
         h_pages_[(size_t)seq * max_pages_ + s.pages.size()] = free_pages_.back();
         s.pages.push_back(free_pages_.back());
         free_pages_.pop_back();
         pages_dirty_ = true;
     }
-    return true;
 }
 
 bool TkLayeredSession::upload_pages() {
@@ -201,27 +203,37 @@ bool TkLayeredSession::describe(int nrows, const int32_t* seq, const int32_t* po
     const int R = row_cap_;
     int32_t *h_seq = h_tab_, *h_pos = h_seq + R, *h_tok = h_pos + R, *h_seg = h_tok + R, *row0 = h_seg + R, *sn = row0 + max_seq, *sin = sn + max_seq, *sout = sin + max_seq,
             *tiles = sout + max_seq + R;
-    std::vector<char> seen((size_t)max_seq, 0);
     p->nrows = nrows; p->nseg = 0; p->ntiles = 0; p->single = true;
+    /* first whether the rows are allowed at all, with nothing changed */
+    struct Run { int r, n, side; };
+    std::vector<Run> runs;
+    std::vector<char> seen((size_t)max_seq, 0);
     for (int r = 0; r < nrows;) {
         int n = 1;
         while (r + n < nrows && seq[r + n] == seq[r] && pos[r + n] == pos[r] + n) ++n;
         const int id = seq[r];
-        Seq& s = seqs_[(size_t)id];
+        const Seq& s = seqs_[(size_t)id];
         if (seen[(size_t)id]) { error = "the rows of a sequence must be one run of consecutive positions"; return false; }
         seen[(size_t)id] = 1;
-        int side = s.side;
-        if (pos[r] == 0) { /* a new sequence in this slot */
-            for (auto it = s.pages.rbegin(); it != s.pages.rend(); ++it) free_pages_.push_back(*it);
-            s.pages.clear();
-            s.len = 0; s.prev = -1;
-        } else if (pos[r] == s.prev) {
-            side ^= 1; /* the sequence's last pass is taken back */
-        } else if (pos[r] != s.len) {
+        if (pos[r] != 0 && pos[r] != s.prev && pos[r] != s.len) {
             error = "sequence " + std::to_string(id) + " stands at position " + std::to_string(s.len) + ": its rows must continue there or start at 0";
             return false;
         }
-        if (!need_pages(s, id, pos[r] + n - 1)) return false;
+        /* a run at the position where the sequence's last pass began takes that pass back */
+        runs.push_back(Run{r, n, pos[r] != 0 && pos[r] == s.prev ? s.side ^ 1 : s.side});
+        r += n;
+    }
+    for (const Run& u : runs)
+        if (pos[u.r] == 0) give_back(seqs_[(size_t)seq[u.r]]); /* a new sequence in this slot */
+    size_t need = 0;
+    for (const Run& u : runs) {
+        const size_t want = (size_t)(pos[u.r] + u.n - 1) / TK_PAGE + 1, have = seqs_[(size_t)seq[u.r]].pages.size();
+        need += want > have ? want - have : 0;
+    }
+    if (need > free_pages_.size()) { error = "cache pool exhausted: " + std::to_string(need) + " more pages wanted, " + std::to_string(free_pages_.size()) + " of " + std::to_string(n_pages_) + " are free"; return false; }
+    for (const Run& u : runs) {
+        const int r = u.r, n = u.n, id = seq[r], side = u.side;
+        need_pages(seqs_[(size_t)id], id, pos[r] + n - 1);
         row0[p->nseg] = r; sn[p->nseg] = n;
         sin[p->nseg] = pos[r] == 0 ? -1 : 2 * id + side;
         sout[p->nseg] = 2 * id + (side ^ 1);
@@ -229,7 +241,6 @@ bool TkLayeredSession::describe(int nrows, const int32_t* seq, const int32_t* po
         for (int i = 0; i < n; ++i) { h_seq[r + i] = id; h_pos[r + i] = pos[r + i]; h_tok[r + i] = tok[r + i]; h_seg[r + i] = p->nseg; }
         if (n > 1) p->single = false;
         ++p->nseg;
-        r += n;
     }
     return upload_pages();
 }
@@ -480,11 +491,15 @@ bool TkLayeredSession::prefill(int nseq, int n_prompt, const int32_t* tokens, in
 bool TkLayeredSession::begin_decode(int nrows, const int32_t* pos, int n_steps) {
     std::lock_guard<std::mutex> lk(mu_);
     if (nrows > (int)live_.size()) { error = "decode() continues the rows of the previous decode step or forward() that sampled every row"; return false; }
+    size_t need = 0;
     for (int r = 0; r < nrows; ++r) {
-        Seq& s = seqs_[(size_t)live_[(size_t)r]];
+        const Seq& s = seqs_[(size_t)live_[(size_t)r]];
         if (s.len != pos[r]) { error = "a sequence has been released or moved since its row was sampled"; return false; }
-        if (!need_pages(s, live_[(size_t)r], pos[r] + n_steps - 1)) return false;
+        const size_t want = (size_t)(pos[r] + n_steps - 1) / TK_PAGE + 1;
+        need += want > s.pages.size() ? want - s.pages.size() : 0;
     }
+    if (need > free_pages_.size()) { error = "cache pool exhausted: the decode loop wants " + std::to_string(need) + " more pages"; return false; }
+    for (int r = 0; r < nrows; ++r) need_pages(seqs_[(size_t)live_[(size_t)r]], live_[(size_t)r], pos[r] + n_steps - 1);
     return upload_pages();
 }
 

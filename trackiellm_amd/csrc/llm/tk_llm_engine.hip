@@ -305,8 +305,8 @@ bool TkLlmSession::init(TkLlmModel* m, int mseq, int mctx) {
 }
 
 TkLlmSession::~TkLlmSession() {
-    if (model && counted_) tk_attention_note_session(model->device, -1);
-    if (model) (void)hipSetDevice(model->device);
+    if (counted_) tk_attention_note_session(device_, -1);
+    (void)hipSetDevice(device_); /* the model may be gone already */
     if (stream) (void)hipStreamSynchronize(stream);
     for (auto& v : graph_exec) for (auto& g : v) if (g) (void)hipGraphExecDestroy(g);
     for (auto& v : graph_prefill) for (auto& g : v) if (g) (void)hipGraphExecDestroy(g);
