@@ -125,7 +125,6 @@ private:
     void enqueue_layers(const Pass& p);
     void enqueue_head(int n, const int32_t* d_rows, int32_t* tok, int32_t* pos);
     void enqueue_moe(const TkLayerSpec& s, const TkLayeredLayer& L, int nrows);
-    int attn_splits(const TkAttnSpec& a, int pages, int nrows) const;
     bool run(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, float* logits_host, int32_t* argmax_host, bool head,
              const uint32_t* const* row_masks, const TkSampleRow* row_samp, int n_out, const int32_t* out_rows);
 };

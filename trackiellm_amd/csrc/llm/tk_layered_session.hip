@@ -28,12 +28,6 @@ bool TkLayeredSession::alloc(void** p, size_t bytes, bool zero) {
     return true;
 }
 
-/* workgroups of the row attention per (row, head group): enough to cover the chip, at least four pages each */
-int TkLayeredSession::attn_splits(const TkAttnSpec& a, int pages, int nrows) const {
-    const int wgs = nrows * a.kv_heads * ((a.heads / a.kv_heads + 15) / 16);
-    return std::max(1, std::min({(512 + wgs - 1) / wgs, pages / 4, 32}));
-}
-
 bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_tokens) {
     m_ = m;
     max_seq = mseq;
@@ -93,8 +87,8 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
                 const int64_t seen = a.window > 0 ? (int64_t)a.window / TK_PAGE + 2 + (a.keep_first + TK_PAGE - 1) / TK_PAGE : max_pages_;
                 bs.splits_pages = (int)std::min<int64_t>(seen, max_pages_);
                 TkAttnArgs aa{};
-                aa.heads = a.heads; aa.kv = bs.kv;
-                for (int n = 1; n <= TK_MAX_ROWS; ++n) scratch = std::max(scratch, tk_attn_rows_scratch_floats(aa, n, attn_splits(a, bs.splits_pages, n)));
+                aa.heads = a.heads; aa.kv_heads = a.kv_heads; aa.kv = bs.kv;
+                for (int n = 1; n <= TK_MAX_ROWS; ++n) scratch = std::max(scratch, tk_attn_rows_scratch_floats(aa, n, tk_attn_rows_splits(aa, bs.splits_pages, n)));
                 if (a.rot_dims > 0) {
                     Rope& r = rope_[{a.rot_dims, a.rot_base}];
                     if (!r.c) { /* double precision on the host */
@@ -310,6 +304,7 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
         /* attention and delta branches are prepared in pairs: one launch when a layer has one of each */
         std::vector<TkAttnArgs> as;
         std::vector<TkDeltaArgs> ds;
+        std::vector<int> visible; /* pages an attention branch may see at most */
         for (size_t b = 0; b < spec.branches.size(); ++b) {
             const TkBranchSpec& bs = spec.branches[b];
             const TkLayeredBranch& B = L.branches[b];
@@ -321,6 +316,7 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
                 a.scale = sp.scale; a.out_scale = bs.scale; a.eps = c.eps; a.col = B.col; a.bias = B.bias; a.q_norm = B.q_norm; a.k_norm = B.k_norm;
                 a.rope_cos = st.rope.c; a.rope_sin = st.rope.s; a.q = q_; a.kv = st.kv; a.out_img = img_mix_; a.out_k0 = B.out_k0; a.out_ktiles = L.out.K / kt;
                 as.push_back(a);
+                visible.push_back(st.splits_pages);
             } else {
                 const TkDeltaSpec& sp = bs.delta;
                 TkDeltaArgs d{};
@@ -336,17 +332,15 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
             const TkAttnArgs* a = ai < as.size() ? &as[ai] : nullptr;
             const TkDeltaArgs* d = di < ds.size() ? &ds[di] : nullptr;
             tk_launch_mixer_prep(type, proj_, L.in.N, a, d, tab_, n, s);
-            if (a) {
-                size_t b = 0;
-                for (size_t k = 0, seen = 0; k < spec.branches.size(); ++k)
-                    if (spec.branches[k].kind == TkBranchSpec::ATTENTION && seen++ == ai) b = k;
-                if (p.single) tk_launch_attn_rows(type, *a, tab_, n, attn_splits(spec.branches[b].attn, st_[l][b].splits_pages, n), scratch_, s);
-                else tk_launch_attn_tiles(type, *a, tab_, d_tiles_, p.ntiles, s);
+            if (!p.single) {
+                if (a) tk_launch_attn_tiles(type, *a, tab_, d_tiles_, p.ntiles, s);
+                if (d) tk_launch_delta_scan(type, *d, tab_, p.nseg, n, s);
+                continue;
             }
-            if (d) {
-                if (p.single) tk_launch_delta_step(type, *d, tab_, n, s);
-                else tk_launch_delta_scan(type, *d, tab_, p.nseg, n, s);
-            }
+            const int splits = a ? tk_attn_rows_splits(*a, visible[ai], n) : 1;
+            if (a && d && splits == 1 && tk_launch_mixers_step(type, *a, *d, tab_, n, s)) continue;
+            if (a) tk_launch_attn_rows(type, *a, tab_, n, splits, scratch_, s);
+            if (d) tk_launch_delta_step(type, *d, tab_, n, s);
         }
         TkImgGemm o{};
         o.type = type; o.w = L.out.img; o.a = img_mix_; o.K = L.out.K; o.N = L.out.N; o.nrows = n; o.out = y_; o.ldc = D; o.n_valid = D;

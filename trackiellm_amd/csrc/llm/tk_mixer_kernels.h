@@ -67,12 +67,16 @@ void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs*
 void tk_launch_attn_tiles(int type, const TkAttnArgs& a, const TkPassTab& t, const int32_t* tiles, int n_tiles, hipStream_t s);
 /* one row at a time (decoding): `splits` workgroups per (row, group of query heads) share the row's pages; scratch for splits > 1 */
 void tk_launch_attn_rows(int type, const TkAttnArgs& a, const TkPassTab& t, int nrows, int splits, float* scratch, hipStream_t s);
+int tk_attn_rows_splits(const TkAttnArgs& a, int pages, int nrows); /* for at most `pages` visible pages */
 size_t tk_attn_rows_scratch_floats(const TkAttnArgs& a, int nrows, int splits);
 
 /* the recurrence over every segment, token by token, and the gated per-head norm of its output */
 void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, int n_segments, int nrows, hipStream_t s);
 /* the same for passes whose segments are single rows: one launch */
 void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s);
+
+/* tk_launch_attn_rows and tk_launch_delta_step in one launch, side by side; false (nothing launched): sizes it has no form for */
+bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s);
 
 /* where a sublayer's output comes from: a product's rows, or the chosen experts' rows, weighted */
 struct TkSubOut {

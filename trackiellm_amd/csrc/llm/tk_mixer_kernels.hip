@@ -14,13 +14,30 @@ constexpr float LOG2E = 1.44269504088896340736f;
 
 /* ------------------------------------------------------------------ embedding, norms ------- */
 
-template <typename T>
+/* VEC: eight consecutive elements per thread (width a multiple of eight), else one */
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void k_layer_embed(const uint16_t* table, int width, const int32_t* tok, float* x, T* img, int ktiles) {
     const int row = blockIdx.x;
     const uint16_t* e = table + (size_t)tok[row] * width;
+    float* xr = x + (size_t)row * width;
+    if (VEC) {
+        for (int k = threadIdx.x * 8; k < width; k += 256 * 8) {
+            const tk_v4u u = *(const tk_v4u*)(e + k);
+            tk_v4f a, b;
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                a[2 * i] = __uint_as_float(u[i] << 16); a[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
+                b[2 * i] = __uint_as_float(u[2 + i] << 16); b[2 * i + 1] = __uint_as_float(u[2 + i] & 0xffff0000u);
+            }
+            *(tk_v4f*)(xr + k) = a;
+            *(tk_v4f*)(xr + k + 4) = b;
+            tk_img_put8(img, row, k, ktiles, a, b);
+        }
+        return;
+    }
     for (int k = threadIdx.x; k < width; k += 256) {
         const float v = tk_bf16_float(e[k]);
-        x[(size_t)row * width + k] = v;
+        xr[k] = v;
         tk_img_put(img, row, k, ktiles, v);
     }
 }
@@ -36,148 +53,238 @@ __device__ __forceinline__ float block_sum(float v, float* red /* [16] */) {
     return t;
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void k_post_norm(TkSubOut o, const float* w, float eps, int width, float* x, T* img, int ktiles) {
+__device__ __forceinline__ float dot4(tk_v4f a, tk_v4f b) { return fmaf(a[0], b[0], fmaf(a[1], b[1], fmaf(a[2], b[2], a[3] * b[3]))); }
+
+template <typename T, bool VEC>
+__global__ __launch_bounds__(512) void k_post_norm(TkSubOut o, const float* w, float eps, int width, float* x, T* img, int ktiles) {
     extern __shared__ __attribute__((aligned(16))) float ybuf[];
     __shared__ float red[16];
-    const int row = blockIdx.x;
+    const int row = blockIdx.x, nt = blockDim.x;
+    float* xr = x + (size_t)row * width;
     float ss = 0.0f;
-    if (o.top > 0) {
-        for (int k = threadIdx.x; k < width; k += 256) {
-            float y = 0.0f;
-            for (int j = 0; j < o.top; ++j) y += o.weight[row * o.top + j] * o.y[(size_t)o.slot[row * o.top + j] * o.ld + k];
-            ybuf[k] = y;
-            ss += y * y;
+    if (VEC) {
+        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
+            tk_v4f a, b;
+            if (o.top > 0) {
+                a = b = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+                for (int j = 0; j < o.top; ++j) {
+                    const float* p = o.y + (size_t)o.slot[row * o.top + j] * o.ld + k;
+                    const float c = o.weight[row * o.top + j];
+                    a += *(const tk_v4f*)p * c;
+                    b += *(const tk_v4f*)(p + 4) * c;
+                }
+            } else {
+                const float* p = o.y + (size_t)row * o.ld + k;
+                a = *(const tk_v4f*)p; b = *(const tk_v4f*)(p + 4);
+                if (o.bias) { a += *(const tk_v4f*)(o.bias + k) * o.bias_scale; b += *(const tk_v4f*)(o.bias + k + 4) * o.bias_scale; }
+            }
+            *(tk_v4f*)(ybuf + k) = a;
+            *(tk_v4f*)(ybuf + k + 4) = b;
+            ss += dot4(a, a) + dot4(b, b);
         }
     } else {
-        for (int k = threadIdx.x; k < width; k += 256) {
-            float y = o.y[(size_t)row * o.ld + k];
-            if (o.bias) y += o.bias[k] * o.bias_scale;
+        for (int k = threadIdx.x; k < width; k += nt) {
+            float y = 0.0f;
+            if (o.top > 0)
+                for (int j = 0; j < o.top; ++j) y += o.weight[row * o.top + j] * o.y[(size_t)o.slot[row * o.top + j] * o.ld + k];
+            else y = o.y[(size_t)row * o.ld + k] + (o.bias ? o.bias[k] * o.bias_scale : 0.0f);
             ybuf[k] = y;
             ss += y * y;
         }
     }
-    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps); /* block_sum synchronises: ybuf is whole; a thread re-reads its own elements */
-    for (int k = threadIdx.x; k < width; k += 256) {
-        const float v = x[(size_t)row * width + k] + ybuf[k] * r * w[k];
-        x[(size_t)row * width + k] = v;
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps); /* a thread re-reads its own elements of ybuf only */
+    if (VEC) {
+        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
+            const tk_v4f a = *(const tk_v4f*)(xr + k) + *(const tk_v4f*)(ybuf + k) * r * *(const tk_v4f*)(w + k);
+            const tk_v4f b = *(const tk_v4f*)(xr + k + 4) + *(const tk_v4f*)(ybuf + k + 4) * r * *(const tk_v4f*)(w + k + 4);
+            *(tk_v4f*)(xr + k) = a;
+            *(tk_v4f*)(xr + k + 4) = b;
+            tk_img_put8(img, row, k, ktiles, a, b);
+        }
+        return;
+    }
+    for (int k = threadIdx.x; k < width; k += nt) {
+        const float v = xr[k] + ybuf[k] * r * w[k];
+        xr[k] = v;
         tk_img_put(img, row, k, ktiles, v);
     }
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void k_rows_norm(const float* x, const int32_t* rows, const float* w, float eps, int width, T* img, int ktiles) {
+template <typename T, bool VEC>
+__global__ __launch_bounds__(512) void k_rows_norm(const float* x, const int32_t* rows, const float* w, float eps, int width, T* img, int ktiles) {
     __shared__ float red[16];
-    const int i = blockIdx.x;
+    const int i = blockIdx.x, nt = blockDim.x;
     const float* xr = x + (size_t)(rows ? rows[i] : i) * width;
     float ss = 0.0f;
-    for (int k = threadIdx.x; k < width; k += 256) ss += xr[k] * xr[k];
+    if (VEC)
+        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
+            const tk_v4f a = *(const tk_v4f*)(xr + k), b = *(const tk_v4f*)(xr + k + 4);
+            ss += dot4(a, a) + dot4(b, b);
+        }
+    else
+        for (int k = threadIdx.x; k < width; k += nt) ss += xr[k] * xr[k];
     const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
-    for (int k = threadIdx.x; k < width; k += 256) tk_img_put(img, i, k, ktiles, xr[k] * r * w[k]);
+    if (VEC)
+        for (int k = threadIdx.x * 8; k < width; k += nt * 8)
+            tk_img_put8(img, i, k, ktiles, *(const tk_v4f*)(xr + k) * r * *(const tk_v4f*)(w + k), *(const tk_v4f*)(xr + k + 4) * r * *(const tk_v4f*)(w + k + 4));
+    else
+        for (int k = threadIdx.x; k < width; k += nt) tk_img_put(img, i, k, ktiles, xr[k] * r * w[k]);
 }
 
 /* ------------------------------------------------------------------ between projections and mixers ---- */
 
-/* one wave: one head of q, k or v of one row */
-template <typename T>
-__device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* p, int row, int u, int lane) {
+/* one wave: one head of q, k or v of RW consecutive rows (rows past the pass repeat its last one and store nothing); all loads come first */
+template <typename T, int RW>
+__device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* proj, int ld, int row0, int nrows, int u, int lane) {
     const bool is_q = u < a.heads, is_v = u >= a.heads + a.kv_heads;
     const int n = is_v ? a.vdim : a.dim;
     const int head = is_q ? u : is_v ? u - a.heads - a.kv_heads : u - a.heads;
     const int off = is_q ? head * a.dim : is_v ? (a.heads + a.kv_heads) * a.dim + head * a.vdim : (a.heads + head) * a.dim;
-    const float* src = p + a.col + off;
     const float* b = a.bias ? a.bias + off : nullptr;
     const float* w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
-    float v[4];
-    float ss = 0.0f;
+    const int half = is_v ? 0 : a.rot_dims / 2;
+    float v[RW][4], z[RW][4], c[RW][4], s[RW][4]; /* element, its rotation partner, cosine, signed sine */
+    int pos[RW];
+    size_t page[RW];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int e = lane + 64 * i;
-        v[i] = e < n ? src[e] + (b ? b[e] : 0.0f) : 0.0f;
-        ss += v[i] * v[i];
-    }
-    const float r = w ? 1.0f / sqrtf(tk_wave_sum(ss) / (float)n + a.eps) : 1.0f;
-    const int pos = t.pos[row], half = is_v ? 0 : a.rot_dims / 2;
-    const size_t page = is_q ? 0 : (size_t)t.page_of[(size_t)t.seq[row] * t.max_pages + pos / TK_PAGE];
+    for (int r = 0; r < RW; ++r) {
+        const int row = row0 + r < nrows ? row0 + r : nrows - 1;
+        pos[r] = t.pos[row];
+        page[r] = is_q ? 0 : (size_t)t.page_of[(size_t)t.seq[row] * t.max_pages + pos[r] / TK_PAGE];
+        const float* src = proj + (size_t)row * ld + a.col + off;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int e = lane + 64 * i;
-        if (e >= n) break;
-        float y = w ? v[i] * r * w[e] : v[i];
-        if (e < 2 * half) { /* the other half of the pair: its value times the head's common factor */
-            const int f = e < half ? e + half : e - half, j = e < half ? e : e - half;
-            float z = src[f] + (b ? b[f] : 0.0f);
-            if (w) z = z * r * w[f];
-            const float c = a.rope_cos[(size_t)pos * half + j], s = a.rope_sin[(size_t)pos * half + j];
-            y = e < half ? y * c - z * s : y * c + z * s;
+        for (int i = 0; i < 4; ++i) {
+            const int e = lane + 64 * i;
+            v[r][i] = z[r][i] = s[r][i] = 0.0f;
+            c[r][i] = 1.0f;
+            if (64 * i < n && e < n) {
+                v[r][i] = src[e] + (b ? b[e] : 0.0f);
+                if (e < 2 * half) {
+                    const int f = e < half ? e + half : e - half, j = e < half ? e : f;
+                    z[r][i] = (src[f] + (b ? b[f] : 0.0f)) * (w ? w[f] : 1.0f);
+                    c[r][i] = a.rope_cos[(size_t)pos[r] * half + j];
+                    s[r][i] = a.rope_sin[(size_t)pos[r] * half + j] * (e < half ? -1.0f : 1.0f);
+                }
+            }
         }
-        if (is_q) ((T*)a.q)[((size_t)row * a.heads + head) * a.kv.dim_pad + e] = TkImg<T>::from(y);
-        else if (is_v) ((T*)a.kv.v)[((page * a.kv_heads + head) * a.kv.vdim_pad + e) * TK_PAGE + pos % TK_PAGE] = TkImg<T>::from(y);
-        else ((T*)a.kv.k)[((page * a.kv_heads + head) * TK_PAGE + pos % TK_PAGE) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+    }
+    float wv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) wv[i] = w && lane + 64 * i < n ? w[lane + 64 * i] : 1.0f;
+#pragma unroll
+    for (int r = 0; r < RW; ++r) {
+        if (row0 + r >= nrows) break;
+        float f = 1.0f;
+        if (w) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) ss += v[r][i] * v[r][i];
+            f = 1.0f / sqrtf(tk_wave_sum(ss) / (float)n + a.eps);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int e = lane + 64 * i;
+            if (e >= n) break;
+            const float y = (v[r][i] * f * wv[i]) * c[r][i] + (z[r][i] * f) * s[r][i];
+            if (is_q) ((T*)a.q)[((size_t)(row0 + r) * a.heads + head) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+            else if (is_v) ((T*)a.kv.v)[((page[r] * a.kv_heads + head) * a.kv.vdim_pad + e) * TK_PAGE + pos[r] % TK_PAGE] = TkImg<T>::from(y);
+            else ((T*)a.kv.k)[((page[r] * a.kv_heads + head) * TK_PAGE + pos[r] % TK_PAGE) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+        }
     }
 }
 
-/* one wave: one head of q, k or v after its convolution, or one head's decays and step size */
-__device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab& t, const float* proj, int ld, int row, int u, int lane) {
+/* one wave: one head of q, k or v after its convolution, or one head's decays and step size, of RW consecutive rows */
+template <int RW>
+__device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab& t, const float* proj, int ld, int rowb, int nrows, int u, int lane) {
     const int qk = d.kv_heads * d.dim, channels = 2 * qk + d.heads * d.vdim;
     if (u >= 2 * d.kv_heads + d.heads) {
         const int h = u - 2 * d.kv_heads - d.heads;
         const float rate = -expf(d.a_log[h]);
-        for (int e = lane; e < d.dim; e += 64) {
-            const float z = d.low[(size_t)row * d.low_ld + d.low_a + h * d.dim + e] + d.dt_bias[h * d.dim + e];
-            const float sp = fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); /* softplus */
-            d.g[((size_t)row * d.heads + h) * d.dim + e] = expf(rate * sp);
+#pragma unroll
+        for (int r = 0; r < RW; ++r) {
+            const int row = rowb + r;
+            if (row >= nrows) break;
+            for (int e = lane; e < d.dim; e += 64) {
+                const float z = d.low[(size_t)row * d.low_ld + d.low_a + h * d.dim + e] + d.dt_bias[h * d.dim + e];
+                const float sp = fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); /* softplus */
+                d.g[((size_t)row * d.heads + h) * d.dim + e] = expf(rate * sp);
+            }
+            if (lane == 0) d.beta[(size_t)row * d.heads + h] = tk_sigmoid32(proj[(size_t)row * ld + d.col + channels + h]);
         }
-        if (lane == 0) d.beta[(size_t)row * d.heads + h] = tk_sigmoid32(proj[(size_t)row * ld + d.col + channels + h]);
         return;
     }
     const int which = u < d.kv_heads ? 0 : u < 2 * d.kv_heads ? 1 : 2;
     const int head = which == 2 ? u - 2 * d.kv_heads : which == 1 ? u - d.kv_heads : u;
     const int n = which == 2 ? d.vdim : d.dim, c0 = which == 2 ? 2 * qk + head * d.vdim : which * qk + head * d.dim;
-    const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0, last = t.seg_n[seg] - 1;
-    const int in = t.seg_in[seg], hist = d.taps - 1;
-    /* input of channel c at time `s` of the segment; negative times are the state's */
-    auto input = [&](int c, int s) -> float {
-        if (s >= 0) return proj[(size_t)(row0 + s) * ld + d.col + c];
-        return in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
-    };
-    float v[4];
-    float ss = 0.0f;
+    const int hist = d.taps - 1;
+    float* dst = which == 0 ? d.q + head * d.dim : which == 1 ? d.k + head * d.dim : d.v + (size_t)head * d.vdim;
+    const size_t pitch = which == 2 ? (size_t)d.heads * d.vdim : qk;
+    float y[RW][4];
+    const int seg0 = t.seg[rowb], first = rowb - t.seg_row0[seg0];
+    if (RW > 1 && first >= hist && first + RW <= t.seg_n[seg0]) { /* every input is a row of this pass */
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int e = lane + 64 * i;
-        v[i] = 0.0f;
-        if (e < n) {
-            const int c = c0 + e;
-            float y = 0.0f;
-            for (int j = 0; j < d.taps; ++j) y += d.conv[(size_t)c * d.taps + j] * input(c, at - hist + j);
-            v[i] = tk_silu32(y);
-            ss += v[i] * v[i];
-            if (at == last) {
-                float* out = d.conv_state + ((size_t)t.seg_out[seg] * channels + c) * hist;
-                for (int j = 0; j < hist; ++j) out[j] = input(c, at + 1 - hist + j);
+        for (int i = 0; i < 4; ++i) {
+#pragma unroll
+            for (int r = 0; r < RW; ++r) y[r][i] = 0.0f;
+            const int c = c0 + lane + 64 * i;
+            if (64 * i < n && lane + 64 * i < n)
+                for (int j = 0; j < d.taps; ++j) {
+                    const float tap = d.conv[(size_t)c * d.taps + j];
+#pragma unroll
+                    for (int r = 0; r < RW; ++r) y[r][i] = fmaf(tap, proj[(size_t)(rowb + r - hist + j) * ld + d.col + c], y[r][i]);
+                }
+        }
+    } else {
+#pragma unroll
+        for (int r = 0; r < RW; ++r) {
+            const int row = rowb + r < nrows ? rowb + r : nrows - 1;
+            const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0, in = t.seg_in[seg];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                y[r][i] = 0.0f;
+                const int c = c0 + lane + 64 * i;
+                if (64 * i < n && lane + 64 * i < n)
+                    for (int j = 0; j < d.taps; ++j) {
+                        const int s = at - hist + j; /* time inside the segment; before it: the history, zeros before the sequence */
+                        const float x = s >= 0 ? proj[(size_t)(row0 + s) * ld + d.col + c] : in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
+                        y[r][i] = fmaf(d.conv[(size_t)c * d.taps + j], x, y[r][i]);
+                    }
             }
         }
     }
-    float r = 1.0f;
-    if (which < 2) {
-        r = 1.0f / sqrtf(tk_wave_sum(ss) + d.unit_eps);
-        if (which == 0) r *= 1.0f / sqrtf((float)d.dim);
-    }
-    float* dst = which == 0 ? d.q + (size_t)row * qk + head * d.dim : which == 1 ? d.k + (size_t)row * qk + head * d.dim : d.v + ((size_t)row * d.heads + head) * d.vdim;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int e = lane + 64 * i;
-        if (e < n) dst[e] = v[i] * r;
+    for (int r = 0; r < RW; ++r) {
+        const int row = rowb + r;
+        if (row >= nrows) break;
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { y[r][i] = tk_silu32(y[r][i]); ss += y[r][i] * y[r][i]; } /* silu(0) = 0 past the head */
+        float f = 1.0f;
+        if (which < 2) {
+            f = 1.0f / sqrtf(tk_wave_sum(ss) + d.unit_eps);
+            if (which == 0) f *= 1.0f / sqrtf((float)d.dim);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (lane + 64 * i < n) dst[row * pitch + lane + 64 * i] = y[r][i] * f;
+        const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0;
+        if (at + 1 == t.seg_n[seg]) { /* the segment's last row leaves the history behind */
+            const int in = t.seg_in[seg], out = t.seg_out[seg];
+            for (int e = lane; e < n; e += 64)
+                for (int j = 0; j < hist; ++j) {
+                    const int c = c0 + e, s = at + 1 - hist + j;
+                    d.conv_state[((size_t)out * channels + c) * hist + j] = s >= 0 ? proj[(size_t)(row0 + s) * ld + d.col + c] : in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
+                }
+        }
     }
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void k_mixer_prep(const float* proj, int ld, TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int nd) {
-    const int row = blockIdx.y, lane = threadIdx.x & 63;
+template <typename T, int RW>
+__global__ __launch_bounds__(256) void k_mixer_prep(const float* proj, int ld, TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int nd, int nrows) {
+    const int row = blockIdx.y * RW, lane = threadIdx.x & 63;
     const int u = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
-    if (u < na) attn_unit<T>(a, t, proj + (size_t)row * ld, row, u, lane);
-    else if (u < na + nd) delta_unit(d, t, proj, ld, row, u - na, lane);
+    if (u < na) attn_unit<T, RW>(a, t, proj, ld, row, nrows, u, lane);
+    else if (u < na + nd) delta_unit<RW>(d, t, proj, ld, row, nrows, u - na, lane);
 }
 
 /* ------------------------------------------------------------------ attention -------------- */
@@ -215,8 +322,7 @@ struct Flash {
         for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[j][r]);
-        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        mx = tk_quad_max(mx);
         const float mn = fmaxf(m, mx), ms = mn == -INFINITY ? 0.0f : mn;
         const float al = __builtin_amdgcn_exp2f(m - ms);
         m = mn;
@@ -226,9 +332,7 @@ struct Flash {
         for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int r = 0; r < 4; ++r) { p[j][r] = __builtin_amdgcn_exp2f(s[j][r] - ms); sum += p[j][r]; }
-        sum += __shfl_xor(sum, 16, 64);
-        sum += __shfl_xor(sum, 32, 64);
-        l = l * al + sum;
+        l = l * al + tk_quad_sum(sum);
 #pragma unroll
         for (int i = 0; i < VT; ++i) o[i] *= al;
         accumulate(p, nv, vfrag);
@@ -362,15 +466,14 @@ __global__ __launch_bounds__(256) void k_attn_tiles(TkAttnArgs a, TkPassTab t, c
 }
 
 /* decoding: one row x up to 16 query heads of one kv head per workgroup, pages dealt to the waves (and to `splits` workgroups), merged in LDS */
-template <typename T, int B>
-__global__ __launch_bounds__(256) void k_attn_rows(TkAttnArgs a, TkPassTab t, int splits, float* scratch) {
+template <typename T, int B, int WAVES>
+__device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t, int block, int row, int split, int splits, float* scratch, uint8_t* lds) {
     constexpr int DT = B / TkImg<T>::KT, VT = B / 16, SZ = sizeof(T);
+    constexpr bool AHEAD = SZ == 2 && B <= 128; /* a page's values are requested together with its keys */
     typedef typename VFrag<T>::type VF;
-    __shared__ tk_v4f so[2][VT][64];
-    __shared__ float sm[2][64], sl[2][64];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4;
-    const int row = blockIdx.y, split = blockIdx.z, gq = a.heads / a.kv_heads, per = (gq + 15) / 16;
-    const int kvh = blockIdx.x / per, q = (blockIdx.x % per) * 16 + (lane & 15);
+    const int gq = a.heads / a.kv_heads, per = (gq + 15) / 16;
+    const int kvh = block / per, q = (block % per) * 16 + (lane & 15);
     const int h = kvh * gq + (q < gq ? q : 0);
     const int nd = a.kv.dim_pad / TkImg<T>::KT, nv = a.kv.vdim_pad / 16;
     const int pos = t.pos[row], seq = t.seq[row];
@@ -381,18 +484,33 @@ __global__ __launch_bounds__(256) void k_attn_rows(TkAttnArgs a, TkPassTab t, in
     Flash<T, VT> f;
     f.init();
     const PageWalk walk(pos, pos, a.window, a.keep_first);
-    for (int i = split * 4 + wave; i < walk.count; i += 4 * splits) {
+    for (int i = split * WAVES + wave; i < walk.count; i += WAVES * splits) {
         const size_t page = (size_t)t.page_of[(size_t)seq * t.max_pages + walk.page(i)] * a.kv_heads + kvh;
         const uint8_t* kp = (const uint8_t*)a.kv.k + (page * TK_PAGE + (lane & 15)) * a.kv.dim_pad * SZ + g * 16;
         const uint8_t* vp = (const uint8_t*)a.kv.v + (page * a.kv.vdim_pad + (lane & 15)) * TK_PAGE * SZ + 4 * g * SZ;
         const int k0 = walk.page(i) * TK_PAGE;
+        auto vload = [&](int vt, int j) { return *(const VF*)(vp + ((size_t)16 * vt * TK_PAGE + 16 * j) * SZ); };
+        tk_v4u kf[AHEAD ? 4 : 1][AHEAD ? DT : 1];
+        VF vf[AHEAD ? VT : 1][4];
+        if (AHEAD) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int d = 0; d < DT; ++d)
+                    if (d < nd) kf[j][d] = *(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64);
+#pragma unroll
+            for (int i2 = 0; i2 < VT; ++i2)
+                if (i2 < nv)
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) vf[i2][j] = vload(i2, j);
+        }
         tk_v4f s[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             s[j] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
             for (int d = 0; d < DT; ++d)
-                if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64), qf[d], s[j]);
+                if (d < nd) s[j] = TkImg<T>::mma(AHEAD ? kf[AHEAD ? j : 0][AHEAD ? d : 0] : *(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64), qf[d], s[j]);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int key = k0 + 16 * j + 4 * g + r;
@@ -400,24 +518,26 @@ __global__ __launch_bounds__(256) void k_attn_rows(TkAttnArgs a, TkPassTab t, in
                 s[j][r] = see ? s[j][r] * (a.scale * LOG2E) : -INFINITY;
             }
         }
-        f.update(s, nv, [&](int vt, int j) { return *(const VF*)(vp + ((size_t)16 * vt * TK_PAGE + 16 * j) * SZ); });
+        f.update(s, nv, [&](int vt, int j) { return AHEAD ? vf[AHEAD ? vt : 0][j] : vload(vt, j); });
     }
-    /* waves 2, 3 into 0, 1, then 1 into 0 */
+    /* the upper half of the waves into the lower half, and again */
+    tk_v4f* so = (tk_v4f*)lds; /* [WAVES / 2][VT][64] */
+    float *sm = (float*)(so + WAVES / 2 * VT * 64), *sl = sm + WAVES / 2 * 64;
 #pragma unroll
-    for (int half = 2; half >= 1; half >>= 1) {
+    for (int half = WAVES / 2; half >= 1; half >>= 1) {
         if (wave >= half && wave < 2 * half) {
 #pragma unroll
-            for (int i = 0; i < VT; ++i) so[wave - half][i][lane] = f.o[i];
-            sm[wave - half][lane] = f.m; sl[wave - half][lane] = f.l;
+            for (int i = 0; i < VT; ++i) so[((wave - half) * VT + i) * 64 + lane] = f.o[i];
+            sm[(wave - half) * 64 + lane] = f.m; sl[(wave - half) * 64 + lane] = f.l;
         }
         __syncthreads();
         if (wave < half) {
-            const float m2 = sm[wave][lane], mn = fmaxf(f.m, m2), ms = mn == -INFINITY ? 0.0f : mn;
+            const float m2 = sm[wave * 64 + lane], mn = fmaxf(f.m, m2), ms = mn == -INFINITY ? 0.0f : mn;
             const float c1 = __builtin_amdgcn_exp2f(f.m - ms), c2 = __builtin_amdgcn_exp2f(m2 - ms);
-            f.l = f.l * c1 + sl[wave][lane] * c2;
+            f.l = f.l * c1 + sl[wave * 64 + lane] * c2;
             f.m = mn;
 #pragma unroll
-            for (int i = 0; i < VT; ++i) f.o[i] = f.o[i] * c1 + so[wave][i][lane] * c2;
+            for (int i = 0; i < VT; ++i) f.o[i] = f.o[i] * c1 + so[(wave * VT + i) * 64 + lane] * c2;
         }
         __syncthreads();
     }
@@ -430,6 +550,13 @@ __global__ __launch_bounds__(256) void k_attn_rows(TkAttnArgs a, TkPassTab t, in
         if (i < nv)
 #pragma unroll
             for (int r = 0; r < 4; ++r) out[2 + 16 * i + 4 * g + r] = f.o[i][r];
+}
+template <int B, int WAVES> constexpr size_t attn_row_lds() { return (size_t)WAVES / 2 * (B / 16 * 1024 + 512); }
+
+template <typename T, int B, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void k_attn_rows(TkAttnArgs a, TkPassTab t, int splits, float* scratch) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    attn_row<T, B, WAVES>(a, t, blockIdx.x, blockIdx.y, blockIdx.z, splits, scratch, lds);
 }
 
 template <typename T>
@@ -450,27 +577,17 @@ __global__ __launch_bounds__(64) void k_attn_merge(TkAttnArgs a, int splits, con
 
 /* ------------------------------------------------------------------ gated delta rule ------- */
 
-template <int CTRL> __device__ __forceinline__ float dpp_row(float v) { return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false)); }
-/* sum over the 16 lanes of a DPP row (row_ror 8, 4, 2, 1) */
-__device__ __forceinline__ float row16_sum(float v) {
-    v += dpp_row<0x128>(v);
-    v += dpp_row<0x124>(v);
-    v += dpp_row<0x122>(v);
-    v += dpp_row<0x121>(v);
-    return v;
-}
-
-/* A workgroup walks 16 columns of one head's state through a segment; a column is 16 lanes x RPL key rows, so the column's recurrence never
- * leaves the wave.  q, k, decays, v and step sizes of TC tokens at a time go through LDS, the next TC in flight in registers. */
-template <int RPL>
+/* A workgroup walks 4 * 64 / LN columns of one head's state through a segment; a column is LN lanes x RPL key rows, so the column's recurrence
+ * never leaves the wave.  q, k, decays, v and step sizes of TC tokens at a time go through LDS, the next TC in flight in registers. */
+template <int LN, int RPL>
 __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) {
-    constexpr int DP = 16 * RPL, TC = RPL > 8 ? 8 : 16, NL = TC * DP / 256;
+    constexpr int DP = LN * RPL, TC = DP > 128 ? 8 : 16, NL = TC * DP / 256, CW = 64 / LN, NC = 4 * CW;
     __shared__ __attribute__((aligned(16))) float lq[2][TC][DP], lk[2][TC][DP], lg[2][TC][DP];
-    __shared__ float lv[2][TC][16], lb[2][TC];
+    __shared__ float lv[2][TC][NC], lb[2][TC];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int h = blockIdx.y, seg = blockIdx.z, kvh = h / (d.heads / d.kv_heads), vp = (d.vdim + 3) & ~3;
     const int row0 = t.seg_row0[seg], n = t.seg_n[seg], in = t.seg_in[seg], out = t.seg_out[seg];
-    const int cl = wave * 4 + (lane >> 4), col = blockIdx.x * 16 + cl, r0 = (lane & 15) * RPL;
+    const int cl = wave * CW + lane / LN, col = blockIdx.x * NC + cl, r0 = (lane % LN) * RPL;
     const bool live = col < d.vdim;
     float S[RPL];
 #pragma unroll
@@ -487,10 +604,10 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
             rk[i] = ok ? d.k[(row * d.kv_heads + kvh) * d.dim + e] : 0.0f;
             rg[i] = ok ? d.g[(row * d.heads + h) * d.dim + e] : 1.0f;
         }
-        if (tid < TC * 16) {
-            const int tt = t0 + tid / 16, c = blockIdx.x * 16 + tid % 16;
+        if (tid < TC * NC) {
+            const int tt = t0 + tid / NC, c = blockIdx.x * NC + tid % NC;
             rv = tt < n && c < d.vdim ? d.v[((size_t)(row0 + tt) * d.heads + h) * d.vdim + c] : 0.0f;
-            if (tid % 16 == 0) rb = tt < n ? d.beta[(size_t)(row0 + tt) * d.heads + h] : 0.0f;
+            if (tid % NC == 0) rb = tt < n ? d.beta[(size_t)(row0 + tt) * d.heads + h] : 0.0f;
         }
     };
     auto put = [&](int b) {
@@ -499,7 +616,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
             const int idx = tid + 256 * i;
             (&lq[b][0][0])[idx] = rq[i]; (&lk[b][0][0])[idx] = rk[i]; (&lg[b][0][0])[idx] = rg[i];
         }
-        if (tid < TC * 16) { lv[b][tid / 16][tid % 16] = rv; if (tid % 16 == 0) lb[b][tid / 16] = rb; }
+        if (tid < TC * NC) { lv[b][tid / NC][tid % NC] = rv; if (tid % NC == 0) lb[b][tid / NC] = rb; }
     };
     fetch(0);
     put(0);
@@ -507,17 +624,29 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
     for (int t0 = 0, b = 0; t0 < n; t0 += TC, b ^= 1) {
         if (t0 + TC < n) fetch(t0 + TC);
         const int m = n - t0 < TC ? n - t0 : TC;
+        float cq[RPL], ck[RPL], cg[RPL], cv, cb; /* this token's operands; the next one's are read while this one is used */
+        auto read = [&](int i) {
+#pragma unroll
+            for (int e = 0; e < RPL; ++e) { cq[e] = lq[b][i][r0 + e]; ck[e] = lk[b][i][r0 + e]; cg[e] = lg[b][i][r0 + e]; }
+            cv = lv[b][i][cl]; cb = lb[b][i];
+        };
+        read(0);
         for (int i = 0; i < m; ++i) {
+            float q[RPL], k[RPL], g[RPL];
+#pragma unroll
+            for (int e = 0; e < RPL; ++e) { q[e] = cq[e]; k[e] = ck[e]; g[e] = cg[e]; }
+            const float v = cv, beta = cb;
+            if (i + 1 < m) read(i + 1);
             float sk = 0.0f;
 #pragma unroll
-            for (int e = 0; e < RPL; ++e) { S[e] *= lg[b][i][r0 + e]; sk += S[e] * lk[b][i][r0 + e]; }
-            sk = row16_sum(sk);
-            const float u = lb[b][i] * (lv[b][i][cl] - sk);
+            for (int e = 0; e < RPL; ++e) { S[e] *= g[e]; sk = fmaf(S[e], k[e], sk); }
+            sk = LN == 16 ? tk_row16_sum(sk) : tk_row32_sum(sk);
+            const float u = beta * (v - sk);
             float so = 0.0f;
 #pragma unroll
-            for (int e = 0; e < RPL; ++e) { S[e] += lk[b][i][r0 + e] * u; so += S[e] * lq[b][i][r0 + e]; }
-            so = row16_sum(so);
-            if ((lane & 15) == 0 && live) d.o[((size_t)(row0 + t0 + i) * d.heads + h) * d.vdim + col] = so;
+            for (int e = 0; e < RPL; ++e) { S[e] = fmaf(k[e], u, S[e]); so = fmaf(S[e], q[e], so); }
+            so = LN == 16 ? tk_row16_sum(so) : tk_row32_sum(so);
+            if (lane % LN == 0 && live) d.o[((size_t)(row0 + t0 + i) * d.heads + h) * d.vdim + col] = so;
         }
         if (t0 + TC < n) put(b ^ 1); /* the other buffer was last read one iteration ago, before the barrier below */
         __syncthreads();
@@ -550,14 +679,12 @@ __global__ __launch_bounds__(256) void k_delta_out(TkDeltaArgs d) {
 /* one token of one head: the state is read once and written once, a thread holds RPT rows x 4 columns of it.
  * o = S_new^T q = (g S)^T q + (k . q) u, so both reductions over the key rows run on the decayed old state at once. */
 template <typename T, int THREADS, int RPT>
-__global__ __launch_bounds__(THREADS) void k_delta_step(TkDeltaArgs d, TkPassTab t, int ct_log2) {
-    extern __shared__ __attribute__((aligned(16))) float step_lds[];
-    __shared__ float red[16];
-    const int tid = threadIdx.x, row = blockIdx.y, h = blockIdx.x, kvh = h / (d.heads / d.kv_heads), vp = (d.vdim + 3) & ~3;
+__device__ __forceinline__ void delta_row(const TkDeltaArgs& d, const TkPassTab& t, int h, int row, int ct_log2, float* step_lds) {
+    const int tid = threadIdx.x, kvh = h / (d.heads / d.kv_heads), vp = (d.vdim + 3) & ~3;
     const int ct = tid & ((1 << ct_log2) - 1), rg = tid >> ct_log2, RG = THREADS >> ct_log2;
     const bool live = 4 * ct < vp;
     const int seg = t.seg[row], in = t.seg_in[seg], out = t.seg_out[seg];
-    float *lq = step_lds, *lk = lq + d.dim, *lg = lk + d.dim, *lu = step_lds + (3 * d.dim + 3) / 4 * 4, *pk = lu + vp, *pq = pk + RG * vp;
+    float *red = step_lds, *lq = red + 16, *lk = lq + d.dim, *lg = lk + d.dim, *lu = red + 16 + (3 * d.dim + 3) / 4 * 4, *pk = lu + vp, *pq = pk + RG * vp;
     tk_v4f S[RPT];
     const float* sin = d.state + ((size_t)(in < 0 ? 0 : in) * d.heads + h) * d.dim * vp + 4 * ct;
 #pragma unroll
@@ -606,6 +733,25 @@ __global__ __launch_bounds__(THREADS) void k_delta_step(TkDeltaArgs d, TkPassTab
         const float gate = tk_sigmoid32(d.low[(size_t)row * d.low_ld + d.low_g + h * d.vdim + tid]);
         tk_img_put((T*)d.out_img, row, d.out_k0 + h * d.vdim + tid, d.out_ktiles, o * r * d.norm[tid] * gate * d.out_scale);
     }
+}
+
+static size_t delta_row_lds(const TkDeltaArgs& d, int threads, int ct_log2) {
+    const size_t vp = (d.vdim + 3) & ~3;
+    return (16 + (size_t)(3 * d.dim + 3) / 4 * 4 + vp + 2 * (size_t)(threads >> ct_log2) * vp) * sizeof(float);
+}
+
+template <typename T, int THREADS, int RPT>
+__global__ __launch_bounds__(THREADS) void k_delta_step(TkDeltaArgs d, TkPassTab t, int ct_log2) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    delta_row<T, THREADS, RPT>(d, t, blockIdx.x, blockIdx.y, ct_log2, (float*)lds);
+}
+
+/* a decode step's attention and delta rule side by side: the first na workgroups of a row are attention's, the others one delta head each */
+template <typename T, int B, int WAVES, int RPT>
+__global__ __launch_bounds__(64 * WAVES) void k_mixers_step(TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int ct_log2) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    if ((int)blockIdx.x < na) attn_row<T, B, WAVES>(a, t, blockIdx.x, blockIdx.y, 0, 1, nullptr, lds);
+    else delta_row<T, 64 * WAVES, RPT>(d, t, blockIdx.x - na, blockIdx.y, ct_log2, (float*)lds);
 }
 
 __global__ void k_swap_state(TkPassTab t, int n) {
@@ -706,15 +852,20 @@ __global__ __launch_bounds__(256) void k_moe_gather(const tk_v4u* img, tk_v4u* o
 
 #define TK_TYPED(type, ...) do { if ((type) == TK_IMG_F32) { typedef float T; __VA_ARGS__; } else { typedef TkBf16 T; __VA_ARGS__; } } while (0)
 
+#define TK_VEC(vec, ...) do { if (vec) { constexpr bool VEC = true; __VA_ARGS__; } else { constexpr bool VEC = false; __VA_ARGS__; } } while (0)
+static int norm_threads(int width) { return width > 2048 ? 512 : 256; }
+
 void tk_launch_layer_embed(int type, const uint16_t* table, int width, const int32_t* tok, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, hipLaunchKernelGGL((k_layer_embed<T>), dim3(nrows), dim3(256), 0, s, table, width, tok, x, (T*)img, ktiles));
+    TK_TYPED(type, TK_VEC(width % 8 == 0, hipLaunchKernelGGL((k_layer_embed<T, VEC>), dim3(nrows), dim3(256), 0, s, table, width, tok, x, (T*)img, ktiles)));
 }
 
 void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs* attn, const TkDeltaArgs* delta, const TkPassTab& t, int nrows, hipStream_t s) {
     const TkAttnArgs a = attn ? *attn : TkAttnArgs{};
     const TkDeltaArgs d = delta ? *delta : TkDeltaArgs{};
     const int na = attn ? a.heads + 2 * a.kv_heads : 0, nd = delta ? 2 * d.kv_heads + 2 * d.heads : 0;
-    TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T>), dim3((na + nd + 3) / 4, nrows), dim3(256), 0, s, proj, ld, a, d, t, na, nd));
+    const int gx = (na + nd + 3) / 4;
+    if (nrows >= 512) TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, 4>), dim3(gx, (nrows + 3) / 4), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows));
+    else TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, 1>), dim3(gx, nrows), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows));
 }
 
 static int attn_bucket(const TkAttnArgs& a) {
@@ -735,49 +886,91 @@ void tk_launch_attn_tiles(int type, const TkAttnArgs& a, const TkPassTab& t, con
 
 size_t tk_attn_rows_scratch_floats(const TkAttnArgs& a, int nrows, int splits) { return splits > 1 ? (size_t)nrows * a.heads * splits * (a.kv.vdim_pad + 2) : 0; }
 
+static int attn_row_blocks(const TkAttnArgs& a) { return a.kv_heads * ((a.heads / a.kv_heads + 15) / 16); }
+/* waves of a row's workgroup: eight where the pass has few workgroups (a latency chain of pages), four where it has many */
+static int attn_row_waves(const TkAttnArgs& a, int nrows) { return nrows * attn_row_blocks(a) < 512 && attn_bucket(a) < 256 ? 8 : 4; }
+
+int tk_attn_rows_splits(const TkAttnArgs& a, int pages, int nrows) {
+    const int wgs = nrows * attn_row_blocks(a), want = (512 + wgs - 1) / wgs, most = pages / (2 * attn_row_waves(a, nrows));
+    const int s = want < most ? want : most;
+    return s < 1 ? 1 : s > 32 ? 32 : s;
+}
+
+#define TK_ROWS(B, W) hipLaunchKernelGGL((k_attn_rows<T, B, W>), grid, dim3(64 * W), (attn_row_lds<B, W>()), s, a, t, splits, scratch)
 void tk_launch_attn_rows(int type, const TkAttnArgs& a, const TkPassTab& t, int nrows, int splits, float* scratch, hipStream_t s) {
-    const int b = attn_bucket(a), gq = a.heads / a.kv_heads;
+    const int b = attn_bucket(a);
+    const bool eight = attn_row_waves(a, nrows) == 8;
     TK_TYPED(type, {
-        const dim3 grid(a.kv_heads * ((gq + 15) / 16), nrows, splits);
-        if (b == 64) hipLaunchKernelGGL((k_attn_rows<T, 64>), grid, dim3(256), 0, s, a, t, splits, scratch);
-        else if (b == 128) hipLaunchKernelGGL((k_attn_rows<T, 128>), grid, dim3(256), 0, s, a, t, splits, scratch);
-        else hipLaunchKernelGGL((k_attn_rows<T, 256>), grid, dim3(256), 0, s, a, t, splits, scratch);
+        const dim3 grid(attn_row_blocks(a), nrows, splits);
+        if (b == 64) { if (eight) TK_ROWS(64, 8); else TK_ROWS(64, 4); }
+        else if (b == 128) { if (eight) TK_ROWS(128, 8); else TK_ROWS(128, 4); }
+        else TK_ROWS(256, 4);
         if (splits > 1) hipLaunchKernelGGL((k_attn_merge<T>), dim3(a.heads, nrows), dim3(64), 0, s, a, splits, scratch);
     });
 }
 
+#undef TK_ROWS
+
+/* column threads of a delta row: the power of two that covers vdim in fours */
+static int delta_ct_log2(const TkDeltaArgs& d) {
+    int l = 0;
+    while ((4 << l) < d.vdim) ++l;
+    return l;
+}
+
+bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s) {
+    const int b = attn_bucket(a), ctl = delta_ct_log2(d), waves = attn_row_waves(a, nrows), threads = 64 * waves;
+    const int rg = threads >> ctl, rpt = rg ? (d.dim + rg - 1) / rg : 1 << 20;
+    if (type != TK_IMG_BF16 || b > 128 || rpt > (waves == 8 ? 8 : 16) || d.vdim > threads) return false;
+    const dim3 grid(attn_row_blocks(a) + d.heads, nrows);
+    const size_t dl = delta_row_lds(d, threads, ctl);
+#define TK_STEP(B, W, R) do { const size_t al = attn_row_lds<B, W>(); \
+        hipLaunchKernelGGL((k_mixers_step<TkBf16, B, W, R>), grid, dim3(threads), al > dl ? al : dl, s, a, d, t, attn_row_blocks(a), ctl); } while (0)
+    if (b == 64) { if (waves == 8) TK_STEP(64, 8, 8); else TK_STEP(64, 4, 16); }
+    else { if (waves == 8) TK_STEP(128, 8, 8); else TK_STEP(128, 4, 16); }
+#undef TK_STEP
+    return true;
+}
+
 void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, int n_segments, int nrows, hipStream_t s) {
-    const dim3 grid((d.vdim + 15) / 16, d.heads, n_segments);
-    const int rpl = (d.dim + 15) / 16;
-    if (rpl <= 2) hipLaunchKernelGGL((k_delta_scan<2>), grid, dim3(256), 0, s, d, t);
-    else if (rpl <= 4) hipLaunchKernelGGL((k_delta_scan<4>), grid, dim3(256), 0, s, d, t);
-    else if (rpl <= 8) hipLaunchKernelGGL((k_delta_scan<8>), grid, dim3(256), 0, s, d, t);
-    else hipLaunchKernelGGL((k_delta_scan<16>), grid, dim3(256), 0, s, d, t);
+    /* few columns over all: 32 lanes each, half the key rows per lane */
+    const bool thin = (int64_t)((d.vdim + 15) / 16) * d.heads * n_segments < 512;
+    const dim3 grid(thin ? (d.vdim + 7) / 8 : (d.vdim + 15) / 16, d.heads, n_segments);
+#define TK_SCAN(LN, RPL) hipLaunchKernelGGL((k_delta_scan<LN, RPL>), grid, dim3(256), 0, s, d, t)
+    if (thin) {
+        if (d.dim <= 32) TK_SCAN(32, 1);
+        else if (d.dim <= 64) TK_SCAN(32, 2);
+        else if (d.dim <= 128) TK_SCAN(32, 4);
+        else TK_SCAN(32, 8);
+    } else {
+        if (d.dim <= 32) TK_SCAN(16, 2);
+        else if (d.dim <= 64) TK_SCAN(16, 4);
+        else if (d.dim <= 128) TK_SCAN(16, 8);
+        else TK_SCAN(16, 16);
+    }
+#undef TK_SCAN
     TK_TYPED(type, hipLaunchKernelGGL((k_delta_out<T>), dim3((d.heads + 3) / 4, nrows), dim3(256), 0, s, d));
 }
 
 void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s) {
-    const int vp = (d.vdim + 3) & ~3;
-    int ctl = 0;
-    while ((4 << ctl) < vp) ++ctl;
+    const int ctl = delta_ct_log2(d);
     const dim3 grid(d.heads, nrows);
     auto rpt = [&](int threads) { const int rg = threads >> ctl; return (d.dim + rg - 1) / rg; };
-    auto lds = [&](int threads) { return ((size_t)(3 * d.dim + 3) / 4 * 4 + vp + 2 * (size_t)(threads >> ctl) * vp) * sizeof(float); };
     TK_TYPED(type, {
-        if (rpt(256) <= 4) hipLaunchKernelGGL((k_delta_step<T, 256, 4>), grid, dim3(256), lds(256), s, d, t, ctl);
-        else if (rpt(256) <= 8) hipLaunchKernelGGL((k_delta_step<T, 256, 8>), grid, dim3(256), lds(256), s, d, t, ctl);
-        else if (rpt(256) <= 16) hipLaunchKernelGGL((k_delta_step<T, 256, 16>), grid, dim3(256), lds(256), s, d, t, ctl);
-        else if (rpt(256) <= 32) hipLaunchKernelGGL((k_delta_step<T, 256, 32>), grid, dim3(256), lds(256), s, d, t, ctl);
-        else hipLaunchKernelGGL((k_delta_step<T, 1024, 16>), grid, dim3(1024), lds(1024), s, d, t, ctl);
+        if (rpt(256) <= 4) hipLaunchKernelGGL((k_delta_step<T, 256, 4>), grid, dim3(256), delta_row_lds(d, 256, ctl), s, d, t, ctl);
+        else if (rpt(256) <= 8) hipLaunchKernelGGL((k_delta_step<T, 256, 8>), grid, dim3(256), delta_row_lds(d, 256, ctl), s, d, t, ctl);
+        else if (rpt(256) <= 16) hipLaunchKernelGGL((k_delta_step<T, 256, 16>), grid, dim3(256), delta_row_lds(d, 256, ctl), s, d, t, ctl);
+        else if (rpt(256) <= 32) hipLaunchKernelGGL((k_delta_step<T, 256, 32>), grid, dim3(256), delta_row_lds(d, 256, ctl), s, d, t, ctl);
+        else hipLaunchKernelGGL((k_delta_step<T, 1024, 16>), grid, dim3(1024), delta_row_lds(d, 1024, ctl), s, d, t, ctl);
     });
 }
 
 void tk_launch_post_norm(int type, const TkSubOut& o, const float* w, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, hipLaunchKernelGGL((k_post_norm<T>), dim3(nrows), dim3(256), (size_t)width * sizeof(float), s, o, w, eps, width, x, (T*)img, ktiles));
+    TK_TYPED(type, TK_VEC(width % 8 == 0 && o.ld % 4 == 0, hipLaunchKernelGGL((k_post_norm<T, VEC>), dim3(nrows), dim3(norm_threads(width)), (size_t)width * sizeof(float), s, o, w, eps, width, x, (T*)img, ktiles)));
 }
 
 void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const float* w, float eps, int width, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, hipLaunchKernelGGL((k_rows_norm<T>), dim3(n), dim3(256), 0, s, x, rows, w, eps, width, (T*)img, ktiles));
+    TK_TYPED(type, TK_VEC(width % 8 == 0, hipLaunchKernelGGL((k_rows_norm<T, VEC>), dim3(n), dim3(norm_threads(width)), 0, s, x, rows, w, eps, width, (T*)img, ktiles)));
 }
 
 void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, const TkMoeTab& t, hipStream_t s) {

@@ -57,11 +57,43 @@ __device__ __forceinline__ void tk_img_put4(TkBf16* img, int64_t row, int k, int
     *(tk_v2u*)(img + tk_img_index<TkBf16>(row, k, ktiles)) = p;
 }
 
-__device__ __forceinline__ float tk_wave_sum(float v) {
+/* eight consecutive k, k % 8 == 0 */
+__device__ __forceinline__ void tk_img_put8(float* img, int64_t row, int k, int ktiles, tk_v4f a, tk_v4f b) { tk_img_put4(img, row, k, ktiles, a); tk_img_put4(img, row, k + 4, ktiles, b); }
+__device__ __forceinline__ void tk_img_put8(TkBf16* img, int64_t row, int k, int ktiles, tk_v4f a, tk_v4f b) {
+    tk_v4u p;
 #pragma unroll
-    for (int s = 32; s >= 1; s >>= 1) v += __shfl_xor(v, s, 64);
+    for (int i = 0; i < 2; ++i) {
+        p[i] = (uint32_t)tk_bf16_bits(a[2 * i]) | (uint32_t)tk_bf16_bits(a[2 * i + 1]) << 16;
+        p[2 + i] = (uint32_t)tk_bf16_bits(b[2 * i]) | (uint32_t)tk_bf16_bits(b[2 * i + 1]) << 16;
+    }
+    *(tk_v4u*)(img + tk_img_index<TkBf16>(row, k, ktiles)) = p;
+}
+
+/* lane exchanges on the vector pipe: DPP rotations inside a row of 16 lanes, row and half-wave swaps between rows */
+template <int CTRL> __device__ __forceinline__ float tk_dpp(float v) { return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false)); }
+/* sum over the 16 lanes of a row, in every lane of it (row_ror 8, 4, 2, 1) */
+__device__ __forceinline__ float tk_row16_sum(float v) {
+    v += tk_dpp<0x128>(v);
+    v += tk_dpp<0x124>(v);
+    v += tk_dpp<0x122>(v);
+    v += tk_dpp<0x121>(v);
     return v;
 }
+/* the values of a pair of rows (lanes l, l ^ 16) or of the two halves (l, l ^ 32), in every lane */
+struct TkPair { float a, b; };
+__device__ __forceinline__ TkPair tk_rows(float v) {
+    const auto p = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return TkPair{__uint_as_float(p[0]), __uint_as_float(p[1])};
+}
+__device__ __forceinline__ TkPair tk_halves(float v) {
+    const auto p = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return TkPair{__uint_as_float(p[0]), __uint_as_float(p[1])};
+}
+__device__ __forceinline__ float tk_row32_sum(float v) { const TkPair p = tk_rows(tk_row16_sum(v)); return p.a + p.b; }
+__device__ __forceinline__ float tk_wave_sum(float v) { const TkPair p = tk_halves(tk_row32_sum(v)); return p.a + p.b; }
+/* over the four lanes l % 16 + 16 g */
+__device__ __forceinline__ float tk_quad_sum(float v) { const TkPair p = tk_rows(v); const TkPair q = tk_halves(p.a + p.b); return q.a + q.b; }
+__device__ __forceinline__ float tk_quad_max(float v) { const TkPair p = tk_rows(v); const TkPair q = tk_halves(fmaxf(p.a, p.b)); return fmaxf(q.a, q.b); }
 __device__ __forceinline__ float tk_sigmoid32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float tk_silu32(float z) { return z / (1.0f + expf(-z)); }
 
