@@ -229,6 +229,30 @@ def test_unequal_requests_share_passes_pages_and_slots(cases, dtype, tol):
     assert s.cache_usage() == (0, 8)
 
 
+@pytest.mark.parametrize("dim,vdim", [(20, 20), (40, 36), (70, 17), (130, 20)])
+def test_many_heads_and_sequences(gpu, tmp_path, dim, vdim):
+    """the recurrence's form for many columns at once: eight sequences of unequal length x 32 heads in one pass, then portions and single tokens"""
+    cfg = config(40, 50, [layer(attention(2, 2, 8, 8, 4, 7, 1), delta(32, 16, dim, vdim, 4), dense(24))])
+    c = Case(gpu, tmp_path, cfg, seed=dim)
+    prompts = [tokens_for(cfg, 21 + 5 * i, i) for i in range(8)]
+    s = c.session("float32", 8, 64)
+    got = [[] for _ in prompts]
+    for lo, hi in ((0, 19), (19, 21), (21, 60)):
+        seq, pos, tok = [], [], []
+        for i, p in enumerate(prompts):
+            part = p[lo:hi]
+            seq += [i] * len(part)
+            pos += range(lo, lo + len(part))
+            tok += part
+        if lo == 21:  # the first sequence has ended
+            assert 0 not in seq
+        lg, _ = s.forward_rows(seq, pos, tok, range(len(seq)))
+        for r, i in enumerate(seq):
+            got[i].append(lg[r])
+    for p, rows in zip(prompts, got):
+        assert close(np.array(rows), c.want(p)[0], F32)
+
+
 def test_wanted_rows_only(cases):
     c = cases("odd")
     toks = tokens_for(c.cfg, 100)

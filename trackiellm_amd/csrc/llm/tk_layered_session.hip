@@ -265,11 +265,10 @@ void TkLayeredSession::enqueue_moe(const TkLayerSpec& s, const TkLayeredLayer& L
     g.type = type; g.w = L.router.img; g.a = img_x_; g.K = L.router.K; g.N = L.router.N; g.nrows = nrows;
     g.out = router_; g.ldc = L.router.N; g.n_valid = f.experts;
     gemm(g);
-    tk_launch_moe_select(router_, L.router.N, f.experts, f.top, f.groups, f.keep, nrows, moe_, stream);
     const int64_t assign = (int64_t)nrows * f.top;
     const int64_t per = assign / f.experts;
     const int bt = per <= 16 ? 1 : per <= 32 ? 2 : per <= 64 ? 4 : 8;
-    tk_launch_moe_plan(f.experts, bt, moe_, stream);
+    tk_launch_moe_select(router_, L.router.N, f.experts, f.top, f.groups, f.keep, nrows, bt, moe_, stream);
     tk_launch_moe_gather(img_x_, img_gather_, xkt, f.top, nrows, moe_, stream);
     TkImgGemm u{};
     u.type = type; u.w = L.gate_up.img; u.a = img_gather_; u.K = L.gate_up.K; u.N = L.gate_up.N;

@@ -99,8 +99,8 @@ struct TkMoeTab {
     TkImgBlock* blocks;
     int32_t* n_blocks;
 };
-void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, const TkMoeTab& t, hipStream_t s);
-void tk_launch_moe_plan(int experts, int block_tiles, const TkMoeTab& t, hipStream_t s);
+/* router logits -> chosen experts, weights, ranks, first tiles and row blocks of at most block_tiles tiles */
+void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, int block_tiles, const TkMoeTab& t, hipStream_t s);
 void tk_launch_moe_gather(const void* img, void* gathered, int ktiles, int top, int nrows, const TkMoeTab& t, hipStream_t s);
 
 /* end of a pass in a device-driven loop: every single-row segment reads next what it has just written */

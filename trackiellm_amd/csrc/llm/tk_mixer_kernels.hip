@@ -577,8 +577,9 @@ __global__ __launch_bounds__(64) void k_attn_merge(TkAttnArgs a, int splits, con
 
 /* ------------------------------------------------------------------ gated delta rule ------- */
 
-/* A workgroup walks 4 * 64 / LN columns of one head's state through a segment; a column is LN lanes x RPL key rows, so the column's recurrence
- * never leaves the wave.  q, k, decays, v and step sizes of TC tokens at a time go through LDS, the next TC in flight in registers. */
+/* A workgroup walks 4 * 64 / LN columns of one head's state through a segment; a column is LN lanes x RPL key rows, so its recurrence never
+ * leaves the wave.  q, k, decays, v and step sizes of TC tokens at a time go through LDS, the next TC in flight in registers.  32 lanes a column
+ * where columns are few (the shorter chain), 16 where they are many (fewer operand reads per column). */
 template <int LN, int RPL>
 __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) {
     constexpr int DP = LN * RPL, TC = DP > 128 ? 8 : 16, NL = TC * DP / 256, CW = 64 / LN, NC = 4 * CW;
@@ -607,8 +608,8 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
         if (tid < TC * NC) {
             const int tt = t0 + tid / NC, c = blockIdx.x * NC + tid % NC;
             rv = tt < n && c < d.vdim ? d.v[((size_t)(row0 + tt) * d.heads + h) * d.vdim + c] : 0.0f;
-            if (tid % NC == 0) rb = tt < n ? d.beta[(size_t)(row0 + tt) * d.heads + h] : 0.0f;
         }
+        if (tid < TC) rb = t0 + tid < n ? d.beta[(size_t)(row0 + t0 + tid) * d.heads + h] : 0.0f;
     };
     auto put = [&](int b) {
 #pragma unroll
@@ -616,7 +617,8 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
             const int idx = tid + 256 * i;
             (&lq[b][0][0])[idx] = rq[i]; (&lk[b][0][0])[idx] = rk[i]; (&lg[b][0][0])[idx] = rg[i];
         }
-        if (tid < TC * NC) { lv[b][tid / NC][tid % NC] = rv; if (tid % NC == 0) lb[b][tid / NC] = rb; }
+        if (tid < TC * NC) lv[b][tid / NC][tid % NC] = rv;
+        if (tid < TC) lb[b][tid] = rb;
     };
     fetch(0);
     put(0);
@@ -624,27 +626,14 @@ __global__ __launch_bounds__(256) void k_delta_scan(TkDeltaArgs d, TkPassTab t) 
     for (int t0 = 0, b = 0; t0 < n; t0 += TC, b ^= 1) {
         if (t0 + TC < n) fetch(t0 + TC);
         const int m = n - t0 < TC ? n - t0 : TC;
-        float cq[RPL], ck[RPL], cg[RPL], cv, cb; /* this token's operands; the next one's are read while this one is used */
-        auto read = [&](int i) {
-#pragma unroll
-            for (int e = 0; e < RPL; ++e) { cq[e] = lq[b][i][r0 + e]; ck[e] = lk[b][i][r0 + e]; cg[e] = lg[b][i][r0 + e]; }
-            cv = lv[b][i][cl]; cb = lb[b][i];
-        };
-        read(0);
         for (int i = 0; i < m; ++i) {
-            float q[RPL], k[RPL], g[RPL];
+            float sk = 0.0f, so = 0.0f;
 #pragma unroll
-            for (int e = 0; e < RPL; ++e) { q[e] = cq[e]; k[e] = ck[e]; g[e] = cg[e]; }
-            const float v = cv, beta = cb;
-            if (i + 1 < m) read(i + 1);
-            float sk = 0.0f;
-#pragma unroll
-            for (int e = 0; e < RPL; ++e) { S[e] *= g[e]; sk = fmaf(S[e], k[e], sk); }
+            for (int e = 0; e < RPL; ++e) { S[e] *= lg[b][i][r0 + e]; sk = fmaf(S[e], lk[b][i][r0 + e], sk); }
             sk = LN == 16 ? tk_row16_sum(sk) : tk_row32_sum(sk);
-            const float u = beta * (v - sk);
-            float so = 0.0f;
+            const float u = lb[b][i] * (lv[b][i][cl] - sk);
 #pragma unroll
-            for (int e = 0; e < RPL; ++e) { S[e] = fmaf(k[e], u, S[e]); so = fmaf(S[e], q[e], so); }
+            for (int e = 0; e < RPL; ++e) { S[e] = fmaf(lk[b][i][r0 + e], u, S[e]); so = fmaf(S[e], lq[b][i][r0 + e], so); }
             so = LN == 16 ? tk_row16_sum(so) : tk_row32_sum(so);
             if (lane % LN == 0 && live) d.o[((size_t)(row0 + t0 + i) * d.heads + h) * d.vdim + col] = so;
         }
@@ -761,13 +750,45 @@ __global__ void k_swap_state(TkPassTab t, int n) {
 
 /* ------------------------------------------------------------------ mixture of experts ----- */
 
-__global__ __launch_bounds__(64) void k_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, TkMoeTab t) {
-    __shared__ float sc[TK_MAX_EXPERTS], gs[64];
-    __shared__ int on[64];
-    const int row = blockIdx.x, lane = threadIdx.x, per = experts / groups;
-    for (int e = lane; e < experts; e += 64) sc[e] = tk_sigmoid32(logits[(size_t)row * ld + e]);
+/* experts' tile counts (threads 0 .. 255, one expert each) -> first tiles and row blocks.  Every thread of the workgroup calls it. */
+__device__ __forceinline__ void moe_plan(int experts, int block_tiles, int count, const TkMoeTab& t, int* st /* [512] LDS */) {
+    const int e = threadIdx.x;
+    const int tiles = e < experts ? (count + 15) / 16 : 0, nb = (tiles + block_tiles - 1) / block_tiles;
+    int* sb = st + 256;
+    if (e < 256) { st[e] = tiles; sb[e] = nb; }
     __syncthreads();
-    if (lane < groups) { /* a group's score: the sum of its two best */
+    for (int s = 1; s < 256; s <<= 1) { /* inclusive sums */
+        const int a = e < 256 && e >= s ? st[e - s] : 0, b = e < 256 && e >= s ? sb[e - s] : 0;
+        __syncthreads();
+        if (e < 256) { st[e] += a; sb[e] += b; }
+        __syncthreads();
+    }
+    if (e < experts) {
+        const int tile0 = st[e] - tiles, b0 = sb[e] - nb;
+        t.tile0[e] = tile0;
+        for (int i = 0; i < nb; ++i) {
+            const int left = tiles - i * block_tiles;
+            t.blocks[b0 + i] = TkImgBlock{e, tile0 + i * block_tiles, left < block_tiles ? left : block_tiles, 0};
+        }
+    }
+    if (e == 255) *t.n_blocks = sb[255];
+}
+
+/* one wave per row, 16 rows per workgroup; an expert's rows are counted in LDS first, one global addition per workgroup and expert.  A launch of
+ * one workgroup goes on to the plan itself. */
+__global__ __launch_bounds__(1024) void k_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, int block_tiles, TkMoeTab t) {
+    __shared__ float sc_[16][TK_MAX_EXPERTS], gs_[16][64];
+    __shared__ uint8_t on_[16][64];
+    __shared__ int cnt[TK_MAX_EXPERTS], base[TK_MAX_EXPERTS], st[512];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, row = blockIdx.x * 16 + wave, per = experts / groups;
+    const bool live = row < nrows;
+    float *sc = sc_[wave], *gs = gs_[wave];
+    uint8_t* on = on_[wave];
+    if (threadIdx.x < TK_MAX_EXPERTS) cnt[threadIdx.x] = 0;
+    if (live)
+        for (int e = lane; e < experts; e += 64) sc[e] = tk_sigmoid32(logits[(size_t)row * ld + e]);
+    __syncthreads();
+    if (live && lane < groups) { /* a group's score: the sum of its two best */
         float a = -INFINITY, b = -INFINITY;
         for (int e = lane * per; e < (lane + 1) * per; ++e) {
             const float v = sc[e];
@@ -776,64 +797,60 @@ __global__ __launch_bounds__(64) void k_moe_select(const float* logits, int ld, 
         gs[lane] = per > 1 ? a + b : a;
     }
     __syncthreads();
-    if (lane < groups) {
+    if (live && lane < groups) {
         int better = 0;
         for (int j = 0; j < groups; ++j) better += gs[j] > gs[lane] || (gs[j] == gs[lane] && j < lane);
         on[lane] = better < keep;
     }
     __syncthreads();
-    float c[TK_MAX_EXPERTS / 64]; /* this lane's candidates */
+    int mine = 0, rank = 0; /* lane j keeps the row's j-th choice */
+    if (live) {
+        float c[TK_MAX_EXPERTS / 64]; /* this lane's candidates */
 #pragma unroll
-    for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i) {
-        const int e = lane + 64 * i;
-        c[i] = e < experts && on[e / per] ? sc[e] : -INFINITY;
-    }
-    for (int j = 0; j < top; ++j) {
-        float best = -INFINITY;
-        int id = 0x7fffffff;
-#pragma unroll
-        for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
-            if (c[i] > best) { best = c[i]; id = lane + 64 * i; }
-        for (int s = 32; s >= 1; s >>= 1) {
-            const float ov = __shfl_xor(best, s, 64);
-            const int oi = __shfl_xor(id, s, 64);
-            if (ov > best || (ov == best && oi < id)) { best = ov; id = oi; }
+        for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i) {
+            const int e = lane + 64 * i;
+            c[i] = e < experts && on[e / per] ? sc[e] : -INFINITY;
         }
-        if (id >= experts) id = 0; /* no finite score is left: a defined expert all the same */
+        for (int j = 0; j < top; ++j) {
+            float best = -INFINITY;
+            int id = 0x7fffffff;
 #pragma unroll
-        for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
-            if (lane + 64 * i == id) c[i] = -INFINITY;
-        if (lane == 0) {
-            t.expert[row * top + j] = id;
-            t.weight[row * top + j] = sc[id];
-            t.rank[row * top + j] = atomicAdd(t.count + id, 1);
+            for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
+                if (c[i] > best) { best = c[i]; id = lane + 64 * i; }
+            for (int s = 32; s >= 1; s >>= 1) {
+                const float ov = __shfl_xor(best, s, 64);
+                const int oi = __shfl_xor(id, s, 64);
+                if (ov > best || (ov == best && oi < id)) { best = ov; id = oi; }
+            }
+            if (id >= experts) id = 0; /* no finite score is left: a defined expert all the same */
+#pragma unroll
+            for (int i = 0; i < TK_MAX_EXPERTS / 64; ++i)
+                if (lane + 64 * i == id) c[i] = -INFINITY;
+            if (lane == j) mine = id;
         }
+        if (lane < top) rank = atomicAdd(&cnt[mine], 1);
     }
+    __syncthreads();
+    if ((int)threadIdx.x < experts) {
+        const int n = cnt[threadIdx.x];
+        base[threadIdx.x] = gridDim.x > 1 && n > 0 ? atomicAdd(t.count + threadIdx.x, n) : 0;
+    }
+    __syncthreads();
+    if (live && lane < top) {
+        const int i = row * top + lane;
+        t.expert[i] = mine;
+        t.weight[i] = sc[mine];
+        t.rank[i] = base[mine] + rank;
+    }
+    if (gridDim.x == 1) moe_plan(experts, block_tiles, (int)threadIdx.x < experts ? cnt[threadIdx.x] : 0, t, st);
 }
 
-/* experts' row counts -> first tiles and row blocks; the counts are cleared for the next layer */
+/* the plan of a launch of several workgroups; the counts are cleared for the next layer */
 __global__ __launch_bounds__(256) void k_moe_plan(int experts, int block_tiles, TkMoeTab t) {
-    __shared__ int st[256], sb[256];
-    const int e = threadIdx.x;
-    const int tiles = e < experts ? (t.count[e] + 15) / 16 : 0, nb = (tiles + block_tiles - 1) / block_tiles;
-    st[e] = tiles; sb[e] = nb;
-    __syncthreads();
-    for (int s = 1; s < 256; s <<= 1) { /* inclusive sums */
-        const int a = e >= s ? st[e - s] : 0, b = e >= s ? sb[e - s] : 0;
-        __syncthreads();
-        st[e] += a; sb[e] += b;
-        __syncthreads();
-    }
-    const int tile0 = st[e] - tiles, b0 = sb[e] - nb;
-    if (e < experts) {
-        t.tile0[e] = tile0;
-        t.count[e] = 0;
-        for (int i = 0; i < nb; ++i) {
-            const int left = tiles - i * block_tiles;
-            t.blocks[b0 + i] = TkImgBlock{e, tile0 + i * block_tiles, left < block_tiles ? left : block_tiles, 0};
-        }
-    }
-    if (e == 255) *t.n_blocks = sb[255];
+    __shared__ int st[512];
+    const int e = threadIdx.x, n = e < experts ? t.count[e] : 0;
+    if (e < experts) t.count[e] = 0;
+    moe_plan(experts, block_tiles, n, t, st);
 }
 
 /* 16-byte pieces of a row of the image to its places among the experts' rows */
@@ -933,21 +950,13 @@ bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, 
 }
 
 void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, int n_segments, int nrows, hipStream_t s) {
-    /* few columns over all: 32 lanes each, half the key rows per lane */
-    const bool thin = (int64_t)((d.vdim + 15) / 16) * d.heads * n_segments < 512;
-    const dim3 grid(thin ? (d.vdim + 7) / 8 : (d.vdim + 15) / 16, d.heads, n_segments);
-#define TK_SCAN(LN, RPL) hipLaunchKernelGGL((k_delta_scan<LN, RPL>), grid, dim3(256), 0, s, d, t)
-    if (thin) {
-        if (d.dim <= 32) TK_SCAN(32, 1);
-        else if (d.dim <= 64) TK_SCAN(32, 2);
-        else if (d.dim <= 128) TK_SCAN(32, 4);
-        else TK_SCAN(32, 8);
-    } else {
-        if (d.dim <= 32) TK_SCAN(16, 2);
-        else if (d.dim <= 64) TK_SCAN(16, 4);
-        else if (d.dim <= 128) TK_SCAN(16, 8);
-        else TK_SCAN(16, 16);
-    }
+    const bool many = (int64_t)((d.vdim + 15) / 16) * d.heads * n_segments >= 512;
+    const dim3 grid(many ? (d.vdim + 15) / 16 : (d.vdim + 7) / 8, d.heads, n_segments);
+#define TK_SCAN(RPL) do { if (many) hipLaunchKernelGGL((k_delta_scan<16, 2 * RPL>), grid, dim3(256), 0, s, d, t); else hipLaunchKernelGGL((k_delta_scan<32, RPL>), grid, dim3(256), 0, s, d, t); } while (0)
+    if (d.dim <= 32) TK_SCAN(1);
+    else if (d.dim <= 64) TK_SCAN(2);
+    else if (d.dim <= 128) TK_SCAN(4);
+    else TK_SCAN(8);
 #undef TK_SCAN
     TK_TYPED(type, hipLaunchKernelGGL((k_delta_out<T>), dim3((d.heads + 3) / 4, nrows), dim3(256), 0, s, d));
 }
@@ -973,10 +982,11 @@ void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, c
     TK_TYPED(type, TK_VEC(width % 8 == 0, hipLaunchKernelGGL((k_rows_norm<T, VEC>), dim3(n), dim3(norm_threads(width)), 0, s, x, rows, w, eps, width, (T*)img, ktiles)));
 }
 
-void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, const TkMoeTab& t, hipStream_t s) {
-    hipLaunchKernelGGL(k_moe_select, dim3(nrows), dim3(64), 0, s, logits, ld, experts, top, groups, keep, t);
+void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, int block_tiles, const TkMoeTab& t, hipStream_t s) {
+    const int wgs = (nrows + 15) / 16;
+    hipLaunchKernelGGL(k_moe_select, dim3(wgs), dim3(1024), 0, s, logits, ld, experts, top, groups, keep, nrows, block_tiles, t);
+    if (wgs > 1) hipLaunchKernelGGL(k_moe_plan, dim3(1), dim3(256), 0, s, experts, block_tiles, t);
 }
-void tk_launch_moe_plan(int experts, int block_tiles, const TkMoeTab& t, hipStream_t s) { hipLaunchKernelGGL(k_moe_plan, dim3(1), dim3(256), 0, s, experts, block_tiles, t); }
 void tk_launch_moe_gather(const void* img, void* gathered, int ktiles, int top, int nrows, const TkMoeTab& t, hipStream_t s) {
     hipLaunchKernelGGL(k_moe_gather, dim3(nrows * top, (ktiles * 4 + 255) / 256), dim3(256), 0, s, (const tk_v4u*)img, (tk_v4u*)gathered, ktiles, top, t);
 }
