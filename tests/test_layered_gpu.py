@@ -25,6 +25,10 @@ CONFIGS = {
     # wide heads, one head, one tap, experts without groups, kept positions over more than one page
     "wide": config(64, 96, [layer(attention(1, 1, 128, 16, 128, 70, 5, base=500.0), delta(3, 3, 130, 8, 1), moe(16, 4, 1)),
                             layer(attention(2, 1, 160, 200, 32, 40, 70), delta(1, 1, 16, 256, 4), moe(33, 8, 4, (4, 4)), 0.5, 2.0)]),
+    # head sizes that fill the attention kernels' tiles exactly
+    "full": config(72, 80, [layer(attention(4, 2, 64, 64, 16, 50, 4), delta(2, 1, 32, 64, 4), dense(64)),
+                            layer(attention(2, 1, 128, 128, 64, 90, 1), delta(1, 1, 64, 128, 4), None),
+                            layer(attention(1, 1, 256, 256, 256, 66, 0), delta(1, 1, 128, 128, 4), moe(24, 4, 2))]),
     # more query heads per key head than a tile has rows, a large state
     "grouped": config(80, 64, [layer(attention(34, 2, 16, 16, 8, 130, 2, scale=0.4), delta(2, 1, 256, 256, 6), dense(48), 1.0, 1.0)]),
 }

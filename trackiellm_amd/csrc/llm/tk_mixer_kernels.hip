@@ -303,6 +303,24 @@ struct PageWalk {
     __device__ __forceinline__ int page(int i) const { return i < nkeep ? i : first + i - nkeep; }
 };
 
+/* scores of one page (raw products, keys k0 + 16 j + 4 g + r) -> log2 units, -inf where the query at position pq may not look.  lo .. hi: the lowest
+ * and highest query position of the wave; a page that all of them see whole is not masked. */
+__device__ __forceinline__ void mask_scores(tk_v4f (&s)[4], const TkAttnArgs& a, int k0, int g, int pq, int lo, int hi) {
+    const float c = a.scale * LOG2E;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) s[j] *= c;
+    if (k0 + TK_PAGE - 1 <= lo && (a.window <= 0 || hi - k0 < a.window || k0 + TK_PAGE <= a.keep_first)) return;
+    const int first = a.window > 0 ? pq - a.window + 1 : 0;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int key = k0 + 16 * j + 4 * g + r;
+            const bool see = (key <= pq) & ((key >= first) | (key < a.keep_first));
+            s[j][r] = see ? s[j][r] : -INFINITY;
+        }
+}
+
 /* running softmax of one wave: 16 queries (lane % 16), VT 16-wide tiles of the output (rows 4 (lane / 16) + r) */
 template <typename T, int VT>
 struct Flash {
@@ -397,76 +415,96 @@ __device__ __forceinline__ void attn_store(const TkAttnArgs& a, const tk_v4f (&o
     }
 }
 
-/* prompts: 64 consecutive positions of a sequence x one head per workgroup, 16 per wave; pages go through LDS (next page's loads are in flight
- * in registers while this one is used) */
-template <typename T, int B>
-__global__ __launch_bounds__(256) void k_attn_tiles(TkAttnArgs a, TkPassTab t, const int32_t* tiles) {
+/* prompts: 64 consecutive positions of a sequence x one head per workgroup, 16 per wave.  Pages go through two LDS buffers (one where two do not
+ * fit): while page i is used, page i + 1 is written to the other one and page i + 2 is on its way to registers. */
+template <typename T, int B> constexpr bool attn_two_buffers() { return sizeof(T) == 2 || B < 256; }
+
+template <typename T, int B, bool FULL /* head sizes fill the bucket */>
+__global__ __launch_bounds__(256, B * sizeof(T) >= 512 ? 1 : 2) void k_attn_tiles(TkAttnArgs a, TkPassTab t, const int32_t* tiles) {
     constexpr int DT = B / TkImg<T>::KT, VT = B / 16, SZ = sizeof(T);
     typedef typename VFrag<T>::type VF;
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4;
     const int row0 = tiles[2 * blockIdx.x], n = tiles[2 * blockIdx.x + 1], h = blockIdx.y, kvh = h / (a.heads / a.kv_heads);
-    const int nd = a.kv.dim_pad / TkImg<T>::KT, nv = a.kv.vdim_pad / 16;
+    const int nd = FULL ? DT : a.kv.dim_pad / TkImg<T>::KT, nv = FULL ? VT : a.kv.vdim_pad / 16;
     const int krow = a.kv.dim_pad * SZ + 16, vrow = TK_PAGE * SZ + 16; /* LDS pitches: rows start in different banks */
-    uint8_t *lk = lds, *lv = lds + TK_PAGE * krow;
+    const int buf = TK_PAGE * krow + a.kv.vdim_pad * vrow;
+    constexpr bool TWO = attn_two_buffers<T, B>();
     const int p0 = t.pos[row0], seq = t.seq[row0];
     const int q = wave * 16 + (lane & 15), live = q < n ? q : 0;
     const int pq = q < n ? p0 + q : -1; /* rows past the tile see nothing and store nothing */
+    const PageWalk walk(p0, p0 + n - 1, a.window, a.keep_first);
+    const int32_t* pages = t.page_of + (size_t)seq * t.max_pages;
+    int ids = pages[walk.page(lane < walk.count ? lane : 0)], ids0 = 0; /* lane l: page id of step ids0 + l */
+    const int kc = TK_PAGE * a.kv.dim_pad * SZ / 16, vc = a.kv.vdim_pad * TK_PAGE * SZ / 16; /* 16-byte pieces of a page */
+    constexpr int KP = TK_PAGE * B * SZ / 16 / 256, VP = B * TK_PAGE * SZ / 16 / 256;
+    tk_v4u kr[KP], vr[VP];
+    auto fetch = [&](int i) {
+        if (i - ids0 >= 64) {
+            ids0 = i;
+            ids = pages[walk.page(i + lane < walk.count ? i + lane : i)];
+        }
+        const size_t page = (size_t)__builtin_amdgcn_readlane(ids, i - ids0) * a.kv_heads + kvh;
+        const uint8_t* kp = (const uint8_t*)a.kv.k + page * TK_PAGE * a.kv.dim_pad * SZ;
+        const uint8_t* vp = (const uint8_t*)a.kv.v + page * a.kv.vdim_pad * TK_PAGE * SZ;
+#pragma unroll
+        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (FULL || p < kc) kr[c] = *(const tk_v4u*)(kp + (size_t)p * 16); }
+#pragma unroll
+        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (FULL || p < vc) vr[c] = *(const tk_v4u*)(vp + (size_t)p * 16); }
+    };
+    const int kpr = FULL ? B * SZ / 16 : a.kv.dim_pad * SZ / 16, vpr = TK_PAGE * SZ / 16; /* pieces of a row */
+    auto put = [&](int i) {
+        uint8_t *lk = lds + (TWO ? (i & 1) * buf : 0), *lv = lk + TK_PAGE * krow;
+#pragma unroll
+        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (FULL || p < kc) *(tk_v4u*)(lk + (p / kpr) * krow + (p % kpr) * 16) = kr[c]; }
+#pragma unroll
+        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (FULL || p < vc) *(tk_v4u*)(lv + (p / vpr) * vrow + (p % vpr) * 16) = vr[c]; }
+    };
+    fetch(0);
     tk_v4u qf[DT];
 #pragma unroll
     for (int d = 0; d < DT; ++d)
         if (d < nd) qf[d] = *(const tk_v4u*)((const uint8_t*)a.q + (((size_t)(row0 + live) * a.heads + h) * a.kv.dim_pad) * SZ + d * 64 + g * 16);
     Flash<T, VT> f;
     f.init();
-    const PageWalk walk(p0, p0 + n - 1, a.window, a.keep_first);
     const int wave_lo = p0 + wave * 16, wave_hi = p0 + (wave * 16 + 15 < n ? wave * 16 + 15 : n - 1);
-    const int kc = TK_PAGE * a.kv.dim_pad * SZ / 16, vc = a.kv.vdim_pad * TK_PAGE * SZ / 16; /* 16-byte pieces of a page */
-    constexpr int KP = TK_PAGE * B * SZ / 16 / 256, VP = B * TK_PAGE * SZ / 16 / 256;
-    tk_v4u kr[KP], vr[VP];
-    auto fetch = [&](int i) {
-        const size_t page = (size_t)t.page_of[(size_t)seq * t.max_pages + walk.page(i)] * a.kv_heads + kvh;
-        const uint8_t* kp = (const uint8_t*)a.kv.k + page * TK_PAGE * a.kv.dim_pad * SZ;
-        const uint8_t* vp = (const uint8_t*)a.kv.v + page * a.kv.vdim_pad * TK_PAGE * SZ;
-#pragma unroll
-        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (p < kc) kr[c] = *(const tk_v4u*)(kp + (size_t)p * 16); }
-#pragma unroll
-        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (p < vc) vr[c] = *(const tk_v4u*)(vp + (size_t)p * 16); }
-    };
-    const int kpr = a.kv.dim_pad * SZ / 16, vpr = TK_PAGE * SZ / 16; /* pieces of a row */
-    fetch(0);
+    put(0);
+    if (walk.count > 1) fetch(1);
+    __syncthreads();
     for (int i = 0; i < walk.count; ++i) {
-        __syncthreads();
-#pragma unroll
-        for (int c = 0; c < KP; ++c) { const int p = threadIdx.x + 256 * c; if (p < kc) *(tk_v4u*)(lk + (p / kpr) * krow + (p % kpr) * 16) = kr[c]; }
-#pragma unroll
-        for (int c = 0; c < VP; ++c) { const int p = threadIdx.x + 256 * c; if (p < vc) *(tk_v4u*)(lv + (p / vpr) * vrow + (p % vpr) * 16) = vr[c]; }
-        __syncthreads();
-        if (i + 1 < walk.count) fetch(i + 1);
-        const int k0 = walk.page(i) * TK_PAGE;
-        /* nothing of this page for this wave's rows */
-        if (wave * 16 >= n || k0 > wave_hi || (a.window > 0 && wave_lo - (k0 + TK_PAGE - 1) >= a.window && k0 >= a.keep_first)) continue;
-        tk_v4f s[4];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            s[j] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
-            const uint8_t* kp = lk + (16 * j + (lane & 15)) * krow + g * 16;
-#pragma unroll
-            for (int d = 0; d < DT; ++d)
-                if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + d * 64), qf[d], s[j]);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int key = k0 + 16 * j + 4 * g + r;
-                const bool see = key <= pq && (a.window <= 0 || pq - key < a.window || key < a.keep_first);
-                s[j][r] = see ? s[j][r] * (a.scale * LOG2E) : -INFINITY;
-            }
+        if (i > 0) { /* page i is in its buffer; every wave is done with page i - 1 */
+            if (!TWO) put(i);
+            __syncthreads();
         }
-        f.update(s, nv, [&](int vt, int j) { return *(const VF*)(lv + (16 * vt + (lane & 15)) * vrow + (16 * j + 4 * g) * SZ); });
+        if (TWO) {
+            if (i + 1 < walk.count) put(i + 1);
+            if (i + 2 < walk.count) fetch(i + 2);
+        } else if (i > 0 && i + 1 < walk.count) {
+            fetch(i + 1);
+        }
+        const uint8_t *lk = lds + (TWO ? (i & 1) * buf : 0), *lv = lk + TK_PAGE * krow;
+        const int k0 = walk.page(i) * TK_PAGE;
+        /* not a page that none of this wave's rows reads */
+        if (wave * 16 < n && k0 <= wave_hi && (a.window <= 0 || wave_lo - (k0 + TK_PAGE - 1) < a.window || k0 < a.keep_first)) {
+            tk_v4f s[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                s[j] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+                const uint8_t* kp = lk + (16 * j + (lane & 15)) * krow + g * 16;
+#pragma unroll
+                for (int d = 0; d < DT; ++d)
+                    if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + d * 64), qf[d], s[j]);
+            }
+            mask_scores(s, a, k0, g, pq, wave_lo, wave * 16 + 15 < n ? wave_hi : 0x40000000);
+            f.update(s, nv, [&](int vt, int j) { return *(const VF*)(lv + (16 * vt + (lane & 15)) * vrow + (16 * j + 4 * g) * SZ); });
+        }
+        if (!TWO) __syncthreads(); /* the only buffer is free again */
     }
     if (q < n) attn_store<T, VT>(a, f.o, row0 + q, h, g, a.out_scale / f.l);
 }
 
 /* decoding: one row x up to 16 query heads of one kv head per workgroup, pages dealt to the waves (and to `splits` workgroups), merged in LDS */
-template <typename T, int B, int WAVES>
+template <typename T, int B, int WAVES, bool FULL>
 __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t, int block, int row, int split, int splits, float* scratch, uint8_t* lds) {
     constexpr int DT = B / TkImg<T>::KT, VT = B / 16, SZ = sizeof(T);
     constexpr bool AHEAD = SZ == 2 && B <= 128; /* a page's values are requested together with its keys */
@@ -475,7 +513,7 @@ __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t
     const int gq = a.heads / a.kv_heads, per = (gq + 15) / 16;
     const int kvh = block / per, q = (block % per) * 16 + (lane & 15);
     const int h = kvh * gq + (q < gq ? q : 0);
-    const int nd = a.kv.dim_pad / TkImg<T>::KT, nv = a.kv.vdim_pad / 16;
+    const int nd = FULL ? DT : a.kv.dim_pad / TkImg<T>::KT, nv = FULL ? VT : a.kv.vdim_pad / 16;
     const int pos = t.pos[row], seq = t.seq[row];
     tk_v4u qf[DT];
 #pragma unroll
@@ -511,13 +549,8 @@ __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t
 #pragma unroll
             for (int d = 0; d < DT; ++d)
                 if (d < nd) s[j] = TkImg<T>::mma(AHEAD ? kf[AHEAD ? j : 0][AHEAD ? d : 0] : *(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64), qf[d], s[j]);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int key = k0 + 16 * j + 4 * g + r;
-                const bool see = key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
-                s[j][r] = see ? s[j][r] * (a.scale * LOG2E) : -INFINITY;
-            }
         }
+        mask_scores(s, a, k0, g, pos, pos, pos);
         f.update(s, nv, [&](int vt, int j) { return AHEAD ? vf[AHEAD ? vt : 0][j] : vload(vt, j); });
     }
     /* the upper half of the waves into the lower half, and again */
@@ -553,10 +586,10 @@ __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t
 }
 template <int B, int WAVES> constexpr size_t attn_row_lds() { return (size_t)WAVES / 2 * (B / 16 * 1024 + 512); }
 
-template <typename T, int B, int WAVES>
-__global__ __launch_bounds__(64 * WAVES) void k_attn_rows(TkAttnArgs a, TkPassTab t, int splits, float* scratch) {
+template <typename T, int B, int WAVES, bool FULL>
+__global__ __launch_bounds__(64 * WAVES, B == 256 ? 1 : 2) void k_attn_rows(TkAttnArgs a, TkPassTab t, int splits, float* scratch) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    attn_row<T, B, WAVES>(a, t, blockIdx.x, blockIdx.y, blockIdx.z, splits, scratch, lds);
+    attn_row<T, B, WAVES, FULL>(a, t, blockIdx.x, blockIdx.y, blockIdx.z, splits, scratch, lds);
 }
 
 template <typename T>
@@ -736,10 +769,10 @@ __global__ __launch_bounds__(THREADS) void k_delta_step(TkDeltaArgs d, TkPassTab
 }
 
 /* a decode step's attention and delta rule side by side: the first na workgroups of a row are attention's, the others one delta head each */
-template <typename T, int B, int WAVES, int RPT>
-__global__ __launch_bounds__(64 * WAVES) void k_mixers_step(TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int ct_log2) {
+template <typename T, int B, int WAVES, int RPT, bool FULL>
+__global__ __launch_bounds__(64 * WAVES, 2) void k_mixers_step(TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int ct_log2) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    if ((int)blockIdx.x < na) attn_row<T, B, WAVES>(a, t, blockIdx.x, blockIdx.y, 0, 1, nullptr, lds);
+    if ((int)blockIdx.x < na) attn_row<T, B, WAVES, FULL>(a, t, blockIdx.x, blockIdx.y, 0, 1, nullptr, lds);
     else delta_row<T, 64 * WAVES, RPT>(d, t, blockIdx.x - na, blockIdx.y, ct_log2, (float*)lds);
 }
 
@@ -890,15 +923,19 @@ static int attn_bucket(const TkAttnArgs& a) {
     return m <= 64 ? 64 : m <= 128 ? 128 : 256;
 }
 
+static bool attn_full(const TkAttnArgs& a) { return a.kv.dim_pad == attn_bucket(a) && a.kv.vdim_pad == attn_bucket(a); }
+
 void tk_launch_attn_tiles(int type, const TkAttnArgs& a, const TkPassTab& t, const int32_t* tiles, int n_tiles, hipStream_t s) {
     const int b = attn_bucket(a);
-    TK_TYPED(type, {
-        const size_t lds = (size_t)TK_PAGE * (a.kv.dim_pad * sizeof(T) + 16) + (size_t)a.kv.vdim_pad * (TK_PAGE * sizeof(T) + 16);
-        const dim3 grid(n_tiles, a.heads);
-        if (b == 64) hipLaunchKernelGGL((k_attn_tiles<T, 64>), grid, dim3(256), lds, s, a, t, tiles);
-        else if (b == 128) hipLaunchKernelGGL((k_attn_tiles<T, 128>), grid, dim3(256), lds, s, a, t, tiles);
-        else hipLaunchKernelGGL((k_attn_tiles<T, 256>), grid, dim3(256), lds, s, a, t, tiles);
-    });
+    const dim3 grid(n_tiles, a.heads);
+    const size_t sz = type == TK_IMG_F32 ? 4 : 2, lds = (TK_PAGE * (a.kv.dim_pad * sz + 16) + a.kv.vdim_pad * (TK_PAGE * sz + 16)) * (type == TK_IMG_F32 && b == 256 ? 1 : 2);
+#define TK_TILES(T, B, F) hipLaunchKernelGGL((k_attn_tiles<T, B, F>), grid, dim3(256), lds, s, a, t, tiles)
+#define TK_TILES_B(T, F) do { if (b == 64) TK_TILES(T, 64, F); else if (b == 128) TK_TILES(T, 128, F); else TK_TILES(T, 256, F); } while (0)
+    if (type == TK_IMG_F32) TK_TILES_B(float, false);
+    else if (attn_full(a)) TK_TILES_B(TkBf16, true);
+    else TK_TILES_B(TkBf16, false);
+#undef TK_TILES_B
+#undef TK_TILES
 }
 
 size_t tk_attn_rows_scratch_floats(const TkAttnArgs& a, int nrows, int splits) { return splits > 1 ? (size_t)nrows * a.heads * splits * (a.kv.vdim_pad + 2) : 0; }
@@ -913,20 +950,22 @@ int tk_attn_rows_splits(const TkAttnArgs& a, int pages, int nrows) {
     return s < 1 ? 1 : s > 32 ? 32 : s;
 }
 
-#define TK_ROWS(B, W) hipLaunchKernelGGL((k_attn_rows<T, B, W>), grid, dim3(64 * W), (attn_row_lds<B, W>()), s, a, t, splits, scratch)
 void tk_launch_attn_rows(int type, const TkAttnArgs& a, const TkPassTab& t, int nrows, int splits, float* scratch, hipStream_t s) {
     const int b = attn_bucket(a);
     const bool eight = attn_row_waves(a, nrows) == 8;
-    TK_TYPED(type, {
-        const dim3 grid(attn_row_blocks(a), nrows, splits);
-        if (b == 64) { if (eight) TK_ROWS(64, 8); else TK_ROWS(64, 4); }
-        else if (b == 128) { if (eight) TK_ROWS(128, 8); else TK_ROWS(128, 4); }
-        else TK_ROWS(256, 4);
-        if (splits > 1) hipLaunchKernelGGL((k_attn_merge<T>), dim3(a.heads, nrows), dim3(64), 0, s, a, splits, scratch);
-    });
-}
-
+    const dim3 grid(attn_row_blocks(a), nrows, splits);
+#define TK_ROWS(T, B, W, F) hipLaunchKernelGGL((k_attn_rows<T, B, W, F>), grid, dim3(64 * W), (attn_row_lds<B, W>()), s, a, t, splits, scratch)
+#define TK_ROWS_B(T, F) do { \
+        if (b == 64) { if (eight) TK_ROWS(T, 64, 8, F); else TK_ROWS(T, 64, 4, F); } \
+        else if (b == 128) { if (eight) TK_ROWS(T, 128, 8, F); else TK_ROWS(T, 128, 4, F); } \
+        else TK_ROWS(T, 256, 4, F); } while (0)
+    if (type == TK_IMG_F32) TK_ROWS_B(float, false);
+    else if (attn_full(a)) TK_ROWS_B(TkBf16, true);
+    else TK_ROWS_B(TkBf16, false);
+#undef TK_ROWS_B
 #undef TK_ROWS
+    if (splits > 1) TK_TYPED(type, hipLaunchKernelGGL((k_attn_merge<T>), dim3(a.heads, nrows), dim3(64), 0, s, a, splits, scratch));
+}
 
 /* column threads of a delta row: the power of two that covers vdim in fours */
 static int delta_ct_log2(const TkDeltaArgs& d) {
@@ -942,7 +981,8 @@ bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, 
     const dim3 grid(attn_row_blocks(a) + d.heads, nrows);
     const size_t dl = delta_row_lds(d, threads, ctl);
 #define TK_STEP(B, W, R) do { const size_t al = attn_row_lds<B, W>(); \
-        hipLaunchKernelGGL((k_mixers_step<TkBf16, B, W, R>), grid, dim3(threads), al > dl ? al : dl, s, a, d, t, attn_row_blocks(a), ctl); } while (0)
+        if (attn_full(a)) hipLaunchKernelGGL((k_mixers_step<TkBf16, B, W, R, true>), grid, dim3(threads), al > dl ? al : dl, s, a, d, t, attn_row_blocks(a), ctl); \
+        else hipLaunchKernelGGL((k_mixers_step<TkBf16, B, W, R, false>), grid, dim3(threads), al > dl ? al : dl, s, a, d, t, attn_row_blocks(a), ctl); } while (0)
     if (b == 64) { if (waves == 8) TK_STEP(64, 8, 8); else TK_STEP(64, 4, 16); }
     else { if (waves == 8) TK_STEP(128, 8, 8); else TK_STEP(128, 4, 16); }
 #undef TK_STEP
@@ -1001,8 +1041,9 @@ const char* tk_mixer_prepare_device() {
     std::lock_guard<std::mutex> lk(mu);
     hipError_t e = hipSuccess;
     auto opt = [&](const void* f) { if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); };
-    opt((const void*)k_attn_tiles<float, 64>); opt((const void*)k_attn_tiles<float, 128>); opt((const void*)k_attn_tiles<float, 256>);
-    opt((const void*)k_attn_tiles<TkBf16, 64>); opt((const void*)k_attn_tiles<TkBf16, 128>); opt((const void*)k_attn_tiles<TkBf16, 256>);
+    opt((const void*)k_attn_tiles<float, 64, false>); opt((const void*)k_attn_tiles<float, 128, false>); opt((const void*)k_attn_tiles<float, 256, false>);
+    opt((const void*)k_attn_tiles<TkBf16, 64, false>); opt((const void*)k_attn_tiles<TkBf16, 128, false>); opt((const void*)k_attn_tiles<TkBf16, 256, false>);
+    opt((const void*)k_attn_tiles<TkBf16, 64, true>); opt((const void*)k_attn_tiles<TkBf16, 128, true>); opt((const void*)k_attn_tiles<TkBf16, 256, true>);
     if (e != hipSuccess) return hipGetErrorString(e);
     done[dev].store(true, std::memory_order_release);
     return nullptr;
