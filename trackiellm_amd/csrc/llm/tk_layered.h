@@ -121,7 +121,8 @@ private:
     void need_pages(Seq& s, int seq, int last_pos);
     void give_back(Seq& s);
     bool upload_pages();
-    void gemm(const TkImgGemm& g);
+    void gemm(const TkImgGemm& g, int* slabs = nullptr);
+    size_t y_floats_ = 0;
     void enqueue_layers(const Pass& p);
     void enqueue_head(int n, const int32_t* d_rows, int32_t* tok, int32_t* pos);
     void enqueue_moe(const TkLayerSpec& s, const TkLayeredLayer& L, int nrows);

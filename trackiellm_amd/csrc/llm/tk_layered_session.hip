@@ -129,7 +129,8 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
             moe_ff = std::max(moe_ff, tk_img_bytes(type, (int64_t)rows, f.ff));
         }
     }
-    const size_t yrows = std::max<size_t>((size_t)R, moe_rows);
+    const size_t yrows = std::max<size_t>({(size_t)R, moe_rows, 8 * TK_MAX_ROWS}); /* a product of up to 256 rows may be split over k into eight slabs */
+    y_floats_ = yrows * c.width;
     if (!alloc((void**)&x_, (size_t)R * c.width * 4) || !alloc((void**)&proj_, (size_t)R * proj * 4, true) || !alloc((void**)&low_, (size_t)R * low * 4, true) ||
         !alloc((void**)&y_, yrows * c.width * 4, true) || !alloc(&img_x_, tk_img_bytes(type, R, c.width), true) || !alloc(&img_low_, lowk, true) ||
         !alloc(&img_mix_, mix, true) || !alloc(&img_ff_, std::max(ff, moe_ff), true) || !alloc(&img_head_, tk_img_bytes(type, TK_MAX_ROWS, c.width), true) ||
@@ -140,6 +141,7 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
               !alloc((void**)&moe_.expert, assign * 4) || !alloc((void**)&moe_.rank, assign * 4) || !alloc((void**)&moe_.weight, assign * 4) || !alloc((void**)&moe_.tile0, E * 4) ||
               !alloc((void**)&moe_.slot, assign * 4) || !alloc((void**)&moe_.blocks, (E + assign / 16 + 1) * sizeof(TkImgBlock), true) || !alloc((void**)&moe_.n_blocks, 4, true)))
         return false;
+    if (const char* e = tk_gemm_image_prepare_device()) { error = std::string("LDS opt-in failed: ") + e; return false; }
     if (const char* e = tk_mixer_prepare_device()) { error = std::string("LDS opt-in failed: ") + e; return false; }
     HIPQ(hipDeviceSynchronize());
     return true;
@@ -253,8 +255,8 @@ void TkLayeredSession::commit(int nrows, const int32_t* seq, const int32_t* pos)
 
 /* ------------------------------------------------------------------ the layers ------------- */
 
-void TkLayeredSession::gemm(const TkImgGemm& g) {
-    if (const char* e = tk_launch_gemm_image(g, stream))
+void TkLayeredSession::gemm(const TkImgGemm& g, int* slabs) {
+    if (const char* e = tk_launch_gemm_image(g, stream, slabs))
         if (launch_error.empty()) launch_error = e;
 }
 
@@ -343,8 +345,13 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
         }
         TkImgGemm o{};
         o.type = type; o.w = L.out.img; o.a = img_mix_; o.K = L.out.K; o.N = L.out.N; o.nrows = n; o.out = y_; o.ldc = D; o.n_valid = D;
-        gemm(o);
-        tk_launch_post_norm(type, TkSubOut{y_, D, L.out_bias, 1.0f, nullptr, nullptr, 0}, L.norm1, c.eps, D, n, x_, img_x_, xkt, s);
+        /* products whose result goes to a norm may come in slabs, as many as y_ holds */
+        const size_t slab = (size_t)n * D;
+        const int most = slab % 4 == 0 ? (int)std::min<size_t>(8, y_floats_ / slab) : 1;
+        int slabs = 1;
+        o.max_slabs = most; o.slab_floats = slab;
+        gemm(o, &slabs);
+        tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, L.out_bias, 1.0f, nullptr, nullptr, 0}, L.norm1, c.eps, D, n, x_, img_x_, xkt, s);
         if (spec.mlp.kind == TkMlpSpec::DENSE) {
             TkImgGemm u{};
             u.type = type; u.w = L.gate_up.img; u.a = img_x_; u.K = L.gate_up.K; u.N = L.gate_up.N; u.nrows = n;
@@ -352,11 +359,12 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
             gemm(u);
             TkImgGemm w{};
             w.type = type; w.w = L.down.img; w.a = img_ff_; w.K = L.down.K; w.N = L.down.N; w.nrows = n; w.out = y_; w.ldc = D; w.n_valid = D;
-            gemm(w);
-            tk_launch_post_norm(type, TkSubOut{y_, D, nullptr, 0.0f, nullptr, nullptr, 0}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
+            w.max_slabs = most; w.slab_floats = slab;
+            gemm(w, &slabs);
+            tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, nullptr, 0.0f, nullptr, nullptr, 0}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
         } else if (spec.mlp.kind == TkMlpSpec::MOE) {
             enqueue_moe(spec, L, n);
-            tk_launch_post_norm(type, TkSubOut{y_, D, nullptr, 0.0f, moe_.slot, moe_.weight, spec.mlp.top}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
+            tk_launch_post_norm(type, TkSubOut{y_, D, 1, 0, nullptr, 0.0f, moe_.slot, moe_.weight, spec.mlp.top}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
         }
         if (streams_) (void)hipMemcpyAsync(streams_ + l * (size_t)n * D, x_, (size_t)n * D * 4, hipMemcpyDeviceToHost, s);
     }

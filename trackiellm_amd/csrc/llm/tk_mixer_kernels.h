@@ -81,6 +81,7 @@ bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, 
 /* where a sublayer's output comes from: a product's rows, or the chosen experts' rows, weighted */
 struct TkSubOut {
     const float* y; int ld;
+    int slabs; size_t slab_floats; /* partial results of a product split over k, added in order (1: whole) */
     const float* bias; float bias_scale; /* bias may be null */
     const int32_t* slot; const float* weight; int top; /* top > 0: y[slot[row * top + j]] * weight[row * top + j] summed over j */
 };

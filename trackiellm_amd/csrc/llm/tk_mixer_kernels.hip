@@ -76,6 +76,7 @@ __global__ __launch_bounds__(512) void k_post_norm(TkSubOut o, const float* w, f
             } else {
                 const float* p = o.y + (size_t)row * o.ld + k;
                 a = *(const tk_v4f*)p; b = *(const tk_v4f*)(p + 4);
+                for (int i = 1; i < o.slabs; ++i) { a += *(const tk_v4f*)(p + i * o.slab_floats); b += *(const tk_v4f*)(p + i * o.slab_floats + 4); }
                 if (o.bias) { a += *(const tk_v4f*)(o.bias + k) * o.bias_scale; b += *(const tk_v4f*)(o.bias + k + 4) * o.bias_scale; }
             }
             *(tk_v4f*)(ybuf + k) = a;
@@ -87,7 +88,11 @@ __global__ __launch_bounds__(512) void k_post_norm(TkSubOut o, const float* w, f
             float y = 0.0f;
             if (o.top > 0)
                 for (int j = 0; j < o.top; ++j) y += o.weight[row * o.top + j] * o.y[(size_t)o.slot[row * o.top + j] * o.ld + k];
-            else y = o.y[(size_t)row * o.ld + k] + (o.bias ? o.bias[k] * o.bias_scale : 0.0f);
+            else {
+                y = o.y[(size_t)row * o.ld + k];
+                for (int i = 1; i < o.slabs; ++i) y += o.y[i * o.slab_floats + (size_t)row * o.ld + k];
+                if (o.bias) y += o.bias[k] * o.bias_scale;
+            }
             ybuf[k] = y;
             ss += y * y;
         }

@@ -41,6 +41,10 @@ struct TkImgGemm {
     /* f32 output: out[row][n], n < n_valid; columns [copy0, copy1) are also written, as T, to the image copy_img at k = n - copy0 */
     float* out;
     int ldc, n_valid;
+    /* K-split (wide kernel, f32 output without copied columns): up to max_slabs partial results, slab i at out + i * slab_floats, which the
+     * consumer adds in ascending order; the launcher reports how many it wrote.  0 / 1: none. */
+    int max_slabs;
+    size_t slab_floats;
     void* copy_img;
     int copy0, copy1, copy_ktiles;
     /* swiglu: the weight image alternates 16 gate rows and 16 up rows; silu(gate) * up goes, as T, to the image act_img [rows][N / 2] */
@@ -55,7 +59,10 @@ struct TkImgGemm {
 };
 
 /* nullptr, or why the arguments are refused (nothing is launched then) */
-const char* tk_launch_gemm_image(const TkImgGemm& g, hipStream_t s);
+const char* tk_launch_gemm_image(const TkImgGemm& g, hipStream_t s, int* slabs = nullptr);
+
+/* opts the kernels into their dynamic LDS on the calling thread's current device; nullptr or an error string.  Idempotent, thread-safe. */
+const char* tk_gemm_image_prepare_device();
 
 /* src: row-major [N][K] (device), bf16 (src_f32 = 0) or f32 -> rows n0 .. and columns k0 .. of an image with `ktiles` k tiles.  Row n of the
  * source lands in row  (n0 + n) of the image, or, with interleave = 0 or 1, in 16-row group 2 * (n / 16) + interleave (gate / up). */

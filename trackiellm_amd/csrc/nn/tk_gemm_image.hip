@@ -1,6 +1,9 @@
 /* tk_gemm_image.hip — see tk_gemm_image.h */
 #include "tk_gemm_image.h"
 
+#include <atomic>
+#include <mutex>
+
 #include "tk_image_device.h"
 
 namespace {
@@ -119,23 +122,28 @@ __global__ __launch_bounds__(64 * WAVES) void k_gemm_skinny(TkImgGemm a) {
     }
 }
 
-/* ---- wide: 128 rows x 16 * NBT columns per workgroup, waves 2 x 2, two k tiles per stage, double-buffered LDS ---- */
+/* s_waitcnt vmcnt(N): all but this wave's N youngest vector-memory requests are done */
+template <int N> __device__ __forceinline__ void wait_vm() { __builtin_amdgcn_s_waitcnt(0x0F70 | (N & 15) | (N >> 4) << 14); }
+
+/* ---- wide: 128 rows x 16 * NBT columns per workgroup, waves 2 x 2, two k tiles per stage, a ring of LDS stages filled by LDS-DMA ---- */
+template <int NBT> constexpr int wide_ring() { return NBT == 8 ? 2 : NBT == 4 ? 3 : 4; } /* stages: as many as let two workgroups share a CU */
 template <typename T, int NBT /* column tiles of the workgroup: 2, 4, 8 */, bool SWIGLU, bool GROUPED>
-__global__ __launch_bounds__(256) void k_gemm_wide(TkImgGemm a, int nblk_n, int nblk_m) {
+__global__ __launch_bounds__(256) void k_gemm_wide(TkImgGemm a, int nblk_n, int nblk_m, int ks) {
     constexpr int MBT = 8, NW = NBT / 2, MW = MBT / 2; /* tiles of one wave */
-    constexpr int STAGE = (MBT + NBT) * 2 * 1024;
+    constexpr int STAGE = (MBT + NBT) * 2 * 1024, RING = wide_ring<NBT>();
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     /* workgroups go to the eight XCDs in turn: give each XCD a contiguous range of blocks (row blocks fastest) so that it re-reads the same
      * columns of W from its own L2 */
     int id = blockIdx.x;
-    const int total = nblk_n * nblk_m;
+    const int total = nblk_n * nblk_m * ks;
     {
         const int per = total / 8, rem = total % 8, x = id % 8, i = id / 8;
         id = x * per + (x < rem ? x : rem) + i;
     }
-    const int bn = id / nblk_m, bm = id % nblk_m;
-    const int ktiles = a.K / TkImg<T>::KT, stages = ktiles / 2;
+    const int slab = id / (nblk_n * nblk_m), bn = id / nblk_m % nblk_n, bm = id % nblk_m;
+    const int ktiles = a.K / TkImg<T>::KT, s0 = (int)((int64_t)(ktiles / 2) * slab / ks), stages = (int)((int64_t)(ktiles / 2) * (slab + 1) / ks) - s0;
+    a.out += slab * a.slab_floats;
     int m0 = bm * MBT, mlive = (a.nrows + 15) / 16 - m0;
     const uint8_t* wbase = (const uint8_t*)a.w;
     if (GROUPED) {
@@ -150,11 +158,11 @@ __global__ __launch_bounds__(256) void k_gemm_wide(TkImgGemm a, int nblk_n, int 
     const uint8_t* src[PPW];
 #pragma unroll
     for (int i = 0; i < PPW; ++i) { /* piece p: tile p / 2 (M-tiles first, then column tiles), k tile p % 2 of the stage */
-        const int p = wave * PPW + i, t = p >> 1;
-        if (t < MBT) src[i] = (const uint8_t*)a.a + ((size_t)(m0 + (t < mlive ? t : 0)) * ktiles + (p & 1)) * 1024 + lane * 16;
+        const int p = wave * PPW + i, t = p >> 1, k0 = 2 * s0 + (p & 1);
+        if (t < MBT) src[i] = (const uint8_t*)a.a + ((size_t)(m0 + (t < mlive ? t : 0)) * ktiles + k0) * 1024 + lane * 16;
         else {
             const int nt = n0 + t - MBT < ntot ? n0 + t - MBT : ntot - 1;
-            src[i] = wbase + ((size_t)nt * ktiles + (p & 1)) * 1024 + lane * 16;
+            src[i] = wbase + ((size_t)nt * ktiles + k0) * 1024 + lane * 16;
         }
     }
     auto stage = [&](int buf) {
@@ -171,13 +179,18 @@ __global__ __launch_bounds__(256) void k_gemm_wide(TkImgGemm a, int nblk_n, int 
     for (int n = 0; n < NW; ++n)
 #pragma unroll
         for (int m = 0; m < MW; ++m) acc[n][m] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
-    stage(0);
+    for (int s = 0; s < RING - 1 && s < stages; ++s) stage(s);
+    int cur = 0, fill = RING - 1;
 #pragma unroll 1
     for (int s = 0; s < stages; ++s) {
-        __builtin_amdgcn_s_waitcnt(0x0F70); /* vmcnt(0): this wave's pieces of stage s have landed */
-        __syncthreads();
-        if (s + 1 < stages) stage((s + 1) & 1);
-        const uint8_t* b = lds + (s & 1) * STAGE + lane * 16;
+        /* stage s has landed when at most the RING - 2 younger ones are outstanding (at the end there are fewer: wait for all) */
+        if (s + RING - 1 <= stages) wait_vm<(RING - 2) * PPW>();
+        else wait_vm<0>();
+        asm volatile("s_barrier" ::: "memory"); /* every wave's pieces of stage s have landed, and every wave has read stage s - 1, whose place is filled next */
+        if (s + RING - 1 < stages) stage(fill);
+        const uint8_t* b = lds + cur * STAGE + lane * 16;
+        cur = cur + 1 < RING ? cur + 1 : 0;
+        fill = fill + 1 < RING ? fill + 1 : 0;
 #pragma unroll
         for (int k = 0; k < 2; ++k) {
             tk_v4u av[MW], wv[NW];
@@ -219,7 +232,7 @@ __global__ void k_put_image(const void* src, int src_f32, int64_t N, int64_t K, 
 }
 
 template <typename T, bool SWIGLU, bool GROUPED>
-const char* launch(const TkImgGemm& g, hipStream_t s) {
+const char* launch(const TkImgGemm& g, hipStream_t s, int* slabs) {
     const int ntiles = g.N / 16;
     const int mtiles = GROUPED ? g.block_tiles : (g.nrows + 15) / 16;
     if (mtiles <= 4) {
@@ -237,9 +250,18 @@ const char* launch(const TkImgGemm& g, hipStream_t s) {
         return nullptr;
     }
     const int nblk_m = GROUPED ? g.max_blocks : (g.nrows + 127) / 128;
-    int nb = 8;
-    while (nb > (SWIGLU ? 4 : 2) && (int64_t)nblk_m * ((ntiles + nb - 1) / nb) < 256) nb /= 2;
-#define TK_WD(NB) do { const int nbn = (ntiles + NB - 1) / NB; hipLaunchKernelGGL((k_gemm_wide<T, NB, SWIGLU, GROUPED>), dim3(nbn * nblk_m), dim3(256), (size_t)2 * (8 + NB) * 2048, s, g, nbn, nblk_m); } while (0)
+    int nb = 8, ks = 1;
+    const int64_t full = (int64_t)nblk_m * ((ntiles + 7) / 8);
+    if (!SWIGLU && !GROUPED && g.max_slabs > 1 && full < 256) { /* large blocks of a part of K rather than small blocks of all of it: at least eight stages each */
+        ks = (int)(512 / full);
+        if (ks > g.max_slabs) ks = g.max_slabs;
+        const int most = g.K / TkImg<T>::KT / 16;
+        if (ks > most) ks = most;
+        if (ks < 1) ks = 1;
+    }
+    while (nb > (SWIGLU ? 4 : 2) && (int64_t)nblk_m * ((ntiles + nb - 1) / nb) * ks < 200) nb /= 2;
+    if (slabs) *slabs = ks;
+#define TK_WD(NB) do { const int nbn = (ntiles + NB - 1) / NB; hipLaunchKernelGGL((k_gemm_wide<T, NB, SWIGLU, GROUPED>), dim3(nbn * nblk_m * ks), dim3(256), (size_t)wide_ring<NB>() * (8 + NB) * 2048, s, g, nbn, nblk_m, ks); } while (0)
     if (nb == 8) TK_WD(8);
     else if (nb == 4 || SWIGLU) TK_WD(4);
     else TK_WD((SWIGLU ? 4 : 2));
@@ -249,16 +271,42 @@ const char* launch(const TkImgGemm& g, hipStream_t s) {
 
 } // namespace
 
-const char* tk_launch_gemm_image(const TkImgGemm& g, hipStream_t s) {
+const char* tk_launch_gemm_image(const TkImgGemm& g, hipStream_t s, int* slabs) {
+    if (slabs) *slabs = 1;
     if (g.type != TK_IMG_BF16 && g.type != TK_IMG_F32) return "gemm_image: unknown element type";
     if (!g.w || !g.a || g.K <= 0 || g.K % (2 * tk_img_kt(g.type))) return "gemm_image: K is not a multiple of two tiles";
     if (g.N <= 0 || g.N % (g.swiglu ? 32 : 16)) return "gemm_image: N is not a multiple of its tile";
     if (g.swiglu ? (!g.act_img || g.act_ktiles * tk_img_kt(g.type) < g.N / 2) : (!g.out || g.n_valid > g.N || g.ldc < g.n_valid)) return "gemm_image: output does not fit";
     if (g.copy_img && g.copy_ktiles * tk_img_kt(g.type) < g.copy1 - g.copy0) return "gemm_image: copied columns do not fit their image";
+    if (g.max_slabs > 1 && (!slabs || g.swiglu || g.copy_img || g.slab_floats % 4)) return "gemm_image: this product cannot be split over k";
     if (g.blocks ? (!g.n_blocks || g.max_blocks < 1 || g.block_tiles < 1 || g.block_tiles > 8) : g.nrows < 1) return "gemm_image: no rows";
-#define TK_GI(T) (g.swiglu ? (g.blocks ? launch<T, true, true>(g, s) : launch<T, true, false>(g, s)) : (g.blocks ? launch<T, false, true>(g, s) : launch<T, false, false>(g, s)))
+#define TK_GI(T) (g.swiglu ? (g.blocks ? launch<T, true, true>(g, s, slabs) : launch<T, true, false>(g, s, slabs)) : (g.blocks ? launch<T, false, true>(g, s, slabs) : launch<T, false, false>(g, s, slabs)))
     return g.type == TK_IMG_F32 ? TK_GI(float) : TK_GI(TkBf16);
 #undef TK_GI
+}
+
+template <typename T>
+static hipError_t opt_in_wide() {
+    hipError_t e = hipSuccess;
+#define TK_OPT(NB, S, G) if (e == hipSuccess) e = hipFuncSetAttribute((const void*)k_gemm_wide<T, NB, S, G>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024)
+    TK_OPT(2, false, false); TK_OPT(2, false, true);
+    TK_OPT(4, false, false); TK_OPT(4, false, true); TK_OPT(4, true, false); TK_OPT(4, true, true);
+#undef TK_OPT
+    return e;
+}
+
+const char* tk_gemm_image_prepare_device() {
+    static std::atomic<bool> done[64];
+    static std::mutex mu;
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return "no current device";
+    if (done[dev].load(std::memory_order_acquire)) return nullptr;
+    std::lock_guard<std::mutex> lk(mu);
+    hipError_t e = opt_in_wide<TkBf16>();
+    if (e == hipSuccess) e = opt_in_wide<float>();
+    if (e != hipSuccess) return hipGetErrorString(e);
+    done[dev].store(true, std::memory_order_release);
+    return nullptr;
 }
 
 void tk_launch_put_image(int type, const void* src, int src_f32, int64_t N, int64_t K, void* img, int ktiles, int64_t n0, int64_t k0, int interleave, hipStream_t s) {
