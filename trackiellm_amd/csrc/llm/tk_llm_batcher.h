@@ -5,7 +5,8 @@
  * (src/ai_models/tk_runner_streaming.c:57-85, contract src/ai_models/tk_model_runner.h:164-181).  Behind the same calls, all runners
  * created on one model share ONE decode session here: a runner owns a sequence slot of the session's KV cache; prepare_generation /
  * generate_next_token / add_tool_response enqueue their (sequence, position, token) rows and block; one scheduler thread per model
- * coalesces whatever is ready — prompt chunks and single decode rows of different runners alike — into passes of up to 256 rows, so
+ * coalesces whatever is ready — prompt chunks and single decode rows of different runners alike — into passes of up to 256 rows (the session's
+ * row_capacity()), so
  * K host threads that each drive "their" runner read the 4.3 GB of weights once per step instead of K times.
  * A row's result does not depend on which other rows share its pass (bit-identical logits at any pass width:
  * tests/test_llm_gpu.py::test_full_7b_pass_width_invariance), so a runner sees exactly the tokens it would see alone.
@@ -16,7 +17,7 @@
  * owner's next call then finds its row in flight or already done.  Not for rows sampled under a grammar mask (the next mask depends on
  * the accepted token), not after EOS, not at the end of the context.  An owner that comes back with something else (a tool response, a
  * new prompt) or not at all costs one wasted row: the cache row it wrote is overwritten before anything attends to it, because positions
- * are fed in order.  Tokens are unchanged — a row's result does not depend on when or with whom it runs.
+ * are fed in order (a session with recurrent state takes its last pass back when the same position is fed again).  Tokens are unchanged — a row's result does not depend on when or with whom it runs.
  */
 #ifndef TK_LLM_BATCHER_H
 #define TK_LLM_BATCHER_H
