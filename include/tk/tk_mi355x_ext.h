@@ -66,7 +66,7 @@ TK_API uint64_t tk_mi355x_llm_model_weight_bytes(const tk_mi355x_llm_model_t* m)
 TK_API void tk_mi355x_llm_model_destroy(tk_mi355x_llm_model_t** m);
 
 /* ---- decoders described layer by layer (csrc/llm/tk_layered.h): a folder with config.json — "architecture" names the design, registered in
- * csrc/llm/tk_layer_spec.cpp (Vuvulorn) — and model.safetensors.  tk_model_loader_load_model takes such a folder as its path (with
+ * csrc/llm/tk_layer_spec.cpp (Vuvulorn, Kaparax) — and model.safetensors.  tk_model_loader_load_model takes such a folder as its path (with
  * "?dtype=float32" behind it for 32-bit); sessions, runners, the scheduler, sampling and the decode loop are the ones of every other model.
  *   load_dir: dtype "bfloat16" (NULL / "": the default; matrix products in bf16 with 32-bit accumulation, norms, scores, routers, the residual
  *     stream and recurrent state in 32-bit) or "float32" (everything in 32-bit);

@@ -158,9 +158,7 @@ def moe(cfg, w, p, h):
     return out
 
 
-def forward(cfg, w, tokens):
-    """(logits [T, vocab], residual stream after every layer [layers, T, width]) of one sequence"""
-    w = {k: np.asarray(v, np.float64) for k, v in w.items()}
+def vuvulorn(cfg, w, tokens):
     eps = cfg["norm"]["eps"]
     x = w["embed"][np.asarray(tokens)]
     stream = []
@@ -177,3 +175,102 @@ def forward(cfg, w, tokens):
             x = x + rms(y, eps) * w[p + "norm2"]
         stream.append(x)
     return (rms(x, eps) * w["final.norm"]) @ w["head"].T, np.array(stream)
+
+
+# ---- Kaparax: retention and chunked attention layers between layer norms ----
+
+def layer_norm(x, gain, shift, eps):
+    """x less its mean, over the root of its variance, per row"""
+    c = x - x.mean(axis=-1, keepdims=True)
+    return c / np.sqrt(np.mean(c * c, axis=-1, keepdims=True) + eps) * gain + shift
+
+
+def retention(q, k, v, decay):
+    """q, k [T, H, dim], v [T, H, vdim], decay [H]: a state [dim, vdim] per head that fades by a constant and gains k v^T; read by q after the gain"""
+    T, H, dim = k.shape
+    S = np.zeros((H, dim, v.shape[2]))
+    o = np.zeros((T, H, v.shape[2]))
+    for t in range(T):
+        for h in range(H):
+            S[h] = decay[h] * S[h] + np.outer(k[t, h], v[t, h])
+            o[t, h] = q[t, h] @ S[h]
+    return o
+
+
+def retention_mixer(cfg, w, p, h, eps):
+    T = h.shape[0]
+    H, dim, vdim = cfg["heads"], cfg["dim"], cfg["vdim"]
+    pos = np.arange(T, dtype=np.float64)
+    q, k = ((h @ w[p + n].T).reshape(T, H, dim) for n in "qk")
+    q, k = (rotate_half(z, pos, cfg["rot"]["dims"], cfg["rot"]["base"]) for z in (q, k))
+    o = retention(q, k * dim ** -0.5, (h @ w[p + "v"].T).reshape(T, H, vdim), cfg["decay"])
+    return (rms(o, eps).reshape(T, H * vdim) * silu(h @ w[p + "g"].T)) @ w[p + "o"].T
+
+
+def same_chunk(i, j, size):
+    """may position i read position j: a chunk of `size` positions, counted from the sequence's start (0: no chunks), is closed to the next ones"""
+    return j <= i and (not size or i // size == j // size)
+
+
+def capped(score, cap):
+    """scores pressed into (-cap, cap); None: left as they are"""
+    return cap * np.tanh(score / cap) if cap else score
+
+
+def chunked_attention(q, k, v, scale, size, cap):
+    """q [T, H, dim], k [T, G, dim], v [T, G, vdim]"""
+    T, H, _ = q.shape
+    per = H // k.shape[1]
+    out = np.zeros((T, H, v.shape[2]))
+    for i in range(T):
+        js = [j for j in range(i + 1) if same_chunk(i, j, size)]
+        for h in range(H):
+            sc = capped(k[js, h // per] @ q[i, h] * scale, cap)
+            e = np.exp(sc - sc.max())
+            out[i, h] = (e / e.sum()) @ v[js, h // per]
+    return out
+
+
+def chunked_attention_mixer(cfg, w, p, h):
+    T = h.shape[0]
+    H, G, dim, vdim = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
+    q, k, v = (causal_conv(h @ w[p + n].T, w[p + n + ".conv"]) for n in "qkv")
+    pos = np.arange(T, dtype=np.float64)
+    q = rotate_half(q.reshape(T, H, dim), pos, cfg["rot"]["dims"], cfg["rot"]["base"])
+    k = rotate_half(k.reshape(T, G, dim), pos, cfg["rot"]["dims"], cfg["rot"]["base"])
+    o = chunked_attention(q, k, v.reshape(T, G, vdim), cfg["scale"], (cfg.get("mask") or {}).get("size"), cfg.get("softcap"))
+    return o.reshape(T, H * vdim) @ w[p + "o"].T
+
+
+def clamped_glu(w, p, h, limit):
+    """the gate is cut above, the linear side on both sides and moved by one"""
+    g = np.minimum(h @ w[p + "gate"].T, limit)
+    u = np.clip(h @ w[p + "up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[p + "down"].T
+
+
+def kaparax(cfg, w, tokens):
+    eps = cfg["norm"]["eps"]
+
+    def norm(name, z):
+        return layer_norm(z, w[name], w[name + ".b"], eps)
+
+    x = w["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
+    stream = []
+    for i, L in enumerate(cfg["layers"]):
+        while cfg["layers"][i].get("weights_of") is not None:
+            i = cfg["layers"][i]["weights_of"]
+        p = "l%d." % i
+        h = norm(p + "norm1", x)
+        y = retention_mixer(L["mixer"], w, p + "mix.", h, eps) if L["type"] == "retention" else chunked_attention_mixer(L["mixer"], w, p + "mix.", h)
+        x = x + norm(p + "norm1b", y)
+        if L.get("mlp"):
+            x = x + norm(p + "norm2b", clamped_glu(w, p + "mlp.", norm(p + "norm2", x), L["mlp"]["limit"]))
+        stream.append(x)
+    return norm("final.norm", x) @ w["head"].T, np.array(stream)
+
+
+def forward(cfg, w, tokens):
+    """(logits [T, vocab], residual stream after every layer [layers, T, width]) of one sequence"""
+    w = {k: np.asarray(v, np.float64) for k, v in w.items()}
+    return {"Vuvulorn": vuvulorn, "Kaparax": kaparax}[cfg["architecture"]](cfg, w, tokens)

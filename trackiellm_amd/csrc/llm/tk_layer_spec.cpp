@@ -48,12 +48,21 @@ bool read_heads(Reader& r, const JVal* m, const std::string& w, int max_dim, int
     return *heads % *kv == 0 || r.fail(w + ".heads is not a multiple of kv_heads");
 }
 
+bool read_rotation(Reader& r, const JVal* m, const std::string& w, int dim, int* dims, double* base) {
+    const JVal* rot = m->get("rot");
+    if (!is_set(rot)) return true;
+    if (!r.integer(rot, "dims", w + ".rot", 0, dim, dims) || !r.num(rot, "base", w + ".rot", base)) return false;
+    if (*dims % 2) return r.fail(w + ".rot.dims is odd");
+    return *base > 0.0 || r.fail(w + ".rot.base is not positive");
+}
+
+/* sizes, score scale and rotation: what every attention has */
 bool read_attention(Reader& r, const JVal* m, const std::string& w, TkAttnSpec* a) {
-    if (!read_heads(r, m, w, TK_MAX_HEAD_DIM, TK_MAX_HEAD_DIM, &a->heads, &a->kv_heads, &a->dim, &a->vdim) || !r.real(m, "scale", w, &a->scale)) return false;
-    if (const JVal* rot = m->get("rot"); is_set(rot)) {
-        if (!r.integer(rot, "dims", w + ".rot", 0, a->dim, &a->rot_dims) || !r.num(rot, "base", w + ".rot", &a->rot_base)) return false;
-        if (a->rot_dims % 2) return r.fail(w + ".rot.dims is odd");
-    }
+    return read_heads(r, m, w, TK_MAX_HEAD_DIM, TK_MAX_HEAD_DIM, &a->heads, &a->kv_heads, &a->dim, &a->vdim) && r.real(m, "scale", w, &a->scale) &&
+           read_rotation(r, m, w, a->dim, &a->rot_dims, &a->rot_base);
+}
+
+bool read_window(Reader& r, const JVal* m, const std::string& w, TkAttnSpec* a) {
     if (const JVal* mask = m->get("mask"); is_set(mask)) {
         if (is_set(mask->get("size")) && !r.integer(mask, "size", w + ".mask", 1, 1 << 30, &a->window)) return false;
         if (is_set(mask->get("keep_first")) && !r.integer(mask, "keep_first", w + ".mask", 0, 1 << 30, &a->keep_first)) return false;
@@ -64,6 +73,27 @@ bool read_attention(Reader& r, const JVal* m, const std::string& w, TkAttnSpec* 
 bool read_delta(Reader& r, const JVal* m, const std::string& w, TkDeltaSpec* d) {
     return read_heads(r, m, w, TK_MAX_DELTA_DIM, TK_MAX_DELTA_VDIM, &d->heads, &d->kv_heads, &d->dim, &d->vdim) &&
            r.integer(m, "conv", w, 1, TK_MAX_CONV_TAPS, &d->taps);
+}
+
+/* chunks, capped scores, a convolution ahead of the rotation */
+bool read_chunks(Reader& r, const JVal* m, const std::string& w, TkAttnSpec* a) {
+    if (const JVal* mask = m->get("mask"); is_set(mask) && is_set(mask->get("size")) && !r.integer(mask, "size", w + ".mask", 1, 1 << 30, &a->chunk)) return false;
+    if (is_set(m->get("softcap")) && !r.real(m, "softcap", w, &a->softcap)) return false;
+    if (is_set(m->get("conv")) && !r.integer(m, "conv", w, 1, TK_MAX_CONV_TAPS, &a->taps)) return false;
+    return a->softcap >= 0.0f || r.fail(w + ".softcap is negative");
+}
+
+bool read_retention(Reader& r, const JVal* m, const std::string& w, TkRetentionSpec* o) {
+    if (!r.integer(m, "heads", w, 1, 4096, &o->heads) || !r.integer(m, "dim", w, 1, TK_MAX_RETENTION_DIM, &o->dim) || !r.integer(m, "vdim", w, 1, TK_MAX_RETENTION_VDIM, &o->vdim) ||
+        !read_rotation(r, m, w, o->dim, &o->rot_dims, &o->rot_base))
+        return false;
+    const JVal* d = m->get("decay");
+    if (!d || d->kind != JVal::JARR || (int)d->arr.size() != o->heads) return r.fail(w + ".decay is not a list of one number per head");
+    for (const JVal& v : d->arr) {
+        if (v.kind != JVal::JNUM || !(v.num >= 0.0 && v.num <= 1.0)) return r.fail(w + ".decay has a value outside 0 .. 1");
+        o->decay.push_back(v.num);
+    }
+    return true;
 }
 
 bool read_mlp(Reader& r, const JVal* m, const std::string& w, TkMlpSpec* o) {
@@ -86,14 +116,21 @@ bool read_mlp(Reader& r, const JVal* m, const std::string& w, TkMlpSpec* o) {
     return o->top <= o->experts / o->groups * o->keep || r.fail(w + ".router.top is larger than the experts that can be chosen");
 }
 
+/* what every design gives: width, vocabulary, norm constant; null or the list of layers */
+const JVal* read_model(Reader& r, const JVal& root, TkLayeredConfig* c) {
+    if (!r.integer(&root, "width", "config", 1, 1 << 20, &c->width) || !r.integer(&root, "vocab", "config", 1, 1 << 24, &c->vocab)) return nullptr;
+    const JVal* norm = r.obj(&root, "norm", "config");
+    if (!norm || !r.real(norm, "eps", "norm", &c->eps)) return nullptr;
+    const JVal* layers = root.get("layers");
+    if (!layers || layers->kind != JVal::JARR || layers->arr.empty()) { r.fail("layers is missing"); return nullptr; }
+    return layers;
+}
+
 /* Vuvulorn: every layer runs window attention and a gated delta rule side by side on the un-normed stream; norms on the sublayers' outputs */
 bool parse_vuvulorn(const JVal& root, TkLayeredConfig* c, std::string* err) {
     Reader r{err};
-    if (!r.integer(&root, "width", "config", 1, 1 << 20, &c->width) || !r.integer(&root, "vocab", "config", 1, 1 << 24, &c->vocab)) return false;
-    const JVal* norm = r.obj(&root, "norm", "config");
-    if (!norm || !r.real(norm, "eps", "norm", &c->eps)) return false;
-    const JVal* layers = root.get("layers");
-    if (!layers || layers->kind != JVal::JARR || layers->arr.empty()) return r.fail("layers is missing");
+    const JVal* layers = read_model(r, root, c);
+    if (!layers) return false;
     for (size_t i = 0; i < layers->arr.size(); ++i) {
         const JVal* L = &layers->arr[i];
         const std::string w = "layers[" + std::to_string(i) + "]", p = "l" + std::to_string(i) + ".";
@@ -109,7 +146,7 @@ bool parse_vuvulorn(const JVal& root, TkLayeredConfig* c, std::string* err) {
         a.kind = TkBranchSpec::ATTENTION; a.prefix = p + "mix.left."; a.attn.bias = a.attn.qk_norm = true;
         d.kind = TkBranchSpec::DELTA; d.prefix = p + "mix.right.";
         if (!r.real(m, "left_scale", w + ".mixer", &a.scale) || !r.real(m, "right_scale", w + ".mixer", &d.scale) ||
-            !read_attention(r, left, w + ".mixer.left", &a.attn) || !read_delta(r, right, w + ".mixer.right", &d.delta))
+            !read_attention(r, left, w + ".mixer.left", &a.attn) || !read_window(r, left, w + ".mixer.left", &a.attn) || !read_delta(r, right, w + ".mixer.right", &d.delta))
             return false;
         if (const JVal* mlp = L->get("mlp"); is_set(mlp)) {
             s.mlp.prefix = p + "mlp.";
@@ -120,8 +157,72 @@ bool parse_vuvulorn(const JVal& root, TkLayeredConfig* c, std::string* err) {
     return true;
 }
 
+/* do two layers' tensors have the same shapes? */
+bool same_shapes(const TkLayerSpec& x, const TkLayerSpec& y) {
+    if (x.branches.size() != y.branches.size()) return false;
+    for (size_t i = 0; i < x.branches.size(); ++i) {
+        const TkBranchSpec &a = x.branches[i], &b = y.branches[i];
+        if (a.kind != b.kind || a.attn.heads != b.attn.heads || a.attn.kv_heads != b.attn.kv_heads || a.attn.dim != b.attn.dim || a.attn.vdim != b.attn.vdim ||
+            a.attn.taps != b.attn.taps || a.delta.heads != b.delta.heads || a.delta.kv_heads != b.delta.kv_heads || a.delta.dim != b.delta.dim ||
+            a.delta.vdim != b.delta.vdim || a.delta.taps != b.delta.taps || a.retention.heads != b.retention.heads || a.retention.dim != b.retention.dim ||
+            a.retention.vdim != b.retention.vdim)
+            return false;
+    }
+    return x.mlp.kind == y.mlp.kind && x.mlp.ff == y.mlp.ff && x.mlp.experts == y.mlp.experts;
+}
+
+/* Kaparax: retention and chunked attention layers in any order, layer norms before and after every sublayer, a clamped gate in the feed-forward
+ * (or none), layers that run another layer's tensors once more */
+bool parse_kaparax(const JVal& root, TkLayeredConfig* c, std::string* err) {
+    Reader r{err};
+    const JVal *layers = read_model(r, root, c), *embedding = layers ? r.obj(&root, "embedding", "config") : nullptr;
+    if (!embedding || !r.real(embedding, "scale", "embedding", &c->embed_scale)) return false;
+    c->norm = TkLayeredConfig::LAYER;
+    const int n = (int)layers->arr.size();
+    for (int i = 0; i < n; ++i) {
+        const JVal* L = &layers->arr[i];
+        const std::string w = "layers[" + std::to_string(i) + "]";
+        TkLayerSpec s;
+        int owner = i;
+        for (int hops = 0; is_set(layers->arr[owner].get("weights_of")); ++hops) {
+            const std::string at = "layers[" + std::to_string(owner) + "]";
+            if (!r.integer(&layers->arr[owner], "weights_of", at, 0, n - 1, &owner)) return false;
+            if (hops > n) return r.fail(w + ".weights_of leads back to itself");
+        }
+        if (owner != i) s.weights_of = owner;
+        const std::string p = "l" + std::to_string(owner) + ".";
+        s.pre1 = p + "norm1"; s.norm1 = p + "norm1b"; s.pre2 = p + "norm2"; s.norm2 = p + "norm2b";
+        const JVal *type = L->get("type"), *m = r.obj(L, "mixer", w);
+        if (!m) return false;
+        s.branches.resize(1);
+        TkBranchSpec& b = s.branches[0];
+        b.prefix = p + "mix.";
+        if (type && type->kind == JVal::JSTR && type->str == "retention") {
+            b.kind = TkBranchSpec::RETENTION;
+            if (!read_retention(r, m, w + ".mixer", &b.retention)) return false;
+        } else if (type && type->kind == JVal::JSTR && type->str == "attention") {
+            if (!read_attention(r, m, w + ".mixer", &b.attn) || !read_chunks(r, m, w + ".mixer", &b.attn)) return false;
+        } else {
+            return r.fail(w + ".type is unknown");
+        }
+        if (const JVal* mlp = L->get("mlp"); is_set(mlp)) {
+            s.mlp.prefix = p + "mlp.";
+            if (!read_mlp(r, mlp, w + ".mlp", &s.mlp) || !r.real(mlp, "limit", w + ".mlp", &s.mlp.limit)) return false;
+            if (s.mlp.kind != TkMlpSpec::DENSE) return r.fail(w + ".mlp.kind is unknown");
+            s.mlp.act = TkMlpSpec::CLAMPED;
+            s.mlp.slope = 1.702f;
+            s.mlp.shift = 1.0f;
+        }
+        c->layers.push_back(std::move(s));
+    }
+    for (int i = 0; i < n; ++i)
+        if (c->layers[i].weights_of >= 0 && !same_shapes(c->layers[i], c->layers[c->layers[i].weights_of]))
+            return r.fail("layers[" + std::to_string(i) + "] has other sizes than the layer whose weights it uses");
+    return true;
+}
+
 struct Entry { const char* name; bool (*parse)(const JVal&, TkLayeredConfig*, std::string*); };
-const Entry g_architectures[] = {{"Vuvulorn", parse_vuvulorn}};
+const Entry g_architectures[] = {{"Vuvulorn", parse_vuvulorn}, {"Kaparax", parse_kaparax}};
 
 } // namespace
 

@@ -5,6 +5,8 @@
  * projections that read a layer's input side by side (one launch), the branches' output projections side by side in k (their sum is one
  * product; a branch's scale is applied to its activations), gate and up interleaved, an expert's matrices behind one another.
  *
+ * A layer may run another layer's tensors (TkLayerSpec::weights_of): the model holds them once, the session keeps a cache and a state for each.
+ *
  * Session: keys and values in pages of 64 positions shared by all sequences (one page table for all layers), recurrent state in two copies per
  * sequence and layer: a pass reads one and writes the other, so the last pass of a sequence can be taken back (the scheduler's run-ahead rows)
  * and nothing is copied.  A pass is any mix of runs of consecutive positions, one run per sequence; each run continues where its sequence
@@ -31,7 +33,7 @@ struct TkLayeredBranch {
     int out_k0 = 0; /* first k of the output projection */
     /* attention */
     float *bias = nullptr, *q_norm = nullptr, *k_norm = nullptr;
-    /* delta rule */
+    /* delta rule; the convolution may be attention's too */
     float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *norm = nullptr;
     int rank_a = 0, rank_g = 0, low_a = 0, low_g = 0;
 };
@@ -40,7 +42,9 @@ struct TkLayeredLayer {
     std::vector<TkLayeredBranch> branches;
     TkMat in, low, out, gate_up, down, router; /* gate_up, down: of all experts when the layer has experts (bytes = one expert's) */
     int low_col = 0, low_cols = 0;             /* projection columns that feed `low` */
-    float *out_bias = nullptr, *norm1 = nullptr, *norm2 = nullptr;
+    uint64_t bytes = 0;                        /* of the matrices */
+    float* out_bias = nullptr;
+    TkNorm pre1{}, norm1{}, pre2{}, norm2{}; /* on the sublayers' inputs (w null: none) and outputs */
 };
 
 class TkLayeredModel : public TkDecoderModel {
@@ -49,7 +53,7 @@ public:
     int type = TK_IMG_BF16; /* element type of weights' and activations' images and of the cache */
     uint16_t* embed = nullptr; /* [vocab][width] bf16 */
     TkMat head;
-    float* final_norm = nullptr;
+    TkNorm final_norm{};
     std::vector<TkLayeredLayer> layers;
 
     ~TkLayeredModel() override;
@@ -92,7 +96,7 @@ protected:
 
 private:
     struct Seq { int len = 0, prev = -1, side = 0; std::vector<int32_t> pages; };
-    struct Pass { int nrows = 0, nseg = 0, ntiles = 0; bool single = true; };
+    struct Pass { int nrows = 0, nseg = 0, ntiles = 0, nblocks = 0, nsums = 0; bool single = true, singles = true; }; /* all segments, or any, are single rows */
     TkLayeredModel* m_ = nullptr;
     std::mutex mu_; /* seqs_, free_pages_, host page table */
     std::vector<Seq> seqs_;
@@ -101,21 +105,25 @@ private:
     int n_pages_ = 0, max_pages_ = 0;
     std::vector<int32_t> live_; /* sequences of rows 0 .. of the last pass decode() may continue from */
     std::vector<void*> owned_;
-    int32_t *h_tab_ = nullptr, *d_tab_ = nullptr, *d_pages_ = nullptr, *d_out_rows_ = nullptr, *d_tiles_ = nullptr, *d_otok_ = nullptr;
+    int32_t *h_tab_ = nullptr, *d_tab_ = nullptr, *d_pages_ = nullptr, *d_out_rows_ = nullptr, *d_tiles_ = nullptr, *d_blocks_ = nullptr, *d_otok_ = nullptr;
+    int ret_heads_ = 0; /* most heads of a retention layer (0: none) */
+    int retention_rows(int nrows) const;
     size_t tab_ints_ = 0;
     TkPassTab tab_{};
     float *x_ = nullptr, *proj_ = nullptr, *low_ = nullptr, *y_ = nullptr, *router_ = nullptr, *scratch_ = nullptr;
+    float* sums_ = nullptr;
     float *dq_ = nullptr, *dk_ = nullptr, *dv_ = nullptr, *dg_ = nullptr, *db_ = nullptr, *do_ = nullptr;
     void *img_x_ = nullptr, *img_low_ = nullptr, *img_mix_ = nullptr, *img_ff_ = nullptr, *img_gather_ = nullptr, *img_head_ = nullptr, *q_ = nullptr;
     TkMoeTab moe_{};
     struct Rope { float *c, *s; };
     std::map<std::pair<int, double>, Rope> rope_;
-    struct BranchState { TkKvPool kv{}; float *conv = nullptr, *state = nullptr; Rope rope{}; int splits_pages = 1; };
+    struct BranchState { TkKvPool kv{}; float *conv = nullptr, *state = nullptr, *decay = nullptr; Rope rope{}; int splits_pages = 1; };
     std::vector<std::vector<BranchState>> st_;
     hipGraphExec_t graphs_[TK_MAX_ROWS + 1] = {};
     float* streams_ = nullptr; /* forward_streams(): destination of the layers' streams */
 
     bool alloc(void** p, size_t bytes, bool zero = false);
+    bool rotation(int dims, double base, Rope* out);
     bool describe(int nrows, const int32_t* seq, const int32_t* pos, const int32_t* tok, Pass* p);
     void commit(int nrows, const int32_t* seq, const int32_t* pos);
     void need_pages(Seq& s, int seq, int last_pos);

@@ -113,6 +113,11 @@ struct TkLayeredModel::Source {
         std::vector<float> v;
         return values(name, shape, &v, lo, hi) && upload(v, dst);
     }
+    bool norm(const std::string& name, TkNorm* n) {
+        if (name.empty()) return true;
+        n->layer = m->cfg.norm == TkLayeredConfig::LAYER;
+        return vec(name, {m->cfg.width}, (float**)&n->w, 0.8f, 1.2f) && (!n->layer || vec(name + ".b", {m->cfg.width}, (float**)&n->b, -0.1f, 0.1f));
+    }
 };
 
 TkLayeredModel::~TkLayeredModel() {
@@ -168,6 +173,8 @@ bool TkLayeredModel::build(Source& src) {
     for (size_t i = 0; i < layers.size(); ++i) {
         const TkLayerSpec& s = cfg.layers[i];
         TkLayeredLayer& L = layers[i];
+        if (s.weights_of >= 0) continue;
+        const uint64_t before = matrix_bytes_;
         L.branches.resize(s.branches.size());
         /* columns: every branch's own projections, then the inner sides of the low-rank gates */
         int col = 0, out_k = 0, low_k = 0, low_n = 0;
@@ -179,6 +186,10 @@ bool TkLayeredModel::build(Source& src) {
                 const TkAttnSpec& a = bs.attn;
                 col += a.heads * a.dim + a.kv_heads * (a.dim + a.vdim);
                 out_k += a.heads * a.vdim;
+            } else if (bs.kind == TkBranchSpec::RETENTION) {
+                const TkRetentionSpec& t = bs.retention;
+                col += 2 * t.heads * (t.dim + t.vdim);
+                out_k += t.heads * t.vdim;
             } else {
                 const TkDeltaSpec& d = bs.delta;
                 if (!(B.rank_a = src.rows_of(bs.prefix + "a1")) || !(B.rank_g = src.rows_of(bs.prefix + "g1"))) return false;
@@ -211,7 +222,20 @@ bool TkLayeredModel::build(Source& src) {
                     out_bias.resize((size_t)D, 0.0f);
                     for (int k = 0; k < D; ++k) out_bias[(size_t)k] += bs.scale * o[(size_t)k];
                 }
+                if (a.taps > 0) {
+                    std::vector<float> conv;
+                    if (!src.values(p + "q.conv", {nq, a.taps}, &conv, -0.9f, 0.9f) || !src.values(p + "k.conv", {nk, a.taps}, &conv, -0.9f, 0.9f) ||
+                        !src.values(p + "v.conv", {nv, a.taps}, &conv, -0.9f, 0.9f) || !src.upload(conv, &B.conv))
+                        return false;
+                }
                 if (a.qk_norm && (!src.vec(p + "q.norm", {a.dim}, &B.q_norm, 0.8f, 1.2f) || !src.vec(p + "k.norm", {a.dim}, &B.k_norm, 0.8f, 1.2f))) return false;
+            } else if (bs.kind == TkBranchSpec::RETENTION) {
+                const TkRetentionSpec& t = bs.retention;
+                const int nk = t.heads * t.dim, nv = t.heads * t.vdim, c0 = B.col;
+                if (!src.put(p + "q", nk, D, L.in.img, L.in.K, c0, 0) || !src.put(p + "k", nk, D, L.in.img, L.in.K, c0 + nk, 0) ||
+                    !src.put(p + "v", nv, D, L.in.img, L.in.K, c0 + 2 * nk, 0) || !src.put(p + "g", nv, D, L.in.img, L.in.K, c0 + 2 * nk + nv, 0) ||
+                    !src.put(p + "o", D, nv, L.out.img, L.out.K, 0, B.out_k0))
+                    return false;
             } else {
                 const TkDeltaSpec& d = bs.delta;
                 const int nk = d.kv_heads * d.dim, nv = d.heads * d.vdim, c0 = B.col;
@@ -230,10 +254,11 @@ bool TkLayeredModel::build(Source& src) {
             }
         }
         if (!out_bias.empty() && !src.upload(out_bias, &L.out_bias)) return false;
-        if (!src.vec(s.norm1, {D}, &L.norm1, 0.8f, 1.2f)) return false;
+        if (!src.norm(s.pre1, &L.pre1) || !src.norm(s.norm1, &L.norm1)) return false;
         const TkMlpSpec& f = s.mlp;
+        L.bytes = matrix_bytes_ - before;
         if (f.kind == TkMlpSpec::NONE) continue;
-        if (!src.vec(s.norm2, {D}, &L.norm2, 0.8f, 1.2f)) return false;
+        if (!src.norm(s.pre2, &L.pre2) || !src.norm(s.norm2, &L.norm2)) return false;
         const int E = f.kind == TkMlpSpec::MOE ? f.experts : 1, ffp = (f.ff + 15) / 16 * 16;
         if (!mat(&L.gate_up, 2 * ffp, D, E) || !mat(&L.down, D, f.ff, E)) return false;
         for (int e = 0; e < E; ++e) {
@@ -243,8 +268,14 @@ bool TkLayeredModel::build(Source& src) {
                 return false;
         }
         if (f.kind == TkMlpSpec::MOE && (!mat(&L.router, f.experts, D) || !src.put(f.prefix + "router", f.experts, D, L.router.img, L.router.K, 0, 0))) return false;
+        L.bytes = matrix_bytes_ - before;
     }
-    return src.vec("final.norm", {D}, &final_norm, 0.8f, 1.2f) && mat(&head, cfg.vocab, D) && src.put("head", cfg.vocab, D, head.img, head.K, 0, 0);
+    for (size_t i = 0; i < layers.size(); ++i)
+        if (cfg.layers[i].weights_of >= 0) {
+            layers[i] = layers[(size_t)cfg.layers[i].weights_of]; /* the model owns the memory, layers only point to it */
+            matrix_bytes_ += layers[i].bytes;                     /* streamed once more */
+        }
+    return src.norm("final.norm", &final_norm) && mat(&head, cfg.vocab, D) && src.put("head", cfg.vocab, D, head.img, head.K, 0, 0);
 }
 
 bool TkLayeredModel::load(const std::string& dir, const std::string& dtype, int dev) {

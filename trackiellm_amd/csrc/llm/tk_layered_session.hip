@@ -28,6 +28,34 @@ bool TkLayeredSession::alloc(void** p, size_t bytes, bool zero) {
     return true;
 }
 
+/* cosines and sines of the positions, double precision on the host; one table per (dims, base) */
+bool TkLayeredSession::rotation(int dims, double base, Rope* out) {
+    if (dims <= 0) return true;
+    Rope& r = rope_[{dims, base}];
+    if (!r.c) {
+        const int half = dims / 2;
+        std::vector<float> cs((size_t)max_ctx * half), sn(cs.size());
+        for (int t = 0; t < max_ctx; ++t)
+            for (int i = 0; i < half; ++i) {
+                const double ang = (double)t * pow(base, -2.0 * i / (double)dims);
+                cs[(size_t)t * half + i] = (float)cos(ang);
+                sn[(size_t)t * half + i] = (float)sin(ang);
+            }
+        if (!alloc((void**)&r.c, cs.size() * 4) || !alloc((void**)&r.s, sn.size() * 4)) return false;
+        HIPQ(hipMemcpy(r.c, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
+        HIPQ(hipMemcpy(r.s, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
+    }
+    *out = r;
+    return true;
+}
+
+/* rows of a retention scan's blocks: about 512 workgroups (heads x blocks) in a pass */
+int TkLayeredSession::retention_rows(int nrows) const {
+    int n = TK_RETENTION_BLOCK;
+    while ((int64_t)(nrows / n) * ret_heads_ > 512) n *= 2;
+    return n;
+}
+
 bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_tokens) {
     m_ = m;
     max_seq = mseq;
@@ -41,9 +69,9 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
     const int64_t want = ((int64_t)mseq * mctx + 63) / 64 * 64;
     const int R = (int)std::max<int64_t>(TK_MAX_ROWS, std::min<int64_t>(PASS_ROWS, want));
     const int max_tiles = R / 64 + mseq;
-    /* tables behind the base's rows: segment of a row, segments, wanted rows, attention tiles, ids of wanted rows */
+    /* tables behind the base's rows: segment of a row, segments, wanted rows, attention tiles, retention blocks */
     int32_t* ext = nullptr;
-    const size_t extra = (size_t)R + 4 * (size_t)mseq + R + 2 * (size_t)max_tiles;
+    const size_t block_ints = sizeof(TkRetentionBlock) / 4, extra = (size_t)R + 4 * (size_t)mseq + R + (2 + block_ints) * (size_t)max_tiles;
     if (!init_tables(m->device, c.vocab, R, extra, &ext)) return false;
     tab_ints_ = 3 * (size_t)R + extra;
     d_tab_ = d_seq;
@@ -55,7 +83,8 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
     tab_.seg_in = p; p += mseq;
     tab_.seg_out = p; p += mseq;
     d_out_rows_ = p; p += R;
-    d_tiles_ = p;
+    d_tiles_ = p; p += 2 * (size_t)max_tiles;
+    d_blocks_ = p;
     HIPQ(hipHostMalloc((void**)&h_tab_, tab_ints_ * 4, hipHostMallocDefault));
     memset(h_tab_, 0, tab_ints_ * 4);
     if (!alloc((void**)&d_pages_, (size_t)mseq * max_pages_ * 4, true) || !alloc((void**)&d_otok_, TK_MAX_ROWS * 4, true)) return false;
@@ -65,7 +94,12 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
     h_pages_.assign((size_t)mseq * max_pages_, 0);
     for (int i = n_pages_ - 1; i >= 0; --i) free_pages_.push_back(i);
 
-    size_t proj = 16, low = 16, mix = 0, lowk = 0, q = 0, dq = 0, dv = 0, dg = 0, dh = 0, ff = 0, scratch = 0, E = 0, gather = 0, moe_ff = 0, assign = 0, moe_rows = 0;
+    size_t proj = 16, low = 16, mix = 0, lowk = 0, q = 0, dq = 0, dv = 0, dg = 0, dh = 0, ff = 0, scratch = 0, E = 0, gather = 0, moe_ff = 0, assign = 0, moe_rows = 0, sums = 0;
+    for (const TkLayerSpec& s : c.layers)
+        for (const TkBranchSpec& b : s.branches)
+            if (b.kind == TkBranchSpec::RETENTION) ret_heads_ = std::max(ret_heads_, b.retention.heads);
+    int ret_slots = 0;
+    for (int n = 1; ret_heads_ && n <= R; ++n) ret_slots = std::max(ret_slots, n / retention_rows(n));
     st_.resize(c.layers.size());
     for (size_t l = 0; l < c.layers.size(); ++l) {
         const TkLayeredLayer& L = m->layers[l];
@@ -84,28 +118,23 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
                 if (!alloc(&bs.kv.k, (size_t)n_pages_ * a.kv_heads * TK_PAGE * bs.kv.dim_pad * esz, true) || !alloc(&bs.kv.v, (size_t)n_pages_ * a.kv_heads * TK_PAGE * bs.kv.vdim_pad * esz, true))
                     return false;
                 q = std::max(q, (size_t)a.heads * bs.kv.dim_pad);
-                const int64_t seen = a.window > 0 ? (int64_t)a.window / TK_PAGE + 2 + (a.keep_first + TK_PAGE - 1) / TK_PAGE : max_pages_;
+                int64_t seen = a.window > 0 ? (int64_t)a.window / TK_PAGE + 2 + (a.keep_first + TK_PAGE - 1) / TK_PAGE : max_pages_;
+                if (a.chunk > 0) seen = std::min<int64_t>(seen, (int64_t)a.chunk / TK_PAGE + 2);
                 bs.splits_pages = (int)std::min<int64_t>(seen, max_pages_);
                 TkAttnArgs aa{};
                 aa.heads = a.heads; aa.kv_heads = a.kv_heads; aa.kv = bs.kv;
                 for (int n = 1; n <= TK_MAX_ROWS; ++n) scratch = std::max(scratch, tk_attn_rows_scratch_floats(aa, n, tk_attn_rows_splits(aa, bs.splits_pages, n)));
-                if (a.rot_dims > 0) {
-                    Rope& r = rope_[{a.rot_dims, a.rot_base}];
-                    if (!r.c) { /* double precision on the host */
-                        const int half = a.rot_dims / 2;
-                        std::vector<float> cs((size_t)mctx * half), sn(cs.size());
-                        for (int t = 0; t < mctx; ++t)
-                            for (int i = 0; i < half; ++i) {
-                                const double ang = (double)t * pow(a.rot_base, -2.0 * i / (double)a.rot_dims);
-                                cs[(size_t)t * half + i] = (float)cos(ang);
-                                sn[(size_t)t * half + i] = (float)sin(ang);
-                            }
-                        if (!alloc((void**)&r.c, cs.size() * 4) || !alloc((void**)&r.s, sn.size() * 4)) return false;
-                        HIPQ(hipMemcpy(r.c, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
-                        HIPQ(hipMemcpy(r.s, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
-                    }
-                    bs.rope = r;
-                }
+                if (!rotation(a.rot_dims, a.rot_base, &bs.rope)) return false;
+                if (a.taps > 0 && !alloc((void**)&bs.conv, 2 * (size_t)mseq * ((size_t)a.heads * a.dim + (size_t)a.kv_heads * (a.dim + a.vdim)) * (a.taps - 1) * 4, true)) return false;
+            } else if (s.branches[b].kind == TkBranchSpec::RETENTION) {
+                const TkRetentionSpec& t = s.branches[b].retention;
+                const size_t state = (size_t)t.heads * t.dim * ((t.vdim + 3) / 4 * 4);
+                std::vector<float> powers;
+                for (double x : t.decay)
+                    for (int n = 0; n <= TK_RETENTION_BLOCK; ++n) powers.push_back((float)pow(x, n));
+                if (!rotation(t.rot_dims, t.rot_base, &bs.rope) || !alloc((void**)&bs.state, 2 * (size_t)mseq * state * 4, true) || !alloc((void**)&bs.decay, powers.size() * 4)) return false;
+                HIPQ(hipMemcpy(bs.decay, powers.data(), powers.size() * 4, hipMemcpyHostToDevice));
+                sums = std::max(sums, (size_t)ret_slots * state);
             } else {
                 const TkDeltaSpec& d = s.branches[b].delta;
                 const size_t ch = 2 * (size_t)d.kv_heads * d.dim + (size_t)d.heads * d.vdim;
@@ -135,7 +164,7 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
         !alloc((void**)&y_, yrows * c.width * 4, true) || !alloc(&img_x_, tk_img_bytes(type, R, c.width), true) || !alloc(&img_low_, lowk, true) ||
         !alloc(&img_mix_, mix, true) || !alloc(&img_ff_, std::max(ff, moe_ff), true) || !alloc(&img_head_, tk_img_bytes(type, TK_MAX_ROWS, c.width), true) ||
         !alloc(&q_, (size_t)R * q * esz, true) || !alloc((void**)&dq_, (size_t)R * dq * 4) || !alloc((void**)&dk_, (size_t)R * dq * 4) || !alloc((void**)&dv_, (size_t)R * dv * 4) ||
-        !alloc((void**)&dg_, (size_t)R * dg * 4) || !alloc((void**)&db_, (size_t)R * dh * 4) || !alloc((void**)&do_, (size_t)R * dv * 4) || !alloc((void**)&scratch_, scratch * 4))
+        !alloc((void**)&sums_, sums * 4) || !alloc((void**)&dg_, (size_t)R * dg * 4) || !alloc((void**)&db_, (size_t)R * dh * 4) || !alloc((void**)&do_, (size_t)R * dv * 4) || !alloc((void**)&scratch_, scratch * 4))
         return false;
     if (E && (!alloc((void**)&router_, (size_t)R * ((E + 15) / 16 * 16) * 4) || !alloc(&img_gather_, gather, true) || !alloc((void**)&moe_.count, E * 4, true) ||
               !alloc((void**)&moe_.expert, assign * 4) || !alloc((void**)&moe_.rank, assign * 4) || !alloc((void**)&moe_.weight, assign * 4) || !alloc((void**)&moe_.tile0, E * 4) ||
@@ -199,7 +228,10 @@ bool TkLayeredSession::describe(int nrows, const int32_t* seq, const int32_t* po
     const int R = row_cap_;
     int32_t *h_seq = h_tab_, *h_pos = h_seq + R, *h_tok = h_pos + R, *h_seg = h_tok + R, *row0 = h_seg + R, *sn = row0 + max_seq, *sin = sn + max_seq, *sout = sin + max_seq,
             *tiles = sout + max_seq + R;
-    p->nrows = nrows; p->nseg = 0; p->ntiles = 0; p->single = true;
+    TkRetentionBlock* blocks = (TkRetentionBlock*)(h_tab_ + (d_blocks_ - d_tab_));
+    *p = Pass();
+    p->nrows = nrows; p->singles = false;
+    const int per = retention_rows(nrows);
     /* first whether the rows are allowed at all, with nothing changed */
     struct Run { int r, n, side; };
     std::vector<Run> runs;
@@ -235,7 +267,15 @@ bool TkLayeredSession::describe(int nrows, const int32_t* seq, const int32_t* po
         sout[p->nseg] = 2 * id + (side ^ 1);
         for (int t = 0; t < n; t += 64, ++p->ntiles) { tiles[2 * p->ntiles] = r + t; tiles[2 * p->ntiles + 1] = std::min(64, n - t); }
         for (int i = 0; i < n; ++i) { h_seq[r + i] = id; h_pos[r + i] = pos[r + i]; h_tok[r + i] = tok[r + i]; h_seg[r + i] = p->nseg; }
-        if (n > 1) p->single = false;
+        if (n > 1) {
+            p->single = false;
+            const int nb = (n + per - 1) / per;
+            if (ret_heads_)
+                for (int b = 0; b < nb; ++b) blocks[p->nblocks++] = TkRetentionBlock{r + b * per, std::min(per, n - b * per), p->nseg, p->nsums, b, b + 1 == nb};
+            p->nsums += nb - 1;
+        } else {
+            p->singles = true;
+        }
         ++p->nseg;
     }
     return upload_pages();
@@ -288,10 +328,11 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
     const TkLayeredConfig& c = m_->cfg;
     const int type = m_->type, D = c.width, kt = tk_img_kt(type), xkt = tk_img_pad_k(type, D) / kt, n = p.nrows;
     hipStream_t s = stream;
-    tk_launch_layer_embed(type, m_->embed, D, d_tok, n, x_, img_x_, xkt, s);
+    tk_launch_layer_embed(type, m_->embed, D, c.embed_scale, d_tok, n, x_, m_->layers[0].pre1, c.eps, img_x_, xkt, s);
     for (size_t l = 0; l < c.layers.size(); ++l) {
         const TkLayerSpec& spec = c.layers[l];
         const TkLayeredLayer& L = m_->layers[l];
+        const TkNorm after = l + 1 < c.layers.size() ? m_->layers[l + 1].pre1 : TkNorm{}; /* on the next layer's input: fused into this layer's last kernel */
         TkImgGemm g{};
         g.type = type; g.w = L.in.img; g.a = img_x_; g.K = L.in.K; g.N = L.in.N; g.nrows = n;
         g.out = proj_; g.ldc = L.in.N; g.n_valid = L.in.rows;
@@ -314,10 +355,19 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
                 const TkAttnSpec& sp = bs.attn;
                 TkAttnArgs a{};
                 a.heads = sp.heads; a.kv_heads = sp.kv_heads; a.dim = sp.dim; a.vdim = sp.vdim; a.rot_dims = sp.rot_dims; a.window = sp.window; a.keep_first = sp.keep_first;
+                a.chunk = sp.chunk; a.softcap = sp.softcap; a.taps = sp.taps; a.conv = B.conv; a.conv_state = st.conv;
                 a.scale = sp.scale; a.out_scale = bs.scale; a.eps = c.eps; a.col = B.col; a.bias = B.bias; a.q_norm = B.q_norm; a.k_norm = B.k_norm;
                 a.rope_cos = st.rope.c; a.rope_sin = st.rope.s; a.q = q_; a.kv = st.kv; a.out_img = img_mix_; a.out_k0 = B.out_k0; a.out_ktiles = L.out.K / kt;
                 as.push_back(a);
                 visible.push_back(st.splits_pages);
+            } else if (bs.kind == TkBranchSpec::RETENTION) { /* reads the projections itself */
+                const TkRetentionSpec& sp = bs.retention;
+                TkRetentionArgs a{};
+                a.heads = sp.heads; a.dim = sp.dim; a.vdim = sp.vdim; a.rot_dims = sp.rot_dims; a.out_scale = bs.scale; a.eps = c.eps; a.col = B.col;
+                a.rope_cos = st.rope.c; a.rope_sin = st.rope.s; a.decay = st.decay; a.state = st.state; a.sums = sums_;
+                a.out_img = img_mix_; a.out_k0 = B.out_k0; a.out_ktiles = L.out.K / kt;
+                if (p.nblocks) tk_launch_retention_scan(type, a, proj_, L.in.N, tab_, (const TkRetentionBlock*)d_blocks_, p.nblocks, p.nsums, s);
+                if (p.singles) tk_launch_retention_step(type, a, proj_, L.in.N, tab_, p.nseg, s);
             } else {
                 const TkDeltaSpec& sp = bs.delta;
                 TkDeltaArgs d{};
@@ -351,20 +401,21 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
         int slabs = 1;
         o.max_slabs = most; o.slab_floats = slab;
         gemm(o, &slabs);
-        tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, L.out_bias, 1.0f, nullptr, nullptr, 0}, L.norm1, c.eps, D, n, x_, img_x_, xkt, s);
+        tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, L.out_bias, 1.0f, nullptr, nullptr, 0}, L.norm1, spec.mlp.kind == TkMlpSpec::NONE ? after : L.pre2, c.eps, D, n, x_, img_x_, xkt, s);
         if (spec.mlp.kind == TkMlpSpec::DENSE) {
             TkImgGemm u{};
             u.type = type; u.w = L.gate_up.img; u.a = img_x_; u.K = L.gate_up.K; u.N = L.gate_up.N; u.nrows = n;
             u.swiglu = 1; u.act_img = img_ff_; u.act_ktiles = L.down.K / kt; u.act_valid = spec.mlp.ff;
+            if (spec.mlp.act == TkMlpSpec::CLAMPED) { u.act_clamped = 1; u.act_limit = spec.mlp.limit; u.act_slope = spec.mlp.slope; u.act_shift = spec.mlp.shift; }
             gemm(u);
             TkImgGemm w{};
             w.type = type; w.w = L.down.img; w.a = img_ff_; w.K = L.down.K; w.N = L.down.N; w.nrows = n; w.out = y_; w.ldc = D; w.n_valid = D;
             w.max_slabs = most; w.slab_floats = slab;
             gemm(w, &slabs);
-            tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, nullptr, 0.0f, nullptr, nullptr, 0}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
+            tk_launch_post_norm(type, TkSubOut{y_, D, slabs, slab, nullptr, 0.0f, nullptr, nullptr, 0}, L.norm2, after, c.eps, D, n, x_, img_x_, xkt, s);
         } else if (spec.mlp.kind == TkMlpSpec::MOE) {
             enqueue_moe(spec, L, n);
-            tk_launch_post_norm(type, TkSubOut{y_, D, 1, 0, nullptr, 0.0f, moe_.slot, moe_.weight, spec.mlp.top}, L.norm2, c.eps, D, n, x_, img_x_, xkt, s);
+            tk_launch_post_norm(type, TkSubOut{y_, D, 1, 0, nullptr, 0.0f, moe_.slot, moe_.weight, spec.mlp.top}, L.norm2, after, c.eps, D, n, x_, img_x_, xkt, s);
         }
         if (streams_) (void)hipMemcpyAsync(streams_ + l * (size_t)n * D, x_, (size_t)n * D * 4, hipMemcpyDeviceToHost, s);
     }

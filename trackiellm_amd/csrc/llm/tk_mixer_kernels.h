@@ -1,7 +1,7 @@
 /*
  * tk_mixer_kernels.h — launch wrappers of the layer-list decoders' kernels (tk_layered.h): paged attention with a sliding window and kept first
- * positions, the gated delta rule with its short convolutions, output norms on the residual stream, the grouped sigmoid router.  Sizes and
- * constants are arguments throughout.  Wrappers only enqueue on `s`.
+ * positions, or with chunks, the gated delta rule and retention, short convolutions, norms around the residual stream, the grouped sigmoid router.
+ * Sizes and constants are arguments throughout.  Wrappers only enqueue on `s`.
  *
  * Activations that feed a matrix product are operand images (nn/tk_gemm_image.h) of the session's element type; everything else — projections'
  * results, the residual stream, gates, decays, recurrent state — is f32.
@@ -31,9 +31,12 @@ struct TkPassTab {
 struct TkKvPool { void *k, *v; int dim_pad, vdim_pad; };
 
 struct TkAttnArgs {
-    int heads, kv_heads, dim, vdim, rot_dims, window, keep_first;
-    float scale, out_scale, eps;
+    int heads, kv_heads, dim, vdim, rot_dims, window, keep_first, chunk;
+    float scale, softcap, out_scale, eps;
     int col;                          /* first column of q | k | v in the projections */
+    int taps;                         /* > 0: a causal convolution on every channel of q | k | v, before the rotation (no biases and norms then) */
+    const float* conv;                /* [channels][taps] */
+    float* conv_state;                /* [copies][channels][taps - 1] */
     const float *bias;                /* q | k | v biases or null */
     const float *q_norm, *k_norm;     /* null: no norm */
     const float *rope_cos, *rope_sin; /* [max_ctx][rot_dims / 2] */
@@ -58,7 +61,26 @@ struct TkDeltaArgs {
     int out_k0, out_ktiles;
 };
 
-void tk_launch_layer_embed(int type, const uint16_t* table, int width, const int32_t* tok, int nrows, float* x, void* img, int ktiles, hipStream_t s);
+/* linear attention with one constant decay per head: S <- decay S + k v^T, o = S^T q; q and k rotated, k times dim^-1/2; o over its root mean square,
+ * times silu(gate) */
+#define TK_RETENTION_BLOCK 64 /* rows of a scan's blocks are multiples of this */
+struct TkRetentionArgs {
+    int heads, dim, vdim, rot_dims;
+    float out_scale, eps;
+    int col;                          /* first column of q | k | v | gate in the projections */
+    const float *rope_cos, *rope_sin; /* [max_ctx][rot_dims / 2] */
+    const float* decay;               /* [heads][TK_RETENTION_BLOCK + 1] powers 0 .. TK_RETENTION_BLOCK */
+    float* state;                     /* [copies][heads][dim][vdim padded to 4] */
+    float* sums;                      /* [slots][heads][dim][vdim padded to 4] what a block of rows adds to the state */
+    void* out_img;
+    int out_k0, out_ktiles;
+};
+
+/* a norm's tensors; w null: no norm.  layer: mean taken off, b added; otherwise over the root mean square */
+struct TkNorm { const float *w, *b; int layer; };
+
+/* x = table[tok] * scale; the image of next(x) */
+void tk_launch_layer_embed(int type, const uint16_t* table, int width, float scale, const int32_t* tok, int nrows, float* x, const TkNorm& next, float eps, void* img, int ktiles, hipStream_t s);
 
 /* everything between the projections and the mixers: biases, per-head norms, rotation, cache append; convolutions, unit norms, decays, step sizes */
 void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs* attn, const TkDeltaArgs* delta, const TkPassTab& t, int nrows, hipStream_t s);
@@ -75,6 +97,13 @@ void tk_launch_delta_scan(int type, const TkDeltaArgs& d, const TkPassTab& t, in
 /* the same for passes whose segments are single rows: one launch */
 void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s);
 
+/* blocks: [n_blocks] runs of rows of one segment; every block but a segment's last has the same number of rows, a multiple of TK_RETENTION_BLOCK.
+ * n_sums: how many of them are followed by another block of their segment (their own share of the state goes through args.sums) */
+struct TkRetentionBlock { int32_t row0, n, seg, slot0, index, last; }; /* slot0: of the segment's first block in args.sums; index: of the block in its segment */
+void tk_launch_retention_scan(int type, const TkRetentionArgs& d, const float* proj, int ld, const TkPassTab& t, const TkRetentionBlock* blocks, int n_blocks, int n_sums, hipStream_t s);
+/* the segments that are single rows (others are left alone) */
+void tk_launch_retention_step(int type, const TkRetentionArgs& d, const float* proj, int ld, const TkPassTab& t, int n_segments, hipStream_t s);
+
 /* tk_launch_attn_rows and tk_launch_delta_step in one launch, side by side; false (nothing launched): sizes it has no form for */
 bool tk_launch_mixers_step(int type, const TkAttnArgs& a, const TkDeltaArgs& d, const TkPassTab& t, int nrows, hipStream_t s);
 
@@ -85,10 +114,10 @@ struct TkSubOut {
     const float* bias; float bias_scale; /* bias may be null */
     const int32_t* slot; const float* weight; int top; /* top > 0: y[slot[row * top + j]] * weight[row * top + j] summed over j */
 };
-/* x += norm(output) * w; the image of the new x */
-void tk_launch_post_norm(int type, const TkSubOut& o, const float* w, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s);
+/* x += norm(output); the image of next(x), the next sublayer's input */
+void tk_launch_post_norm(int type, const TkSubOut& o, const TkNorm& norm, const TkNorm& next, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s);
 /* norm of the listed rows (null: rows 0 .. n - 1) as an image */
-void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const float* w, float eps, int width, void* img, int ktiles, hipStream_t s);
+void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const TkNorm& norm, float eps, int width, void* img, int ktiles, hipStream_t s);
 
 struct TkMoeTab {
     int32_t* count;      /* [experts], zero between passes */

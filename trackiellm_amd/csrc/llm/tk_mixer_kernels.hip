@@ -14,34 +14,6 @@ constexpr float LOG2E = 1.44269504088896340736f;
 
 /* ------------------------------------------------------------------ embedding, norms ------- */
 
-/* VEC: eight consecutive elements per thread (width a multiple of eight), else one */
-template <typename T, bool VEC>
-__global__ __launch_bounds__(256) void k_layer_embed(const uint16_t* table, int width, const int32_t* tok, float* x, T* img, int ktiles) {
-    const int row = blockIdx.x;
-    const uint16_t* e = table + (size_t)tok[row] * width;
-    float* xr = x + (size_t)row * width;
-    if (VEC) {
-        for (int k = threadIdx.x * 8; k < width; k += 256 * 8) {
-            const tk_v4u u = *(const tk_v4u*)(e + k);
-            tk_v4f a, b;
-#pragma unroll
-            for (int i = 0; i < 2; ++i) {
-                a[2 * i] = __uint_as_float(u[i] << 16); a[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
-                b[2 * i] = __uint_as_float(u[2 + i] << 16); b[2 * i + 1] = __uint_as_float(u[2 + i] & 0xffff0000u);
-            }
-            *(tk_v4f*)(xr + k) = a;
-            *(tk_v4f*)(xr + k + 4) = b;
-            tk_img_put8(img, row, k, ktiles, a, b);
-        }
-        return;
-    }
-    for (int k = threadIdx.x; k < width; k += 256) {
-        const float v = tk_bf16_float(e[k]);
-        xr[k] = v;
-        tk_img_put(img, row, k, ktiles, v);
-    }
-}
-
 __device__ __forceinline__ float block_sum(float v, float* red /* [16] */) {
     v = tk_wave_sum(v);
     const int w = threadIdx.x >> 6, nw = blockDim.x >> 6;
@@ -53,94 +25,226 @@ __device__ __forceinline__ float block_sum(float v, float* red /* [16] */) {
     return t;
 }
 
-__device__ __forceinline__ float dot4(tk_v4f a, tk_v4f b) { return fmaf(a[0], b[0], fmaf(a[1], b[1], fmaf(a[2], b[2], a[3] * b[3]))); }
-
-template <typename T, bool VEC>
-__global__ __launch_bounds__(512) void k_post_norm(TkSubOut o, const float* w, float eps, int width, float* x, T* img, int ktiles) {
-    extern __shared__ __attribute__((aligned(16))) float ybuf[];
-    __shared__ float red[16];
-    const int row = blockIdx.x, nt = blockDim.x;
-    float* xr = x + (size_t)row * width;
-    float ss = 0.0f;
-    if (VEC) {
-        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
-            tk_v4f a, b;
-            if (o.top > 0) {
-                a = b = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
-                for (int j = 0; j < o.top; ++j) {
-                    const float* p = o.y + (size_t)o.slot[row * o.top + j] * o.ld + k;
-                    const float c = o.weight[row * o.top + j];
-                    a += *(const tk_v4f*)p * c;
-                    b += *(const tk_v4f*)(p + 4) * c;
-                }
+/* A row of `width` elements over a workgroup, NV groups of eight a thread.  VEC (width a multiple of eight): a group is eight consecutive
+ * elements; otherwise elements a workgroup apart. */
+template <bool VEC, int NV>
+struct Row {
+    float v[NV][8];
+    __device__ static __forceinline__ int at(int j, int e) { return VEC ? (int)(j * blockDim.x + threadIdx.x) * 8 + e : (int)((j * 8 + e) * blockDim.x + threadIdx.x); }
+    /* f(group, element, k) of the thread's elements below width */
+    template <typename F>
+    __device__ static __forceinline__ void each(int width, F f) {
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+            if (VEC && at(j, 0) >= width) break;
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                if (VEC || at(j, e) < width) f(j, e, at(j, e));
+        }
+    }
+    __device__ __forceinline__ void load(const float* p, int width) {
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+            if (VEC) {
+                if (at(j, 0) >= width) break;
+                const tk_v4f a = *(const tk_v4f*)(p + at(j, 0)), b = *(const tk_v4f*)(p + at(j, 0) + 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { v[j][e] = a[e]; v[j][4 + e] = b[e]; }
             } else {
-                const float* p = o.y + (size_t)row * o.ld + k;
-                a = *(const tk_v4f*)p; b = *(const tk_v4f*)(p + 4);
-                for (int i = 1; i < o.slabs; ++i) { a += *(const tk_v4f*)(p + i * o.slab_floats); b += *(const tk_v4f*)(p + i * o.slab_floats + 4); }
-                if (o.bias) { a += *(const tk_v4f*)(o.bias + k) * o.bias_scale; b += *(const tk_v4f*)(o.bias + k + 4) * o.bias_scale; }
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[j][e] = at(j, e) < width ? p[at(j, e)] : 0.0f;
             }
-            *(tk_v4f*)(ybuf + k) = a;
-            *(tk_v4f*)(ybuf + k + 4) = b;
-            ss += dot4(a, a) + dot4(b, b);
+        }
+    }
+    __device__ __forceinline__ void store(float* p, int width) const {
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+            if (VEC) {
+                if (at(j, 0) >= width) break;
+                *(tk_v4f*)(p + at(j, 0)) = tk_v4f{v[j][0], v[j][1], v[j][2], v[j][3]};
+                *(tk_v4f*)(p + at(j, 0) + 4) = tk_v4f{v[j][4], v[j][5], v[j][6], v[j][7]};
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; ++e)
+                    if (at(j, e) < width) p[at(j, e)] = v[j][e];
+            }
+        }
+    }
+    template <typename T>
+    __device__ __forceinline__ void image(T* img, int64_t row, int ktiles, int width) const {
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+            if (VEC) {
+                if (at(j, 0) >= width) break;
+                tk_img_put8(img, row, at(j, 0), ktiles, tk_v4f{v[j][0], v[j][1], v[j][2], v[j][3]}, tk_v4f{v[j][4], v[j][5], v[j][6], v[j][7]});
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; ++e)
+                    if (at(j, e) < width) tk_img_put(img, row, at(j, e), ktiles, v[j][e]);
+            }
+        }
+    }
+    /* the row over its root mean square, or less its mean over its deviation; red: [24], of this call only.  The variance is merged from the waves'
+     * own means and squared deviations. */
+    __device__ __forceinline__ void normalise(const TkNorm& n, float eps, int width, float* red) {
+        Row w, b;
+        w.load(n.w, width);
+        if (n.layer) b.load(n.b, width);
+        const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+        float mean = 0.0f, r;
+        if (n.layer) {
+            float s = 0.0f, c = 0.0f, d = 0.0f;
+            each(width, [&](int j, int e, int) { s += v[j][e]; c += 1.0f; });
+            s = tk_wave_sum(s);
+            c = tk_wave_sum(c);
+            const float m = c > 0.0f ? s / c : 0.0f;
+            each(width, [&](int j, int e, int) { d += (v[j][e] - m) * (v[j][e] - m); });
+            d = tk_wave_sum(d);
+            if ((threadIdx.x & 63) == 0) { red[wave] = s; red[8 + wave] = c; red[16 + wave] = d; }
+            __syncthreads();
+            for (int i = 0; i < nw; ++i) mean += red[i];
+            mean /= (float)width;
+            float var = 0.0f;
+            for (int i = 0; i < nw; ++i) {
+                const float ci = red[8 + i], off = ci > 0.0f ? red[i] / ci - mean : 0.0f;
+                var += red[16 + i] + ci * off * off;
+            }
+            r = 1.0f / sqrtf(var / (float)width + eps);
+        } else {
+            float d = 0.0f;
+            each(width, [&](int j, int e, int) { d += v[j][e] * v[j][e]; });
+            d = tk_wave_sum(d);
+            if ((threadIdx.x & 63) == 0) red[wave] = d;
+            __syncthreads();
+            float t = 0.0f;
+            for (int i = 0; i < nw; ++i) t += red[i];
+            r = 1.0f / sqrtf(t / (float)width + eps);
+        }
+        each(width, [&](int j, int e, int) { v[j][e] = (v[j][e] - mean) * r * w.v[j][e] + (n.layer ? b.v[j][e] : 0.0f); });
+    }
+};
+
+template <typename T, bool VEC, int NV>
+__global__ __launch_bounds__(512) void k_layer_embed(const uint16_t* table, int width, float scale, const int32_t* tok, float* x, TkNorm next, float eps, T* img, int ktiles) {
+    __shared__ float red[24];
+    const int row = blockIdx.x;
+    const uint16_t* e = table + (size_t)tok[row] * width;
+    Row<VEC, NV> v;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        if (VEC) {
+            if (v.at(j, 0) >= width) break;
+            const tk_v4u u = *(const tk_v4u*)(e + v.at(j, 0));
+#pragma unroll
+            for (int i = 0; i < 4; ++i) { v.v[j][2 * i] = __uint_as_float(u[i] << 16) * scale; v.v[j][2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u) * scale; }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v.v[j][i] = v.at(j, i) < width ? tk_bf16_float(e[v.at(j, i)]) * scale : 0.0f;
+        }
+    }
+    v.store(x + (size_t)row * width, width);
+    if (next.w) v.normalise(next, eps, width, red);
+    v.image(img, row, ktiles, width);
+}
+
+template <typename T, bool VEC, int NV>
+__global__ __launch_bounds__(512) void k_post_norm(TkSubOut o, TkNorm norm, TkNorm next, float eps, int width, float* x, T* img, int ktiles) {
+    __shared__ float red[2][24];
+    const int row = blockIdx.x;
+    float* xr = x + (size_t)row * width;
+    Row<VEC, NV> y, z;
+    if (o.top > 0) {
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) y.v[j][e] = 0.0f;
+        for (int j = 0; j < o.top; ++j) {
+            z.load(o.y + (size_t)o.slot[row * o.top + j] * o.ld, width);
+            const float c = o.weight[row * o.top + j];
+            y.each(width, [&](int g, int e, int) { y.v[g][e] += z.v[g][e] * c; });
         }
     } else {
-        for (int k = threadIdx.x; k < width; k += nt) {
-            float y = 0.0f;
-            if (o.top > 0)
-                for (int j = 0; j < o.top; ++j) y += o.weight[row * o.top + j] * o.y[(size_t)o.slot[row * o.top + j] * o.ld + k];
-            else {
-                y = o.y[(size_t)row * o.ld + k];
-                for (int i = 1; i < o.slabs; ++i) y += o.y[i * o.slab_floats + (size_t)row * o.ld + k];
-                if (o.bias) y += o.bias[k] * o.bias_scale;
-            }
-            ybuf[k] = y;
-            ss += y * y;
+        y.load(o.y + (size_t)row * o.ld, width);
+        for (int i = 1; i < o.slabs; ++i) {
+            z.load(o.y + i * o.slab_floats + (size_t)row * o.ld, width);
+            y.each(width, [&](int g, int e, int) { y.v[g][e] += z.v[g][e]; });
+        }
+        if (o.bias) {
+            z.load(o.bias, width);
+            y.each(width, [&](int g, int e, int) { y.v[g][e] += z.v[g][e] * o.bias_scale; });
         }
     }
-    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps); /* a thread re-reads its own elements of ybuf only */
-    if (VEC) {
-        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
-            const tk_v4f a = *(const tk_v4f*)(xr + k) + *(const tk_v4f*)(ybuf + k) * r * *(const tk_v4f*)(w + k);
-            const tk_v4f b = *(const tk_v4f*)(xr + k + 4) + *(const tk_v4f*)(ybuf + k + 4) * r * *(const tk_v4f*)(w + k + 4);
-            *(tk_v4f*)(xr + k) = a;
-            *(tk_v4f*)(xr + k + 4) = b;
-            tk_img_put8(img, row, k, ktiles, a, b);
-        }
-        return;
-    }
-    for (int k = threadIdx.x; k < width; k += nt) {
-        const float v = xr[k] + ybuf[k] * r * w[k];
-        xr[k] = v;
-        tk_img_put(img, row, k, ktiles, v);
-    }
+    z.load(xr, width);
+    y.normalise(norm, eps, width, red[0]);
+    y.each(width, [&](int g, int e, int) { y.v[g][e] += z.v[g][e]; });
+    y.store(xr, width);
+    if (next.w) y.normalise(next, eps, width, red[1]);
+    y.image(img, row, ktiles, width);
 }
 
-template <typename T, bool VEC>
-__global__ __launch_bounds__(512) void k_rows_norm(const float* x, const int32_t* rows, const float* w, float eps, int width, T* img, int ktiles) {
-    __shared__ float red[16];
-    const int i = blockIdx.x, nt = blockDim.x;
-    const float* xr = x + (size_t)(rows ? rows[i] : i) * width;
-    float ss = 0.0f;
-    if (VEC)
-        for (int k = threadIdx.x * 8; k < width; k += nt * 8) {
-            const tk_v4f a = *(const tk_v4f*)(xr + k), b = *(const tk_v4f*)(xr + k + 4);
-            ss += dot4(a, a) + dot4(b, b);
-        }
-    else
-        for (int k = threadIdx.x; k < width; k += nt) ss += xr[k] * xr[k];
-    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
-    if (VEC)
-        for (int k = threadIdx.x * 8; k < width; k += nt * 8)
-            tk_img_put8(img, i, k, ktiles, *(const tk_v4f*)(xr + k) * r * *(const tk_v4f*)(w + k), *(const tk_v4f*)(xr + k + 4) * r * *(const tk_v4f*)(w + k + 4));
-    else
-        for (int k = threadIdx.x; k < width; k += nt) tk_img_put(img, i, k, ktiles, xr[k] * r * w[k]);
+template <typename T, bool VEC, int NV>
+__global__ __launch_bounds__(512) void k_rows_norm(const float* x, const int32_t* rows, TkNorm norm, float eps, int width, T* img, int ktiles) {
+    __shared__ float red[24];
+    const int i = blockIdx.x;
+    Row<VEC, NV> v;
+    v.load(x + (size_t)(rows ? rows[i] : i) * width, width);
+    v.normalise(norm, eps, width, red);
+    v.image(img, i, ktiles, width);
 }
+
+/* ------------------------------------------------------------------ short convolutions ----- */
+
+/* a causal convolution over the rows of a sequence; what came before the pass is in the history (zeros before the sequence) */
+struct Conv {
+    const float* w; /* [channels][taps] */
+    float* state;   /* [copies][channels][taps - 1] */
+    int channels, taps, col;
+    __device__ __forceinline__ float input(const TkPassTab& t, const float* proj, int ld, int seg, int s, int c) const {
+        if (s >= 0) return proj[(size_t)(t.seg_row0[seg] + s) * ld + col + c]; /* s: time inside the segment */
+        const int in = t.seg_in[seg], hist = taps - 1;
+        return in < 0 ? 0.0f : state[((size_t)in * channels + c) * hist + hist + s];
+    }
+    /* channels c0 + lane + 64 i (< c0 + n) of RW rows from rowb on (rows past the pass repeat its last one) */
+    template <int RW>
+    __device__ __forceinline__ void rows(const TkPassTab& t, const float* proj, int ld, int rowb, int nrows, int c0, int n, int lane, float (&y)[RW][4]) const {
+        const int hist = taps - 1, seg0 = t.seg[rowb], first = rowb - t.seg_row0[seg0];
+        const bool inside = RW > 1 && first >= hist && first + RW <= t.seg_n[seg0]; /* every input is a row of this pass */
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+#pragma unroll
+            for (int r = 0; r < RW; ++r) y[r][i] = 0.0f;
+            const int c = c0 + lane + 64 * i;
+            if (64 * i >= n || lane + 64 * i >= n) continue;
+            if (inside) {
+                for (int j = 0; j < taps; ++j) {
+                    const float tap = w[(size_t)c * taps + j];
+#pragma unroll
+                    for (int r = 0; r < RW; ++r) y[r][i] = fmaf(tap, proj[(size_t)(rowb + r - hist + j) * ld + col + c], y[r][i]);
+                }
+            } else {
+#pragma unroll
+                for (int r = 0; r < RW; ++r) {
+                    const int row = rowb + r < nrows ? rowb + r : nrows - 1, seg = t.seg[row], at = row - t.seg_row0[seg];
+                    for (int j = 0; j < taps; ++j) y[r][i] = fmaf(w[(size_t)c * taps + j], input(t, proj, ld, seg, at - hist + j, c), y[r][i]);
+                }
+            }
+        }
+    }
+    /* a segment's last row leaves the history behind */
+    __device__ __forceinline__ void leave(const TkPassTab& t, const float* proj, int ld, int row, int c0, int n, int lane) const {
+        const int seg = t.seg[row], at = row - t.seg_row0[seg], hist = taps - 1;
+        if (at + 1 != t.seg_n[seg]) return;
+        for (int e = lane; e < n; e += 64)
+            for (int j = 0; j < hist; ++j) state[((size_t)t.seg_out[seg] * channels + c0 + e) * hist + j] = input(t, proj, ld, seg, at + 1 - hist + j, c0 + e);
+    }
+};
 
 /* ------------------------------------------------------------------ between projections and mixers ---- */
 
-/* one wave: one head of q, k or v of RW consecutive rows (rows past the pass repeat its last one and store nothing); all loads come first */
-template <typename T, int RW>
-__device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* proj, int ld, int row0, int nrows, int u, int lane) {
+/* one wave: one head of q, k or v of RW consecutive rows (rows past the pass repeat its last one and store nothing); all loads come first.
+ * CONV: the elements are convolved ones; rotation partners meet in `ex`, [RW][TK_MAX_HEAD_DIM] of LDS of this wave's own */
+template <typename T, int RW, bool CONV>
+__device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* proj, int ld, int row0, int nrows, int u, int lane, float* ex) {
     const bool is_q = u < a.heads, is_v = u >= a.heads + a.kv_heads;
     const int n = is_v ? a.vdim : a.dim;
     const int head = is_q ? u : is_v ? u - a.heads - a.kv_heads : u - a.heads;
@@ -151,6 +255,20 @@ __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& 
     float v[RW][4], z[RW][4], c[RW][4], s[RW][4]; /* element, its rotation partner, cosine, signed sine */
     int pos[RW];
     size_t page[RW];
+    const Conv conv{a.conv, a.conv_state, (a.heads + a.kv_heads) * a.dim + a.kv_heads * a.vdim, a.taps, a.col};
+    if (CONV) {
+        conv.rows<RW>(t, proj, ld, row0, nrows, off, n, lane, v);
+        if (half > 0) {
+#pragma unroll
+            for (int r = 0; r < RW; ++r)
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (lane + 64 * i < 2 * half) ex[r * TK_MAX_HEAD_DIM + lane + 64 * i] = v[r][i];
+            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+            __builtin_amdgcn_wave_barrier();
+            __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+        }
+    }
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
         const int row = row0 + r < nrows ? row0 + r : nrows - 1;
@@ -160,13 +278,14 @@ __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& 
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int e = lane + 64 * i;
-            v[r][i] = z[r][i] = s[r][i] = 0.0f;
+            if (!CONV) v[r][i] = 0.0f;
+            z[r][i] = s[r][i] = 0.0f;
             c[r][i] = 1.0f;
             if (64 * i < n && e < n) {
-                v[r][i] = src[e] + (b ? b[e] : 0.0f);
+                if (!CONV) v[r][i] = src[e] + (b ? b[e] : 0.0f);
                 if (e < 2 * half) {
                     const int f = e < half ? e + half : e - half, j = e < half ? e : f;
-                    z[r][i] = (src[f] + (b ? b[f] : 0.0f)) * (w ? w[f] : 1.0f);
+                    z[r][i] = CONV ? ex[r * TK_MAX_HEAD_DIM + f] : (src[f] + (b ? b[f] : 0.0f)) * (w ? w[f] : 1.0f);
                     c[r][i] = a.rope_cos[(size_t)pos[r] * half + j];
                     s[r][i] = a.rope_sin[(size_t)pos[r] * half + j] * (e < half ? -1.0f : 1.0f);
                 }
@@ -195,6 +314,7 @@ __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& 
             else if (is_v) ((T*)a.kv.v)[((page[r] * a.kv_heads + head) * a.kv.vdim_pad + e) * TK_PAGE + pos[r] % TK_PAGE] = TkImg<T>::from(y);
             else ((T*)a.kv.k)[((page[r] * a.kv_heads + head) * TK_PAGE + pos[r] % TK_PAGE) * a.kv.dim_pad + e] = TkImg<T>::from(y);
         }
+        if (CONV) conv.leave(t, proj, ld, row0 + r, off, n, lane);
     }
 }
 
@@ -221,42 +341,11 @@ __device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab
     const int which = u < d.kv_heads ? 0 : u < 2 * d.kv_heads ? 1 : 2;
     const int head = which == 2 ? u - 2 * d.kv_heads : which == 1 ? u - d.kv_heads : u;
     const int n = which == 2 ? d.vdim : d.dim, c0 = which == 2 ? 2 * qk + head * d.vdim : which * qk + head * d.dim;
-    const int hist = d.taps - 1;
     float* dst = which == 0 ? d.q + head * d.dim : which == 1 ? d.k + head * d.dim : d.v + (size_t)head * d.vdim;
     const size_t pitch = which == 2 ? (size_t)d.heads * d.vdim : qk;
+    const Conv conv{d.conv, d.conv_state, channels, d.taps, d.col};
     float y[RW][4];
-    const int seg0 = t.seg[rowb], first = rowb - t.seg_row0[seg0];
-    if (RW > 1 && first >= hist && first + RW <= t.seg_n[seg0]) { /* every input is a row of this pass */
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-#pragma unroll
-            for (int r = 0; r < RW; ++r) y[r][i] = 0.0f;
-            const int c = c0 + lane + 64 * i;
-            if (64 * i < n && lane + 64 * i < n)
-                for (int j = 0; j < d.taps; ++j) {
-                    const float tap = d.conv[(size_t)c * d.taps + j];
-#pragma unroll
-                    for (int r = 0; r < RW; ++r) y[r][i] = fmaf(tap, proj[(size_t)(rowb + r - hist + j) * ld + d.col + c], y[r][i]);
-                }
-        }
-    } else {
-#pragma unroll
-        for (int r = 0; r < RW; ++r) {
-            const int row = rowb + r < nrows ? rowb + r : nrows - 1;
-            const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0, in = t.seg_in[seg];
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                y[r][i] = 0.0f;
-                const int c = c0 + lane + 64 * i;
-                if (64 * i < n && lane + 64 * i < n)
-                    for (int j = 0; j < d.taps; ++j) {
-                        const int s = at - hist + j; /* time inside the segment; before it: the history, zeros before the sequence */
-                        const float x = s >= 0 ? proj[(size_t)(row0 + s) * ld + d.col + c] : in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
-                        y[r][i] = fmaf(d.conv[(size_t)c * d.taps + j], x, y[r][i]);
-                    }
-            }
-        }
-    }
+    conv.rows<RW>(t, proj, ld, rowb, nrows, c0, n, lane, y);
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
         const int row = rowb + r;
@@ -272,34 +361,35 @@ __device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab
 #pragma unroll
         for (int i = 0; i < 4; ++i)
             if (lane + 64 * i < n) dst[row * pitch + lane + 64 * i] = y[r][i] * f;
-        const int seg = t.seg[row], row0 = t.seg_row0[seg], at = row - row0;
-        if (at + 1 == t.seg_n[seg]) { /* the segment's last row leaves the history behind */
-            const int in = t.seg_in[seg], out = t.seg_out[seg];
-            for (int e = lane; e < n; e += 64)
-                for (int j = 0; j < hist; ++j) {
-                    const int c = c0 + e, s = at + 1 - hist + j;
-                    d.conv_state[((size_t)out * channels + c) * hist + j] = s >= 0 ? proj[(size_t)(row0 + s) * ld + d.col + c] : in < 0 ? 0.0f : d.conv_state[((size_t)in * channels + c) * hist + hist + s];
-                }
-        }
+        conv.leave(t, proj, ld, row, c0, n, lane);
     }
 }
 
-template <typename T, int RW>
+template <typename T, int RW, bool CONV>
 __global__ __launch_bounds__(256) void k_mixer_prep(const float* proj, int ld, TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int nd, int nrows) {
+    __shared__ float ex[CONV ? 4 * RW * TK_MAX_HEAD_DIM : 1];
     const int row = blockIdx.y * RW, lane = threadIdx.x & 63;
     const int u = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
-    if (u < na) attn_unit<T, RW>(a, t, proj, ld, row, nrows, u, lane);
+    if (u < na) attn_unit<T, RW, CONV>(a, t, proj, ld, row, nrows, u, lane, ex + (CONV ? (threadIdx.x >> 6) * RW * TK_MAX_HEAD_DIM : 0));
     else if (u < na + nd) delta_unit<RW>(d, t, proj, ld, row, nrows, u - na, lane);
 }
 
 /* ------------------------------------------------------------------ attention -------------- */
 
-/* the pages a range of query positions [p0, p1] reads: the kept first ones, then the window's */
+/* the lowest position (kept first ones aside) that a query at position p reads; never falls as p grows */
+__device__ __forceinline__ int first_visible(const TkAttnArgs& a, int p) {
+    int lo = 0;
+    if (a.window > 0) lo = p - a.window + 1;
+    if (a.chunk > 0) { const int c = p - (int)((unsigned)p % (unsigned)a.chunk); lo = c > lo ? c : lo; }
+    return lo > 0 ? lo : 0;
+}
+
+/* the pages a range of query positions [p0, p1] reads: the kept first ones, then the window's or chunk's */
 struct PageWalk {
     int nkeep, first, count;
-    __device__ __forceinline__ PageWalk(int p0, int p1, int window, int keep) {
-        const int lo = window > 0 && p0 - window + 1 > 0 ? p0 - window + 1 : 0;
-        first = lo / TK_PAGE;
+    __device__ __forceinline__ PageWalk(const TkAttnArgs& a, int p0, int p1) {
+        const int keep = a.keep_first;
+        first = first_visible(a, p0) / TK_PAGE;
         const int k = keep < p1 + 1 ? keep : p1 + 1;
         const int kp = (k + TK_PAGE - 1) / TK_PAGE;
         nkeep = kp < first ? kp : first;
@@ -308,14 +398,31 @@ struct PageWalk {
     __device__ __forceinline__ int page(int i) const { return i < nkeep ? i : first + i - nkeep; }
 };
 
-/* scores of one page (raw products, keys k0 + 16 j + 4 g + r) -> log2 units, -inf where the query at position pq may not look.  lo .. hi: the lowest
- * and highest query position of the wave; a page that all of them see whole is not masked. */
-__device__ __forceinline__ void mask_scores(tk_v4f (&s)[4], const TkAttnArgs& a, int k0, int g, int pq, int lo, int hi) {
-    const float c = a.scale * LOG2E;
+/* cap * tanh(score / cap), in log2 units; EXACT: the library's function rather than a quotient of exponentials (absolute error 1e-7 of the cap) */
+template <bool EXACT>
+__device__ __forceinline__ float soft_cap(float x, float inv, float cap2) {
+    if (EXACT) return cap2 * tanhf(x * inv);
+    const float e = __builtin_amdgcn_exp2f(x * (inv * 2.0f * LOG2E));
+    return cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(1.0f + e);
+}
+
+/* scores of one page (raw products, keys k0 + 16 j + 4 g + r) -> log2 units, -inf where the query at position pq, which reads `first` on, may not
+ * look.  lo, whole: the lowest query position of the wave, and the first position that all of the wave's queries read; a page that all of them see
+ * whole is not masked. */
+template <typename T>
+__device__ __forceinline__ void mask_scores(tk_v4f (&s)[4], const TkAttnArgs& a, int k0, int g, int pq, int first, int lo, int whole) {
+    if (a.softcap > 0.0f) {
+        const float inv = a.scale / a.softcap, cap2 = a.softcap * LOG2E;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) s[j] *= c;
-    if (k0 + TK_PAGE - 1 <= lo && (a.window <= 0 || hi - k0 < a.window || k0 + TK_PAGE <= a.keep_first)) return;
-    const int first = a.window > 0 ? pq - a.window + 1 : 0;
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s[j][r] = soft_cap<sizeof(T) == 4>(s[j][r], inv, cap2);
+    } else {
+        const float c = a.scale * LOG2E;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[j] *= c;
+    }
+    if (k0 + TK_PAGE - 1 <= lo && (whole <= k0 || k0 + TK_PAGE <= a.keep_first)) return;
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -438,7 +545,7 @@ __global__ __launch_bounds__(256, B * sizeof(T) >= 512 ? 1 : 2) void k_attn_tile
     const int p0 = t.pos[row0], seq = t.seq[row0];
     const int q = wave * 16 + (lane & 15), live = q < n ? q : 0;
     const int pq = q < n ? p0 + q : -1; /* rows past the tile see nothing and store nothing */
-    const PageWalk walk(p0, p0 + n - 1, a.window, a.keep_first);
+    const PageWalk walk(a, p0, p0 + n - 1);
     const int32_t* pages = t.page_of + (size_t)seq * t.max_pages;
     int ids = pages[walk.page(lane < walk.count ? lane : 0)], ids0 = 0; /* lane l: page id of step ids0 + l */
     const int kc = TK_PAGE * a.kv.dim_pad * SZ / 16, vc = a.kv.vdim_pad * TK_PAGE * SZ / 16; /* 16-byte pieces of a page */
@@ -473,6 +580,9 @@ __global__ __launch_bounds__(256, B * sizeof(T) >= 512 ? 1 : 2) void k_attn_tile
     Flash<T, VT> f;
     f.init();
     const int wave_lo = p0 + wave * 16, wave_hi = p0 + (wave * 16 + 15 < n ? wave * 16 + 15 : n - 1);
+    /* what this lane's query reads from on, what any and what all of the wave's queries do (a wave with rows past the tile always masks) */
+    const int first = pq >= 0 ? first_visible(a, pq) : 0, any = first_visible(a, wave_lo);
+    const int whole = wave * 16 + 15 < n || (a.window <= 0 && a.chunk <= 0) ? first_visible(a, wave_hi) : 0x7fffffff;
     put(0);
     if (walk.count > 1) fetch(1);
     __syncthreads();
@@ -490,7 +600,7 @@ __global__ __launch_bounds__(256, B * sizeof(T) >= 512 ? 1 : 2) void k_attn_tile
         const uint8_t *lk = lds + (TWO ? (i & 1) * buf : 0), *lv = lk + TK_PAGE * krow;
         const int k0 = walk.page(i) * TK_PAGE;
         /* not a page that none of this wave's rows reads */
-        if (wave * 16 < n && k0 <= wave_hi && (a.window <= 0 || wave_lo - (k0 + TK_PAGE - 1) < a.window || k0 < a.keep_first)) {
+        if (wave * 16 < n && k0 <= wave_hi && (any < k0 + TK_PAGE || k0 < a.keep_first)) {
             tk_v4f s[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
@@ -500,7 +610,7 @@ __global__ __launch_bounds__(256, B * sizeof(T) >= 512 ? 1 : 2) void k_attn_tile
                 for (int d = 0; d < DT; ++d)
                     if (d < nd) s[j] = TkImg<T>::mma(*(const tk_v4u*)(kp + d * 64), qf[d], s[j]);
             }
-            mask_scores(s, a, k0, g, pq, wave_lo, wave * 16 + 15 < n ? wave_hi : 0x40000000);
+            mask_scores<T>(s, a, k0, g, pq, first, wave_lo, whole);
             f.update(s, nv, [&](int vt, int j) { return *(const VF*)(lv + (16 * vt + (lane & 15)) * vrow + (16 * j + 4 * g) * SZ); });
         }
         if (!TWO) __syncthreads(); /* the only buffer is free again */
@@ -526,7 +636,8 @@ __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t
         if (d < nd) qf[d] = *(const tk_v4u*)((const uint8_t*)a.q + (((size_t)row * a.heads + h) * a.kv.dim_pad) * SZ + d * 64 + g * 16);
     Flash<T, VT> f;
     f.init();
-    const PageWalk walk(pos, pos, a.window, a.keep_first);
+    const PageWalk walk(a, pos, pos);
+    const int low = first_visible(a, pos);
     for (int i = split * WAVES + wave; i < walk.count; i += WAVES * splits) {
         const size_t page = (size_t)t.page_of[(size_t)seq * t.max_pages + walk.page(i)] * a.kv_heads + kvh;
         const uint8_t* kp = (const uint8_t*)a.kv.k + (page * TK_PAGE + (lane & 15)) * a.kv.dim_pad * SZ + g * 16;
@@ -555,7 +666,7 @@ __device__ __forceinline__ void attn_row(const TkAttnArgs& a, const TkPassTab& t
             for (int d = 0; d < DT; ++d)
                 if (d < nd) s[j] = TkImg<T>::mma(AHEAD ? kf[AHEAD ? j : 0][AHEAD ? d : 0] : *(const tk_v4u*)(kp + (size_t)16 * j * a.kv.dim_pad * SZ + d * 64), qf[d], s[j]);
         }
-        mask_scores(s, a, k0, g, pos, pos, pos);
+        mask_scores<T>(s, a, k0, g, pos, low, pos, low);
         f.update(s, nv, [&](int vt, int j) { return AHEAD ? vf[AHEAD ? vt : 0][j] : vload(vt, j); });
     }
     /* the upper half of the waves into the lower half, and again */
@@ -786,6 +897,375 @@ __global__ void k_swap_state(TkPassTab t, int n) {
     if (i < n) { const int o = t.seg_out[i]; t.seg_in[i] = o; t.seg_out[i] = o ^ 1; }
 }
 
+/* ------------------------------------------------------------------ retention -------------- */
+
+/* Prompts.  With pw(n) = decay^n, a chunk of up to C tokens that starts from the state S0 gives
+ *     o_i = pw(i + 1) S0^T q_i + sum over j <= i of pw(i - j) (q_i . k_j) v_j,      S = pw(n) S0 + sum over j of pw(n - 1 - j) k_j v_j^T:
+ * four matrix products.  A workgroup walks one head's block of rows; every wave owns NT 16-column tiles of the state, in the registers that the
+ * products leave it in: an accumulator tile [key dimension][value column] is at once the operand of S^T q, because the key dimensions of q (and k)
+ * lie in LDS in the order in which a lane's accumulators hold them.  Scores go through LDS.  bf16 sessions: q, k and v are bf16 (as in attention);
+ * what is 32-bit by nature (the state, decayed scores, decayed values) enters a product as the sum of two bf16 numbers.
+ * SUMS: only what the block adds to the state, into args.sums: blocks of a segment run side by side, each starts from the segment's state and the
+ * sums of the blocks before it. */
+template <typename T> struct RetChunk { static constexpr int C = sizeof(T) == 2 ? 64 : 32; };
+
+/* where element e of a key row lies: see above (f32 accumulators are in order already) */
+template <typename T> __device__ __forceinline__ int ret_place(int e) { return sizeof(T) == 2 ? (e & ~31) | (e & 12) << 1 | (e & 16) >> 2 | (e & 3) : e; }
+
+/* x as operand words: one bf16 pair per word, hi and the rest lo; f32 as it is (lo unused) */
+template <typename T> struct Split;
+template <> struct Split<TkBf16> {
+    tk_v4u hi, lo;
+    __device__ __forceinline__ Split(tk_v4f a, tk_v4f b) {
+        const float x[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const uint16_t p = tk_bf16_bits(x[2 * i]), q = tk_bf16_bits(x[2 * i + 1]);
+            hi[i] = (uint32_t)p | (uint32_t)q << 16;
+            lo[i] = (uint32_t)tk_bf16_bits(x[2 * i] - tk_bf16_float(p)) | (uint32_t)tk_bf16_bits(x[2 * i + 1] - tk_bf16_float(q)) << 16;
+        }
+    }
+};
+
+template <typename T, int DIM, int VB>
+struct RetLds { /* byte offsets */
+    static constexpr int C = RetChunk<T>::C, SZ = sizeof(T), RP = DIM * SZ + 16, TP = C * SZ + 16;
+    static constexpr int q = 0, k = q + C * RP, kt = k + C * RP, vt = kt + DIM * TP, p = vt + VB * TP, lo = p + C * TP, pw = lo + (SZ == 2 ? C * TP : 0),
+                         red = pw + (TK_RETENTION_BLOCK + 4) * 4, bytes = red + 16 * C * 4;
+};
+
+/* two tokens' elements side by side; four */
+__device__ __forceinline__ void ret_put4(TkBf16* p, const float (&x)[4]) {
+    *(tk_v2u*)p = tk_v2u{(uint32_t)tk_bf16_bits(x[0]) | (uint32_t)tk_bf16_bits(x[1]) << 16, (uint32_t)tk_bf16_bits(x[2]) | (uint32_t)tk_bf16_bits(x[3]) << 16};
+}
+__device__ __forceinline__ void ret_put4(float* p, const float (&x)[4]) { *(tk_v4f*)p = tk_v4f{x[0], x[1], x[2], x[3]}; }
+
+template <typename T, int DIM, int WAVES, int NT, bool SUMS>
+__global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a, const float* proj, int ld, TkPassTab t, const TkRetentionBlock* blocks) {
+    constexpr int C = RetChunk<T>::C, KT = TkImg<T>::KT, EP = TkImg<T>::EP, SZ = sizeof(T), THREADS = 64 * WAVES, VB = 16 * WAVES * NT;
+    constexpr int DT = DIM / KT, DS = DIM / 16, CT = C / 16, CK = C / KT;
+    typedef RetLds<T, DIM, VB> L;
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, r16 = lane & 15, h = blockIdx.x;
+    const TkRetentionBlock b = blocks[blockIdx.y];
+    if (SUMS && b.last) return;
+    const int vp = (a.vdim + 3) & ~3, in = t.seg_in[b.seg], pos0 = t.pos[b.row0];
+    const size_t head_floats = (size_t)a.dim * vp;
+    for (int i = tid; i < L::bytes / 16; i += THREADS) *(tk_v4u*)(lds + i * 16) = tk_v4u{0, 0, 0, 0}; /* paddings stay zero */
+    __syncthreads();
+    float *pw = (float*)(lds + L::pw), *red = (float*)(lds + L::red);
+    if (tid <= TK_RETENTION_BLOCK) pw[tid] = a.decay[(size_t)h * (TK_RETENTION_BLOCK + 1) + tid];
+    int col[NT]; /* this lane's value columns */
+#pragma unroll
+    for (int n = 0; n < NT; ++n) col[n] = (wave * NT + n) * 16 + r16;
+    tk_v4f S[NT][DS]; /* [key dimension 16 d + 4 g + r][column col[n]] */
+    auto state_at = [&](float* base, auto f) {
+#pragma unroll
+        for (int n = 0; n < NT; ++n)
+#pragma unroll
+            for (int d = 0; d < DS; ++d)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int e = 16 * d + 4 * g + r;
+                    if (e < a.dim && col[n] < a.vdim) S[n][d][r] = f(S[n][d][r], base[(size_t)e * vp + col[n]]);
+                }
+    };
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int d = 0; d < DS; ++d) S[n][d] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+    if (!SUMS) {
+        if (in >= 0) state_at(a.state + ((size_t)in * a.heads + h) * head_floats, [](float, float& m) { return m; });
+        if (b.index > 0) {
+            __syncthreads();
+            float fade = 1.0f; /* over a block */
+            for (int n = 0; n < blocks[blockIdx.y - 1].n; n += TK_RETENTION_BLOCK) fade *= pw[TK_RETENTION_BLOCK];
+            for (int i = 0; i < b.index; ++i) state_at(a.sums + ((size_t)(b.slot0 + i) * a.heads + h) * head_floats, [&](float s, float& m) { return fmaf(s, fade, m); });
+        }
+    }
+    const int half = a.rot_dims / 2, units = a.dim - half, qk = a.heads * a.dim;
+    const float kscale = 1.0f / sqrtf((float)a.dim);
+    const float *qp = proj + a.col + h * a.dim, *kp = qp + qk, *vsrc = proj + a.col + 2 * qk + h * a.vdim, *gsrc = vsrc + a.heads * a.vdim;
+    for (int c0 = 0; c0 < b.n; c0 += C) {
+        const int n = b.n - c0 < C ? b.n - c0 : C, base = b.row0 + c0;
+        const bool more = c0 + C < b.n;
+        /* ---- rotated q and k, v into LDS; a unit is a rotating pair or a single element of four tokens ---- */
+        for (int it = tid; it < units * (C / 4); it += THREADS) {
+            const int u = it % units, t0 = it / units * 4;
+            const bool pair = u < half;
+            const int e0 = pair ? u : u + half, e1 = pair ? u + half : e0;
+            float q0[4], q1[4], k0[4], k1[4], cs[4], sn[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int tt = t0 + r < n ? t0 + r : n - 1;
+                const size_t row = (size_t)(base + tt) * ld;
+                if (!SUMS) { q0[r] = qp[row + e0]; q1[r] = qp[row + e1]; }
+                k0[r] = kp[row + e0];
+                k1[r] = kp[row + e1];
+                const size_t at = (size_t)(pos0 + c0 + tt) * half + (pair ? u : 0);
+                cs[r] = pair ? a.rope_cos[at] : 1.0f;
+                sn[r] = pair ? a.rope_sin[at] : 0.0f;
+            }
+            float ka[4], kb[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const bool ok = t0 + r < n;
+                ka[r] = ok ? (k0[r] * cs[r] - k1[r] * sn[r]) * kscale : 0.0f;
+                kb[r] = ok ? (k1[r] * cs[r] + k0[r] * sn[r]) * kscale : 0.0f;
+                if (!SUMS) {
+                    T *lq = (T*)(lds + L::q + (t0 + r) * L::RP), *lk = (T*)(lds + L::k + (t0 + r) * L::RP);
+                    lq[ret_place<T>(e0)] = TkImg<T>::from(q0[r] * cs[r] - q1[r] * sn[r]);
+                    lk[ret_place<T>(e0)] = TkImg<T>::from(ka[r]);
+                    if (pair) {
+                        lq[ret_place<T>(e1)] = TkImg<T>::from(q1[r] * cs[r] + q0[r] * sn[r]);
+                        lk[ret_place<T>(e1)] = TkImg<T>::from(kb[r]);
+                    }
+                }
+            }
+            ret_put4((T*)(lds + L::kt + e0 * L::TP) + t0, ka);
+            if (pair) ret_put4((T*)(lds + L::kt + e1 * L::TP) + t0, kb);
+        }
+        for (int it = tid; it < a.vdim * (C / 4); it += THREADS) {
+            const int e = it % a.vdim, t0 = it / a.vdim * 4;
+            float v[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = vsrc[(size_t)(base + (t0 + r < n ? t0 + r : n - 1)) * ld + e];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = t0 + r < n ? v[r] : 0.0f;
+            ret_put4((T*)(lds + L::vt + e * L::TP) + t0, v);
+        }
+        __syncthreads();
+        tk_v4f o[SUMS ? 1 : NT][SUMS ? 1 : CT]; /* [column 4 g + r of tile n][query 16 m + lane % 16] */
+        if constexpr (!SUMS) {
+            /* ---- decayed scores, tiles of 16 queries x 16 keys dealt to the waves ---- */
+            for (int i = wave; i < CT * (CT + 1) / 2; i += WAVES) {
+                const int m = i < 1 ? 0 : i < 3 ? 1 : i < 6 ? 2 : 3, j = i - m * (m + 1) / 2;
+                if (16 * m >= n) continue;
+                tk_v4f s = {0.0f, 0.0f, 0.0f, 0.0f};
+                const uint8_t *lk = lds + L::k + (16 * j + r16) * L::RP + g * 16, *lq = lds + L::q + (16 * m + r16) * L::RP + g * 16;
+#pragma unroll
+                for (int d = 0; d < DT; ++d) s = TkImg<T>::mma(*(const tk_v4u*)(lk + d * 64), *(const tk_v4u*)(lq + d * 64), s);
+                const int age = 16 * (m - j) + r16 - 4 * g;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) s[r] = age - r >= 0 ? s[r] * pw[age - r >= 0 ? age - r : 0] : 0.0f;
+                const int at = (16 * m + r16) * L::TP + (16 * j + 4 * g) * SZ;
+                if constexpr (SZ == 2) {
+                    const Split<TkBf16> w(s, s);
+                    *(tk_v2u*)(lds + L::p + at) = tk_v2u{w.hi[0], w.hi[1]};
+                    *(tk_v2u*)(lds + L::lo + at) = tk_v2u{w.lo[0], w.lo[1]};
+                } else {
+                    *(tk_v4f*)(lds + L::p + at) = s;
+                }
+            }
+            /* ---- what the state gives ---- */
+#pragma unroll
+            for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+                for (int m = 0; m < CT; ++m) o[nt][m] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+            if (in >= 0 || b.index > 0 || c0 > 0) {
+#pragma unroll
+                for (int d = 0; d < DT; ++d) {
+                    tk_v4u qf[CT];
+#pragma unroll
+                    for (int m = 0; m < CT; ++m) qf[m] = *(const tk_v4u*)(lds + L::q + (16 * m + r16) * L::RP + d * 64 + g * 16);
+#pragma unroll
+                    for (int nt = 0; nt < NT; ++nt) {
+                        if constexpr (SZ == 2) {
+                            const Split<TkBf16> w(S[nt][2 * d], S[nt][2 * d + 1]);
+#pragma unroll
+                            for (int m = 0; m < CT; ++m) {
+                                o[nt][m] = TkImg<T>::mma(w.hi, qf[m], o[nt][m]);
+                                o[nt][m] = TkImg<T>::mma(w.lo, qf[m], o[nt][m]);
+                            }
+                        } else {
+#pragma unroll
+                            for (int m = 0; m < CT; ++m) o[nt][m] = TkImg<T>::mma(__builtin_bit_cast(tk_v4u, S[nt][d]), qf[m], o[nt][m]);
+                        }
+                    }
+                }
+#pragma unroll
+                for (int m = 0; m < CT; ++m) {
+                    const float f = pw[16 * m + r16 + 1];
+#pragma unroll
+                    for (int nt = 0; nt < NT; ++nt) o[nt][m] *= f;
+                }
+            }
+            __syncthreads();
+        }
+        /* ---- what the chunk's own tokens give, and the state after them ---- */
+        tk_v4u vf[NT][CK];
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+            for (int k = 0; k < CK; ++k) vf[nt][k] = *(const tk_v4u*)(lds + L::vt + col[nt] * L::TP + k * 64 + g * 16);
+        if constexpr (!SUMS) {
+#pragma unroll
+            for (int k = 0; k < CK; ++k)
+#pragma unroll
+                for (int m = 0; m < CT; ++m)
+                    if (k * KT < 16 * m + 16) {
+                        const int at = (16 * m + r16) * L::TP + k * 64 + g * 16;
+                        const tk_v4u hi = *(const tk_v4u*)(lds + L::p + at), lo = SZ == 2 ? *(const tk_v4u*)(lds + L::lo + at) : hi;
+#pragma unroll
+                        for (int nt = 0; nt < NT; ++nt) {
+                            o[nt][m] = TkImg<T>::mma(vf[nt][k], hi, o[nt][m]);
+                            if (SZ == 2) o[nt][m] = TkImg<T>::mma(vf[nt][k], lo, o[nt][m]);
+                        }
+                    }
+        }
+        if (SUMS || more || b.last) {
+            const float fade = pw[n];
+#pragma unroll
+            for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+                for (int d = 0; d < DS; ++d) S[nt][d] *= fade;
+#pragma unroll
+            for (int k = 0; k < CK; ++k) {
+                float w[EP];
+#pragma unroll
+                for (int e = 0; e < EP; ++e) { const int left = n - 1 - (k * KT + g * EP + e); w[e] = pw[left >= 0 ? left : 0]; } /* past n: v is zero */
+                if constexpr (SZ == 2) {
+                    tk_v4u hi[NT], lo[NT];
+#pragma unroll
+                    for (int nt = 0; nt < NT; ++nt) {
+                        tk_v4f x, y;
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) {
+                            x[e] = tk_bf16_float((uint16_t)(vf[nt][k][e >> 1] >> 16 * (e & 1))) * w[e];
+                            y[e] = tk_bf16_float((uint16_t)(vf[nt][k][2 + (e >> 1)] >> 16 * (e & 1))) * w[EP - 4 + e];
+                        }
+                        const Split<TkBf16> z(x, y);
+                        hi[nt] = z.hi; lo[nt] = z.lo;
+                    }
+#pragma unroll
+                    for (int d = 0; d < DS; ++d) {
+                        const tk_v4u kf = *(const tk_v4u*)(lds + L::kt + (16 * d + r16) * L::TP + k * 64 + g * 16);
+#pragma unroll
+                        for (int nt = 0; nt < NT; ++nt) { S[nt][d] = TkImg<T>::mma(kf, hi[nt], S[nt][d]); S[nt][d] = TkImg<T>::mma(kf, lo[nt], S[nt][d]); }
+                    }
+                } else {
+                    tk_v4f x[NT];
+#pragma unroll
+                    for (int nt = 0; nt < NT; ++nt) {
+                        x[nt] = __builtin_bit_cast(tk_v4f, vf[nt][k]);
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) x[nt][e] *= w[e];
+                    }
+#pragma unroll
+                    for (int d = 0; d < DS; ++d) {
+                        const tk_v4u kf = *(const tk_v4u*)(lds + L::kt + (16 * d + r16) * L::TP + k * 64 + g * 16);
+#pragma unroll
+                        for (int nt = 0; nt < NT; ++nt) S[nt][d] = TkImg<T>::mma(kf, __builtin_bit_cast(tk_v4u, x[nt]), S[nt][d]);
+                    }
+                }
+            }
+        }
+        if constexpr (!SUMS) {
+            /* ---- each head's output over its root mean square, times the gate ---- */
+#pragma unroll
+            for (int m = 0; m < CT; ++m) {
+                float ss = 0.0f;
+#pragma unroll
+                for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) ss += o[nt][m][r] * o[nt][m][r];
+                ss = tk_quad_sum(ss);
+                if (g == 0) red[wave * C + 16 * m + r16] = ss;
+            }
+            __syncthreads();
+#pragma unroll
+            for (int m = 0; m < CT; ++m) {
+                const int i = 16 * m + r16;
+                float ss = 0.0f;
+#pragma unroll
+                for (int w = 0; w < WAVES; ++w) ss += red[w * C + i];
+                if (i >= n) continue;
+                const float f = a.out_scale / sqrtf(ss / (float)a.vdim + a.eps);
+                const int64_t row = base + i;
+#pragma unroll
+                for (int nt = 0; nt < NT; ++nt) {
+                    const int e = (wave * NT + nt) * 16 + 4 * g, at = a.out_k0 + h * a.vdim + e;
+                    if (e >= a.vdim) continue;
+                    const float* gp = gsrc + (size_t)row * ld + e;
+                    if (((uintptr_t)gp & 15) == 0 && (at & 3) == 0 && e + 3 < a.vdim) {
+                        const tk_v4f z = *(const tk_v4f*)gp;
+                        tk_v4f y;
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) y[r] = o[nt][m][r] * f * tk_silu32(z[r]);
+                        tk_img_put4((T*)a.out_img, row, at, a.out_ktiles, y);
+                    } else {
+#pragma unroll
+                        for (int r = 0; r < 4; ++r)
+                            if (e + r < a.vdim) tk_img_put((T*)a.out_img, row, at + r, a.out_ktiles, o[nt][m][r] * f * tk_silu32(gp[r]));
+                    }
+                }
+            }
+        } else {
+            __syncthreads(); /* the next chunk takes the operands' place (outputs: every wave is past them at the barrier above) */
+        }
+    }
+    if (SUMS) state_at(a.sums + ((size_t)(b.slot0 + b.index) * a.heads + h) * head_floats, [](float s, float& m) { return m = s; });
+    else if (b.last) state_at(a.state + ((size_t)t.seg_out[b.seg] * a.heads + h) * head_floats, [](float s, float& m) { return m = s; });
+}
+
+/* One token of one head: the state is read once and written once, a thread holds RPT rows x 4 columns of it.  Rotation, output norm and gate with it. */
+template <typename T, int THREADS, int RPT>
+__global__ __launch_bounds__(THREADS) void k_retention_step(TkRetentionArgs a, const float* proj, int ld, TkPassTab t, int ct_log2) {
+    extern __shared__ __attribute__((aligned(16))) float ret_lds[];
+    const int h = blockIdx.x, seg = blockIdx.y, tid = threadIdx.x, vp = (a.vdim + 3) & ~3;
+    if (t.seg_n[seg] != 1) return;
+    const int row = t.seg_row0[seg], in = t.seg_in[seg], out = t.seg_out[seg], pos = t.pos[row];
+    const int ct = tid & ((1 << ct_log2) - 1), rg = tid >> ct_log2, RG = THREADS >> ct_log2;
+    const bool live = 4 * ct < vp;
+    float *red = ret_lds, *lv = red + 16, *po = lv + vp, *lq = po + RG * vp, *lk = lq + a.dim;
+    tk_v4f S[RPT];
+    const float* sin = a.state + ((size_t)(in < 0 ? 0 : in) * a.heads + h) * a.dim * vp + 4 * ct;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const int e = rg + RG * i;
+        S[i] = in >= 0 && live && e < a.dim ? *(const tk_v4f*)(sin + (size_t)e * vp) : tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+    const int half = a.rot_dims / 2, qk = a.heads * a.dim;
+    const float *qp = proj + (size_t)row * ld + a.col + h * a.dim, *kp = qp + qk, *vsrc = proj + (size_t)row * ld + a.col + 2 * qk + h * a.vdim;
+    const float gate = tid < a.vdim ? vsrc[a.heads * a.vdim + tid] : 0.0f; /* vdim <= 256 <= THREADS: one column per thread */
+    const float kscale = 1.0f / sqrtf((float)a.dim), decay = a.decay[(size_t)h * (TK_RETENTION_BLOCK + 1) + 1];
+    for (int e = tid; e < a.dim; e += THREADS) {
+        float q = qp[e], k = kp[e];
+        if (e < 2 * half) {
+            const int f = e < half ? e + half : e - half, j = e < half ? e : f;
+            const float c = a.rope_cos[(size_t)pos * half + j], s = a.rope_sin[(size_t)pos * half + j] * (e < half ? -1.0f : 1.0f);
+            q = q * c + qp[f] * s;
+            k = k * c + kp[f] * s;
+        }
+        lq[e] = q;
+        lk[e] = k * kscale;
+    }
+    if (tid < vp) lv[tid] = tid < a.vdim ? vsrc[tid] : 0.0f;
+    __syncthreads();
+    tk_v4f ao = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (live) {
+        const tk_v4f v = *(const tk_v4f*)(lv + 4 * ct);
+        float* so = a.state + ((size_t)out * a.heads + h) * a.dim * vp + 4 * ct;
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) {
+            const int e = rg + RG * i;
+            if (e < a.dim) {
+                S[i] = S[i] * decay + v * lk[e];
+                *(tk_v4f*)(so + (size_t)e * vp) = S[i];
+                ao += S[i] * lq[e];
+            }
+        }
+        *(tk_v4f*)(po + rg * vp + 4 * ct) = ao;
+    }
+    __syncthreads();
+    float o = 0.0f;
+    if (tid < a.vdim)
+        for (int i = 0; i < RG; ++i) o += po[i * vp + tid];
+    const float ss = block_sum(o * o, red);
+    if (tid < a.vdim)
+        tk_img_put((T*)a.out_img, row, a.out_k0 + h * a.vdim + tid, a.out_ktiles, o * (a.out_scale / sqrtf(ss / (float)a.vdim + a.eps)) * tk_silu32(gate));
+}
+
 /* ------------------------------------------------------------------ mixture of experts ----- */
 
 /* experts' tile counts (threads 0 .. 255, one expert each) -> first tiles and row blocks.  Every thread of the workgroup calls it. */
@@ -907,11 +1387,14 @@ __global__ __launch_bounds__(256) void k_moe_gather(const tk_v4u* img, tk_v4u* o
 
 #define TK_TYPED(type, ...) do { if ((type) == TK_IMG_F32) { typedef float T; __VA_ARGS__; } else { typedef TkBf16 T; __VA_ARGS__; } } while (0)
 
-#define TK_VEC(vec, ...) do { if (vec) { constexpr bool VEC = true; __VA_ARGS__; } else { constexpr bool VEC = false; __VA_ARGS__; } } while (0)
+/* threads and register groups that hold a row */
 static int norm_threads(int width) { return width > 2048 ? 512 : 256; }
+#define TK_ROW(vec, width, ...) do { \
+        if (vec) { constexpr bool VEC = true; if ((width) <= 8 * norm_threads(width)) { constexpr int NV = 1; __VA_ARGS__; } else { constexpr int NV = 4; __VA_ARGS__; } } \
+        else { constexpr bool VEC = false; if ((width) <= 8 * norm_threads(width)) { constexpr int NV = 1; __VA_ARGS__; } else { constexpr int NV = 4; __VA_ARGS__; } } } while (0)
 
-void tk_launch_layer_embed(int type, const uint16_t* table, int width, const int32_t* tok, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, TK_VEC(width % 8 == 0, hipLaunchKernelGGL((k_layer_embed<T, VEC>), dim3(nrows), dim3(256), 0, s, table, width, tok, x, (T*)img, ktiles)));
+void tk_launch_layer_embed(int type, const uint16_t* table, int width, float scale, const int32_t* tok, int nrows, float* x, const TkNorm& next, float eps, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, TK_ROW(width % 8 == 0, width, hipLaunchKernelGGL((k_layer_embed<T, VEC, NV>), dim3(nrows), dim3(norm_threads(width)), 0, s, table, width, scale, tok, x, next, eps, (T*)img, ktiles)));
 }
 
 void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs* attn, const TkDeltaArgs* delta, const TkPassTab& t, int nrows, hipStream_t s) {
@@ -919,8 +1402,10 @@ void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs*
     const TkDeltaArgs d = delta ? *delta : TkDeltaArgs{};
     const int na = attn ? a.heads + 2 * a.kv_heads : 0, nd = delta ? 2 * d.kv_heads + 2 * d.heads : 0;
     const int gx = (na + nd + 3) / 4;
-    if (nrows >= 512) TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, 4>), dim3(gx, (nrows + 3) / 4), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows));
-    else TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, 1>), dim3(gx, nrows), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows));
+#define TK_PREP(RW, CV) TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, RW, CV>), dim3(gx, (nrows + RW - 1) / RW), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows))
+    if (nrows >= 512) { if (a.taps > 0) TK_PREP(4, true); else TK_PREP(4, false); }
+    else { if (a.taps > 0) TK_PREP(1, true); else TK_PREP(1, false); }
+#undef TK_PREP
 }
 
 static int attn_bucket(const TkAttnArgs& a) {
@@ -1019,12 +1504,44 @@ void tk_launch_delta_step(int type, const TkDeltaArgs& d, const TkPassTab& t, in
     });
 }
 
-void tk_launch_post_norm(int type, const TkSubOut& o, const float* w, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, TK_VEC(width % 8 == 0 && o.ld % 4 == 0, hipLaunchKernelGGL((k_post_norm<T, VEC>), dim3(nrows), dim3(norm_threads(width)), (size_t)width * sizeof(float), s, o, w, eps, width, x, (T*)img, ktiles)));
+void tk_launch_post_norm(int type, const TkSubOut& o, const TkNorm& norm, const TkNorm& next, float eps, int width, int nrows, float* x, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, TK_ROW(width % 8 == 0 && o.ld % 4 == 0, width, hipLaunchKernelGGL((k_post_norm<T, VEC, NV>), dim3(nrows), dim3(norm_threads(width)), 0, s, o, norm, next, eps, width, x, (T*)img, ktiles)));
 }
 
-void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const float* w, float eps, int width, void* img, int ktiles, hipStream_t s) {
-    TK_TYPED(type, TK_VEC(width % 8 == 0, hipLaunchKernelGGL((k_rows_norm<T, VEC>), dim3(n), dim3(norm_threads(width)), 0, s, x, rows, w, eps, width, (T*)img, ktiles)));
+void tk_launch_rows_norm(int type, const float* x, const int32_t* rows, int n, const TkNorm& norm, float eps, int width, void* img, int ktiles, hipStream_t s) {
+    TK_TYPED(type, TK_ROW(width % 8 == 0, width, hipLaunchKernelGGL((k_rows_norm<T, VEC, NV>), dim3(n), dim3(norm_threads(width)), 0, s, x, rows, norm, eps, width, (T*)img, ktiles)));
+}
+
+/* the forms of the scan: key dimensions 64, 128, 256 x value columns 64, 128, 256 */
+#define TK_RET_FORMS(X, T) X(T, 64, 4, 1) X(T, 64, 8, 1) X(T, 64, 8, 2) X(T, 128, 4, 1) X(T, 128, 8, 1) X(T, 128, 8, 2) X(T, 256, 4, 1) X(T, 256, 8, 1) X(T, 256, 8, 2)
+
+void tk_launch_retention_scan(int type, const TkRetentionArgs& a, const float* proj, int ld, const TkPassTab& t, const TkRetentionBlock* blocks, int n_blocks, int n_sums, hipStream_t s) {
+    const int dim = a.dim <= 64 ? 64 : a.dim <= 128 ? 128 : 256, vb = a.vdim <= 64 ? 64 : a.vdim <= 128 ? 128 : 256;
+    const dim3 grid(a.heads, n_blocks);
+#define TK_RET(T, D, W, N) \
+    if (dim == D && vb == 16 * W * N) { \
+        constexpr size_t lds = RetLds<T, D, 16 * W * N>::bytes; \
+        if (n_sums) hipLaunchKernelGGL((k_retention_scan<T, D, W, N, true>), grid, dim3(64 * W), lds, s, a, proj, ld, t, blocks); \
+        hipLaunchKernelGGL((k_retention_scan<T, D, W, N, false>), grid, dim3(64 * W), lds, s, a, proj, ld, t, blocks); \
+    }
+    if (type == TK_IMG_F32) { TK_RET_FORMS(TK_RET, float) } else { TK_RET_FORMS(TK_RET, TkBf16) }
+#undef TK_RET
+}
+
+void tk_launch_retention_step(int type, const TkRetentionArgs& a, const float* proj, int ld, const TkPassTab& t, int n_segments, hipStream_t s) {
+    int ctl = 0;
+    while ((4 << ctl) < a.vdim) ++ctl;
+    const dim3 grid(a.heads, n_segments);
+    const size_t vp = (a.vdim + 3) & ~3;
+    auto lds = [&](int threads) { return (16 + vp + (size_t)(threads >> ctl) * vp + 2 * (size_t)a.dim) * sizeof(float); };
+    auto rpt = [&](int threads) { const int rg = threads >> ctl; return (a.dim + rg - 1) / rg; };
+    TK_TYPED(type, {
+        if (rpt(256) <= 4) hipLaunchKernelGGL((k_retention_step<T, 256, 4>), grid, dim3(256), lds(256), s, a, proj, ld, t, ctl);
+        else if (rpt(256) <= 8) hipLaunchKernelGGL((k_retention_step<T, 256, 8>), grid, dim3(256), lds(256), s, a, proj, ld, t, ctl);
+        else if (rpt(256) <= 16) hipLaunchKernelGGL((k_retention_step<T, 256, 16>), grid, dim3(256), lds(256), s, a, proj, ld, t, ctl);
+        else if (rpt(256) <= 32) hipLaunchKernelGGL((k_retention_step<T, 256, 32>), grid, dim3(256), lds(256), s, a, proj, ld, t, ctl);
+        else hipLaunchKernelGGL((k_retention_step<T, 1024, 16>), grid, dim3(1024), lds(1024), s, a, proj, ld, t, ctl);
+    });
 }
 
 void tk_launch_moe_select(const float* logits, int ld, int experts, int top, int groups, int keep, int nrows, int block_tiles, const TkMoeTab& t, hipStream_t s) {
@@ -1049,6 +1566,9 @@ const char* tk_mixer_prepare_device() {
     opt((const void*)k_attn_tiles<float, 64, false>); opt((const void*)k_attn_tiles<float, 128, false>); opt((const void*)k_attn_tiles<float, 256, false>);
     opt((const void*)k_attn_tiles<TkBf16, 64, false>); opt((const void*)k_attn_tiles<TkBf16, 128, false>); opt((const void*)k_attn_tiles<TkBf16, 256, false>);
     opt((const void*)k_attn_tiles<TkBf16, 64, true>); opt((const void*)k_attn_tiles<TkBf16, 128, true>); opt((const void*)k_attn_tiles<TkBf16, 256, true>);
+#define TK_RET_OPT(T, D, W, N) opt((const void*)k_retention_scan<T, D, W, N, true>); opt((const void*)k_retention_scan<T, D, W, N, false>);
+    TK_RET_FORMS(TK_RET_OPT, float) TK_RET_FORMS(TK_RET_OPT, TkBf16)
+#undef TK_RET_OPT
     if (e != hipSuccess) return hipGetErrorString(e);
     done[dev].store(true, std::memory_order_release);
     return nullptr;

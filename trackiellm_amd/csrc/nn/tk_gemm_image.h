@@ -47,8 +47,10 @@ struct TkImgGemm {
     size_t slab_floats;
     void* copy_img;
     int copy0, copy1, copy_ktiles;
-    /* swiglu: the weight image alternates 16 gate rows and 16 up rows; silu(gate) * up goes, as T, to the image act_img [rows][N / 2] */
-    int swiglu;
+    /* swiglu: the weight image alternates 16 gate rows and 16 up rows; silu(gate) * up goes, as T, to the image act_img [rows][N / 2].
+     * act_clamped: g = min(gate, limit), u = clamp(up, -limit, limit), then g * sigmoid(act_slope * g) * (u + act_shift) instead */
+    int swiglu, act_clamped;
+    float act_limit, act_slope, act_shift;
     void* act_img;
     int act_ktiles, act_valid; /* columns >= act_valid are not stored */
     /* grouped: row blocks from a device table of at most max_blocks entries, *n_blocks of them live; block_tiles = the largest ntiles (<= 8) */

@@ -26,12 +26,21 @@ __device__ __forceinline__ void store_f32(const TkImgGemm& a, int64_t row, int n
             if (n + r >= a.copy0 && n + r < a.copy1) tk_img_put((T*)a.copy_img, row, n + r - a.copy0, a.copy_ktiles, v[r]);
 }
 
-/* gate and up tiles of the same 16 columns -> silu(gate) * up in the next product's operand image */
+/* gate and up tiles of the same 16 columns -> the gated activation in the next product's operand image */
 template <typename T>
 __device__ __forceinline__ void store_act(const TkImgGemm& a, int64_t row, int n, tk_v4f gate, tk_v4f up) {
     tk_v4f h;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) h[r] = n + r < a.act_valid ? tk_silu32(gate[r]) * up[r] : 0.0f;
+    for (int r = 0; r < 4; ++r) {
+        float y;
+        if (a.act_clamped) {
+            const float g = fminf(gate[r], a.act_limit), u = fminf(fmaxf(up[r], -a.act_limit), a.act_limit);
+            y = g * tk_sigmoid32(a.act_slope * g) * (u + a.act_shift);
+        } else {
+            y = tk_silu32(gate[r]) * up[r];
+        }
+        h[r] = n + r < a.act_valid ? y : 0.0f;
+    }
     if (n < a.act_valid) tk_img_put4((T*)a.act_img, row, n, a.act_ktiles, h);
 }
 
