@@ -658,8 +658,12 @@ def layered_config(width, n_layer, attn, delta, mlp, vocab=32000):
     return {"architecture": "Vuvulorn", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": [layer] * n_layer}
 
 
+def kaparax_config(width, layers, vocab=32000):
+    return {"architecture": "Kaparax", "embedding": {"scale": float(width) ** 0.5}, "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": layers}
+
+
 def layered_sizes():
-    """name -> (configuration, Mistral-class geometry of the same width, depth and active feed-forward)"""
+    """name -> (configuration, Mistral-class geometry of the same width, depth and active feed-forward, name of the layer-list design beside it or None)"""
     from trackiellm_amd import LlmHParams
 
     def attn(heads, kv, window):
@@ -668,11 +672,22 @@ def layered_sizes():
     def delta(heads):
         return {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}
     moe = {"kind": "moe", "expert": {"ff": 1024}, "router": {"experts": 64, "top": 8, "groups": {"count": 8, "keep": 4}}}
-    return {"dense-4096": (layered_config(4096, 4, attn(16, 4, 1024), delta(16), {"kind": "dense", "ff": 14336}),
-                           LlmHParams(4, 4096, 32, 8, 128, 14336, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1)),
+
+    def kaparax(width, n_layer, heads, kv, chunk, ff):
+        """retention and attention layers in turn, each with a feed-forward: heads of 128 that together are as wide as the stream"""
+        n = width // 128
+        mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+        ret = {"type": "retention", "mlp": mlp, "mixer": {"heads": n, "dim": 128, "vdim": 128, "rot": {"dims": 128, "base": 10000.0}, "decay": [1.0 - 2.0 ** (-5 - 4.0 * i / n) for i in range(n)]}}
+        att = {"type": "attention", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "rot": {"dims": 64, "base": 10000.0}, "scale": 128 ** -0.5,
+                                                        "mask": {"size": chunk}, "conv": 4, "softcap": 30.0}}
+        return kaparax_config(width, [ret, att] * (n_layer // 2))
+    return {"kaparax-4096": (kaparax(4096, 4, 32, 8, 1024, 14336), LlmHParams(4, 4096, 32, 8, 128, 14336, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1), "dense-4096"),
+            "kaparax-2048": (kaparax(2048, 8, 16, 4, 512, 8192), LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1), "dense-2048"),
+            "dense-4096": (layered_config(4096, 4, attn(16, 4, 1024), delta(16), {"kind": "dense", "ff": 14336}),
+                           LlmHParams(4, 4096, 32, 8, 128, 14336, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1), None),
             "dense-2048": (layered_config(2048, 8, attn(8, 2, 512), delta(8), {"kind": "dense", "ff": 8192}),
-                           LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1)),
-            "moe-2048": (layered_config(2048, 8, attn(8, 2, 512), delta(8), moe), LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1))}
+                           LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1), None),
+            "moe-2048": (layered_config(2048, 8, attn(8, 2, 512), delta(8), moe), LlmHParams(8, 2048, 16, 4, 128, 8192, 32000, 1e-5, 10000.0, 0, 0, 0, 0, 1), None)}
 
 
 def layered_point(tk, model, prompts, batches, context, steps):
@@ -701,15 +716,20 @@ def layered_point(tk, model, prompts, batches, context, steps):
 
 def run_layered(args, tk, device):
     """--layered: the layer-list decoders at sizes that resemble a real model's layers, random weights, beside the Mistral-class model of the same
-    width, depth and active feed-forward (its fp16 and its Q4_K_M checkpoints)"""
+    width, depth and active feed-forward (its fp16 and its Q4_K_M checkpoints); Kaparax beside Vuvulorn of the same width, depth and feed-forward too"""
     prompts, batches = (512, 2048), (1, 16, 64, 256)
     res = {}
-    for name, (cfg, hp) in layered_sizes().items():
+    sizes = layered_sizes()
+    for name, (cfg, hp, beside) in sizes.items():
         if args.layered not in ("all", name):
             continue
         m = tk.LlmModel(config=cfg, device=device, gate_rank=128)
         res[name] = {"layered_bf16": layered_point(tk, m, prompts, batches, 512, 24)}
         m.close()
+        if beside:
+            m = tk.LlmModel(config=sizes[beside][0], device=device, gate_rank=128)
+            res[name]["vuvulorn_bf16"] = layered_point(tk, m, prompts, batches, 512, 24)
+            m.close()
         if not args.layered_only:
             for tag, f16 in (("mistral_f16", True), ("mistral_q4_k_m", False)):
                 m = tk.LlmModel(hp, device=device).fill_synthetic(4, f16=f16)
@@ -720,8 +740,8 @@ def run_layered(args, tk, device):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--layered", default="", choices=["", "all"] + ["dense-4096", "dense-2048", "moe-2048"],
-                    help="instead of the headline: prefill and decode throughput of the layer-list decoders (Vuvulorn) beside the Mistral-class model of equal size; one JSON line of its own")
+    ap.add_argument("--layered", default="", choices=["", "all", "kaparax-4096", "kaparax-2048", "dense-4096", "dense-2048", "moe-2048"],
+                    help="instead of the headline: prefill and decode throughput of the layer-list decoders (Kaparax, Vuvulorn) beside the Mistral-class model of equal size; one JSON line of its own")
     ap.add_argument("--layered-only", action="store_true", help="with --layered: leave the Mistral-class models out (profiling)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)

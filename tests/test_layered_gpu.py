@@ -9,13 +9,11 @@ import numpy as np
 import pytest
 
 import layered_util as U
-from layered_util import LO, attention, config, delta, dense, layer, moe
+from layered_util import BF16, F32, LO, Case, attention, close, config, delta, dense, greedy, layer, moe, no_end, runner_ids, tokens_for
 
 pytestmark = pytest.mark.gpu
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-F32 = 2e-5   # worst row's rms difference in units of the logits' spread
-BF16 = 0.06  # of nine rows in ten: where a router's choice is close, bf16 inputs may take another expert than the restatement
 
 CONFIGS = {
     # nothing a multiple of anything: padded tiles in every product
@@ -32,35 +30,6 @@ CONFIGS = {
     # more query heads per key head than a tile has rows, a large state
     "grouped": config(80, 64, [layer(attention(34, 2, 16, 16, 8, 130, 2, scale=0.4), delta(2, 1, 256, 256, 6), dense(48), 1.0, 1.0)]),
 }
-
-
-def close(got, want, tol):
-    return U.rel_rms(got, want, 1.0 if tol < 1e-3 else 0.9) < tol
-
-
-def tokens_for(cfg, n, seed=11):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
-
-
-class Case:
-    """a checkpoint on disk, its restatement, and models per dtype"""
-
-    def __init__(self, tk, path, cfg, seed=7, w=None):
-        self.tk, self.cfg = tk, cfg
-        self.w = w if w is not None else U.random_weights(cfg, seed)
-        self.dir = U.write_folder(path, cfg, self.w)
-        self.models, self.known = {}, {}
-
-    def session(self, dtype, max_seq=4, max_ctx=512, pool=0):
-        if dtype not in self.models:
-            self.models[dtype] = self.tk.LlmModel(folder=self.dir, dtype=dtype)
-        return self.tk.LlmSession(self.models[dtype], max_seq, max_ctx, pool_tokens=pool)
-
-    def want(self, tokens):
-        k = tuple(tokens)
-        if k not in self.known:
-            self.known[k] = LO.forward(self.cfg, self.w, tokens)
-        return self.known[k]
 
 
 @pytest.fixture(scope="module")
@@ -323,17 +292,6 @@ def test_more_rows_than_a_pass_holds(gpu, tmp_path):
 
 # ---- generation ----
 
-def greedy(session, slot, prompt, n):
-    out, at, nxt = [], len(prompt), None
-    _, ids = session.forward_rows([slot] * at, range(at), prompt, [at - 1], want_logits=False, want_ids=True)
-    for _ in range(n):
-        nxt = int(ids[0])
-        out.append(nxt)
-        _, ids = session.forward_rows([slot], [at], [nxt], [0], want_logits=False, want_ids=True)
-        at += 1
-    return out
-
-
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_device_driven_decode_loop(cases, dtype, monkeypatch):
     """the captured loop against one pass per token, over 300 steps and several replays, with passes of the host in between; and without graphs"""
@@ -370,22 +328,6 @@ def test_decode_loop_keeps_to_what_it_continues(cases):
     s.forward_rows([0, 0], [0, 1], [1, 2], [1])
     with pytest.raises(c.tk.TkError, match="continues"):
         s.decode(1, 3)
-
-
-def runner_ids(runner, prompt, n):
-    runner.prepare_ids(prompt)
-    out = []
-    for _ in range(n):
-        i = runner.pending_id
-        if runner.next_token() is None:
-            break
-        out.append(i)
-    return out
-
-
-def no_end(ids, n):
-    """what a runner yields of a greedy continuation: it stops at the end-of-sequence id"""
-    return ids[:ids.index(2)] if 2 in ids[:n] else ids[:n]
 
 
 def test_runners_share_the_scheduler(cases):

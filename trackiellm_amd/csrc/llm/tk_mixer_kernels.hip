@@ -931,7 +931,7 @@ template <typename T, int DIM, int VB>
 struct RetLds { /* byte offsets */
     static constexpr int C = RetChunk<T>::C, SZ = sizeof(T), RP = DIM * SZ + 16, TP = C * SZ + 16;
     static constexpr int q = 0, k = q + C * RP, kt = k + C * RP, vt = kt + DIM * TP, p = vt + VB * TP, lo = p + C * TP, pw = lo + (SZ == 2 ? C * TP : 0),
-                         red = pw + (TK_RETENTION_BLOCK + 4) * 4, bytes = red + 16 * C * 4;
+                         red = pw + (TK_RETENTION_BLOCK + 4) * 4, bytes = red + 8 * C * 4; /* eight waves at most */
 };
 
 /* two tokens' elements side by side; four */
@@ -945,6 +945,7 @@ __global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a
     constexpr int C = RetChunk<T>::C, KT = TkImg<T>::KT, EP = TkImg<T>::EP, SZ = sizeof(T), THREADS = 64 * WAVES, VB = 16 * WAVES * NT;
     constexpr int DT = DIM / KT, DS = DIM / 16, CT = C / 16, CK = C / KT;
     typedef RetLds<T, DIM, VB> L;
+    static_assert(WAVES <= 8 && L::bytes <= 160 * 1024, "a chunk fits the LDS");
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, r16 = lane & 15, h = blockIdx.x;
     const TkRetentionBlock b = blocks[blockIdx.y];
