@@ -21,6 +21,9 @@
 
 static constexpr int PASS_ROWS = 2048; /* rows of one pass at most */
 
+/* floats between two rows of the projections: an odd number of 256-byte lines, so that a head's columns of many rows spread over the memory channels */
+static int proj_pitch(int n) { return ((n + 63) / 64 | 1) * 64; }
+
 bool TkLayeredSession::alloc(void** p, size_t bytes, bool zero) {
     HIPQ(hipMalloc(p, bytes ? bytes : 16));
     owned_.push_back(*p);
@@ -49,10 +52,10 @@ bool TkLayeredSession::rotation(int dims, double base, Rope* out) {
     return true;
 }
 
-/* rows of a retention scan's blocks: about 512 workgroups (heads x blocks) in a pass */
+/* rows of a retention scan's blocks: a workgroup (a head's block) for every compute unit */
 int TkLayeredSession::retention_rows(int nrows) const {
     int n = TK_RETENTION_BLOCK;
-    while ((int64_t)(nrows / n) * ret_heads_ > 512) n *= 2;
+    while ((int64_t)(nrows / n) * ret_heads_ > 256) n *= 2;
     return n;
 }
 
@@ -104,7 +107,7 @@ bool TkLayeredSession::init(TkLayeredModel* m, int mseq, int mctx, int pool_toke
     for (size_t l = 0; l < c.layers.size(); ++l) {
         const TkLayeredLayer& L = m->layers[l];
         const TkLayerSpec& s = c.layers[l];
-        proj = std::max(proj, (size_t)L.in.N);
+        proj = std::max(proj, (size_t)proj_pitch(L.in.N));
         low = std::max(low, (size_t)L.low.N);
         mix = std::max(mix, tk_img_bytes(type, R, L.out.cols));
         if (L.low_cols) lowk = std::max(lowk, tk_img_bytes(type, R, L.low_cols));
@@ -333,9 +336,10 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
         const TkLayerSpec& spec = c.layers[l];
         const TkLayeredLayer& L = m_->layers[l];
         const TkNorm after = l + 1 < c.layers.size() ? m_->layers[l + 1].pre1 : TkNorm{}; /* on the next layer's input: fused into this layer's last kernel */
+        const int pitch = proj_pitch(L.in.N);
         TkImgGemm g{};
         g.type = type; g.w = L.in.img; g.a = img_x_; g.K = L.in.K; g.N = L.in.N; g.nrows = n;
-        g.out = proj_; g.ldc = L.in.N; g.n_valid = L.in.rows;
+        g.out = proj_; g.ldc = pitch; g.n_valid = L.in.rows;
         if (L.low_cols) { g.copy_img = img_low_; g.copy0 = L.low_col; g.copy1 = L.low_col + L.low_cols; g.copy_ktiles = L.low.K / kt; }
         gemm(g);
         if (L.low_cols) { /* outer sides of all low-rank gates: one block-diagonal product */
@@ -366,8 +370,8 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
                 a.heads = sp.heads; a.dim = sp.dim; a.vdim = sp.vdim; a.rot_dims = sp.rot_dims; a.out_scale = bs.scale; a.eps = c.eps; a.col = B.col;
                 a.rope_cos = st.rope.c; a.rope_sin = st.rope.s; a.decay = st.decay; a.state = st.state; a.sums = sums_;
                 a.out_img = img_mix_; a.out_k0 = B.out_k0; a.out_ktiles = L.out.K / kt;
-                if (p.nblocks) tk_launch_retention_scan(type, a, proj_, L.in.N, tab_, (const TkRetentionBlock*)d_blocks_, p.nblocks, p.nsums, s);
-                if (p.singles) tk_launch_retention_step(type, a, proj_, L.in.N, tab_, p.nseg, s);
+                if (p.nblocks) tk_launch_retention_scan(type, a, proj_, pitch, tab_, (const TkRetentionBlock*)d_blocks_, p.nblocks, p.nsums, s);
+                if (p.singles) tk_launch_retention_step(type, a, proj_, pitch, tab_, p.nseg, s);
             } else {
                 const TkDeltaSpec& sp = bs.delta;
                 TkDeltaArgs d{};
@@ -382,7 +386,7 @@ void TkLayeredSession::enqueue_layers(const Pass& p) {
         for (size_t i = 0, ai = 0, di = 0; i < std::max(as.size(), ds.size()); ++i, ++ai, ++di) {
             const TkAttnArgs* a = ai < as.size() ? &as[ai] : nullptr;
             const TkDeltaArgs* d = di < ds.size() ? &ds[di] : nullptr;
-            tk_launch_mixer_prep(type, proj_, L.in.N, a, d, tab_, n, s);
+            tk_launch_mixer_prep(type, proj_, pitch, a, d, tab_, n, s);
             if (!p.single) {
                 if (a) tk_launch_attn_tiles(type, *a, tab_, d_tiles_, p.ntiles, s);
                 if (d) tk_launch_delta_scan(type, *d, tab_, p.nseg, n, s);

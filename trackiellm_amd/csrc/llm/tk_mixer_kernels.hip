@@ -194,6 +194,14 @@ __global__ __launch_bounds__(512) void k_rows_norm(const float* x, const int32_t
 
 /* ------------------------------------------------------------------ short convolutions ----- */
 
+/* V neighbouring elements of a row a lane, i = 0, V, 2 V ..: element(lane, i) + 0 .. V - 1 */
+template <int V> struct TkVf;
+template <> struct TkVf<1> { typedef float type __attribute__((ext_vector_type(1))); };
+template <> struct TkVf<2> { typedef float type __attribute__((ext_vector_type(2))); };
+template <int V> using tk_vf = typename TkVf<V>::type;
+template <int V> __device__ __forceinline__ int element(int lane, int i) { return V * lane + 64 * i; }
+template <int V> __device__ __forceinline__ tk_vf<V> load_v(const float* p) { return *(const tk_vf<V>*)p; } /* V = 2: eight-byte aligned */
+
 /* a causal convolution over the rows of a sequence; what came before the pass is in the history (zeros before the sequence) */
 struct Conv {
     const float* w; /* [channels][taps] */
@@ -204,28 +212,57 @@ struct Conv {
         const int in = t.seg_in[seg], hist = taps - 1;
         return in < 0 ? 0.0f : state[((size_t)in * channels + c) * hist + hist + s];
     }
-    /* channels c0 + lane + 64 i (< c0 + n) of RW rows from rowb on (rows past the pass repeat its last one) */
-    template <int RW>
+    /* channels c0 + element(lane, i) (< c0 + n) of RW rows from rowb on (rows past the pass repeat its last one) */
+    template <int RW, int V>
     __device__ __forceinline__ void rows(const TkPassTab& t, const float* proj, int ld, int rowb, int nrows, int c0, int n, int lane, float (&y)[RW][4]) const {
         const int hist = taps - 1, seg0 = t.seg[rowb], first = rowb - t.seg_row0[seg0];
-        const bool inside = RW > 1 && first >= hist && first + RW <= t.seg_n[seg0]; /* every input is a row of this pass */
+        const bool inside = first >= hist && first + RW <= t.seg_n[seg0]; /* every input is a row of this pass */
+        const int in0 = t.seg_in[seg0];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
+        for (int i = 0; i < 4; i += V) {
 #pragma unroll
-            for (int r = 0; r < RW; ++r) y[r][i] = 0.0f;
-            const int c = c0 + lane + 64 * i;
-            if (64 * i >= n || lane + 64 * i >= n) continue;
-            if (inside) {
-                for (int j = 0; j < taps; ++j) {
-                    const float tap = w[(size_t)c * taps + j];
+            for (int r = 0; r < RW; ++r)
 #pragma unroll
-                    for (int r = 0; r < RW; ++r) y[r][i] = fmaf(tap, proj[(size_t)(rowb + r - hist + j) * ld + col + c], y[r][i]);
+                for (int k = 0; k < V; ++k) y[r][i + k] = 0.0f;
+            const int c = c0 + element<V>(lane, i);
+            if (64 * i >= n || element<V>(lane, i) >= n) continue;
+            if (inside && taps == 4) { /* every input once */
+                tk_vf<V> x[RW + 3];
+#pragma unroll
+                for (int j = 0; j < RW + 3; ++j) x[j] = load_v<V>(proj + (size_t)(rowb - 3 + j) * ld + col + c);
+#pragma unroll
+                for (int k = 0; k < V; ++k) {
+                    const tk_v4f f = *(const tk_v4f*)(w + (size_t)(c + k) * 4);
+#pragma unroll
+                    for (int r = 0; r < RW; ++r)
+#pragma unroll
+                        for (int j = 0; j < 4; ++j) y[r][i + k] = fmaf(f[j], x[r + j][k], y[r][i + k]);
                 }
+            } else if (RW == 1 && first == 0 && taps == 4) { /* decoding: the history and one row */
+                const tk_vf<V> x = load_v<V>(proj + (size_t)rowb * ld + col + c);
+#pragma unroll
+                for (int k = 0; k < V; ++k) {
+                    const tk_v4f f = *(const tk_v4f*)(w + (size_t)(c + k) * 4);
+                    const float* old = state + ((size_t)(in0 < 0 ? 0 : in0) * channels + c + k) * 3;
+                    float past = fmaf(f[2], old[2], fmaf(f[1], old[1], f[0] * old[0]));
+                    if (in0 < 0) past = 0.0f;
+                    y[0][i + k] = fmaf(f[3], x[k], past);
+                }
+            } else if (inside) {
+                for (int j = 0; j < taps; ++j)
+#pragma unroll
+                    for (int k = 0; k < V; ++k) {
+                        const float tap = w[(size_t)(c + k) * taps + j];
+#pragma unroll
+                        for (int r = 0; r < RW; ++r) y[r][i + k] = fmaf(tap, proj[(size_t)(rowb + r - hist + j) * ld + col + c + k], y[r][i + k]);
+                    }
             } else {
 #pragma unroll
                 for (int r = 0; r < RW; ++r) {
                     const int row = rowb + r < nrows ? rowb + r : nrows - 1, seg = t.seg[row], at = row - t.seg_row0[seg];
-                    for (int j = 0; j < taps; ++j) y[r][i] = fmaf(w[(size_t)c * taps + j], input(t, proj, ld, seg, at - hist + j, c), y[r][i]);
+                    for (int j = 0; j < taps; ++j)
+#pragma unroll
+                        for (int k = 0; k < V; ++k) y[r][i + k] = fmaf(w[(size_t)(c + k) * taps + j], input(t, proj, ld, seg, at - hist + j, c + k), y[r][i + k]);
                 }
             }
         }
@@ -242,8 +279,9 @@ struct Conv {
 /* ------------------------------------------------------------------ between projections and mixers ---- */
 
 /* one wave: one head of q, k or v of RW consecutive rows (rows past the pass repeat its last one and store nothing); all loads come first.
- * CONV: the elements are convolved ones; rotation partners meet in `ex`, [RW][TK_MAX_HEAD_DIM] of LDS of this wave's own */
-template <typename T, int RW, bool CONV>
+ * CONV: the elements are convolved ones; rotation partners meet in `ex`, [RW][TK_MAX_HEAD_DIM] of LDS of this wave's own.  V = 2: sizes, columns and
+ * pitch are even, half the rotating dimensions too */
+template <typename T, int RW, bool CONV, int V>
 __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& t, const float* proj, int ld, int row0, int nrows, int u, int lane, float* ex) {
     const bool is_q = u < a.heads, is_v = u >= a.heads + a.kv_heads;
     const int n = is_v ? a.vdim : a.dim;
@@ -256,45 +294,65 @@ __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& 
     int pos[RW];
     size_t page[RW];
     const Conv conv{a.conv, a.conv_state, (a.heads + a.kv_heads) * a.dim + a.kv_heads * a.vdim, a.taps, a.col};
-    if (CONV) {
-        conv.rows<RW>(t, proj, ld, row0, nrows, off, n, lane, v);
-        if (half > 0) {
-#pragma unroll
-            for (int r = 0; r < RW; ++r)
-#pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    if (lane + 64 * i < 2 * half) ex[r * TK_MAX_HEAD_DIM + lane + 64 * i] = v[r][i];
-            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-            __builtin_amdgcn_wave_barrier();
-            __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-        }
-    }
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
         const int row = row0 + r < nrows ? row0 + r : nrows - 1;
         pos[r] = t.pos[row];
         page[r] = is_q ? 0 : (size_t)t.page_of[(size_t)t.seq[row] * t.max_pages + pos[r] / TK_PAGE];
         const float* src = proj + (size_t)row * ld + a.col + off;
+        const float *cosp = a.rope_cos + (size_t)pos[r] * half, *sinp = a.rope_sin + (size_t)pos[r] * half;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int e = lane + 64 * i;
-            if (!CONV) v[r][i] = 0.0f;
-            z[r][i] = s[r][i] = 0.0f;
-            c[r][i] = 1.0f;
+        for (int i = 0; i < 4; i += V) {
+            const int e = element<V>(lane, i);
+            tk_vf<V> x = {}, y = {}, cs, sn = {};
+#pragma unroll
+            for (int k = 0; k < V; ++k) cs[k] = 1.0f;
             if (64 * i < n && e < n) {
-                if (!CONV) v[r][i] = src[e] + (b ? b[e] : 0.0f);
+                const int f = e < half ? e + half : e - half, j = e < half ? e : f;
+                if (!CONV) x = load_v<V>(src + e);
                 if (e < 2 * half) {
-                    const int f = e < half ? e + half : e - half, j = e < half ? e : f;
-                    z[r][i] = CONV ? ex[r * TK_MAX_HEAD_DIM + f] : (src[f] + (b ? b[f] : 0.0f)) * (w ? w[f] : 1.0f);
-                    c[r][i] = a.rope_cos[(size_t)pos[r] * half + j];
-                    s[r][i] = a.rope_sin[(size_t)pos[r] * half + j] * (e < half ? -1.0f : 1.0f);
+                    if (!CONV) y = load_v<V>(src + f);
+                    cs = load_v<V>(cosp + j);
+                    sn = load_v<V>(sinp + j) * (e < half ? -1.0f : 1.0f);
+                }
+#pragma unroll
+                for (int k = 0; k < V; ++k) {
+                    if (b) x[k] += b[e + k];
+                    if (e < 2 * half) y[k] = (y[k] + (b ? b[f + k] : 0.0f)) * (w ? w[f + k] : 1.0f);
                 }
             }
+#pragma unroll
+            for (int k = 0; k < V; ++k) { v[r][i + k] = x[k]; z[r][i + k] = y[k]; c[r][i + k] = cs[k]; s[r][i + k] = sn[k]; }
+        }
+    }
+    if (CONV) {
+        conv.rows<RW, V>(t, proj, ld, row0, nrows, off, n, lane, v);
+        if (half > 0) { /* partners change hands inside the wave */
+#pragma unroll
+            for (int r = 0; r < RW; ++r)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int e = element<V>(lane, i / V * V) + i % V;
+                    if (e < 2 * half) ex[r * TK_MAX_HEAD_DIM + e] = v[r][i];
+                }
+            __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+            __builtin_amdgcn_wave_barrier();
+            __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+            for (int r = 0; r < RW; ++r)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int e = element<V>(lane, i / V * V) + i % V;
+                    if (e < 2 * half) z[r][i] = ex[r * TK_MAX_HEAD_DIM + (e < half ? e + half : e - half)];
+                }
         }
     }
     float wv[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) wv[i] = w && lane + 64 * i < n ? w[lane + 64 * i] : 1.0f;
+    for (int i = 0; i < 4; ++i) {
+        const int e = element<V>(lane, i / V * V) + i % V;
+        wv[i] = w && e < n ? w[e] : 1.0f;
+    }
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
         if (row0 + r >= nrows) break;
@@ -305,14 +363,25 @@ __device__ __forceinline__ void attn_unit(const TkAttnArgs& a, const TkPassTab& 
             for (int i = 0; i < 4; ++i) ss += v[r][i] * v[r][i];
             f = 1.0f / sqrtf(tk_wave_sum(ss) / (float)n + a.eps);
         }
+        T* dst = is_q ? (T*)a.q + ((size_t)(row0 + r) * a.heads + head) * a.kv.dim_pad
+                      : is_v ? (T*)a.kv.v + (page[r] * a.kv_heads + head) * a.kv.vdim_pad * TK_PAGE + pos[r] % TK_PAGE
+                             : (T*)a.kv.k + ((page[r] * a.kv_heads + head) * TK_PAGE + pos[r] % TK_PAGE) * a.kv.dim_pad;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int e = lane + 64 * i;
-            if (e >= n) break;
-            const float y = (v[r][i] * f * wv[i]) * c[r][i] + (z[r][i] * f) * s[r][i];
-            if (is_q) ((T*)a.q)[((size_t)(row0 + r) * a.heads + head) * a.kv.dim_pad + e] = TkImg<T>::from(y);
-            else if (is_v) ((T*)a.kv.v)[((page[r] * a.kv_heads + head) * a.kv.vdim_pad + e) * TK_PAGE + pos[r] % TK_PAGE] = TkImg<T>::from(y);
-            else ((T*)a.kv.k)[((page[r] * a.kv_heads + head) * TK_PAGE + pos[r] % TK_PAGE) * a.kv.dim_pad + e] = TkImg<T>::from(y);
+        for (int i = 0; i < 4; i += V) {
+            const int e = element<V>(lane, i);
+            if (64 * i >= n || e >= n) break;
+            T y[V];
+#pragma unroll
+            for (int k = 0; k < V; ++k) y[k] = TkImg<T>::from((v[r][i + k] * f * wv[i + k]) * c[r][i + k] + (z[r][i + k] * f) * s[r][i + k]);
+            if (is_v) {
+#pragma unroll
+                for (int k = 0; k < V; ++k) dst[(e + k) * TK_PAGE] = y[k];
+            } else if constexpr (V == 2) {
+                struct __attribute__((aligned(2 * sizeof(T)))) Two { T a, b; };
+                *(Two*)(dst + e) = Two{y[0], y[1]};
+            } else {
+                dst[e] = y[0];
+            }
         }
         if (CONV) conv.leave(t, proj, ld, row0 + r, off, n, lane);
     }
@@ -345,7 +414,7 @@ __device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab
     const size_t pitch = which == 2 ? (size_t)d.heads * d.vdim : qk;
     const Conv conv{d.conv, d.conv_state, channels, d.taps, d.col};
     float y[RW][4];
-    conv.rows<RW>(t, proj, ld, rowb, nrows, c0, n, lane, y);
+    conv.rows<RW, 1>(t, proj, ld, rowb, nrows, c0, n, lane, y);
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
         const int row = rowb + r;
@@ -365,12 +434,12 @@ __device__ __forceinline__ void delta_unit(const TkDeltaArgs& d, const TkPassTab
     }
 }
 
-template <typename T, int RW, bool CONV>
+template <typename T, int RW, bool CONV, int V>
 __global__ __launch_bounds__(256) void k_mixer_prep(const float* proj, int ld, TkAttnArgs a, TkDeltaArgs d, TkPassTab t, int na, int nd, int nrows) {
     __shared__ float ex[CONV ? 4 * RW * TK_MAX_HEAD_DIM : 1];
     const int row = blockIdx.y * RW, lane = threadIdx.x & 63;
     const int u = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
-    if (u < na) attn_unit<T, RW, CONV>(a, t, proj, ld, row, nrows, u, lane, ex + (CONV ? (threadIdx.x >> 6) * RW * TK_MAX_HEAD_DIM : 0));
+    if (u < na) attn_unit<T, RW, CONV, V>(a, t, proj, ld, row, nrows, u, lane, ex + (CONV ? (threadIdx.x >> 6) * RW * TK_MAX_HEAD_DIM : 0));
     else if (u < na + nd) delta_unit<RW>(d, t, proj, ld, row, nrows, u - na, lane);
 }
 
@@ -905,9 +974,9 @@ __global__ void k_swap_state(TkPassTab t, int n) {
  * products leave it in: an accumulator tile [key dimension][value column] is at once the operand of S^T q, because the key dimensions of q (and k)
  * lie in LDS in the order in which a lane's accumulators hold them.  Scores go through LDS.  bf16 sessions: q, k and v are bf16 (as in attention);
  * what is 32-bit by nature (the state, decayed scores, decayed values) enters a product as the sum of two bf16 numbers.
- * SUMS: only what the block adds to the state, into args.sums: blocks of a segment run side by side, each starts from the segment's state and the
- * sums of the blocks before it. */
-template <typename T> struct RetChunk { static constexpr int C = sizeof(T) == 2 ? 64 : 32; };
+ * SUMS: only what the block adds to the state, into args.sums; k_retention_prefix turns these into the states that the segment's next blocks start
+ * from, so that all blocks run side by side. */
+template <typename T> struct RetChunk { static constexpr int C = 32; };
 
 /* where element e of a key row lies: see above (f32 accumulators are in order already) */
 template <typename T> __device__ __forceinline__ int ret_place(int e) { return sizeof(T) == 2 ? (e & ~31) | (e & 12) << 1 | (e & 16) >> 2 | (e & 3) : e; }
@@ -927,6 +996,9 @@ template <> struct Split<TkBf16> {
     }
 };
 
+/* a gate on its way into a bf16 image needs no more than the hardware's exponential and reciprocal (1e-7) */
+template <typename T> __device__ __forceinline__ float silu_out(float z) { return sizeof(T) == 4 ? tk_silu32(z) : z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-LOG2E * z)); }
+
 template <typename T, int DIM, int VB>
 struct RetLds { /* byte offsets */
     static constexpr int C = RetChunk<T>::C, SZ = sizeof(T), RP = DIM * SZ + 16, TP = C * SZ + 16;
@@ -941,13 +1013,15 @@ __device__ __forceinline__ void ret_put4(TkBf16* p, const float (&x)[4]) {
 __device__ __forceinline__ void ret_put4(float* p, const float (&x)[4]) { *(tk_v4f*)p = tk_v4f{x[0], x[1], x[2], x[3]}; }
 
 template <typename T, int DIM, int WAVES, int NT, bool SUMS>
-__global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a, const float* proj, int ld, TkPassTab t, const TkRetentionBlock* blocks) {
+__global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) void k_retention_scan(TkRetentionArgs a, const float* proj, int ld, TkPassTab t, const TkRetentionBlock* blocks) {
     constexpr int C = RetChunk<T>::C, KT = TkImg<T>::KT, EP = TkImg<T>::EP, SZ = sizeof(T), THREADS = 64 * WAVES, VB = 16 * WAVES * NT;
     constexpr int DT = DIM / KT, DS = DIM / 16, CT = C / 16, CK = C / KT;
     typedef RetLds<T, DIM, VB> L;
     static_assert(WAVES <= 8 && L::bytes <= 160 * 1024, "a chunk fits the LDS");
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, r16 = lane & 15, h = blockIdx.x;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, r16 = lane & 15;
+    /* workgroups go to the eight XCDs in turn, and the L2 slices of one repeat every 4 KiB of a row: an XCD's heads lie side by side, other ones in the next block */
+    const int per = a.heads / 8, h = a.heads % 8 ? blockIdx.x : (blockIdx.x % 8 * per + blockIdx.x / 8 + blockIdx.y * per) % a.heads;
     const TkRetentionBlock b = blocks[blockIdx.y];
     if (SUMS && b.last) return;
     const int vp = (a.vdim + 3) & ~3, in = t.seg_in[b.seg], pos0 = t.pos[b.row0];
@@ -976,66 +1050,104 @@ __global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a
 #pragma unroll
         for (int d = 0; d < DS; ++d) S[n][d] = tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
     if (!SUMS) {
-        if (in >= 0) state_at(a.state + ((size_t)in * a.heads + h) * head_floats, [](float, float& m) { return m; });
-        if (b.index > 0) {
-            __syncthreads();
-            float fade = 1.0f; /* over a block */
-            for (int n = 0; n < blocks[blockIdx.y - 1].n; n += TK_RETENTION_BLOCK) fade *= pw[TK_RETENTION_BLOCK];
-            for (int i = 0; i < b.index; ++i) state_at(a.sums + ((size_t)(b.slot0 + i) * a.heads + h) * head_floats, [&](float s, float& m) { return fmaf(s, fade, m); });
-        }
+        if (b.index > 0) state_at(a.sums + ((size_t)(b.slot0 + b.index - 1) * a.heads + h) * head_floats, [](float, float& m) { return m; });
+        else if (in >= 0) state_at(a.state + ((size_t)in * a.heads + h) * head_floats, [](float, float& m) { return m; });
     }
-    const int half = a.rot_dims / 2, units = a.dim - half, qk = a.heads * a.dim;
+    const int half = a.rot_dims / 2, units = (a.dim + 1) / 2, qk = a.heads * a.dim;
     const float kscale = 1.0f / sqrtf((float)a.dim);
     const float *qp = proj + a.col + h * a.dim, *kp = qp + qk, *vsrc = proj + a.col + 2 * qk + h * a.vdim, *gsrc = vsrc + a.heads * a.vdim;
-    for (int c0 = 0; c0 < b.n; c0 += C) {
+    /* a thread's share of a chunk, four tokens at a time: pairs of key dimensions (rotation partners, or neighbours among those that do not turn) and
+     * value columns.  Small heads: the next chunk's is on its way to registers while one is used. */
+    constexpr int QI = (DIM / 2 * (C / 4) + THREADS - 1) / THREADS, VI = VB * (C / 4) / THREADS;
+    float q0[QI][4], q1[QI][4], k0[QI][4], k1[QI][4], cs[QI][4], sn[QI][4], vv[VI][4];
+    auto fetch = [&](int c0) {
         const int n = b.n - c0 < C ? b.n - c0 : C, base = b.row0 + c0;
-        const bool more = c0 + C < b.n;
-        /* ---- rotated q and k, v into LDS; a unit is a rotating pair or a single element of four tokens ---- */
-        for (int it = tid; it < units * (C / 4); it += THREADS) {
-            const int u = it % units, t0 = it / units * 4;
-            const bool pair = u < half;
-            const int e0 = pair ? u : u + half, e1 = pair ? u + half : e0;
-            float q0[4], q1[4], k0[4], k1[4], cs[4], sn[4];
+#pragma unroll
+        for (int i = 0; i < QI; ++i) {
+            const int it = tid + i * THREADS, u = it % (DIM / 2) < units ? it % (DIM / 2) : units - 1, t0 = it / (DIM / 2) * 4;
+            const int e0 = u < half ? u : 2 * u, e1 = u < half ? u + half : 2 * u + 1 < a.dim ? 2 * u + 1 : 2 * u;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                const int tt = t0 + r < n ? t0 + r : n - 1;
-                const size_t row = (size_t)(base + tt) * ld;
-                if (!SUMS) { q0[r] = qp[row + e0]; q1[r] = qp[row + e1]; }
-                k0[r] = kp[row + e0];
-                k1[r] = kp[row + e1];
-                const size_t at = (size_t)(pos0 + c0 + tt) * half + (pair ? u : 0);
-                cs[r] = pair ? a.rope_cos[at] : 1.0f;
-                sn[r] = pair ? a.rope_sin[at] : 0.0f;
+                const size_t row = (size_t)(base + (t0 + r < n ? t0 + r : n - 1)) * ld;
+                if (!SUMS) { q0[i][r] = qp[row + e0]; q1[i][r] = qp[row + e1]; }
+                k0[i][r] = kp[row + e0];
+                k1[i][r] = kp[row + e1];
             }
+            if (half > 0)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const size_t at = (size_t)(pos0 + c0 + (t0 + r < n ? t0 + r : n - 1)) * half + (u < half ? u : 0);
+                    cs[i][r] = a.rope_cos[at];
+                    sn[i][r] = a.rope_sin[at];
+                }
+        }
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int it = tid + i * THREADS, e = it % VB < a.vdim ? it % VB : a.vdim - 1, t0 = it / VB * 4;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) vv[i][r] = vsrc[(size_t)(base + (t0 + r < n ? t0 + r : n - 1)) * ld + e];
+        }
+    };
+    auto put = [&](int n) {
+#pragma unroll
+        for (int i = 0; i < QI; ++i) {
+            const int it = tid + i * THREADS, u = it % (DIM / 2), t0 = it / (DIM / 2) * 4;
+            if (u >= units || t0 >= C) break;
+            const bool turns = u < half, two = turns || 2 * u + 1 < a.dim;
+            const int e0 = turns ? u : 2 * u, e1 = turns ? u + half : two ? 2 * u + 1 : 2 * u;
             float ka[4], kb[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const bool ok = t0 + r < n;
-                ka[r] = ok ? (k0[r] * cs[r] - k1[r] * sn[r]) * kscale : 0.0f;
-                kb[r] = ok ? (k1[r] * cs[r] + k0[r] * sn[r]) * kscale : 0.0f;
+                const float c = turns ? cs[i][r] : 1.0f, z = turns ? sn[i][r] : 0.0f;
+                ka[r] = ok ? (k0[i][r] * c - k1[i][r] * z) * kscale : 0.0f;
+                kb[r] = ok ? (k1[i][r] * c + k0[i][r] * z) * kscale : 0.0f;
                 if (!SUMS) {
                     T *lq = (T*)(lds + L::q + (t0 + r) * L::RP), *lk = (T*)(lds + L::k + (t0 + r) * L::RP);
-                    lq[ret_place<T>(e0)] = TkImg<T>::from(q0[r] * cs[r] - q1[r] * sn[r]);
+                    lq[ret_place<T>(e0)] = TkImg<T>::from(q0[i][r] * c - q1[i][r] * z);
                     lk[ret_place<T>(e0)] = TkImg<T>::from(ka[r]);
-                    if (pair) {
-                        lq[ret_place<T>(e1)] = TkImg<T>::from(q1[r] * cs[r] + q0[r] * sn[r]);
+                    if (two) {
+                        lq[ret_place<T>(e1)] = TkImg<T>::from(q1[i][r] * c + q0[i][r] * z);
                         lk[ret_place<T>(e1)] = TkImg<T>::from(kb[r]);
                     }
                 }
             }
             ret_put4((T*)(lds + L::kt + e0 * L::TP) + t0, ka);
-            if (pair) ret_put4((T*)(lds + L::kt + e1 * L::TP) + t0, kb);
+            if (two) ret_put4((T*)(lds + L::kt + e1 * L::TP) + t0, kb);
         }
-        for (int it = tid; it < a.vdim * (C / 4); it += THREADS) {
-            const int e = it % a.vdim, t0 = it / a.vdim * 4;
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int it = tid + i * THREADS, e = it % VB, t0 = it / VB * 4;
             float v[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) v[r] = vsrc[(size_t)(base + (t0 + r < n ? t0 + r : n - 1)) * ld + e];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) v[r] = t0 + r < n ? v[r] : 0.0f;
-            ret_put4((T*)(lds + L::vt + e * L::TP) + t0, v);
+            for (int r = 0; r < 4; ++r) v[r] = t0 + r < n ? vv[i][r] : 0.0f;
+            if (e < a.vdim) ret_put4((T*)(lds + L::vt + e * L::TP) + t0, v);
         }
+    };
+    constexpr bool AHEAD = NT * DIM <= 128; /* as many registers as that takes are free */
+    if (AHEAD) fetch(0);
+    for (int c0 = 0; c0 < b.n; c0 += C) {
+        const int n = b.n - c0 < C ? b.n - c0 : C, base = b.row0 + c0;
+        const bool more = c0 + C < b.n;
+        if (!AHEAD) fetch(c0);
+        put(n);
         __syncthreads();
+        if (AHEAD && more) fetch(c0 + C);
+        tk_v4f gate[SUMS ? 1 : NT][SUMS ? 1 : CT];
+        if constexpr (!SUMS) {
+            const bool vec = ((uintptr_t)gsrc & 15) == 0 && (ld & 3) == 0 && (a.vdim & 3) == 0;
+#pragma unroll
+            for (int m = 0; m < CT; ++m)
+#pragma unroll
+                for (int nt = 0; nt < NT; ++nt) {
+                    const int e = (wave * NT + nt) * 16 + 4 * g;
+                    const float* gp = gsrc + (size_t)(base + (16 * m + r16 < n ? 16 * m + r16 : n - 1)) * ld;
+                    if (vec) gate[nt][m] = *(const tk_v4f*)(gp + (e < a.vdim ? e : 0));
+                    else
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) gate[nt][m][r] = gp[e + r < a.vdim ? e + r : 0];
+                }
+        }
         tk_v4f o[SUMS ? 1 : NT][SUMS ? 1 : CT]; /* [column 4 g + r of tile n][query 16 m + lane % 16] */
         if constexpr (!SUMS) {
             /* ---- decayed scores, tiles of 16 queries x 16 keys dealt to the waves ---- */
@@ -1187,18 +1299,14 @@ __global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a
                 for (int nt = 0; nt < NT; ++nt) {
                     const int e = (wave * NT + nt) * 16 + 4 * g, at = a.out_k0 + h * a.vdim + e;
                     if (e >= a.vdim) continue;
-                    const float* gp = gsrc + (size_t)row * ld + e;
-                    if (((uintptr_t)gp & 15) == 0 && (at & 3) == 0 && e + 3 < a.vdim) {
-                        const tk_v4f z = *(const tk_v4f*)gp;
-                        tk_v4f y;
+                    tk_v4f y;
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) y[r] = o[nt][m][r] * f * tk_silu32(z[r]);
-                        tk_img_put4((T*)a.out_img, row, at, a.out_ktiles, y);
-                    } else {
+                    for (int r = 0; r < 4; ++r) y[r] = o[nt][m][r] * f * silu_out<T>(gate[nt][m][r]);
+                    if ((at & 3) == 0 && e + 3 < a.vdim) tk_img_put4((T*)a.out_img, row, at, a.out_ktiles, y);
+                    else
 #pragma unroll
                         for (int r = 0; r < 4; ++r)
-                            if (e + r < a.vdim) tk_img_put((T*)a.out_img, row, at + r, a.out_ktiles, o[nt][m][r] * f * tk_silu32(gp[r]));
-                    }
+                            if (e + r < a.vdim) tk_img_put((T*)a.out_img, row, at + r, a.out_ktiles, y[r]);
                 }
             }
         } else {
@@ -1207,6 +1315,30 @@ __global__ __launch_bounds__(64 * WAVES) void k_retention_scan(TkRetentionArgs a
     }
     if (SUMS) state_at(a.sums + ((size_t)(b.slot0 + b.index) * a.heads + h) * head_floats, [](float s, float& m) { return m = s; });
     else if (b.last) state_at(a.state + ((size_t)t.seg_out[b.seg] * a.heads + h) * head_floats, [](float s, float& m) { return m = s; });
+}
+
+/* sums of a segment's blocks -> the state behind each of them; one thread per element of a head's state */
+__global__ __launch_bounds__(256) void k_retention_prefix(TkRetentionArgs a, TkPassTab t, const TkRetentionBlock* blocks) {
+    const TkRetentionBlock b = blocks[blockIdx.z];
+    if (b.index > 0 || b.last) return;
+    const int vp = (a.vdim + 3) & ~3, h = blockIdx.y, i = (blockIdx.x * 256 + threadIdx.x) * 4, in = t.seg_in[b.seg], nb = (t.seg_n[b.seg] + b.n - 1) / b.n;
+    const size_t head_floats = (size_t)a.dim * vp;
+    if (i >= (int)head_floats) return;
+    const float step = a.decay[(size_t)h * (TK_RETENTION_BLOCK + 1) + TK_RETENTION_BLOCK];
+    float fade = 1.0f; /* over a block */
+    for (int n = 0; n < b.n; n += TK_RETENTION_BLOCK) fade *= step;
+    tk_v4f S = in >= 0 ? *(const tk_v4f*)(a.state + ((size_t)in * a.heads + h) * head_floats + i) : tk_v4f{0.0f, 0.0f, 0.0f, 0.0f};
+    float* p = a.sums + ((size_t)b.slot0 * a.heads + h) * head_floats + i;
+    const size_t pitch = a.heads * head_floats;
+    for (int k = 0; k + 1 < nb; k += 8) {
+        tk_v4f m[8]; /* loads ahead of the chain */
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (k + j + 1 < nb) m[j] = *(const tk_v4f*)(p + (k + j) * pitch);
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (k + j + 1 < nb) { S = S * fade + m[j]; *(tk_v4f*)(p + (k + j) * pitch) = S; }
+    }
 }
 
 /* One token of one head: the state is read once and written once, a thread holds RPT rows x 4 columns of it.  Rotation, output norm and gate with it. */
@@ -1403,9 +1535,12 @@ void tk_launch_mixer_prep(int type, const float* proj, int ld, const TkAttnArgs*
     const TkDeltaArgs d = delta ? *delta : TkDeltaArgs{};
     const int na = attn ? a.heads + 2 * a.kv_heads : 0, nd = delta ? 2 * d.kv_heads + 2 * d.heads : 0;
     const int gx = (na + nd + 3) / 4;
-#define TK_PREP(RW, CV) TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, RW, CV>), dim3(gx, (nrows + RW - 1) / RW), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows))
-    if (nrows >= 512) { if (a.taps > 0) TK_PREP(4, true); else TK_PREP(4, false); }
-    else { if (a.taps > 0) TK_PREP(1, true); else TK_PREP(1, false); }
+    const bool even = a.dim % 2 == 0 && a.vdim % 2 == 0 && a.rot_dims % 4 == 0 && a.col % 2 == 0 && ld % 2 == 0;
+#define TK_PREP(RW, CV, V) TK_TYPED(type, hipLaunchKernelGGL((k_mixer_prep<T, RW, CV, V>), dim3(gx, (nrows + RW - 1) / RW), dim3(256), 0, s, proj, ld, a, d, t, na, nd, nrows))
+#define TK_PREP_V(RW, CV) do { if (even) TK_PREP(RW, CV, 2); else TK_PREP(RW, CV, 1); } while (0)
+    if (nrows >= 512) { if (a.taps > 0) TK_PREP_V(4, true); else TK_PREP_V(4, false); }
+    else { if (a.taps > 0) TK_PREP_V(1, true); else TK_PREP_V(1, false); }
+#undef TK_PREP_V
 #undef TK_PREP
 }
 
@@ -1522,7 +1657,10 @@ void tk_launch_retention_scan(int type, const TkRetentionArgs& a, const float* p
 #define TK_RET(T, D, W, N) \
     if (dim == D && vb == 16 * W * N) { \
         constexpr size_t lds = RetLds<T, D, 16 * W * N>::bytes; \
-        if (n_sums) hipLaunchKernelGGL((k_retention_scan<T, D, W, N, true>), grid, dim3(64 * W), lds, s, a, proj, ld, t, blocks); \
+        if (n_sums) { \
+            hipLaunchKernelGGL((k_retention_scan<T, D, W, N, true>), grid, dim3(64 * W), lds, s, a, proj, ld, t, blocks); \
+            hipLaunchKernelGGL(k_retention_prefix, dim3((a.dim * ((a.vdim + 3) / 4) + 255) / 256, a.heads, n_blocks), dim3(256), 0, s, a, t, blocks); \
+        } \
         hipLaunchKernelGGL((k_retention_scan<T, D, W, N, false>), grid, dim3(64 * W), lds, s, a, proj, ld, t, blocks); \
     }
     if (type == TK_IMG_F32) { TK_RET_FORMS(TK_RET, float) } else { TK_RET_FORMS(TK_RET, TkBf16) }
