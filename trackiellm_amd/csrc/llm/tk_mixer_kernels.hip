@@ -972,8 +972,8 @@ __global__ void k_swap_state(TkPassTab t, int n) {
  *     o_i = pw(i + 1) S0^T q_i + sum over j <= i of pw(i - j) (q_i . k_j) v_j,      S = pw(n) S0 + sum over j of pw(n - 1 - j) k_j v_j^T:
  * four matrix products.  A workgroup walks one head's block of rows; every wave owns NT 16-column tiles of the state, in the registers that the
  * products leave it in: an accumulator tile [key dimension][value column] is at once the operand of S^T q, because the key dimensions of q (and k)
- * lie in LDS in the order in which a lane's accumulators hold them.  Scores go through LDS.  bf16 sessions: q, k and v are bf16 (as in attention);
- * what is 32-bit by nature (the state, decayed scores, decayed values) enters a product as the sum of two bf16 numbers.
+ * lie in LDS in the order in which a lane's accumulators hold them.  Scores go through LDS.  bf16 sessions: v is bf16; what is 32-bit (rotated q and
+ * k, the state, decayed scores and values) enters a product as the sum of two bf16 numbers, without the product of the two small parts.
  * SUMS: only what the block adds to the state, into args.sums; k_retention_prefix turns these into the states that the segment's next blocks start
  * from, so that all blocks run side by side. */
 template <typename T> struct RetChunk { static constexpr int C = 32; };
@@ -1002,15 +1002,26 @@ template <typename T> __device__ __forceinline__ float silu_out(float z) { retur
 template <typename T, int DIM, int VB>
 struct RetLds { /* byte offsets */
     static constexpr int C = RetChunk<T>::C, SZ = sizeof(T), RP = DIM * SZ + 16, TP = C * SZ + 16;
-    static constexpr int q = 0, k = q + C * RP, kt = k + C * RP, vt = kt + DIM * TP, p = vt + VB * TP, lo = p + C * TP, pw = lo + (SZ == 2 ? C * TP : 0),
+    /* the small parts (bf16) lie behind the large ones */
+    static constexpr int PARTS = SZ == 2 ? 2 : 1, q_lo = C * RP, k_lo = C * RP, kt_lo = DIM * TP, p_lo = C * TP;
+    static constexpr int q = 0, k = q + PARTS * q_lo, kt = k + PARTS * k_lo, vt = kt + PARTS * kt_lo, p = vt + VB * TP, pw = p + PARTS * p_lo,
                          red = pw + (TK_RETENTION_BLOCK + 4) * 4, bytes = red + 8 * C * 4; /* eight waves at most */
 };
 
-/* two tokens' elements side by side; four */
+/* four tokens' elements side by side, and their small parts */
 __device__ __forceinline__ void ret_put4(TkBf16* p, const float (&x)[4]) {
     *(tk_v2u*)p = tk_v2u{(uint32_t)tk_bf16_bits(x[0]) | (uint32_t)tk_bf16_bits(x[1]) << 16, (uint32_t)tk_bf16_bits(x[2]) | (uint32_t)tk_bf16_bits(x[3]) << 16};
 }
 __device__ __forceinline__ void ret_put4(float* p, const float (&x)[4]) { *(tk_v4f*)p = tk_v4f{x[0], x[1], x[2], x[3]}; }
+__device__ __forceinline__ float ret_rest(float x) { return x - tk_bf16_float(tk_bf16_bits(x)); }
+__device__ __forceinline__ void ret_put4_split(uint8_t* p, int lo, TkBf16, const float (&x)[4]) {
+    const float y[4] = {ret_rest(x[0]), ret_rest(x[1]), ret_rest(x[2]), ret_rest(x[3])};
+    ret_put4((TkBf16*)p, x);
+    ret_put4((TkBf16*)(p + lo), y);
+}
+__device__ __forceinline__ void ret_put4_split(uint8_t* p, int, float, const float (&x)[4]) { ret_put4((float*)p, x); }
+__device__ __forceinline__ void ret_put_split(uint8_t* p, int lo, TkBf16, float x) { *(uint16_t*)p = tk_bf16_bits(x); *(uint16_t*)(p + lo) = tk_bf16_bits(ret_rest(x)); }
+__device__ __forceinline__ void ret_put_split(uint8_t* p, int, float, float x) { *(float*)p = x; }
 
 template <typename T, int DIM, int WAVES, int NT, bool SUMS>
 __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) void k_retention_scan(TkRetentionArgs a, const float* proj, int ld, TkPassTab t, const TkRetentionBlock* blocks) {
@@ -1103,17 +1114,17 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                 ka[r] = ok ? (k0[i][r] * c - k1[i][r] * z) * kscale : 0.0f;
                 kb[r] = ok ? (k1[i][r] * c + k0[i][r] * z) * kscale : 0.0f;
                 if (!SUMS) {
-                    T *lq = (T*)(lds + L::q + (t0 + r) * L::RP), *lk = (T*)(lds + L::k + (t0 + r) * L::RP);
-                    lq[ret_place<T>(e0)] = TkImg<T>::from(q0[i][r] * c - q1[i][r] * z);
-                    lk[ret_place<T>(e0)] = TkImg<T>::from(ka[r]);
+                    uint8_t *at0 = lds + (t0 + r) * L::RP + ret_place<T>(e0) * SZ, *at1 = lds + (t0 + r) * L::RP + ret_place<T>(e1) * SZ;
+                    ret_put_split(at0 + L::q, L::q_lo, T(), q0[i][r] * c - q1[i][r] * z);
+                    ret_put_split(at0 + L::k, L::k_lo, T(), ka[r]);
                     if (two) {
-                        lq[ret_place<T>(e1)] = TkImg<T>::from(q1[i][r] * c + q0[i][r] * z);
-                        lk[ret_place<T>(e1)] = TkImg<T>::from(kb[r]);
+                        ret_put_split(at1 + L::q, L::q_lo, T(), q1[i][r] * c + q0[i][r] * z);
+                        ret_put_split(at1 + L::k, L::k_lo, T(), kb[r]);
                     }
                 }
             }
-            ret_put4((T*)(lds + L::kt + e0 * L::TP) + t0, ka);
-            if (two) ret_put4((T*)(lds + L::kt + e1 * L::TP) + t0, kb);
+            ret_put4_split(lds + L::kt + e0 * L::TP + t0 * SZ, L::kt_lo, T(), ka);
+            if (two) ret_put4_split(lds + L::kt + e1 * L::TP + t0 * SZ, L::kt_lo, T(), kb);
         }
 #pragma unroll
         for (int i = 0; i < VI; ++i) {
@@ -1157,7 +1168,14 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                 tk_v4f s = {0.0f, 0.0f, 0.0f, 0.0f};
                 const uint8_t *lk = lds + L::k + (16 * j + r16) * L::RP + g * 16, *lq = lds + L::q + (16 * m + r16) * L::RP + g * 16;
 #pragma unroll
-                for (int d = 0; d < DT; ++d) s = TkImg<T>::mma(*(const tk_v4u*)(lk + d * 64), *(const tk_v4u*)(lq + d * 64), s);
+                for (int d = 0; d < DT; ++d) {
+                    const tk_v4u kf = *(const tk_v4u*)(lk + d * 64), qf = *(const tk_v4u*)(lq + d * 64);
+                    s = TkImg<T>::mma(kf, qf, s);
+                    if constexpr (SZ == 2) {
+                        s = TkImg<T>::mma(*(const tk_v4u*)(lk + L::k_lo + d * 64), qf, s);
+                        s = TkImg<T>::mma(kf, *(const tk_v4u*)(lq + L::q_lo + d * 64), s);
+                    }
+                }
                 const int age = 16 * (m - j) + r16 - 4 * g;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) s[r] = age - r >= 0 ? s[r] * pw[age - r >= 0 ? age - r : 0] : 0.0f;
@@ -1165,7 +1183,7 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                 if constexpr (SZ == 2) {
                     const Split<TkBf16> w(s, s);
                     *(tk_v2u*)(lds + L::p + at) = tk_v2u{w.hi[0], w.hi[1]};
-                    *(tk_v2u*)(lds + L::lo + at) = tk_v2u{w.lo[0], w.lo[1]};
+                    *(tk_v2u*)(lds + L::p + L::p_lo + at) = tk_v2u{w.lo[0], w.lo[1]};
                 } else {
                     *(tk_v4f*)(lds + L::p + at) = s;
                 }
@@ -1189,6 +1207,7 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                             for (int m = 0; m < CT; ++m) {
                                 o[nt][m] = TkImg<T>::mma(w.hi, qf[m], o[nt][m]);
                                 o[nt][m] = TkImg<T>::mma(w.lo, qf[m], o[nt][m]);
+                                o[nt][m] = TkImg<T>::mma(w.hi, *(const tk_v4u*)(lds + L::q + L::q_lo + (16 * m + r16) * L::RP + d * 64 + g * 16), o[nt][m]);
                             }
                         } else {
 #pragma unroll
@@ -1218,7 +1237,7 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                 for (int m = 0; m < CT; ++m)
                     if (k * KT < 16 * m + 16) {
                         const int at = (16 * m + r16) * L::TP + k * 64 + g * 16;
-                        const tk_v4u hi = *(const tk_v4u*)(lds + L::p + at), lo = SZ == 2 ? *(const tk_v4u*)(lds + L::lo + at) : hi;
+                        const tk_v4u hi = *(const tk_v4u*)(lds + L::p + at), lo = SZ == 2 ? *(const tk_v4u*)(lds + L::p + L::p_lo + at) : hi;
 #pragma unroll
                         for (int nt = 0; nt < NT; ++nt) {
                             o[nt][m] = TkImg<T>::mma(vf[nt][k], hi, o[nt][m]);
@@ -1252,9 +1271,14 @@ __global__ __launch_bounds__(64 * WAVES, SUMS && DIM <= 128 && NT == 1 ? 4 : 2) 
                     }
 #pragma unroll
                     for (int d = 0; d < DS; ++d) {
-                        const tk_v4u kf = *(const tk_v4u*)(lds + L::kt + (16 * d + r16) * L::TP + k * 64 + g * 16);
+                        const uint8_t* kat = lds + L::kt + (16 * d + r16) * L::TP + k * 64 + g * 16;
+                        const tk_v4u kf = *(const tk_v4u*)kat, kl = *(const tk_v4u*)(kat + L::kt_lo);
 #pragma unroll
-                        for (int nt = 0; nt < NT; ++nt) { S[nt][d] = TkImg<T>::mma(kf, hi[nt], S[nt][d]); S[nt][d] = TkImg<T>::mma(kf, lo[nt], S[nt][d]); }
+                        for (int nt = 0; nt < NT; ++nt) {
+                            S[nt][d] = TkImg<T>::mma(kf, hi[nt], S[nt][d]);
+                            S[nt][d] = TkImg<T>::mma(kf, lo[nt], S[nt][d]);
+                            S[nt][d] = TkImg<T>::mma(kl, hi[nt], S[nt][d]);
+                        }
                     }
                 } else {
                     tk_v4f x[NT];
